@@ -119,10 +119,10 @@ class LLMEngine:
         self.prefilling: list[SeqState] = []   # admitted, prompt not fully cached
         self.running: list[SeqState] = []
         self.chunk_size = chunk_size
-        # recurrent layers carry a state that is only known at the last
-        # token a sequence has run: a prefix cannot be skipped on the
-        # strength of its cached keys, and rejected proposals cannot be
-        # taken back
+        # recurrent layers and convolutions over time carry a state that is
+        # only known at the last token a sequence has run: a prefix cannot
+        # be skipped on the strength of its cached keys, and rejected
+        # proposals cannot be taken back
         self.states = kv_cache.states
         if self.states is not None and spec_lookup:
             raise ValueError("spec_lookup needs a model without recurrent "

@@ -51,6 +51,13 @@ class KVLayer:
 
 
 @dataclasses.dataclass(frozen=True)
+class LatentLayer:
+    """What one latent attention layer caches per token: one vector that
+    serves all heads as key and value."""
+    dim: int
+
+
+@dataclasses.dataclass(frozen=True)
 class StateLayer:
     """What one recurrent layer carries per sequence (f32)."""
     heads: int
@@ -58,22 +65,53 @@ class StateLayer:
     vdim: int
 
 
-class RecurrentStates:
-    """Per-sequence recurrent states: one slot per live sequence, and in
-    each slot a [heads, dim, vdim] f32 state per recurrent layer (rows
-    padded to 16 bytes).  A slot is not cleared when it changes hands: a
-    sequence's first row starts its recurrence from zero by position."""
+@dataclasses.dataclass(frozen=True)
+class TailLayer:
+    """What a short causal convolution carries per sequence: its last
+    ``rows`` inputs, a ring by position (activation dtype)."""
+    rows: int
+    width: int
 
-    def __init__(self, layers: list, n_slots: int, device) -> None:
+
+def layer_parts(spec) -> tuple:
+    """A layer may keep one thing or several."""
+    return spec if isinstance(spec, tuple) else (spec,)
+
+
+class RecurrentStates:
+    """What live sequences carry from token to token: one slot per live
+    sequence, and in each slot a [heads, dim, vdim] f32 state per recurrent
+    layer (rows padded to 16 bytes) and the tail of each convolution.  A
+    slot is not cleared when it changes hands: what a sequence's first rows
+    would read is zero by position."""
+
+    def __init__(self, layers: list, n_slots: int, device,
+                 dtype: torch.dtype = torch.bfloat16) -> None:
         self.n_slots = n_slots
-        self._layers = {
-            i: torch.zeros((n_slots, s.heads, s.dim, -(-s.vdim // 4) * 4),
-                           dtype=torch.float32, device=device)
-            for i, s in enumerate(layers) if isinstance(s, StateLayer)}
+        self._layers: dict[int, torch.Tensor] = {}
+        self._tails: dict[int, torch.Tensor] = {}
+        for i, spec in enumerate(layers):
+            for s in layer_parts(spec):
+                if isinstance(s, StateLayer):
+                    self._layers[i] = torch.zeros(
+                        (n_slots, s.heads, s.dim, -(-s.vdim // 4) * 4),
+                        dtype=torch.float32, device=device)
+                elif isinstance(s, TailLayer):
+                    self._tails[i] = torch.zeros(
+                        (n_slots, s.rows, s.width), dtype=dtype,
+                        device=device)
         self._free = list(range(n_slots - 1, -1, -1))
+
+    @staticmethod
+    def needed(layers: list) -> bool:
+        return any(isinstance(s, (StateLayer, TailLayer))
+                   for spec in layers for s in layer_parts(spec))
 
     def layer(self, i: int) -> torch.Tensor:
         return self._layers[i]
+
+    def tail(self, i: int) -> Optional[torch.Tensor]:
+        return self._tails.get(i)
 
     @property
     def free_slots(self) -> int:
@@ -87,15 +125,22 @@ class RecurrentStates:
     def free(self, slot: int) -> None:
         self._free.append(slot)
 
+    def cast(self, dtype: torch.dtype) -> None:
+        self._tails = {i: t.to(dtype) for i, t in self._tails.items()}
+
     def export(self, slot: int) -> dict:
-        return {i: t[slot].cpu() for i, t in self._layers.items()}
+        return {"states": {i: t[slot].cpu() for i, t in self._layers.items()},
+                "tails": {i: t[slot].cpu() for i, t in self._tails.items()}}
 
     def import_(self, slot: int, payload: dict) -> None:
         for i, t in self._layers.items():
-            t[slot].copy_(payload[i])
+            t[slot].copy_(payload["states"][i])
+        for i, t in self._tails.items():
+            t[slot].copy_(payload["tails"][i])
 
     def bytes_used(self) -> int:
-        return sum(t.numel() * 4 for t in self._layers.values())
+        return sum(t.numel() * t.element_size() for t in
+                   (*self._layers.values(), *self._tails.values()))
 
 
 class PagedKVCache:
@@ -227,9 +272,11 @@ class PagedKVCache:
 class LayeredKVCache(PagedKVCache):
     """Paged cache of a model whose layers differ: every attention layer
     has its own [num_blocks, kv heads, block, width] K and V (widths may
-    differ, layers may share), recurrent layers have none, and their
-    states live in ``states``.  Blocks are allocated as in the uniform
-    cache: one block id addresses a token range in every layer."""
+    differ, layers may share), a latent attention layer one
+    [num_blocks, 1, block, width] tensor, recurrent layers have none, and
+    what layers carry per sequence lives in ``states``.  Blocks are
+    allocated as in the uniform cache: one block id addresses a token range
+    in every layer."""
 
     def __init__(self, layers: list, num_blocks: int, block_size: int,
                  device="cpu", dtype: torch.dtype = torch.bfloat16,
@@ -238,23 +285,30 @@ class LayeredKVCache(PagedKVCache):
         self._init_blocks(num_blocks, block_size)
         self._kv: dict[int, tuple] = {}
         self._own: list[int] = []
-        for i, s in enumerate(layers):
-            if not isinstance(s, KVLayer):
-                continue
-            if s.share is not None:
-                self._kv[i] = self._kv[s.share]
-                continue
-            self._own.append(i)
-            self._kv[i] = tuple(
-                torch.zeros((num_blocks, s.n_kv_heads, block_size, d),
-                            dtype=dtype, device=device)
-                for d in (s.k_dim, s.v_dim))
-        self._share = {i: s.share for i, s in enumerate(layers)
-                       if isinstance(s, KVLayer) and s.share is not None}
-        if any(isinstance(s, StateLayer) for s in layers):
-            self.states = RecurrentStates(layers, state_slots, device)
+        self._share: dict[int, int] = {}
 
-    def layer(self, i: int) -> tuple[torch.Tensor, torch.Tensor]:
+        def pages(heads, width):
+            return torch.zeros((num_blocks, heads, block_size, width),
+                               dtype=dtype, device=device)
+        for i, spec in enumerate(layers):
+            for s in layer_parts(spec):
+                if isinstance(s, KVLayer) and s.share is not None:
+                    self._kv[i] = self._kv[s.share]
+                    self._share[i] = s.share
+                elif isinstance(s, KVLayer):
+                    self._own.append(i)
+                    self._kv[i] = (pages(s.n_kv_heads, s.k_dim),
+                                   pages(s.n_kv_heads, s.v_dim))
+                elif isinstance(s, LatentLayer):
+                    self._own.append(i)
+                    self._kv[i] = (pages(1, s.dim),)
+        if RecurrentStates.needed(layers):
+            # tails hold activations, also where the cache is 8-bit
+            self.states = RecurrentStates(
+                layers, state_slots, device,
+                dtype if dtype.itemsize > 1 else torch.bfloat16)
+
+    def layer(self, i: int) -> tuple:
         return self._kv[i]
 
     def cast(self, dtype: torch.dtype) -> None:
@@ -262,14 +316,16 @@ class LayeredKVCache(PagedKVCache):
             self._kv[i] = tuple(t.to(dtype) for t in self._kv[i])
         for i, j in self._share.items():
             self._kv[i] = self._kv[j]
+        if self.states is not None:
+            self.states.cast(dtype)
 
     def export_blocks(self, blocks: list):
         return [tuple(t[torch.tensor(blocks, device=t.device)].to("cpu")
                       for t in self._kv[i]) for i in self._own]
 
     def import_blocks(self, blocks: list, payload) -> None:
-        for i, pair in zip(self._own, payload):
-            for dst, src in zip(self._kv[i], pair):
+        for i, own in zip(self._own, payload):
+            for dst, src in zip(self._kv[i], own):
                 idx = torch.tensor(blocks[:src.shape[0]], dtype=torch.long,
                                    device=dst.device)
                 dst.index_copy_(0, idx, src.to(dst.device, dst.dtype))

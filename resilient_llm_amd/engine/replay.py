@@ -65,7 +65,7 @@ def main(argv=None) -> int:
         from ..ops import build
         build.ensure(get_model_class(args.model).EXTENSIONS)
     pool = -(-args.max_tokens // POOL_UNIT) * POOL_UNIT
-    config.max_position = max(pool, POOL_UNIT)
+    config.fit_positions(max(pool, POOL_UNIT))
     model = build_model(config, weights=args.model, device=device,
                         dtype=dtype)
     block_size = 16

@@ -19,9 +19,6 @@ throughout.
 from __future__ import annotations
 
 import dataclasses
-import json
-import math
-import os
 from typing import Optional
 
 import torch
@@ -30,6 +27,7 @@ import torch.nn.functional as F
 from .. import ops
 from ..engine.kv_cache import KVLayer, StateLayer
 from .llama import _linear
+from .mixed import DenseSpec, LayerSpec, MixedConfig, MixedModel
 
 
 @dataclasses.dataclass(frozen=True)
@@ -55,11 +53,6 @@ class GlaSpec:
 
 
 @dataclasses.dataclass(frozen=True)
-class DenseSpec:
-    ff: int
-
-
-@dataclasses.dataclass(frozen=True)
 class MoeSpec:
     experts: int
     top: int
@@ -67,14 +60,8 @@ class MoeSpec:
     limit: float
 
 
-@dataclasses.dataclass(frozen=True)
-class LayerSpec:
-    mixer: object                    # AttentionSpec | GlaSpec
-    mlp: object                      # DenseSpec | MoeSpec | None
-
-
 @dataclasses.dataclass
-class NesizenConfig:
+class NesizenConfig(MixedConfig):
     name: str
     hidden_size: int
     vocab_size: int
@@ -84,10 +71,6 @@ class NesizenConfig:
     decay_rank: int = 16             # random init; a checkpoint's own wins
     max_position: int = 32768        # serving limit, not a model constant
     eos_ids: tuple = ()
-
-    @property
-    def n_layers(self) -> int:
-        return len(self.layers)
 
     def __post_init__(self) -> None:
         if self.hidden_size % 8 or self.hidden_size > 8192:
@@ -147,12 +130,6 @@ class NesizenConfig:
         return cls(name=name, hidden_size=d["width"], vocab_size=d["vocab"],
                    streams=d["streams"], rms_eps=float(d["norm"]["eps"]),
                    layers=tuple(layers), **kw)
-
-    @classmethod
-    def from_dir(cls, path: str, **kw):
-        with open(os.path.join(path, "config.json")) as f:
-            return cls.from_dict(json.load(f), name=os.path.basename(
-                os.path.normpath(path)), **kw)
 
     def cache_layers(self, tp_world: int = 1) -> list:
         """What each layer keeps per token or per sequence."""
@@ -219,58 +196,40 @@ NESIZEN_PRESETS = {
 }
 
 
-class NesizenForCausalLM:
+class NesizenForCausalLM(MixedModel):
     """Inference-only Nesizen.  TP shards heads (attention and recurrent),
     the dense and expert widths column-wise, output projections row-wise,
     with an all-reduce after each sublayer; streams are replicated."""
 
-    # the engine hands prompt rows and state slots to such a model
-    mixed_layers = True
-    EXTENSIONS = ("rlli_mix",)
+    EXTENSIONS = ("rlli_mix", "rlli_rec")
 
-    def __init__(self, config: NesizenConfig, device: str = "cpu",
-                 dtype: torch.dtype = torch.bfloat16,
-                 tp_rank: int = 0, tp_world: int = 1,
-                 tp_group=None, seed: int = 0,
-                 quant: Optional[str] = None,
-                 weights: Optional[str] = None) -> None:
-        if quant is not None:
-            raise ValueError("quant is not available for this model")
-        self.config = config
-        self.device = torch.device(device)
-        self.dtype = dtype
-        self.quant = None
-        self.tp_rank, self.tp_world, self.tp_group = tp_rank, tp_world, tp_group
-        for spec in config.layers:
+    def sharded_sizes(self) -> list:
+        sizes = []
+        for spec in self.config.layers:
             m, f = spec.mixer, spec.mlp
-            sizes = [m.heads]
+            sizes.append(m.heads)
             if isinstance(m, AttentionSpec):
                 sizes.append(m.kv_heads)
             if f is not None:
                 sizes.append(f.ff)
-            assert all(s % tp_world == 0 for s in sizes), \
-                f"TP={tp_world} must divide heads and feed-forward widths"
-        self.params: dict[str, torch.Tensor] = {}
+        return sizes
+
+    def _prepare(self) -> None:
         self._rot: dict[tuple, torch.Tensor] = {}
-        for spec in config.layers:
+        for spec in self.config.layers:
             m = spec.mixer
             if isinstance(m, AttentionSpec):
                 key = (m.rot_dims, m.rot_base)
                 if key not in self._rot:
                     self._rot[key] = ops.build_cos_sin(
-                        config.max_position, m.rot_dims, m.rot_base,
+                        self.config.max_position, m.rot_dims, m.rot_base,
                         device=self.device).contiguous()
-        if weights is not None:
-            self.load_safetensors(weights)
-        else:
-            self._init_weights(seed)
 
     # ------------------------------------------------------------ weights
-    def tensor_shapes(self, rank: Optional[int] = None) -> dict:
+    def tensor_shapes(self) -> dict:
         """Checkpoint names -> shapes (full, unsharded)."""
         c = self.config
-        d, s = c.hidden_size, c.streams
-        rank = c.decay_rank if rank is None else rank
+        d, s, rank = c.hidden_size, c.streams, c.decay_rank
         out = {"embed": (c.vocab_size, d), "embed.norm": (d,)}
         for i, spec in enumerate(c.layers):
             m, f, p = spec.mixer, spec.mlp, f"l{i}."
@@ -307,71 +266,30 @@ class NesizenForCausalLM:
         out["head"] = (c.vocab_size, d)
         return out
 
-    def _init_weights(self, seed: int) -> None:
-        """Every rank draws the full tensors from one seed and keeps its
-        shard, so TP=N computes the same function as TP=1."""
-        gen = torch.Generator(device=self.device)
-        shapes = self.tensor_shapes()
-        std_o = 0.02 / math.sqrt(2 * max(1, self.config.n_layers))
-        order = {n: k for k, n in enumerate(shapes)}
+    def initial(self, leaf: str, shape: tuple):
         s = self.config.streams
+        if leaf == "mix.norm":
+            return torch.ones(shape)
+        if "norm" in leaf or leaf == "mix.sink":
+            return torch.zeros(shape)
+        if leaf.startswith("hc"):
+            if leaf.endswith(".mix"):
+                return torch.eye(s)
+            return torch.full(shape, 1.0 / s if leaf.endswith(".in") else 1.0)
+        if leaf == "mix.a2.b":
+            return torch.full(shape, 2.0)
+        return None
 
-        def draw(name):
-            shape = shapes[name]
-            leaf = name.split(".", 1)[-1]
-            if leaf == "mix.norm":
-                return torch.ones(shape, device=self.device)
-            if "norm" in leaf or leaf == "mix.sink":
-                return torch.zeros(shape, device=self.device)
-            if leaf.startswith("hc"):
-                if leaf.endswith(".mix"):
-                    return torch.eye(s, device=self.device)
-                return torch.full(shape, 1.0 / s if leaf.endswith(".in")
-                                  else 1.0, device=self.device)
-            if leaf == "mix.a2.b":
-                return torch.full(shape, 2.0, device=self.device)
-            gen.manual_seed(seed * 1000003 + order[name] * 1009 + 1)
-            t = torch.empty(shape, dtype=self.dtype, device=self.device)
-            return t.normal_(0.0, std_o if leaf.endswith((".o", ".down"))
-                             else 0.02, generator=gen)
-        self._install(draw)
-
-    def load_safetensors(self, path: str) -> int:
-        """Load a checkpoint directory, TP-sharded; returns the number of
-        tensors consumed."""
-        from safetensors import safe_open
-        files = sorted(f for f in os.listdir(path)
-                       if f.endswith(".safetensors"))
-        if not files:
-            raise FileNotFoundError(f"no .safetensors files under {path}")
-        where, handles = {}, []
-        for f in files:
-            h = safe_open(os.path.join(path, f), framework="pt")
-            handles.append(h)
-            for k in h.keys():
-                where[k] = h
-        loaded: list[str] = []
-        # the decay rank is the one size a tensor's shape gives
-        rank = next((where[n].get_slice(n).get_shape()[0] for n in where
-                     if n.endswith(".mix.a1")), None)
-        shapes = self.tensor_shapes(rank)
-
-        def take(name):
-            if name not in where:
-                raise KeyError(f"{path}: tensor {name!r} is missing")
-            t = where[name].get_tensor(name)
-            want = shapes[name]
-            if name.endswith((".mix.a1", ".mix.a2")):
-                a1 = where[name.rsplit(".", 1)[0] + ".a1"].get_slice(
-                    name.rsplit(".", 1)[0] + ".a1").get_shape()[0]
-                want = (a1, want[1]) if name.endswith("a1") else (want[0], a1)
-            if tuple(t.shape) != tuple(want):
-                raise ValueError(f"{path}: {name} is {tuple(t.shape)}, "
-                                 f"the configuration says {tuple(want)}")
-            loaded.append(name)
-            return t
-        self._install(take)
-        return len(loaded)
+    def _checkpoint_shapes(self, shape_of, names) -> dict:
+        # the decay rank is the one size that a tensor's shape gives
+        shapes = self.tensor_shapes()
+        for n, (_, d) in [(n, s) for n, s in shapes.items()
+                          if n.endswith(".mix.a1") and n in names]:
+            rank = shape_of(n)[0]
+            shapes[n] = (rank, d)
+            a2 = n[:-1] + "2"
+            shapes[a2] = (shapes[a2][0], rank)
+        return shapes
 
     def _install(self, get) -> None:
         """Pack full checkpoint tensors into this rank's parameters:
@@ -380,24 +298,13 @@ class NesizenForCausalLM:
         interleaved in blocks of 16 (the grouped GEMM pairs them in its
         accumulators) with the expert width zero-padded to 64."""
         c, P = self.config, self.params
-        r, n = self.tp_rank, self.tp_world
+        n = self.tp_world
 
-        def mat(name, rows: bool = False, cols: bool = False):
-            t = get(name)
-            if rows:
-                k = t.shape[0] // n
-                t = t[r * k:(r + 1) * k]
-            if cols:
-                k = t.shape[1] // n
-                t = t[:, r * k:(r + 1) * k]
-            return t.to(self.device).to(self.dtype).contiguous()
+        def mat(name, **kw):
+            return self._mat(get(name), **kw)
 
-        def vec(name, rows: bool = False):
-            t = get(name)
-            if rows:
-                k = t.shape[0] // n
-                t = t[r * k:(r + 1) * k]
-            return t.to(self.device).float().contiguous()
+        def vec(name, **kw):
+            return self._vec(get(name), **kw)
 
         P["embed"] = mat("embed")
         P["embed.norm"] = 1 + vec("embed.norm")
@@ -441,9 +348,6 @@ class NesizenForCausalLM:
                 P[p + "w_up"], P[p + "w_down"] = up, down
         P["final.norm"] = 1 + vec("final.norm")
         P["head"] = mat("head")
-
-    def param_bytes(self) -> int:
-        return sum(t.numel() * t.element_size() for t in self.params.values())
 
     # ------------------------------------------------------------ compute
     def _reduce(self, y: torch.Tensor) -> torch.Tensor:

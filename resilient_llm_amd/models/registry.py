@@ -8,15 +8,20 @@ import os
 from typing import Optional
 
 from .llama import MODEL_PRESETS, LlamaConfig, LlamaForCausalLM
+from .mixed import MixedModel
 from .nesizen import NESIZEN_PRESETS, NesizenConfig, NesizenForCausalLM
+from .riruzen import RIRUZEN_PRESETS, RiruzenConfig, RiruzenForCausalLM
 
 # config.json 'architecture' -> (configuration, model)
-ARCHITECTURES = {"Nesizen": (NesizenConfig, NesizenForCausalLM)}
-_MODELS = {LlamaConfig: LlamaForCausalLM, NesizenConfig: NesizenForCausalLM}
+ARCHITECTURES = {"Nesizen": (NesizenConfig, NesizenForCausalLM),
+                 "Riruzen": (RiruzenConfig, RiruzenForCausalLM)}
+_MODELS = {LlamaConfig: LlamaForCausalLM, **dict(ARCHITECTURES.values())}
+# presets that are made when asked for
+_MADE_PRESETS = {**NESIZEN_PRESETS, **RIRUZEN_PRESETS}
 
 
 def model_names() -> list:
-    return sorted([*MODEL_PRESETS, *NESIZEN_PRESETS])
+    return sorted([*MODEL_PRESETS, *_MADE_PRESETS])
 
 
 def checkpoint_architecture(path: Optional[str]) -> Optional[str]:
@@ -39,8 +44,8 @@ def get_config(name: str, weights: Optional[str] = None):
             return ARCHITECTURES[arch][0].from_dir(path)
     if name in MODEL_PRESETS:
         return MODEL_PRESETS[name]
-    if name in NESIZEN_PRESETS:
-        return NESIZEN_PRESETS[name]()
+    if name in _MADE_PRESETS:
+        return _MADE_PRESETS[name]()
     raise KeyError(f"unknown model {name!r}; have {model_names()}")
 
 
@@ -51,7 +56,7 @@ def get_model_class(name: str, weights: Optional[str] = None):
 def build_model(config, weights: Optional[str] = None, **kw):
     """The model of ``config``; with ``weights``, loaded from there."""
     cls = _MODELS[type(config)]
-    if cls is NesizenForCausalLM:
+    if issubclass(cls, MixedModel):
         return cls(config, weights=weights, **kw)
     model = cls(config, **kw)
     if weights:

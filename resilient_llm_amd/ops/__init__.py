@@ -17,9 +17,8 @@ from . import ref  # noqa: F401
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 _SO_PATH = os.path.join(_HERE, "_rlli_hip.so")
-_MIX_SO_PATH = os.path.join(_HERE, "_rlli_mix.so")
 _loaded = False
-_mix_loaded = False
+_loaded_libs: set = set()
 
 
 class ExtensionMissing(RuntimeError):
@@ -51,17 +50,22 @@ def _gpu() -> None:
     load_extension(required=True)
 
 
-def load_mix_extension() -> None:
-    """Load the mixed-layer kernels (idempotent); raises if not built."""
-    global _mix_loaded
-    if _mix_loaded:
-        return
-    if not os.path.exists(_MIX_SO_PATH):
-        raise ExtensionMissing(
-            f"HIP extension not built: {_MIX_SO_PATH} missing. "
-            f"Run `python -m resilient_llm_amd.ops.build`.")
-    torch.ops.load_library(_MIX_SO_PATH)
-    _mix_loaded = True
+def load_libraries(libs) -> None:
+    """Load kernel libraries by name (idempotent); raises if one is not
+    built."""
+    for lib in libs:
+        if lib in _loaded_libs:
+            continue
+        if lib == "rlli_hip":
+            _gpu()
+            continue
+        path = os.path.join(_HERE, f"_{lib}.so")
+        if not os.path.exists(path):
+            raise ExtensionMissing(
+                f"HIP extension not built: {path} missing. "
+                f"Run `python -m resilient_llm_amd.ops.build`.")
+        torch.ops.load_library(path)
+        _loaded_libs.add(lib)
 
 
 # ------------------------------------------------------------------ ops
@@ -273,19 +277,26 @@ build_cos_sin = ref.build_cos_sin
 
 
 # ----------------------------------------------- mixed-layer model ops
-# Residual streams, windowed attention with kept tokens and a sink, gated
-# linear attention, mixture of experts.  f32 or bf16 activations; the
-# GPU side is torch.ops.rlli_mix, the CPU side ops/ref_mix.py.
-from . import ref_mix  # noqa: E402
+# f32 or bf16 activations.  The GPU side is torch.ops.rlli_mix (residual
+# streams, windowed attention with kept tokens and a sink, mixture of
+# experts), rlli_rec (gated linear recurrences) and rlli_lat (parallel
+# blocks, latent attention); the CPU side ref_mix.py and ref_lat.py.
+from . import ref_lat, ref_mix  # noqa: E402
 from .ref_mix import GLA_CHUNK  # noqa: E402,F401
+
+_CPU_FORMS = {"rlli_mix": ref_mix, "rlli_rec": ref_mix, "rlli_lat": ref_lat}
+
+
+def _ns(lib: str, t: torch.Tensor):
+    """The op namespace of ``lib`` for ``t``'s device."""
+    if t.is_cuda:
+        load_libraries((lib,))
+        return getattr(torch.ops, lib)
+    return _CPU_FORMS[lib]
 
 
 def _mix(t: torch.Tensor):
-    """The op namespace for ``t``'s device."""
-    if t.is_cuda:
-        load_mix_extension()
-        return torch.ops.rlli_mix
-    return ref_mix
+    return _ns("rlli_mix", t)
 
 
 def hyper_embed(ids, table, w_embed, x, in_w, gain, eps: float):
@@ -309,7 +320,7 @@ def relu2(x):
 def window_tile_rows(group: int, device) -> int:
     """Prompt-tile height that the tiled attention kernel wants."""
     if torch.device(device).type == "cuda":
-        load_mix_extension()
+        load_libraries(("rlli_mix",))
         return torch.ops.rlli_mix.window_tile_rows(group)
     return 32
 
@@ -337,17 +348,49 @@ def window_decode(qkv, k_cache, v_cache, positions, cos_sin, slots,
         scale, n_q, window, keep_first, has_kv)
 
 
+def _out(proj, state, vdim, out):
+    if out is not None:
+        return out
+    return torch.empty((proj.shape[0], state.shape[1] * vdim),
+                       dtype=proj.dtype, device=proj.device)
+
+
 def gla_decode(proj, a2, a2_bias, norm, state, slots, positions, vdim: int,
-               tau: float, eps: float):
-    return _mix(proj).gla_decode(proj, a2, a2_bias, norm, state, slots,
-                                 positions, vdim, tau, eps)
+               tau: float, eps: float, out=None):
+    """Gated linear attention, one new token per sequence.  ``out`` may be
+    a column range of a wider matrix."""
+    out = _out(proj, state, vdim, out)
+    _ns("rlli_rec", proj).gla_decode(proj, a2, a2_bias, norm, state, slots,
+                                     positions, vdim, tau, eps, out)
+    return out
 
 
 def gla_prefill(proj, a2, a2_bias, norm, state, prompt, vdim: int,
-                tau: float, eps: float):
-    return _mix(proj).gla_prefill(
+                tau: float, eps: float, out=None):
+    out = _out(proj, state, vdim, out)
+    _ns("rlli_rec", proj).gla_prefill(
         proj, a2, a2_bias, norm, state, prompt.tiles(GLA_CHUNK),
-        prompt.seqs(GLA_CHUNK), vdim, tau, eps)
+        prompt.seqs(GLA_CHUNK), vdim, tau, eps, out)
+    return out
+
+
+def hgrn2_decode(proj, bias, lower, norm, state, slots, positions, vdim: int,
+                 eps: float, out=None):
+    """HGRN2: the same recurrence with k = 1 - decay, silu queries and a
+    lower-bounded decay; ``proj`` is q | forget logit | v."""
+    out = _out(proj, state, vdim, out)
+    _ns("rlli_rec", proj).hgrn2_decode(proj, bias, lower, norm, state, slots,
+                                       positions, vdim, eps, out)
+    return out
+
+
+def hgrn2_prefill(proj, bias, lower, norm, state, prompt, vdim: int,
+                  eps: float, out=None):
+    out = _out(proj, state, vdim, out)
+    _ns("rlli_rec", proj).hgrn2_prefill(
+        proj, bias, lower, norm, state, prompt.tiles(GLA_CHUNK),
+        prompt.seqs(GLA_CHUNK), vdim, eps, out)
+    return out
 
 
 def moe_route(h, router, top: int):
@@ -357,3 +400,108 @@ def moe_route(h, router, top: int):
 def moe_experts(h, router, w_up, w_down, top: int, limit: float):
     """[T, top, W]: one row per chosen expert; the consumer sums them."""
     return _mix(h).moe_experts(h, router, w_up, w_down, top, limit)
+
+
+# ------------------------------------------- parallel blocks, latents
+CONV_SPAN = 16        # prompt rows that one convolution workgroup walks
+
+
+def block_embed(ids, table, pos_table, positions, x, gain, groups: int,
+                eps: float, taps=None, tail=None, slots=None,
+                n_decode: int = 0):
+    """Fill the f32 residual with embedding + position and return its
+    grouped norm h and, for the first ``n_decode`` rows (one token per
+    sequence), h + conv(h) from the sequences' tails."""
+    return _ns("rlli_lat", table).block_embed(
+        ids, table, pos_table, positions, x, gain, groups, eps, taps, tail,
+        slots, n_decode)
+
+
+def block_step(x, y, gain, groups: int, eps: float, positions, taps=None,
+               tail=None, slots=None, n_decode: int = 0, rows=None,
+               keep: bool = True):
+    """Add a block's output to the residual; then as block_embed.  ``rows``
+    restricts the result (then keep=False)."""
+    return _ns("rlli_lat", y).block_step(x, y, gain, groups, eps, positions,
+                                         taps, tail, slots, n_decode, rows,
+                                         keep)
+
+
+def conv_prompt(h, taps, tail, prompt, out):
+    """out = h + conv(h) for prompt rows, and their sequences' tails."""
+    _ns("rlli_lat", h).conv_prompt(h, taps, tail, prompt.spans(CONV_SPAN),
+                                   prompt.spans(1 << 30), out)
+
+
+def gate_act(gate_up, out, act: str):
+    """out = act(gate) * up of [rows, gate | up]."""
+    _ns("rlli_lat", gate_up).gate_act(gate_up, out, act)
+    return out
+
+
+def latent_prep(proj, q_norm, kv_norm, eps: float, cache, slots):
+    """Norm both latents of ``proj`` (query | key/value | ...), cache the
+    second, return the first."""
+    return _ns("rlli_lat", proj).latent_prep(proj, q_norm, kv_norm, eps,
+                                             cache, slots)
+
+
+def head_linear(x, w, gate=None, out=None):
+    """out[t, h] = w[h] x[t, h] (times sigmoid(gate)); w [heads, n, k]."""
+    if out is None:
+        out = torch.empty((x.shape[0], w.shape[0] * w.shape[1]),
+                          dtype=x.dtype, device=x.device)
+    _ns("rlli_lat", w).head_linear(x, w, gate, out)
+    return out
+
+
+def latent_decode(q, gate, cache, positions, block_tables, scale: float,
+                  w_uk, w_uv, out):
+    """One new token per sequence: absorbed queries over the cached
+    latents.  w_uk [heads, rank, dim], w_uv [heads, vdim, rank]."""
+    heads = w_uk.shape[0]
+    ns = _ns("rlli_lat", q)
+    c = ns.latent_attn(head_linear(q, w_uk), cache, block_tables, scale,
+                       heads, positions, None, None)
+    return head_linear(c, w_uv, gate, out)
+
+
+def expands(prompt, rank: int, dim: int, vdim: int) -> bool:
+    """Whether a step's prompt rows are cheaper with expanded keys and
+    values: rebuilding them costs a fixed amount per cached token, a score
+    and value row of latent width costs more per (row, token)."""
+    absorbed = expanded = 0
+    for p in prompt.portions:
+        ctx = p.pos0 + p.n
+        absorbed += p.n * ctx * 2 * rank
+        expanded += ctx * (dim + vdim) * (rank + p.n)
+    # the absorbed kernel reaches about half the expanded one's rate
+    return 2 * absorbed > expanded
+
+
+def latent_prefill(q, gate, cache, block_tables, prompt, scale: float, w_uk,
+                   w_uv, w_k, w_v, out, expand=None):
+    """Prompt rows over the cached latents, their own included: with keys
+    and values expanded from the latents (w_k [heads * dim, rank], w_v
+    [heads * vdim, rank]) or with absorbed queries, whichever is cheaper
+    (``expand`` forces one)."""
+    heads, rank, dim = w_uk.shape
+    vdim = w_uv.shape[1]
+    ns = _ns("rlli_lat", q)
+    fast = q.is_cuda and ns.latent_fast(cache, q.dtype == torch.float32)
+    ok = fast and ns.expanded_ok(dim, vdim) and all(
+        t.stride(0) % 4 == 0 and t.data_ptr() % 8 == 0 for t in (gate, out))
+    if expand is None:
+        expand = ok and expands(prompt, rank, dim, vdim)
+    if expand and ok:
+        blocks, kv_off, tokens = prompt.gathered(64)
+        c = ns.latent_gather(cache, block_tables, blocks, tokens)
+        k = torch.nn.functional.linear(c, w_k)
+        vt = torch.nn.functional.linear(w_v, c)      # already transposed
+        ns.expanded_attn(q, k, vt, gate, prompt.tiles(128), kv_off, heads,
+                         scale, out)
+        return out
+    tiles = prompt.vectors(64, heads) if fast else prompt.tiles(32)
+    c = ns.latent_attn(head_linear(q, w_uk), cache, block_tables, scale,
+                       heads, None, tiles, prompt.pos0())
+    return head_linear(c, w_uv, gate, out)

@@ -29,10 +29,10 @@ SAN_FLAGS = {"asan": ["-Xarch_host", "-fsanitize=address"],
              "tsan": ["-Xarch_host", "-fsanitize=thread"], "": []}[_SAN]
 BUILD = os.path.join(HERE, "build" + (f"-{_SAN}" if _SAN else ""))
 
-# Two libraries, so a process compiles and loads what its model needs:
-# rlli_hip has the Llama-family kernels and the sampler, rlli_mix the
-# mixed-layer kernels (residual streams, windowed attention, gated linear
-# attention, mixture of experts).
+# Libraries, so that a process compiles and loads what its model needs:
+# rlli_hip has the Llama-family kernels and the sampler, rlli_mix residual
+# streams, windowed attention and mixture of experts, rlli_rec the gated
+# linear recurrences, rlli_lat parallel blocks and latent attention.
 LIBRARIES = {
     "rlli_hip": [
         "ext.cpp",
@@ -54,12 +54,24 @@ LIBRARIES = {
         "hyper.hip",
         "window_attn.hip",
         "window_prefill.hip",
-        "gla.hip",
         "moe.hip",
     ],
+    "rlli_rec": [
+        "ext_rec.cpp",
+        "gla.hip",
+    ],
+    "rlli_lat": [
+        "ext_lat.cpp",
+        "block.hip",
+        "latent.hip",
+        "latent_prefill.hip",
+    ],
 }
+_MIX_HEADERS = ["common.h", "mix.h", "attn_rows.h", "ext_common.h"]
 HEADERS = {"rlli_hip": ["common.h", "kernels.h"],
-           "rlli_mix": ["common.h", "mix.h"]}
+           "rlli_mix": _MIX_HEADERS,
+           "rlli_rec": _MIX_HEADERS,
+           "rlli_lat": _MIX_HEADERS + ["lat.h"]}
 # some packed f32 instruction forms have returned wrong results on this
 # hardware; keep the compiler from forming them
 CODEGEN = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
@@ -128,7 +140,7 @@ def _link(lib: str, objs: list[str], libs: list[str], force: bool,
 
 
 def build(force: bool = False, verbose: bool = True,
-          libs: tuple = ("rlli_hip", "rlli_mix")) -> str:
+          libs: tuple = tuple(LIBRARIES)) -> str:
     """Compile ``libs`` (incrementally unless ``force``); returns the path
     of the first one."""
     os.makedirs(BUILD, exist_ok=True)

@@ -2,63 +2,12 @@
 // Every shape, dtype and index-table assumption of a kernel is checked
 // here before it is launched.
 
-#include <torch/library.h>
-#include <ATen/ATen.h>
-#include <ATen/hip/impl/HIPStreamMasqueradingAsCUDA.h>
-#include <ATen/hip/impl/HIPGuardImplMasqueradingAsCUDA.h>
-#include <c10/hip/HIPGraphsC10Utils.h>
-
+#include "ext_common.h"
 #include "mix.h"
-
-#include <optional>
 
 namespace {
 
-using at::Tensor;
-using OptTensor = std::optional<Tensor>;
-
-hipStream_t stream_of(const Tensor& t) {
-  return at::hip::getCurrentHIPStreamMasqueradingAsCUDA(
-      t.device().index()).stream();
-}
-
-void check_launch(const char* op) {
-  if (c10::hip::currentStreamCaptureStatusMayInitCtx() !=
-      c10::hip::CaptureStatus::None)
-    return;
-  hipError_t e = hipGetLastError();
-  TORCH_CHECK(e == hipSuccess, op, " launch failed: ", hipGetErrorString(e));
-}
-
-bool act_f32(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.is_contiguous(), name,
-              " must be contiguous and on the GPU");
-  const bool f32 = t.scalar_type() == at::kFloat;
-  TORCH_CHECK(f32 || t.scalar_type() == at::kBFloat16, name,
-              " must be bf16 or f32");
-  return f32;
-}
-
-void same_act(const Tensor& t, const Tensor& like, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.is_contiguous() &&
-              t.scalar_type() == like.scalar_type(), name,
-              " must be contiguous, on the GPU and of the activation dtype");
-}
-
-const float* f32_vec(const Tensor& t, int64_t n, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.is_contiguous() &&
-              t.scalar_type() == at::kFloat && t.numel() == n, name,
-              " must be ", n, " contiguous f32 values on the GPU, got ",
-              t.numel());
-  return t.data_ptr<float>();
-}
-
-const int32_t* i32(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.is_contiguous() &&
-              t.scalar_type() == at::kInt, name,
-              " must be contiguous int32 on the GPU");
-  return t.data_ptr<int32_t>();
-}
+using namespace rlli_ext;
 
 // ---------------------------------------------------------------- hyper
 void check_streams(const Tensor& x) {
@@ -287,90 +236,6 @@ Tensor window_decode(const Tensor& qkv, const Tensor& k_cache,
   return out;
 }
 
-// ------------------------------------------------------------------ gla
-rlli::GlaArgs gla_args(const Tensor& proj, const Tensor& a2,
-                       const Tensor& a2_bias, const Tensor& norm,
-                       const Tensor& state, int64_t vdim, double tau,
-                       double eps) {
-  rlli::GlaArgs a{};
-  a.f32 = act_f32(proj, "proj");
-  same_act(a2, proj, "a2");
-  TORCH_CHECK(state.is_cuda() && state.is_contiguous() && state.dim() == 4 &&
-              state.scalar_type() == at::kFloat,
-              "state must be f32 [slots, heads, dim, vdim padded to 4]");
-  a.rows = int(proj.size(0));
-  a.stride = int(proj.size(1));
-  a.n_slots = int(state.size(0));
-  a.heads = int(state.size(1));
-  a.dim = int(state.size(2));
-  a.vpad = int(state.size(3));
-  a.vdim = int(vdim);
-  TORCH_CHECK(a.vpad % 4 == 0 && a.vpad >= a.vdim && a.vpad < a.vdim + 4);
-  TORCH_CHECK(a.dim <= 256 && a.vdim <= 1024, "gla head sizes out of range");
-  a.dpad = (a.dim + 15) / 16 * 16;
-  TORCH_CHECK(a2.dim() == 2 && a2.size(0) == a.heads * a.dim);
-  a.rank = int(a2.size(1));
-  TORCH_CHECK(a.rank <= 1024, "decay rank out of range");
-  TORCH_CHECK(a.stride == 2 * a.heads * (a.dim + a.vdim) + a.rank,
-              "gla projection width mismatch");
-  a.proj = proj.data_ptr();
-  a.a2 = a2.data_ptr();
-  a.a2_bias = f32_vec(a2_bias, int64_t(a.heads) * a.dim, "a2_bias");
-  a.norm = f32_vec(norm, a.vdim, "norm");
-  a.state = state.data_ptr<float>();
-  a.tau = float(tau);
-  a.eps = float(eps);
-  return a;
-}
-
-Tensor gla_decode(const Tensor& proj, const Tensor& a2, const Tensor& a2_bias,
-                  const Tensor& norm, Tensor state, const Tensor& slots,
-                  const Tensor& positions, int64_t vdim, double tau,
-                  double eps) {
-  auto a = gla_args(proj, a2, a2_bias, norm, state, vdim, tau, eps);
-  a.slots = i32(slots, "slots");
-  a.positions = i32(positions, "positions");
-  TORCH_CHECK(slots.numel() == a.rows && positions.numel() == a.rows);
-  Tensor out = at::empty({a.rows, int64_t(a.heads) * a.vdim}, proj.options());
-  a.out = out.data_ptr();
-  c10::hip::HIPGuardMasqueradingAsCUDA guard(proj.device());
-  rlli::launch_gla_decode(a, stream_of(proj));
-  check_launch("gla_decode");
-  return out;
-}
-
-Tensor gla_prefill(const Tensor& proj, const Tensor& a2,
-                   const Tensor& a2_bias, const Tensor& norm, Tensor state,
-                   const Tensor& tiles, const Tensor& seqs, int64_t vdim,
-                   double tau, double eps) {
-  auto a = gla_args(proj, a2, a2_bias, norm, state, vdim, tau, eps);
-  a.tiles = i32(tiles, "tiles");
-  a.seqs = i32(seqs, "seqs");
-  TORCH_CHECK(tiles.dim() == 2 && tiles.size(0) == 4 && seqs.dim() == 2 &&
-              seqs.size(0) == 4);
-  a.n_tiles = int(tiles.size(1));
-  a.n_seqs = int(seqs.size(1));
-  const int64_t C = rlli::kGlaChunk;
-  const int64_t nh = int64_t(a.n_tiles) * a.heads;
-  auto fo = proj.options().dtype(at::kFloat);
-  Tensor qd = at::empty({nh, C, a.dpad}, fo);
-  Tensor kd = at::empty({nh, a.dpad, C}, fo);
-  Tensor sc = at::empty({nh, C, C}, fo);
-  Tensor dec = at::empty({nh, a.dpad}, fo);
-  Tensor o = at::empty({a.rows, int64_t(a.heads) * a.vdim}, fo);
-  Tensor out = at::empty({a.rows, int64_t(a.heads) * a.vdim}, proj.options());
-  a.qd = qd.data_ptr<float>();
-  a.kd = kd.data_ptr<float>();
-  a.sc = sc.data_ptr<float>();
-  a.dec = dec.data_ptr<float>();
-  a.o = o.data_ptr<float>();
-  a.out = out.data_ptr();
-  c10::hip::HIPGuardMasqueradingAsCUDA guard(proj.device());
-  rlli::launch_gla_prefill(a, stream_of(proj));
-  check_launch("gla_prefill");
-  return out;
-}
-
 // ------------------------------------------------------------------ moe
 void moe_sizes(rlli::MoeArgs& a, const Tensor& h, const Tensor& router,
                int64_t top) {
@@ -474,12 +339,6 @@ TORCH_LIBRARY(rlli_mix, m) {
         "Tensor(c!) v_cache, Tensor positions, Tensor cos_sin, Tensor slots, "
         "Tensor block_tables, Tensor? sink, float scale, int n_q, "
         "int window, int keep_first, bool has_kv) -> Tensor");
-  m.def("gla_decode(Tensor proj, Tensor a2, Tensor a2_bias, Tensor norm, "
-        "Tensor(a!) state, Tensor slots, Tensor positions, int vdim, "
-        "float tau, float eps) -> Tensor");
-  m.def("gla_prefill(Tensor proj, Tensor a2, Tensor a2_bias, Tensor norm, "
-        "Tensor(a!) state, Tensor tiles, Tensor seqs, int vdim, float tau, "
-        "float eps) -> Tensor");
   m.def("moe_route(Tensor h, Tensor router, int top) -> (Tensor, Tensor)");
   m.def("moe_experts(Tensor h, Tensor router, Tensor w_up, Tensor w_down, "
         "int top, float limit) -> Tensor");
@@ -491,8 +350,6 @@ TORCH_LIBRARY_IMPL(rlli_mix, CUDA, m) {
   m.impl("relu2", &relu2);
   m.impl("window_prefill", &window_prefill);
   m.impl("window_decode", &window_decode);
-  m.impl("gla_decode", &gla_decode);
-  m.impl("gla_prefill", &gla_prefill);
   m.impl("moe_route", &moe_route);
   m.impl("moe_experts", &moe_experts);
 }

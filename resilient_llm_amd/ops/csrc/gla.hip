@@ -1,21 +1,27 @@
-// Gated linear attention: S_t = diag(alpha_t) S_{t-1} + k_t v_t^T,
-// o_t = S_t^T q_t per head, alpha = sigmoid(z)^(1/tau) per key channel,
-// z = A2 (A1 h) + b; then RMS norm over the value width, silu gate.
+// Gated linear recurrences: S_t = diag(alpha_t) S_{t-1} + k_t v_t^T,
+// o_t = S_t^T q_t per head, alpha a decay per key channel, then RMS norm
+// over the value width.  Two ways to make q, k and alpha from the
+// projections:
+//   GLA     q | k | v | gate | A1 h:  alpha = sigmoid(z)^(1/tau) with
+//           z = A2 (A1 h) + b, q scaled by dim^-1/2, silu output gate
+//   HGRN2   q | z | v:  alpha = l + (1 - l) sigmoid(z + b) with a lower
+//           bound l per channel, k = 1 - alpha, q = silu(q), no gate
 //
-// The projections q | k | v | gate | A1 h arrive as one GEMM output row;
-// everything from z on is 32-bit, matrix products included (the f32 MFMA
-// forms), and so are the states.
+// The projections arrive as one GEMM output row; everything from z on is
+// 32-bit, matrix products included (the f32 MFMA forms), and so are the
+// states.
 //
 // Decode is one fused kernel per layer: decay, state update, readout,
 // norm and gate; a state is read and written exactly once.
 //
 // Prompts run in chunks of 64 tokens whose four 16-token sub-chunks bound
-// every exponent: with L the running log-decay inside a sub-chunk and B_I
-// its value at the start of sub-chunk I,
-//     A[t,s] = sum_d q_t e^{L_t} * k_s e^{B_I - B_J - L_s}   (J < I)
-// has both factors' exponents <= 0 for any decay.  Inside a sub-chunk
-// e^{L_t} * e^{-L_s} is used while the whole sub-chunk decays by less
-// than e^40; beyond that the pairwise e^{L_t - L_s} is summed directly.
+// every exponent: with L the running log-decay inside a sub-chunk, tot its
+// last row and B_I the running log-decay at the start of sub-chunk I,
+//     A[t,s] = sum_d (q_t e^{L_t} e^{B_I - B_{J+1}}) * (k_s e^{tot_J - L_s})
+// for J < I has only exponents <= 0, whatever the decay.  Inside a
+// sub-chunk the factors are e^{L_t - m} and e^{m - L_s} with m the middle
+// row's log-decay, as long as either half decays by less than e^40; beyond
+// that the pairwise e^{L_t - L_s} is summed directly.
 //   gla_intra   per (chunk, head): A, q e^{b_t}, k e^{b_C - b_s}, e^{b_C}
 //   gla_scan    per (sequence, head, value slice): chunk after chunk,
 //               O = (q e^{b}) S + A V, S = e^{b_C} S + (k e^{b_C-b})^T V,
@@ -44,6 +50,26 @@ DEV_INLINE float log_sigmoid(float x) {
   return fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
 }
 
+DEV_INLINE float silu(float x) { return x / (1.f + expf(-x)); }
+
+// HGRN2: alpha = low + (1 - low) sigmoid(z), k = 1 - alpha without the
+// cancellation
+DEV_INLINE float forget_key(float z, float low, float* alpha) {
+  const float e = expf(-fabsf(z));
+  const float r = 1.f / (1.f + e), er = e * r;
+  *alpha = low + (1.f - low) * (z >= 0.f ? r : er);
+  return (1.f - low) * (z >= 0.f ? er : r);
+}
+
+// its logarithm; e^-80 and less is nothing beside a key of order one
+template <typename T>
+DEV_INLINE float log_forget(float z, float low) {
+  float alpha;
+  const float k = forget_key(z, low, &alpha);
+  if constexpr (sizeof(T) == 2) return fmaxf(__logf(alpha), -80.f);
+  return alpha > 0.5f ? log1pf(-k) : fmaxf(logf(alpha), -80.f);
+}
+
 DEV_INLINE f32x4_t mma4(float a, float b, f32x4_t c) {
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 }
@@ -61,7 +87,7 @@ DEV_INLINE f32x4_t load4_guard(const T* p, int d, int dim, bool row_ok,
 }
 
 // ------------------------------------------------------------- decode
-template <typename T>
+template <typename T, bool FG>
 __global__ __launch_bounds__(256)
 void gla_decode_kernel(GlaArgs a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
@@ -73,13 +99,21 @@ void gla_decode_kernel(GlaArgs a) {
   float* a1 = qs + a.dpad;              // [rank, padded to 4]
   float* red = a1 + (a.rank + 3) / 4 * 4;   // [rows][vpad] then sums
   const T* row = reinterpret_cast<const T*>(a.proj) + int64_t(seq) * a.stride;
-  const int hd = a.heads * a.dim, hv = a.heads * a.vdim;
-  for (int r = tid; r < a.rank; r += 256)
-    a1[r] = act_load(row + 2 * hd + 2 * hv + r);
-  const float qscale = 1.f / sqrtf(float(a.dim));
-  for (int d = tid; d < a.dim; d += 256) {
-    qs[d] = act_load(row + h * a.dim + d) * qscale;
-    ks[d] = act_load(row + hd + h * a.dim + d);
+  const int hv = a.heads * a.vdim;
+  if constexpr (FG) {
+    for (int d = tid; d < a.dim; d += 256) {
+      const int hc = h * a.dim + d;
+      qs[d] = silu(act_load(row + hc));
+      ks[d] = forget_key(act_load(row + a.off_k + hc) + a.a2_bias[hc],
+                         a.lower[hc], al + d);
+    }
+  } else {
+    for (int r = tid; r < a.rank; r += 256) a1[r] = act_load(row + a.off_a + r);
+    const float qscale = 1.f / sqrtf(float(a.dim));
+    for (int d = tid; d < a.dim; d += 256) {
+      qs[d] = act_load(row + h * a.dim + d) * qscale;
+      ks[d] = act_load(row + a.off_k + h * a.dim + d);
+    }
   }
   const int v4n = a.vpad / 4;
   const int n_rows = 256 / v4n;
@@ -87,20 +121,22 @@ void gla_decode_kernel(GlaArgs a) {
   const bool live = vr < n_rows;
   f32x4_t v = f32x4_t{0.f, 0.f, 0.f, 0.f};
   if (live) {
-    const T* vp = row + 2 * hd + h * a.vdim;
+    const T* vp = row + a.off_v + h * a.vdim;
 #pragma unroll
     for (int j = 0; j < 4; ++j)
       if (vc * 4 + j < a.vdim) v[j] = act_load(vp + vc * 4 + j);
   }
   __syncthreads();
-  for (int d = tid; d < a.dim; d += 256) {
-    const T* w = reinterpret_cast<const T*>(a.a2) +
-                 int64_t(h * a.dim + d) * a.rank;
-    float z = a.a2_bias[h * a.dim + d];
-    for (int r = 0; r < a.rank; ++r) z += act_load(w + r) * a1[r];
-    al[d] = expf(log_sigmoid<T>(z) / a.tau);
+  if constexpr (!FG) {
+    for (int d = tid; d < a.dim; d += 256) {
+      const T* w = reinterpret_cast<const T*>(a.a2) +
+                   int64_t(h * a.dim + d) * a.rank;
+      float z = a.a2_bias[h * a.dim + d];
+      for (int r = 0; r < a.rank; ++r) z += act_load(w + r) * a1[r];
+      al[d] = expf(log_sigmoid<T>(z) / a.tau);
+    }
+    __syncthreads();
   }
-  __syncthreads();
 
   const bool fresh = a.positions[seq] == 0;
   float* S = a.state +
@@ -145,29 +181,31 @@ void gla_decode_kernel(GlaArgs a) {
   __syncthreads();
   const float inv =
       1.f / sqrtf((ws[0] + ws[1] + ws[2] + ws[3]) / a.vdim + a.eps);
-  const T* gate = row + 2 * hd + hv + h * a.vdim;
-  T* out = reinterpret_cast<T*>(a.out) + int64_t(seq) * hv + h * a.vdim;
+  T* out = reinterpret_cast<T*>(a.out) + int64_t(seq) * a.out_stride +
+           h * a.vdim;
   for (int e = tid; e < a.vdim; e += 256) {
-    const float g = act_load(gate + e);
-    act_store(out + e, red[e] * inv * a.norm[e] * (g / (1.f + expf(-g))));
+    float o2 = red[e] * inv * a.norm[e];
+    if constexpr (!FG) o2 *= silu(act_load(row + a.off_g + h * a.vdim + e));
+    act_store(out + e, o2);
   }
 }
 
 // -------------------------------------------------------------- intra
-template <typename T>
+// Wave w owns sub-chunk w; MD bounds the key tiles (dpad <= 64 * MD).
+template <typename T, bool FG, int MD>
 __global__ __launch_bounds__(256)
 void gla_intra_kernel(GlaArgs a, bool vec) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
+  constexpr int NT = 4 * MD;
   const int tile = blockIdx.x, h = blockIdx.y;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int lr = lane & 15, g = lane >> 4;
-  const int DP = a.dpad, LR = DP + 4;
-  float* L = sm;                         // [64][LR]
+  const int DP = a.dpad, LR = DP + 4, ndt = DP / 16;
+  float* L = sm;                         // [64][LR], then decayed keys
   float* tot = L + C * LR;               // [4][DP]
   float* B = tot + 4 * DP;               // [5][DP]
   const int row0 = a.tiles[tile];
   const int n = a.tiles[2 * a.n_tiles + tile];
-  const int hd = a.heads * a.dim, hv = a.heads * a.vdim;
   const T* base = reinterpret_cast<const T*>(a.proj) +
                   int64_t(row0) * a.stride;
   const int trow = w * 16 + lr;          // this lane's operand row
@@ -175,41 +213,57 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
 
   // log-decay of sub-chunk w, then its running sum down the rows
   float wmin = 0.f;
-  for (int dt = 0; dt < DP / 16; ++dt) {
+  for (int dt = 0; dt < ndt; ++dt) {
     const int d = dt * 16 + lr;
     f32x4_t z = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    const T* a1 = base + int64_t(trow) * a.stride + 2 * hd + 2 * hv;
-    const T* a2 = reinterpret_cast<const T*>(a.a2) +
-                  int64_t(h * a.dim + d) * a.rank;
-    for (int k0 = 0; k0 < a.rank; k0 += 16) {
-      const f32x4_t av = load4_guard(a1, k0 + g * 4, a.rank, row_ok, false);
-      const f32x4_t bv = load4_guard(a2, k0 + g * 4, a.rank, d < a.dim,
-                                     false);
+    if constexpr (FG) {
 #pragma unroll
-      for (int j = 0; j < 4; ++j) z = mma4(av[j], bv[j], z);
+      for (int r = 0; r < 4; ++r) {
+        const int t = w * 16 + g * 4 + r;
+        if (d < a.dim && t < n)
+          z[r] = act_load(base + int64_t(t) * a.stride + a.off_k +
+                          h * a.dim + d);
+      }
+    } else {
+      const T* a1 = base + int64_t(trow) * a.stride + a.off_a;
+      const T* a2 = reinterpret_cast<const T*>(a.a2) +
+                    int64_t(h * a.dim + d) * a.rank;
+      for (int k0 = 0; k0 < a.rank; k0 += 16) {
+        const f32x4_t av = load4_guard(a1, k0 + g * 4, a.rank, row_ok, false);
+        const f32x4_t bv = load4_guard(a2, k0 + g * 4, a.rank, d < a.dim,
+                                       false);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) z = mma4(av[j], bv[j], z);
+      }
     }
     const float bias = d < a.dim ? a.a2_bias[h * a.dim + d] : 0.f;
+    float low = 0.f;
+    if constexpr (FG) low = d < a.dim ? a.lower[h * a.dim + d] : 0.f;
     float c[4], run = 0.f;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const bool ok = d < a.dim && w * 16 + g * 4 + r < n;
-      run += ok ? log_sigmoid<T>(z[r] + bias) / a.tau : 0.f;
+      float ld;
+      if constexpr (FG) ld = log_forget<T>(z[r] + bias, low);
+      else ld = log_sigmoid<T>(z[r] + bias) / a.tau;
+      run += ok ? ld : 0.f;
       c[r] = run;
     }
     // prefix over the four 4-row lane groups
-    float pre = 0.f, t = run;
-    const float u1 = __shfl_up(t, 16, kWave);
-    const float u2 = __shfl_up(t, 32, kWave);
-    const float u3 = __shfl_up(t, 48, kWave);
+    float pre = 0.f;
+    const float u1 = __shfl_up(run, 16, kWave);
+    const float u2 = __shfl_up(run, 32, kWave);
+    const float u3 = __shfl_up(run, 48, kWave);
     if (g >= 1) pre += u1;
     if (g >= 2) pre += u2;
     if (g >= 3) pre += u3;
 #pragma unroll
     for (int r = 0; r < 4; ++r)
       L[(w * 16 + g * 4 + r) * LR + d] = pre + c[r];
+    const float mid = __shfl(pre + run, 16 + lr, kWave);
     if (g == 3) {
       tot[w * DP + d] = pre + run;
-      wmin = fminf(wmin, pre + run);
+      wmin = fminf(wmin, fminf(mid, pre + run - mid));
     }
   }
   const bool safe = __all(wmin > -kSafeLog);
@@ -230,50 +284,9 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
   const int64_t ch = int64_t(tile) * a.heads + h;
   float* qd = a.qd + ch * C * DP;
   float* kd = a.kd + ch * DP * C;
-  f32x4_t acc[4];
+  f32x4_t acc[4], qh[NT];
 #pragma unroll
   for (int J = 0; J < 4; ++J) acc[J] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  const T* qrow = base + int64_t(trow) * a.stride + h * a.dim;
-  for (int d0 = 0; d0 < DP; d0 += 16) {
-    const int d = d0 + g * 4;
-    f32x4_t q = load4_guard(qrow, d, a.dim, row_ok, vec);
-    const f32x4_t Lt = *reinterpret_cast<const f32x4_t*>(L + trow * LR + d);
-    const f32x4_t BI = *reinterpret_cast<const f32x4_t*>(B + w * DP + d);
-    const f32x4_t BC = *reinterpret_cast<const f32x4_t*>(B + 4 * DP + d);
-    f32x4_t qh, qo;
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      q[j] *= qscale;
-      qh[j] = q[j] * gexp<T>(Lt[j]);
-      qo[j] = q[j] * gexp<T>(BI[j] + Lt[j]);
-    }
-    *reinterpret_cast<f32x4_t*>(qd + trow * DP + d) = qo;
-#pragma unroll
-    for (int J = 0; J < 4; ++J) {
-      if (J > w) break;
-      const int srow = J * 16 + lr;
-      const f32x4_t k = load4_guard(
-          base + int64_t(srow) * a.stride + hd + h * a.dim, d, a.dim,
-          srow < n, vec);
-      const f32x4_t Ls =
-          *reinterpret_cast<const f32x4_t*>(L + srow * LR + d);
-      if (J == w) {
-#pragma unroll
-        for (int j = 0; j < 4; ++j)
-          kd[int64_t(d + j) * C + srow] = k[j] * gexp<T>(BC[j] - BI[j] - Ls[j]);
-        if (safe) {
-#pragma unroll
-          for (int j = 0; j < 4; ++j)
-            acc[J] = mma4(qh[j], k[j] * gexp<T>(-Ls[j]), acc[J]);
-        }
-      } else {
-        const f32x4_t BJ = *reinterpret_cast<const f32x4_t*>(B + J * DP + d);
-#pragma unroll
-        for (int j = 0; j < 4; ++j)
-          acc[J] = mma4(qh[j], k[j] * gexp<T>(BI[j] - BJ[j] - Ls[j]), acc[J]);
-      }
-    }
-  }
   if (!safe) {
     // steep decay: pair by pair, every exponent <= 0
 #pragma unroll
@@ -282,14 +295,92 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
       float sum = 0.f;
       if (s <= t && t < n) {
         const T* qt = base + int64_t(t) * a.stride + h * a.dim;
-        const T* kt = base + int64_t(s) * a.stride + hd + h * a.dim;
-        for (int d = 0; d < a.dim; ++d)
-          sum += act_load(qt + d) * qscale * act_load(kt + d) *
-                 expf(L[t * LR + d] - L[s * LR + d]);
+        const T* kt = base + int64_t(s) * a.stride + a.off_k + h * a.dim;
+        for (int d = 0; d < a.dim; ++d) {
+          float q = act_load(qt + d), k = act_load(kt + d);
+          if constexpr (FG) {
+            float alpha;
+            q = silu(q);
+            k = forget_key(k + a.a2_bias[h * a.dim + d],
+                           a.lower[h * a.dim + d], &alpha);
+          } else {
+            q *= qscale;
+          }
+          sum += q * k * expf(L[t * LR + d] - L[s * LR + d]);
+        }
       }
 #pragma unroll
       for (int J = 0; J < 4; ++J)
         if (J == w) acc[J][r] = sum;
+    }
+  }
+  // this wave's own rows: q e^{L}, k e^{tot - L} and the diagonal block
+  const T* qrow = base + int64_t(trow) * a.stride + h * a.dim;
+  const T* krow = qrow + a.off_k;
+  f32x4_t diag = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int dt = 0; dt < NT; ++dt) {
+    if (dt >= ndt) continue;
+    const int d = dt * 16 + g * 4;
+    f32x4_t q = load4_guard(qrow, d, a.dim, row_ok, vec);
+    f32x4_t k = load4_guard(krow, d, a.dim, row_ok, vec);
+    if constexpr (FG) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int hc = h * a.dim + min(d + j, a.dim - 1);
+        float alpha;
+        q[j] = silu(q[j]);
+        const float kk = forget_key(k[j] + a.a2_bias[hc], a.lower[hc],
+                                    &alpha);
+        k[j] = row_ok && d + j < a.dim ? kk : 0.f;
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) q[j] *= qscale;
+    }
+    const f32x4_t Lt = *reinterpret_cast<const f32x4_t*>(L + trow * LR + d);
+    const f32x4_t Lm =
+        *reinterpret_cast<const f32x4_t*>(L + (w * 16 + 7) * LR + d);
+    const f32x4_t tw = *reinterpret_cast<const f32x4_t*>(tot + w * DP + d);
+    const f32x4_t BI = *reinterpret_cast<const f32x4_t*>(B + w * DP + d);
+    const f32x4_t BN = *reinterpret_cast<const f32x4_t*>(B + (w + 1) * DP + d);
+    const f32x4_t BC = *reinterpret_cast<const f32x4_t*>(B + 4 * DP + d);
+    f32x4_t kt, qo;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      qh[dt][j] = q[j] * gexp<T>(Lt[j]);
+      qo[j] = q[j] * gexp<T>(BI[j] + Lt[j]);
+      kt[j] = k[j] * gexp<T>(tw[j] - Lt[j]);
+      kd[int64_t(d + j) * C + trow] = kt[j] * gexp<T>(BC[j] - BN[j]);
+      if (safe)
+        diag = mma4(q[j] * gexp<T>(Lt[j] - Lm[j]),
+                    k[j] * gexp<T>(Lm[j] - Lt[j]), diag);
+    }
+    *reinterpret_cast<f32x4_t*>(qd + trow * DP + d) = qo;
+    *reinterpret_cast<f32x4_t*>(L + trow * LR + d) = kt;
+  }
+  if (safe) {
+#pragma unroll
+    for (int J = 0; J < 4; ++J)
+      if (J == w) acc[J] = diag;
+  }
+  __syncthreads();
+  // rows of the sub-chunks before
+#pragma unroll
+  for (int dt = 0; dt < NT; ++dt) {
+    if (dt >= ndt) continue;
+    const int d = dt * 16 + g * 4;
+    const f32x4_t BI = *reinterpret_cast<const f32x4_t*>(B + w * DP + d);
+#pragma unroll
+    for (int J = 0; J < 3; ++J) {
+      if (J >= w) break;
+      const f32x4_t BJ =
+          *reinterpret_cast<const f32x4_t*>(B + (J + 1) * DP + d);
+      const f32x4_t kt =
+          *reinterpret_cast<const f32x4_t*>(L + (J * 16 + lr) * LR + d);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        acc[J] = mma4(qh[dt][j] * gexp<T>(BI[j] - BJ[j]), kt[j], acc[J]);
     }
   }
   float* sc = a.sc + ch * C * C;
@@ -325,7 +416,7 @@ void gla_scan_kernel(GlaArgs a) {
   float* state = a.state +
                  (int64_t(a.seqs[3 * a.n_seqs + seq]) * a.heads + h) *
                      a.dim * a.vpad;
-  const int hd = a.heads * a.dim, hv = a.heads * a.vdim;
+  const int hv = a.heads * a.vdim;
 
   f32x4_t S[MD][VT];
 #pragma unroll
@@ -347,7 +438,7 @@ void gla_scan_kernel(GlaArgs a) {
   const int trow = w * 16 + lr;
   f32x4_t qr[NQ], ar[4], kr[MD][4];
   float vr[NV];
-  const T* vb = reinterpret_cast<const T*>(a.proj) + 2 * hd + h * a.vdim;
+  const T* vb = reinterpret_cast<const T*>(a.proj) + a.off_v + h * a.vdim;
   auto load_q = [&](int t) {
     const int64_t ch = int64_t(t) * a.heads + h;
     const float* qd = a.qd + ch * C * DP + trow * DP + g * 4;
@@ -473,7 +564,7 @@ void gla_scan_kernel(GlaArgs a) {
 
 // one wave per (row, head); V4 float4 columns per lane when the width and
 // its offsets allow vectors (V4 = 0: one column at a time)
-template <typename T, int V4>
+template <typename T, bool FG, int V4>
 __global__ __launch_bounds__(256)
 void gla_gate_kernel(GlaArgs a) {
   const int lane = threadIdx.x & 63;
@@ -484,8 +575,8 @@ void gla_gate_kernel(GlaArgs a) {
   const int hv = a.heads * a.vdim;
   const float* o = a.o + row * hv + h * a.vdim;
   const T* gate = reinterpret_cast<const T*>(a.proj) + row * a.stride +
-                  2 * a.heads * a.dim + hv + h * a.vdim;
-  T* out = reinterpret_cast<T*>(a.out) + row * hv + h * a.vdim;
+                  a.off_g + h * a.vdim;
+  T* out = reinterpret_cast<T*>(a.out) + row * a.out_stride + h * a.vdim;
   float ss = 0.f;
   if constexpr (V4 > 0) {
     f32x4_t ov[V4], gv[V4];
@@ -495,7 +586,7 @@ void gla_gate_kernel(GlaArgs a) {
       ov[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
       if (c < a.vdim) {
         ov[i] = *reinterpret_cast<const f32x4_t*>(o + c);
-        gv[i] = act_load4(gate + c);
+        if constexpr (!FG) gv[i] = act_load4(gate + c);
       }
 #pragma unroll
       for (int j = 0; j < 4; ++j) ss += ov[i][j] * ov[i][j];
@@ -508,17 +599,22 @@ void gla_gate_kernel(GlaArgs a) {
       const f32x4_t nv = *reinterpret_cast<const f32x4_t*>(a.norm + c);
       f32x4_t r;
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        r[j] = ov[i][j] * inv * nv[j] *
-               (gv[i][j] / (1.f + gexp<T>(-gv[i][j])));
+      for (int j = 0; j < 4; ++j) {
+        r[j] = ov[i][j] * inv * nv[j];
+        if constexpr (!FG) r[j] *= gv[i][j] / (1.f + gexp<T>(-gv[i][j]));
+      }
       act_store4(out + c, r);
     }
   } else {
     for (int e = lane; e < a.vdim; e += 64) ss += o[e] * o[e];
     const float inv = 1.f / sqrtf(wave_sum(ss) / a.vdim + a.eps);
     for (int e = lane; e < a.vdim; e += 64) {
-      const float g = act_load(gate + e);
-      act_store(out + e, o[e] * inv * a.norm[e] * (g / (1.f + gexp<T>(-g))));
+      float r = o[e] * inv * a.norm[e];
+      if constexpr (!FG) {
+        const float g = act_load(gate + e);
+        r *= g / (1.f + gexp<T>(-g));
+      }
+      act_store(out + e, r);
     }
   }
 }
@@ -540,18 +636,22 @@ void scan_md(const GlaArgs& a, hipStream_t st) {
   else run(gla_scan_kernel<T, VT, 4>);
 }
 
-template <typename T>
+template <typename T, bool FG>
 void prefill(const GlaArgs& a, hipStream_t st) {
   const bool vec = a.dim % 4 == 0 && a.stride % 4 == 0;
   const size_t smem =
       size_t(C * (a.dpad + 4) + 9 * a.dpad) * sizeof(float);
-  auto* k = gla_intra_kernel<T>;
-  if (smem > 65536)
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k),
-                              hipFuncAttributeMaxDynamicSharedMemorySize,
-                              int(smem));
-  hipLaunchKernelGGL(k, dim3(a.n_tiles, a.heads), dim3(256), smem, st, a,
-                     vec);
+  auto intra = [&](auto* k) {
+    if (smem > 65536)
+      (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k),
+                                hipFuncAttributeMaxDynamicSharedMemorySize,
+                                int(smem));
+    hipLaunchKernelGGL(k, dim3(a.n_tiles, a.heads), dim3(256), smem, st, a,
+                       vec);
+  };
+  if (a.dpad <= 64) intra(gla_intra_kernel<T, FG, 1>);
+  else if (a.dpad <= 128) intra(gla_intra_kernel<T, FG, 2>);
+  else intra(gla_intra_kernel<T, FG, 4>);
   // a scan step is latency-bound: narrow value slices, several
   // workgroups per CU, until there are plenty anyway
   const int64_t sh = int64_t(a.n_seqs) * a.heads;
@@ -563,12 +663,13 @@ void prefill(const GlaArgs& a, hipStream_t st) {
   auto gate = [&](auto* kg) {
     hipLaunchKernelGGL(kg, grid, dim3(256), 0, st, a);
   };
-  if (a.vdim % 4 || a.stride % 4 || (a.heads * a.dim) % 2)
-    gate(gla_gate_kernel<T, 0>);
+  if (a.vdim % 4 || a.stride % 4 || a.off_g % 4 || a.out_stride % 4 ||
+      reinterpret_cast<uintptr_t>(a.out) % 16)
+    gate(gla_gate_kernel<T, FG, 0>);
   else if (a.vdim <= 256)
-    gate(gla_gate_kernel<T, 1>);
+    gate(gla_gate_kernel<T, FG, 1>);
   else
-    gate(gla_gate_kernel<T, 4>);
+    gate(gla_gate_kernel<T, FG, 4>);
 }
 
 }  // namespace
@@ -580,18 +681,27 @@ void launch_gla_decode(const GlaArgs& a, hipStream_t st) {
       size_t(3 * a.dpad + (a.rank + 3) / 4 * 4 + n_rows * a.vpad) *
       sizeof(float);
   const dim3 grid(a.rows, a.heads);
-  if (a.f32)
-    hipLaunchKernelGGL(gla_decode_kernel<float>, grid, dim3(256), smem, st,
-                       a);
-  else
-    hipLaunchKernelGGL(gla_decode_kernel<uint16_t>, grid, dim3(256), smem,
-                       st, a);
+  auto go = [&](auto* k) {
+    hipLaunchKernelGGL(k, grid, dim3(256), smem, st, a);
+  };
+  if (a.forget) {
+    if (a.f32) go(gla_decode_kernel<float, true>);
+    else go(gla_decode_kernel<uint16_t, true>);
+  } else {
+    if (a.f32) go(gla_decode_kernel<float, false>);
+    else go(gla_decode_kernel<uint16_t, false>);
+  }
 }
 
 void launch_gla_prefill(const GlaArgs& a, hipStream_t st) {
   if (a.rows == 0 || a.n_seqs == 0) return;
-  if (a.f32) prefill<float>(a, st);
-  else prefill<uint16_t>(a, st);
+  if (a.forget) {
+    if (a.f32) prefill<float, true>(a, st);
+    else prefill<uint16_t, true>(a, st);
+  } else {
+    if (a.f32) prefill<float, false>(a, st);
+    else prefill<uint16_t, false>(a, st);
+  }
 }
 
 }  // namespace rlli

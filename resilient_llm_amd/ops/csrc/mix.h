@@ -156,8 +156,10 @@ int window_prefill_sub_tiles(int group);
 // ---- gla.hip -----------------------------------------------------------
 struct GlaArgs {
   const void* proj;        // [rows, stride]: q | k | v | gate | low-rank
+                           // (HGRN2: q | forget logit | v)
   const void* a2;          // [heads * dim, rank]
   const float* a2_bias;    // [heads * dim]
+  const float* lower;      // [heads * dim] (HGRN2)
   const float* norm;       // [vdim]
   float* state;            // [slots, heads, dim, vpad]
   const int32_t* slots;    // [sequences]
@@ -169,10 +171,12 @@ struct GlaArgs {
   float* sc;               // [n_tiles, heads, 64, 64]
   float* dec;              // [n_tiles, heads, dpad]
   float* o;                // [rows, heads * vdim]
-  void* out;               // [rows, heads * vdim]
+  void* out;               // [rows, heads * vdim], rows out_stride apart
   int rows, n_tiles, n_seqs, heads, dim, vdim, vpad, dpad, rank, stride;
-  int n_slots;
+  int off_k, off_v, off_g, off_a;   // columns of proj
+  int out_stride, n_slots;
   float tau, eps;
+  bool forget;             // HGRN2 instead of GLA
   bool f32;
 };
 constexpr int kGlaChunk = 64;

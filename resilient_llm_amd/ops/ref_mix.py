@@ -133,19 +133,15 @@ def _gla_out(o, g, norm, eps, dtype):
     return (_norm(o, norm, eps) * F.silu(g)).flatten(1).to(dtype)
 
 
-def gla_decode(proj, a2, a2_bias, norm, state, slots, positions, vdim, tau,
-               eps):
-    q, k, v, g, alpha = _gla_parts(proj, a2, a2_bias, state, vdim, tau)
+def _step_states(q, k, v, alpha, state, slots, positions, vdim):
     S = state[slots.long()][..., :vdim]
     S[positions == 0] = 0.0               # a fresh sequence, a used slot
     S = alpha[..., None] * S + k[..., None] * v[:, :, None]
     state[slots.long(), :, :, :vdim] = S
-    return _gla_out(torch.einsum("bhd,bhdv->bhv", q, S), g, norm, eps,
-                    proj.dtype)
+    return torch.einsum("bhd,bhdv->bhv", q, S)
 
 
-def gla_prefill(proj, a2, a2_bias, norm, state, tiles, seqs, vdim, tau, eps):
-    q, k, v, g, alpha = _gla_parts(proj, a2, a2_bias, state, vdim, tau)
+def _scan_states(q, k, v, alpha, state, tiles, seqs, vdim):
     o = torch.empty_like(v)
     for first, count, pos0, slot in seqs.t().tolist():
         S = state[slot, :, :, :vdim].clone()
@@ -157,7 +153,46 @@ def gla_prefill(proj, a2, a2_bias, norm, state, tiles, seqs, vdim, tau, eps):
             S = alpha[t][..., None] * S + k[t][..., None] * v[t][:, None]
             o[t] = torch.einsum("hd,hdv->hv", q[t], S)
         state[slot, :, :, :vdim] = S
-    return _gla_out(o, g, norm, eps, proj.dtype)
+    return o
+
+
+def gla_decode(proj, a2, a2_bias, norm, state, slots, positions, vdim, tau,
+               eps, out):
+    q, k, v, g, alpha = _gla_parts(proj, a2, a2_bias, state, vdim, tau)
+    o = _step_states(q, k, v, alpha, state, slots, positions, vdim)
+    out.copy_(_gla_out(o, g, norm, eps, proj.dtype))
+
+
+def gla_prefill(proj, a2, a2_bias, norm, state, tiles, seqs, vdim, tau, eps,
+                out):
+    q, k, v, g, alpha = _gla_parts(proj, a2, a2_bias, state, vdim, tau)
+    o = _scan_states(q, k, v, alpha, state, tiles, seqs, vdim)
+    out.copy_(_gla_out(o, g, norm, eps, proj.dtype))
+
+
+def _hgrn2_parts(proj, bias, lower, state, vdim):
+    T = proj.shape[0]
+    _, H, D, _ = state.shape
+    q, z, v = torch.split(proj.float(), [H * D, H * D, H * vdim], dim=1)
+    z = z + bias
+    k = (1 - lower) * torch.sigmoid(-z)
+    alpha = lower + (1 - lower) * torch.sigmoid(z)
+    return (F.silu(q).view(T, H, D), k.view(T, H, D), v.view(T, H, vdim),
+            alpha.view(T, H, D))
+
+
+def hgrn2_decode(proj, bias, lower, norm, state, slots, positions, vdim, eps,
+                 out):
+    parts = _hgrn2_parts(proj, bias, lower, state, vdim)
+    o = _step_states(*parts, state, slots, positions, vdim)
+    out.copy_(_norm(o, norm, eps).flatten(1))
+
+
+def hgrn2_prefill(proj, bias, lower, norm, state, tiles, seqs, vdim, eps,
+                  out):
+    parts = _hgrn2_parts(proj, bias, lower, state, vdim)
+    o = _scan_states(*parts, state, tiles, seqs, vdim)
+    out.copy_(_norm(o, norm, eps).flatten(1))
 
 
 # ---------------------------------------------------------------- experts

@@ -54,9 +54,8 @@ def main() -> None:
         from .. import ops
         from ..models import get_model_class
         ops.load_extension(required=True)
-        if getattr(get_model_class(args.model, args.weights), "mixed_layers",
-                   False):
-            ops.load_mix_extension()
+        ops.load_libraries(
+            get_model_class(args.model, args.weights).EXTENSIONS)
 
     from ..utils.logging import log_with_timestamp
     from .engine_worker import EngineWorker
