@@ -176,36 +176,69 @@ class LoadGen:
             self.proc.kill()
 
 
-def design_pairs() -> dict:
-    """size -> (Nesizen config, Llama config of equal width, depth, heads
-    and active feed-forward width)."""
-    from resilient_llm_amd.models import LlamaConfig, NesizenConfig
-    from resilient_llm_amd.models.nesizen import hybrid_layers
+def design_models(design: str) -> dict:
+    """size -> {name: configuration}: the design, then existing models of
+    equal width, depth, heads and (active) feed-forward size."""
+    from resilient_llm_amd.models import (
+        LlamaConfig, NesizenConfig, RiruzenConfig,
+    )
+    from resilient_llm_amd.models import nesizen, riruzen
 
-    def pair(width, layers, heads, kv, gla_heads, experts, top, ff):
-        nz = NesizenConfig.from_dict(
+    def llama(width, layers, heads, kv, ff):
+        return LlamaConfig(name=f"llama-w{width}", hidden_size=width,
+                           n_layers=layers, n_heads=heads, n_kv_heads=kv,
+                           head_dim=128, intermediate_size=ff,
+                           vocab_size=65536, max_position=32768)
+
+    def nesi(width, layers, heads, kv, gla_heads, mlp, first=None):
+        return NesizenConfig.from_dict(
             {"width": width, "vocab": 65536, "streams": 2,
              "norm": {"eps": 1e-5},
-             "layers": hybrid_layers(
+             "layers": nesizen.hybrid_layers(
                  layers, 3,
                  {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128,
                   "scale": 128 ** -0.5, "rot": {"dims": 64, "base": 1e6},
                   "mask": {"size": 1024, "keep_first": 4}},
                  {"heads": gla_heads, "dim": 128, "vdim": 256, "tau": 16.0},
-                 {"kind": "moe", "expert": {"ff": ff, "limit": 7.0},
-                  "router": {"experts": experts, "top": top}},
-                 {"kind": "dense", "ff": 3 * top * ff // 2})},
+                 mlp, first)},
             name=f"nesizen-w{width}")
-        ll = LlamaConfig(name=f"llama-w{width}", hidden_size=width,
-                         n_layers=layers, n_heads=heads, n_kv_heads=kv,
-                         head_dim=128, intermediate_size=top * ff,
-                         vocab_size=65536, max_position=32768)
-        return nz, ll
-    return {"w2048": pair(2048, 12, 16, 4, 8, 32, 4, 1024),
-            "w4096": pair(4096, 6, 32, 8, 16, 16, 2, 3584)}
+
+    def moe(experts, top, ff):
+        return {"kind": "moe", "expert": {"ff": ff, "limit": 7.0},
+                "router": {"experts": experts, "top": top}}
+
+    def riru(width, layers, heads, q_rank, ff):
+        return RiruzenConfig.from_dict(
+            {"width": width, "vocab": 65536, "logit_scale": 1.0,
+             "max_positions": 32768, "canon": {"taps": 4},
+             "norm": {"eps": 1e-5, "groups": 4},
+             "layers": riruzen.hybrid_layers(
+                 layers, 3,
+                 {"heads": heads, "dim": 128, "vdim": 128, "q_rank": q_rank,
+                  "kv_rank": 512, "scale": 128 ** -0.5},
+                 {"heads": heads, "dim": 128, "vdim": 128},
+                 {"kind": "dense", "ff": ff})}, name=f"riruzen-w{width}")
+
+    def dense(ff):
+        return {"kind": "dense", "ff": ff}
+    if design == "nesizen":
+        return {"w2048": {"nesizen": nesi(2048, 12, 16, 4, 8,
+                                          moe(32, 4, 1024), dense(6144)),
+                          "llama": llama(2048, 12, 16, 4, 4096)},
+                "w4096": {"nesizen": nesi(4096, 6, 32, 8, 16,
+                                          moe(16, 2, 3584), dense(10752)),
+                          "llama": llama(4096, 6, 32, 8, 7168)}}
+    # two matrices of 3/2 the width are as large as the gated three
+    return {"w2048": {"riruzen": riru(2048, 12, 16, 768, 4096),
+                      "nesizen": nesi(2048, 12, 16, 4, 8, dense(6144)),
+                      "llama": llama(2048, 12, 16, 4, 4096)},
+            "w4096": {"riruzen": riru(4096, 6, 32, 1536, 7168),
+                      "nesizen": nesi(4096, 6, 32, 8, 16, dense(10752)),
+                      "llama": llama(4096, 6, 32, 8, 7168)}}
 
 
-def run_design(sizes: list, which: list, steps: int, phases: list) -> None:
+def run_design(design: str, sizes: list, which: list, steps: int,
+               phases: list) -> None:
     """Engine-level throughput, no gateway: prefill = prompt tokens/s of
     one full prefill step, decode = output tokens/s of graph-replayed
     steps.  Random weights, synthetic tokens."""
@@ -227,8 +260,8 @@ def run_design(sizes: list, which: list, steps: int, phases: list) -> None:
         return torch.randint(5, 60000, (n,), generator=rng).tolist()
 
     for size in sizes:
-        for kind, cfg in zip(("nesizen", "llama"), design_pairs()[size]):
-            if kind not in which:
+        for kind, cfg in design_models(design)[size].items():
+            if which and kind not in which:
                 continue
             model = build_model(cfg, device="cuda:0", dtype=torch.bfloat16)
             for phase in phases:
@@ -304,20 +337,21 @@ def main() -> None:
                          "headline metric stays bf16)")
     ap.add_argument("--device", default=None,
                     help="override torch device (tests: cpu)")
-    ap.add_argument("--design", default=None, choices=("nesizen",),
+    ap.add_argument("--design", default=None, choices=("nesizen", "riruzen"),
                     help="measure this design's engine throughput beside "
-                         "a Llama of equal size instead of serving")
+                         "existing models of equal size instead of serving")
     ap.add_argument("--design-sizes", default="w2048,w4096")
-    ap.add_argument("--design-models", default="nesizen,llama")
+    ap.add_argument("--design-models", default="",
+                    help="comma list of models to measure (default: all)")
     ap.add_argument("--design-phases", default="prefill:4:2048,"
                     "prefill:1:8192,decode:1:2048,decode:16:2048,"
                     "decode:64:2048",
                     help="comma list of phase:sequences:tokens")
     args = ap.parse_args()
     if args.design:
-        run_design(args.design_sizes.split(","),
-                   args.design_models.split(","), max(1, args.steps),
-                   args.design_phases.split(","))
+        run_design(args.design, args.design_sizes.split(","),
+                   [m for m in args.design_models.split(",") if m],
+                   max(1, args.steps), args.design_phases.split(","))
         return
     globals()["OUTPUT_TOKENS"] = args.output_tokens
 
