@@ -59,40 +59,83 @@ void block_step_kernel(BlockArgs a) {
       pr = reinterpret_cast<const T*>(a.pos_table) +
            int64_t(min(a.positions[n], a.n_positions - 1)) * W;
   }
-  auto value = [&](int c, float (&u)[V]) {
-    float t[V];
+  // the two summands of a row's new value
+  auto summands = [&](int c, float (&u)[V], float (&t)[V]) {
     if constexpr (EMBED) {
       load_v<T, V>(er + c, u);
       if (pr) {
         load_v<T, V>(pr + c, t);
+      } else {
 #pragma unroll
-        for (int j = 0; j < V; ++j) u[j] += t[j];
+        for (int j = 0; j < V; ++j) t[j] = 0.f;
       }
     } else {
       load_v<float, V>(xr + c, u);
       load_v<T, V>(yr + c, t);
-#pragma unroll
-      for (int j = 0; j < V; ++j) u[j] += t[j];
     }
   };
-  float u[IT > 0 ? IT : 1][V];
+  // IT > 0: everything a row needs is asked for up front, so that one
+  // memory latency covers it; long convolutions and the plain walk load
+  // the rest late
+  constexpr int ITS = IT > 0 ? IT : 1;
+  constexpr int EARLY = IT == 1 || IT == 2 ? 4 : 0;      // taps
+  float u[ITS][V], t[ITS][V], gain[ITS][V];
+  float tap[ITS][EARLY + 1][V], past[ITS][EARLY + 1][V];
   auto every = [&](auto body) {           // over this thread's vectors
     if constexpr (IT > 0) {
 #pragma unroll
       for (int i = 0; i < IT; ++i)
-        if (i * NT + int(threadIdx.x) < nv) body(i * NT + threadIdx.x, u[i]);
+        if (i * NT + int(threadIdx.x) < nv) body(i * NT + threadIdx.x, i);
     } else {
-      for (int v = threadIdx.x; v < nv; v += NT) body(v, u[0]);
+      for (int v = threadIdx.x; v < nv; v += NT) body(v, 0);
     }
   };
-  every([&](int v, float (&uu)[V]) {
-    value(v * V, uu);
+  const bool conv = a.hc && n < a.n_decode;
+  const int back = a.n_taps - 1;          // earlier inputs in the ring
+  auto load_tap = [&](int k, int c, float (&w)[V]) {
+    load_v<float, V>(a.taps + int64_t(back - k) * W + c, w);
+  };
+  if constexpr (IT > 0) {
+    every([&](int v, int i) { summands(v * V, u[i], t[i]); });
+    every([&](int v, int i) { load_v<float, V>(a.gain + v * V, gain[i]); });
+    if (conv)
+      every([&](int v, int i) {
+#pragma unroll
+        for (int k = 0; k < EARLY; ++k)
+          if (k <= back) load_tap(k, v * V, tap[i][k]);
+      });
+  }
+  int pos = 0, at = 0;                    // position, its row of the ring
+  T* ring = nullptr;
+  if (conv) {
+    pos = a.positions[n];
+    if (back > 0) {
+      ring = reinterpret_cast<T*>(a.tail) + int64_t(a.slots[n]) * back * W;
+      at = pos % back;
+    }
+  }
+  auto load_ring = [&](int k, int c, float (&e)[V]) {
+    const int r = at - k < 0 ? at - k + back : at - k;
+    load_v<T, V>(ring + int64_t(r) * W + c, e);
+  };
+  if (conv)
+    every([&](int v, int i) {
+#pragma unroll
+      for (int k = 1; k < EARLY; ++k)
+        if (k <= back && k <= pos) load_ring(k, v * V, past[i][k]);
+    });
+
+  every([&](int v, int i) {
+    if constexpr (IT == 0) summands(v * V, u[0], t[0]);
     float s = 0.f;
 #pragma unroll
-    for (int j = 0; j < V; ++j) s += uu[j] * uu[j];
+    for (int j = 0; j < V; ++j) {
+      u[i][j] += t[i][j];
+      s += u[i][j] * u[i][j];
+    }
     sq[v] = s;
     if constexpr (IT > 0)
-      if (a.keep) store_v<float, V>(xr + v * V, uu);
+      if (a.keep) store_v<float, V>(xr + v * V, u[i]);
   });
   __syncthreads();
   for (int g = threadIdx.x >> 6; g < a.groups; g += WAVES) {
@@ -104,42 +147,40 @@ void block_step_kernel(BlockArgs a) {
   }
   __syncthreads();
   T* hr = reinterpret_cast<T*>(a.h) + int64_t(n) * W;
-  const bool conv = a.hc && n < a.n_decode;
-  const int back = a.n_taps - 1;          // earlier inputs in the ring
-  int pos = 0;
-  T* ring = nullptr;
-  if (conv) {
-    pos = a.positions[n];
-    if (back > 0)
-      ring = reinterpret_cast<T*>(a.tail) + int64_t(a.slots[n]) * back * W;
-  }
-  every([&](int v, float (&uu)[V]) {
+  every([&](int v, int i) {
     const int c = v * V;
     if constexpr (IT == 0) {
-      value(c, uu);
-      if (a.keep) store_v<float, V>(xr + c, uu);
+      summands(c, u[0], t[0]);
+#pragma unroll
+      for (int j = 0; j < V; ++j) u[0][j] += t[0][j];
+      if (a.keep) store_v<float, V>(xr + c, u[0]);
+      load_v<float, V>(a.gain + c, gain[0]);
     }
-    float g[V], hv[V];
-    load_v<float, V>(a.gain + c, g);
+    float hv[V];
     const float inv = scale[v / gv];
 #pragma unroll
-    for (int j = 0; j < V; ++j) hv[j] = round_act(T{}, uu[j] * inv * g[j]);
+    for (int j = 0; j < V; ++j)
+      hv[j] = round_act(T{}, u[i][j] * inv * gain[i][j]);
     store_v<T, V>(hr + c, hv);
     if (conv) {
-      float w[V], o[V];
-      load_v<float, V>(a.taps + int64_t(back) * W + c, w);
+      float o[V];
 #pragma unroll
-      for (int j = 0; j < V; ++j) o[j] = hv[j] + w[j] * hv[j];
-      for (int k = 1; k <= back; ++k) {
-        if (pos - k < 0) break;
-        float e[V];
-        load_v<T, V>(ring + int64_t((pos - k) % back) * W + c, e);
-        load_v<float, V>(a.taps + int64_t(back - k) * W + c, w);
+      for (int j = 0; j < V; ++j) o[j] = hv[j];
+      auto add = [&](const float (&w)[V], const float (&e)[V]) {
 #pragma unroll
         for (int j = 0; j < V; ++j) o[j] += w[j] * e[j];
+      };
+#pragma unroll
+      for (int k = 0; k < EARLY; ++k)
+        if (k <= back && k <= pos) add(tap[i][k], k == 0 ? hv : past[i][k]);
+      for (int k = EARLY; k <= back && k <= pos; ++k) {
+        float w[V], e[V];
+        load_tap(k, c, w);
+        if (k > 0) load_ring(k, c, e);
+        add(w, k == 0 ? hv : e);
       }
       store_v<T, V>(reinterpret_cast<T*>(a.hc) + int64_t(n) * W + c, o);
-      if (back > 0) store_v<T, V>(ring + int64_t(pos % back) * W + c, hv);
+      if (back > 0) store_v<T, V>(ring + int64_t(at) * W + c, hv);
     }
   });
 }

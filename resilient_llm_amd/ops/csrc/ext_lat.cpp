@@ -287,7 +287,8 @@ Tensor latent_attn(const Tensor& q, const Tensor& cache,
   a.rows = int(rows);
   a.heads = int(heads);
   a.rank = int(R);
-  a.block_size = int(cache.size(2));
+  const int64_t block = cache.size(2);
+  while ((int64_t(1) << a.block_shift) < block) ++a.block_shift;
   a.max_blocks = int(block_tables.size(1));
   a.scale = float(scale);
   a.out = out.data_ptr();
@@ -302,12 +303,13 @@ Tensor latent_attn(const Tensor& q, const Tensor& cache,
     const int t = rlli::latent_tile(a.heads, true);
     wgs = rows * ((heads + t - 1) / t);
   }
-  // enough workgroups for the chip, at least two key tiles each
-  const int64_t key_tiles =
-      (int64_t(a.max_blocks) * a.block_size + 63) / 64;
+  // enough workgroups for the chip, at least 128 keys each
+  const int64_t most = int64_t(a.max_blocks) * block / 128;
+  const int64_t aim =
+      rlli::latent_tile(a.heads, tiles == std::nullopt) <= 32 ? 512 : 256;
   a.n_split = int(std::max<int64_t>(
-      1, std::min<int64_t>({32, key_tiles / 2,
-                            (512 + wgs - 1) / std::max<int64_t>(wgs, 1)})));
+      1, std::min<int64_t>({32, most, (aim + wgs - 1) /
+                                          std::max<int64_t>(wgs, 1)})));
   Tensor pa, pm;
   if (a.n_split > 1) {
     auto fo = q.options().dtype(at::kFloat);

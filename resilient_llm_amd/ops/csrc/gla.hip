@@ -21,7 +21,7 @@
 // for J < I has only exponents <= 0, whatever the decay.  Inside a
 // sub-chunk the factors are e^{L_t - m} and e^{m - L_s} with m the middle
 // row's log-decay, as long as either half decays by less than e^40; beyond
-// that the pairwise e^{L_t - L_s} is summed directly.
+// that four-row blocks do the same once more.
 //   gla_intra   per (chunk, head): A, q e^{b_t}, k e^{b_C - b_s}, e^{b_C}
 //   gla_scan    per (sequence, head, value slice): chunk after chunk,
 //               O = (q e^{b}) S + A V, S = e^{b_C} S + (k e^{b_C-b})^T V,
@@ -50,24 +50,43 @@ DEV_INLINE float log_sigmoid(float x) {
   return fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
 }
 
-DEV_INLINE float silu(float x) { return x / (1.f + expf(-x)); }
+// 1 / x for x >= 1, good to an ulp where activations are 16-bit
+template <typename T> DEV_INLINE float grcp(float x);
+template <> DEV_INLINE float grcp<uint16_t>(float x) {
+  return __builtin_amdgcn_rcpf(x);
+}
+template <> DEV_INLINE float grcp<float>(float x) { return 1.f / x; }
+
+template <typename T>
+DEV_INLINE float silu(float x) {
+  // (the exponent is bounded so that the reciprocal stays finite)
+  return x * grcp<T>(1.f + gexp<T>(fminf(-x, 80.f)));
+}
 
 // HGRN2: alpha = low + (1 - low) sigmoid(z), k = 1 - alpha without the
 // cancellation
+template <typename T>
 DEV_INLINE float forget_key(float z, float low, float* alpha) {
-  const float e = expf(-fabsf(z));
-  const float r = 1.f / (1.f + e), er = e * r;
+  const float e = gexp<T>(-fabsf(z));
+  const float r = grcp<T>(1.f + e), er = e * r;
   *alpha = low + (1.f - low) * (z >= 0.f ? r : er);
   return (1.f - low) * (z >= 0.f ? er : r);
 }
 
-// its logarithm; e^-80 and less is nothing beside a key of order one
+// log alpha; e^-80 and less is nothing beside a key of order one
 template <typename T>
-DEV_INLINE float log_forget(float z, float low) {
-  float alpha;
-  const float k = forget_key(z, low, &alpha);
+DEV_INLINE float log_forget(float alpha, float k) {
   if constexpr (sizeof(T) == 2) return fmaxf(__logf(alpha), -80.f);
   return alpha > 0.5f ? log1pf(-k) : fmaxf(logf(alpha), -80.f);
+}
+
+// running sum over the 16 lanes of a row
+DEV_INLINE float row_prefix(float v) {
+  v += dpp_mov_f32<0x111>(v);             // row_shr 1, 2, 4, 8: zeros enter
+  v += dpp_mov_f32<0x112>(v);
+  v += dpp_mov_f32<0x114>(v);
+  v += dpp_mov_f32<0x118>(v);
+  return v;
 }
 
 DEV_INLINE f32x4_t mma4(float a, float b, f32x4_t c) {
@@ -103,9 +122,9 @@ void gla_decode_kernel(GlaArgs a) {
   if constexpr (FG) {
     for (int d = tid; d < a.dim; d += 256) {
       const int hc = h * a.dim + d;
-      qs[d] = silu(act_load(row + hc));
-      ks[d] = forget_key(act_load(row + a.off_k + hc) + a.a2_bias[hc],
-                         a.lower[hc], al + d);
+      qs[d] = silu<T>(act_load(row + hc));
+      ks[d] = forget_key<T>(act_load(row + a.off_k + hc) + a.a2_bias[hc],
+                            a.lower[hc], al + d);
     }
   } else {
     for (int r = tid; r < a.rank; r += 256) a1[r] = act_load(row + a.off_a + r);
@@ -185,13 +204,15 @@ void gla_decode_kernel(GlaArgs a) {
            h * a.vdim;
   for (int e = tid; e < a.vdim; e += 256) {
     float o2 = red[e] * inv * a.norm[e];
-    if constexpr (!FG) o2 *= silu(act_load(row + a.off_g + h * a.vdim + e));
+    if constexpr (!FG)
+      o2 *= silu<T>(act_load(row + a.off_g + h * a.vdim + e));
     act_store(out + e, o2);
   }
 }
 
 // -------------------------------------------------------------- intra
-// Wave w owns sub-chunk w; MD bounds the key tiles (dpad <= 64 * MD).
+// Wave w owns sub-chunk w, lane l its row l & 15 and four neighbouring key
+// columns of every 16; MD bounds the key tiles (dpad <= 64 * MD).
 template <typename T, bool FG, int MD>
 __global__ __launch_bounds__(256)
 void gla_intra_kernel(GlaArgs a, bool vec) {
@@ -201,163 +222,180 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int lr = lane & 15, g = lane >> 4;
   const int DP = a.dpad, LR = DP + 4, ndt = DP / 16;
-  float* L = sm;                         // [64][LR], then decayed keys
-  float* tot = L + C * LR;               // [4][DP]
-  float* B = tot + 4 * DP;               // [5][DP]
+  float* kl = sm;                        // [64][LR] decayed keys
+  float* tot = kl + C * LR;              // [4][DP] log-decays of sub-chunks
+  float* EB = tot + 4 * DP;              // [4][DP] e^{B_w}
+  float* ED = EB + 4 * DP;               // [4][DP] e^{B_4 - B_{w+1}}
+  float* EJ = ED + 4 * DP;               // [3][DP] sub-chunks in between
   const int row0 = a.tiles[tile];
   const int n = a.tiles[2 * a.n_tiles + tile];
-  const T* base = reinterpret_cast<const T*>(a.proj) +
-                  int64_t(row0) * a.stride;
-  const int trow = w * 16 + lr;          // this lane's operand row
+  const int trow = w * 16 + lr;          // this lane's row
   const bool row_ok = trow < n;
+  const T* qrow = reinterpret_cast<const T*>(a.proj) +
+                  int64_t(row0 + trow) * a.stride + h * a.dim;
+  const T* krow = qrow + a.off_k;
+  const float* bias = a.a2_bias + h * a.dim;
+  const float* low = FG ? a.lower + h * a.dim : nullptr;
+  const float qscale = 1.f / sqrtf(float(a.dim));
 
-  // log-decay of sub-chunk w, then its running sum down the rows
+  // queries, keys and the running log-decay, all in registers
+  f32x4_t q[NT], k[NT], L[NT];
   float wmin = 0.f;
-  for (int dt = 0; dt < ndt; ++dt) {
-    const int d = dt * 16 + lr;
-    f32x4_t z = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    if constexpr (FG) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = w * 16 + g * 4 + r;
-        if (d < a.dim && t < n)
-          z[r] = act_load(base + int64_t(t) * a.stride + a.off_k +
-                          h * a.dim + d);
+  for (int dt = 0; dt < NT; ++dt) {
+    if (dt >= ndt) continue;
+    const int d = dt * 16 + g * 4;
+    q[dt] = load4_guard(qrow, d, a.dim, row_ok, vec);
+    k[dt] = load4_guard(krow, d, a.dim, row_ok, vec);
+  }
+#pragma unroll
+  for (int dt = 0; dt < NT; ++dt) {
+    if (dt >= ndt) continue;
+    const int d = dt * 16 + g * 4;
+    const f32x4_t bv = load4_guard(bias, d, a.dim, true, a.dim % 4 == 0);
+    if constexpr (FG) {
+      const f32x4_t lv = load4_guard(low, d, a.dim, true, a.dim % 4 == 0);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const bool ok = row_ok && d + j < a.dim;
+        float alpha;
+        const float kk = forget_key<T>(k[dt][j] + bv[j], lv[j], &alpha);
+        k[dt][j] = ok ? kk : 0.f;
+        L[dt][j] = ok ? log_forget<T>(alpha, kk) : 0.f;
+        q[dt][j] = silu<T>(q[dt][j]);
       }
     } else {
-      const T* a1 = base + int64_t(trow) * a.stride + a.off_a;
+      // z transposed: columns down, rows across the lanes
+      f32x4_t z = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      const T* a1 = qrow - h * a.dim + a.off_a;
       const T* a2 = reinterpret_cast<const T*>(a.a2) +
-                    int64_t(h * a.dim + d) * a.rank;
+                    int64_t(h * a.dim + dt * 16 + lr) * a.rank;
       for (int k0 = 0; k0 < a.rank; k0 += 16) {
         const f32x4_t av = load4_guard(a1, k0 + g * 4, a.rank, row_ok, false);
-        const f32x4_t bv = load4_guard(a2, k0 + g * 4, a.rank, d < a.dim,
-                                       false);
+        const f32x4_t wv = load4_guard(a2, k0 + g * 4, a.rank,
+                                       dt * 16 + lr < a.dim, false);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) z = mma4(av[j], bv[j], z);
+        for (int j = 0; j < 4; ++j) z = mma4(wv[j], av[j], z);
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const bool ok = row_ok && d + j < a.dim;
+        L[dt][j] = ok ? log_sigmoid<T>(z[j] + bv[j]) / a.tau : 0.f;
+        q[dt][j] *= qscale;
       }
     }
-    const float bias = d < a.dim ? a.a2_bias[h * a.dim + d] : 0.f;
-    float low = 0.f;
-    if constexpr (FG) low = d < a.dim ? a.lower[h * a.dim + d] : 0.f;
-    float c[4], run = 0.f;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const bool ok = d < a.dim && w * 16 + g * 4 + r < n;
-      float ld;
-      if constexpr (FG) ld = log_forget<T>(z[r] + bias, low);
-      else ld = log_sigmoid<T>(z[r] + bias) / a.tau;
-      run += ok ? ld : 0.f;
-      c[r] = run;
-    }
-    // prefix over the four 4-row lane groups
-    float pre = 0.f;
-    const float u1 = __shfl_up(run, 16, kWave);
-    const float u2 = __shfl_up(run, 32, kWave);
-    const float u3 = __shfl_up(run, 48, kWave);
-    if (g >= 1) pre += u1;
-    if (g >= 2) pre += u2;
-    if (g >= 3) pre += u3;
-#pragma unroll
-    for (int r = 0; r < 4; ++r)
-      L[(w * 16 + g * 4 + r) * LR + d] = pre + c[r];
-    const float mid = __shfl(pre + run, 16 + lr, kWave);
-    if (g == 3) {
-      tot[w * DP + d] = pre + run;
-      wmin = fminf(wmin, fminf(mid, pre + run - mid));
+    for (int j = 0; j < 4; ++j) {
+      L[dt][j] = row_prefix(L[dt][j]);
+      const float mid = __shfl(L[dt][j], g * 16 + 7, kWave);
+      if (lr == 15) {
+        tot[w * DP + d + j] = L[dt][j];
+        wmin = fminf(wmin, fminf(mid, L[dt][j] - mid));
+      }
     }
   }
   const bool safe = __all(wmin > -kSafeLog);
   __syncthreads();
   for (int d = threadIdx.x; d < DP; d += 256) {
-    float b = 0.f;
+    float t[4], b = 0.f;
 #pragma unroll
     for (int s = 0; s < 4; ++s) {
-      B[s * DP + d] = b;
-      b += tot[s * DP + d];
+      t[s] = tot[s * DP + d];
+      EB[s * DP + d] = gexp<T>(b);
+      b += t[s];
     }
-    B[4 * DP + d] = b;
     a.dec[(int64_t(tile) * a.heads + h) * DP + d] = expf(b);
+    float after = 0.f;
+#pragma unroll
+    for (int s = 3; s >= 0; --s) {
+      ED[s * DP + d] = gexp<T>(after);
+      after += t[s];
+    }
+    EJ[d] = gexp<T>(t[1]);                // from 0 to 2
+    EJ[DP + d] = gexp<T>(t[1] + t[2]);    // from 0 to 3
+    EJ[2 * DP + d] = gexp<T>(t[2]);       // from 1 to 3
   }
-  __syncthreads();
-
-  const float qscale = 1.f / sqrtf(float(a.dim));
-  const int64_t ch = int64_t(tile) * a.heads + h;
-  float* qd = a.qd + ch * C * DP;
-  float* kd = a.kd + ch * DP * C;
-  f32x4_t acc[4], qh[NT];
+  f32x4_t acc[4];
 #pragma unroll
   for (int J = 0; J < 4; ++J) acc[J] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   if (!safe) {
-    // steep decay: pair by pair, every exponent <= 0
+    // steep decay: four-row blocks.  Block pairs a > b factor around the
+    // row before a, so every exponent is <= 0; inside a block the three
+    // distances are summed lane by lane.
+    float near[4] = {0.f, 0.f, 0.f, 0.f};  // row lr and the row so far back
+    f32x4_t far = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = w * 16 + g * 4 + r, s = w * 16 + lr;
-      float sum = 0.f;
-      if (s <= t && t < n) {
-        const T* qt = base + int64_t(t) * a.stride + h * a.dim;
-        const T* kt = base + int64_t(s) * a.stride + a.off_k + h * a.dim;
-        for (int d = 0; d < a.dim; ++d) {
-          float q = act_load(qt + d), k = act_load(kt + d);
-          if constexpr (FG) {
-            float alpha;
-            q = silu(q);
-            k = forget_key(k + a.a2_bias[h * a.dim + d],
-                           a.lower[h * a.dim + d], &alpha);
-          } else {
-            q *= qscale;
-          }
-          sum += q * k * expf(L[t * LR + d] - L[s * LR + d]);
-        }
+    for (int dt = 0; dt < NT; ++dt) {
+      if (dt >= ndt) continue;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float Lt = L[dt][j], qv = q[dt][j], kv = k[dt][j];
+        float ref[4];
+#pragma unroll
+        for (int b = 1; b < 4; ++b)
+          ref[b] = __shfl(Lt, g * 16 + 4 * b - 1, kWave);
+        const int own = lr >> 2;
+        const float mine = own == 3 ? ref[3] : own == 2 ? ref[2] : ref[1];
+        const float qa = own > 0 ? qv * gexp<T>(Lt - mine) : 0.f;
+#pragma unroll
+        for (int b = 1; b < 4; ++b)
+          far = mma4(own == b ? qa : 0.f,
+                     lr < 4 * b ? kv * gexp<T>(ref[b] - Lt) : 0.f, far);
+        near[0] += qv * kv;
+        near[1] += qv * dpp_mov_f32<0x111>(kv) *
+                   gexp<T>(fminf(Lt - dpp_mov_f32<0x111>(Lt), 0.f));
+        near[2] += qv * dpp_mov_f32<0x112>(kv) *
+                   gexp<T>(fminf(Lt - dpp_mov_f32<0x112>(Lt), 0.f));
+        near[3] += qv * dpp_mov_f32<0x113>(kv) *
+                   gexp<T>(fminf(Lt - dpp_mov_f32<0x113>(Lt), 0.f));
+      }
+    }
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      near[x] += __shfl_xor(near[x], 16, kWave);
+      near[x] += __shfl_xor(near[x], 32, kWave);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        const float v = __shfl(near[x], g * 4 + r, kWave);
+        if (lr >> 2 == g && g * 4 + r - lr == x) far[r] = v;
       }
 #pragma unroll
-      for (int J = 0; J < 4; ++J)
-        if (J == w) acc[J][r] = sum;
-    }
+    for (int J = 0; J < 4; ++J)
+      if (J == w) acc[J] = far;
   }
+  __syncthreads();
+
   // this wave's own rows: q e^{L}, k e^{tot - L} and the diagonal block
-  const T* qrow = base + int64_t(trow) * a.stride + h * a.dim;
-  const T* krow = qrow + a.off_k;
+  const int64_t ch = int64_t(tile) * a.heads + h;
+  float* qd = a.qd + ch * C * DP;
+  float* kd = a.kd + ch * DP * C;
   f32x4_t diag = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int dt = 0; dt < NT; ++dt) {
     if (dt >= ndt) continue;
     const int d = dt * 16 + g * 4;
-    f32x4_t q = load4_guard(qrow, d, a.dim, row_ok, vec);
-    f32x4_t k = load4_guard(krow, d, a.dim, row_ok, vec);
-    if constexpr (FG) {
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int hc = h * a.dim + min(d + j, a.dim - 1);
-        float alpha;
-        q[j] = silu(q[j]);
-        const float kk = forget_key(k[j] + a.a2_bias[hc], a.lower[hc],
-                                    &alpha);
-        k[j] = row_ok && d + j < a.dim ? kk : 0.f;
-      }
-    } else {
-#pragma unroll
-      for (int j = 0; j < 4; ++j) q[j] *= qscale;
-    }
-    const f32x4_t Lt = *reinterpret_cast<const f32x4_t*>(L + trow * LR + d);
-    const f32x4_t Lm =
-        *reinterpret_cast<const f32x4_t*>(L + (w * 16 + 7) * LR + d);
     const f32x4_t tw = *reinterpret_cast<const f32x4_t*>(tot + w * DP + d);
-    const f32x4_t BI = *reinterpret_cast<const f32x4_t*>(B + w * DP + d);
-    const f32x4_t BN = *reinterpret_cast<const f32x4_t*>(B + (w + 1) * DP + d);
-    const f32x4_t BC = *reinterpret_cast<const f32x4_t*>(B + 4 * DP + d);
+    const f32x4_t eb = *reinterpret_cast<const f32x4_t*>(EB + w * DP + d);
+    const f32x4_t ed = *reinterpret_cast<const f32x4_t*>(ED + w * DP + d);
     f32x4_t kt, qo;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      qh[dt][j] = q[j] * gexp<T>(Lt[j]);
-      qo[j] = q[j] * gexp<T>(BI[j] + Lt[j]);
-      kt[j] = k[j] * gexp<T>(tw[j] - Lt[j]);
-      kd[int64_t(d + j) * C + trow] = kt[j] * gexp<T>(BC[j] - BN[j]);
-      if (safe)
-        diag = mma4(q[j] * gexp<T>(Lt[j] - Lm[j]),
-                    k[j] * gexp<T>(Lm[j] - Lt[j]), diag);
+      const float Lt = L[dt][j];
+      if (safe) {
+        const float Lm = __shfl(Lt, g * 16 + 7, kWave);
+        diag = mma4(q[dt][j] * gexp<T>(Lt - Lm), k[dt][j] * gexp<T>(Lm - Lt),
+                    diag);
+      }
+      q[dt][j] *= gexp<T>(Lt);
+      qo[j] = q[dt][j] * eb[j];
+      kt[j] = k[dt][j] * gexp<T>(tw[j] - Lt);
+      kd[int64_t(d + j) * C + trow] = kt[j] * ed[j];
     }
     *reinterpret_cast<f32x4_t*>(qd + trow * DP + d) = qo;
-    *reinterpret_cast<f32x4_t*>(L + trow * LR + d) = kt;
+    *reinterpret_cast<f32x4_t*>(kl + trow * LR + d) = kt;
   }
   if (safe) {
 #pragma unroll
@@ -370,17 +408,20 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
   for (int dt = 0; dt < NT; ++dt) {
     if (dt >= ndt) continue;
     const int d = dt * 16 + g * 4;
-    const f32x4_t BI = *reinterpret_cast<const f32x4_t*>(B + w * DP + d);
 #pragma unroll
     for (int J = 0; J < 3; ++J) {
       if (J >= w) break;
-      const f32x4_t BJ =
-          *reinterpret_cast<const f32x4_t*>(B + (J + 1) * DP + d);
-      const f32x4_t kt =
-          *reinterpret_cast<const f32x4_t*>(L + (J * 16 + lr) * LR + d);
+      f32x4_t qe = q[dt];
+      if (J + 1 < w) {
+        const f32x4_t e = *reinterpret_cast<const f32x4_t*>(
+            EJ + (J == 1 ? 2 : w - 2) * DP + d);
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        acc[J] = mma4(qh[dt][j] * gexp<T>(BI[j] - BJ[j]), kt[j], acc[J]);
+        for (int j = 0; j < 4; ++j) qe[j] *= e[j];
+      }
+      const f32x4_t kt =
+          *reinterpret_cast<const f32x4_t*>(kl + (J * 16 + lr) * LR + d);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[J] = mma4(qe[j], kt[j], acc[J]);
     }
   }
   float* sc = a.sc + ch * C * C;
@@ -562,13 +603,13 @@ void gla_scan_kernel(GlaArgs a) {
       }
 }
 
-// one wave per (row, head); V4 float4 columns per lane when the width and
+// GL lanes per (row, head); V4 float4 columns per lane when the width and
 // its offsets allow vectors (V4 = 0: one column at a time)
-template <typename T, bool FG, int V4>
+template <typename T, bool FG, int V4, int GL>
 __global__ __launch_bounds__(256)
 void gla_gate_kernel(GlaArgs a) {
-  const int lane = threadIdx.x & 63;
-  const int64_t rh = int64_t(blockIdx.x) * 4 + (threadIdx.x >> 6);
+  const int lane = threadIdx.x % GL;
+  const int64_t rh = int64_t(blockIdx.x) * (256 / GL) + threadIdx.x / GL;
   if (rh >= int64_t(a.rows) * a.heads) return;
   const int64_t row = rh / a.heads;
   const int h = int(rh % a.heads);
@@ -582,7 +623,7 @@ void gla_gate_kernel(GlaArgs a) {
     f32x4_t ov[V4], gv[V4];
 #pragma unroll
     for (int i = 0; i < V4; ++i) {
-      const int c = (i * 64 + lane) * 4;
+      const int c = (i * GL + lane) * 4;
       ov[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
       if (c < a.vdim) {
         ov[i] = *reinterpret_cast<const f32x4_t*>(o + c);
@@ -591,10 +632,10 @@ void gla_gate_kernel(GlaArgs a) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) ss += ov[i][j] * ov[i][j];
     }
-    const float inv = 1.f / sqrtf(wave_sum(ss) / a.vdim + a.eps);
+    const float inv = 1.f / sqrtf(group_sum<GL>(ss) / a.vdim + a.eps);
 #pragma unroll
     for (int i = 0; i < V4; ++i) {
-      const int c = (i * 64 + lane) * 4;
+      const int c = (i * GL + lane) * 4;
       if (c >= a.vdim) break;
       const f32x4_t nv = *reinterpret_cast<const f32x4_t*>(a.norm + c);
       f32x4_t r;
@@ -606,9 +647,9 @@ void gla_gate_kernel(GlaArgs a) {
       act_store4(out + c, r);
     }
   } else {
-    for (int e = lane; e < a.vdim; e += 64) ss += o[e] * o[e];
-    const float inv = 1.f / sqrtf(wave_sum(ss) / a.vdim + a.eps);
-    for (int e = lane; e < a.vdim; e += 64) {
+    for (int e = lane; e < a.vdim; e += GL) ss += o[e] * o[e];
+    const float inv = 1.f / sqrtf(group_sum<GL>(ss) / a.vdim + a.eps);
+    for (int e = lane; e < a.vdim; e += GL) {
       float r = o[e] * inv * a.norm[e];
       if constexpr (!FG) {
         const float g = act_load(gate + e);
@@ -640,7 +681,7 @@ template <typename T, bool FG>
 void prefill(const GlaArgs& a, hipStream_t st) {
   const bool vec = a.dim % 4 == 0 && a.stride % 4 == 0;
   const size_t smem =
-      size_t(C * (a.dpad + 4) + 9 * a.dpad) * sizeof(float);
+      size_t(C * (a.dpad + 4) + 15 * a.dpad) * sizeof(float);
   auto intra = [&](auto* k) {
     if (smem > 65536)
       (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k),
@@ -659,17 +700,22 @@ void prefill(const GlaArgs& a, hipStream_t st) {
   else if (a.vdim > 16 && sh * ((a.vdim + 31) / 32) >= 1024)
     scan_md<T, 2>(a, st);
   else scan_md<T, 1>(a, st);
-  const dim3 grid(uint32_t((int64_t(a.rows) * a.heads + 3) / 4));
-  auto gate = [&](auto* kg) {
-    hipLaunchKernelGGL(kg, grid, dim3(256), 0, st, a);
+  auto gate = [&](auto* kg, int per_wg = 4) {
+    const int64_t rh = int64_t(a.rows) * a.heads;
+    hipLaunchKernelGGL(kg, dim3(uint32_t((rh + per_wg - 1) / per_wg)),
+                       dim3(256), 0, st, a);
   };
   if (a.vdim % 4 || a.stride % 4 || a.off_g % 4 || a.out_stride % 4 ||
       reinterpret_cast<uintptr_t>(a.out) % 16)
-    gate(gla_gate_kernel<T, FG, 0>);
+    gate(gla_gate_kernel<T, FG, 0, 64>);
+  else if (a.vdim <= 64)
+    gate(gla_gate_kernel<T, FG, 1, 16>, 16);
+  else if (a.vdim <= 128)
+    gate(gla_gate_kernel<T, FG, 1, 32>, 8);
   else if (a.vdim <= 256)
-    gate(gla_gate_kernel<T, FG, 1>);
+    gate(gla_gate_kernel<T, FG, 1, 64>);
   else
-    gate(gla_gate_kernel<T, FG, 4>);
+    gate(gla_gate_kernel<T, FG, 4, 64>);
 }
 
 }  // namespace

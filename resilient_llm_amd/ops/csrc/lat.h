@@ -87,7 +87,8 @@ struct LatentAttnArgs {
   void* out;               // [rows * heads, rank]
   float* part_acc;         // [rows * heads, n_split, rank]
   float* part_ml;          // [rows * heads, n_split, 2]
-  int rows, n_tiles, heads, rank, block_size, max_blocks, n_split;
+  int rows, n_tiles, heads, rank, max_blocks, n_split;
+  int block_shift;         // log2 of the page size
   float scale;
   int cache_kind;
 };

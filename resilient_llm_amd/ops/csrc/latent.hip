@@ -10,7 +10,7 @@
 //   head_linear      y[t,h] = W[h] x[t,h], optionally gated; Uk^T before
 //                    and Uv after the attention
 //   latent_attn      (rows x heads) against the latents, split over keys;
-//                    a 64-token latent tile in LDS is both K and V
+//                    a 32-token latent tile in LDS is both K and V
 //   latent_combine   joins the splits
 //   latent_gather    a sequence's latents as one matrix, for the expanded
 //                    form of long portions (latent_prefill.hip)
@@ -167,7 +167,7 @@ void head_linear_kernel(HeadLinearArgs a, bool vec_w, bool vec_x) {
 }
 
 // ------------------------------------------------------- latent_attn
-constexpr int KT = 64;                    // keys of a tile
+constexpr int KT = 32;                    // keys of a tile
 constexpr int SROW = KT + 4;              // score row in LDS
 
 typedef float f32x2_t __attribute__((ext_vector_type(2)));
@@ -190,20 +190,24 @@ DEV_INLINE uint4 to_bf16x8(const typename KC::vec8& raw) {
   }
 }
 
-// MT tiles of 16 query vectors; a wave scores 16 of a tile's 64 keys and
-// accumulates 16 * NC of the output columns
+// MT tiles of 16 query vectors.  Waves pair up over the tile's two groups
+// of 16 keys to score: both of a pair with half of the rank each (MT = 1,
+// the softmax adds the halves) or with half of the query tiles.  Then every
+// wave weighs all keys and accumulates 16 * NC of the output columns.
 template <int MT, int NC, typename KC>
-__global__ __launch_bounds__(256, MT == 1 ? 2 : 1)
+__global__ __launch_bounds__(256, MT == 4 ? 1 : MT == 1 ? 3 : 2)
 void latent_attn_kernel(LatentAttnArgs a) {
   using vec8 = typename KC::vec8;
   using elem = typename KC::elem;
   constexpr int RP = NC * 64, RS = RP + 8, KS = RP / 32;
   constexpr int PF = KT * RP / 8 / 256;   // vectors a thread stages
-  constexpr bool QREG = MT == 1;
+  constexpr int MW = MT > 1 ? MT / 2 : 1; // query tiles a wave scores
+  constexpr int KW = MT > 1 ? KS : KS / 2;
+  constexpr int SP = MT > 1 ? 1 : 2;      // score parts to add
   extern __shared__ __attribute__((aligned(16))) char smem[];
   uint16_t* cs = reinterpret_cast<uint16_t*>(smem);      // [KT][RS]
-  float* sc = reinterpret_cast<float*>(cs + KT * RS);    // [MT*16][SROW]
-  uint16_t* ql = reinterpret_cast<uint16_t*>(sc + MT * 16 * SROW);
+  float* sc = reinterpret_cast<float*>(cs + KT * RS);    // [SP][MT*16][SROW]
+  uint16_t* ql = reinterpret_cast<uint16_t*>(sc + SP * MT * 16 * SROW);
 
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int lr = lane & 15, g = lane >> 4;
@@ -229,62 +233,32 @@ void latent_attn_kernel(LatentAttnArgs a) {
     return decode ? first : first + (off + i) / a.heads;
   };
   // (a padded graph lane's position may run past its table)
-  const int len = min(qpos(cnt - 1) + 1, a.max_blocks * a.block_size);
+  const int len = min(qpos(cnt - 1) + 1, a.max_blocks << a.block_shift);
   const int32_t* bt = a.block_tables + int64_t(seq) * a.max_blocks;
   const elem* cache = reinterpret_cast<const elem*>(a.cache);
+  const int bmask = (1 << a.block_shift) - 1;
 
-  // queries: fragments in registers (one tile) or rows in LDS
-  const uint16_t* q = reinterpret_cast<const uint16_t*>(a.q);
-  s16x8_t qf[QREG ? KS : 1];
-  if constexpr (QREG) {
-#pragma unroll
-    for (int kk = 0; kk < KS; ++kk) {
-      uint4 raw = {0, 0, 0, 0};
-      const int d = kk * 32 + g * 8;
-      if (lr < cnt && d < a.rank)
-        raw = *reinterpret_cast<const uint4*>(q + (vec0 + lr) * a.rank + d);
-      qf[kk] = *reinterpret_cast<s16x8_t*>(&raw);
-    }
-  } else {
-    for (int e = threadIdx.x; e < MT * 16 * (RP / 8); e += 256) {
-      const int i = e / (RP / 8), d = e % (RP / 8) * 8;
-      uint4 raw = {0, 0, 0, 0};
-      if (i < cnt && d < a.rank)
-        raw = *reinterpret_cast<const uint4*>(q + (vec0 + i) * a.rank + d);
-      *reinterpret_cast<uint4*>(ql + i * RS + d) = raw;
-    }
-  }
-  int qp[MT][4];
-#pragma unroll
-  for (int m = 0; m < MT; ++m)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int i = m * 16 + g * 4 + r;
-      qp[m][r] = i < cnt ? qpos(i) : -1;
-    }
-
-  f32x4_t o[MT][NC];
-  float ms[MT], ls[MT];                   // of row lr of each tile
-#pragma unroll
-  for (int m = 0; m < MT; ++m) {
-#pragma unroll
-    for (int c = 0; c < NC; ++c) o[m][c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    ms[m] = kNegInf;
-    ls[m] = 0.f;
-  }
-
+  // this thread's vectors of a tile; the pages of its two 16-token halves
+  // are looked up a tile ahead
   vec8 pf[PF];
+  int page[2];
+  auto lookup = [&](int t) {
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int p = t * KT + i * 16;
+      page[i] = p < len ? bt[p >> a.block_shift] : 0;
+    }
+  };
   auto fetch = [&](int t) {
 #pragma unroll
     for (int i = 0; i < PF; ++i) {
       const int e = i * 256 + threadIdx.x;
       const int p = t * KT + e / (RP / 8), d = e % (RP / 8) * 8;
       pf[i] = vec8{};
-      if (p < len && d < a.rank) {
-        const int64_t tok =
-            int64_t(bt[p / a.block_size]) * a.block_size + p % a.block_size;
-        pf[i] = *reinterpret_cast<const vec8*>(cache + tok * a.rank + d);
-      }
+      if (p < len && d < a.rank)
+        pf[i] = *reinterpret_cast<const vec8*>(
+            cache + ((int64_t(page[2 * i / PF]) << a.block_shift) +
+                     (p & bmask)) * a.rank + d);
     }
   };
   auto stage = [&]() {
@@ -296,114 +270,154 @@ void latent_attn_kernel(LatentAttnArgs a) {
     }
   };
   int t = split;
-  if (t * KT < len) fetch(t);
+  lookup(t);
+  fetch(t);
+  lookup(t + a.n_split);
+
+  // queries: fragments in registers (one tile) or rows in LDS
+  const uint16_t* q = reinterpret_cast<const uint16_t*>(a.q);
+  const int kg = w & 1, half = w >> 1;    // group of keys, half of the work
+  s16x8_t qf[MT == 1 ? KW : 1];
+  if constexpr (MT == 1) {
+#pragma unroll
+    for (int kk = 0; kk < KW; ++kk) {
+      uint4 raw = {0, 0, 0, 0};
+      const int d = (half * KW + kk) * 32 + g * 8;
+      if (lr < cnt && d < a.rank)
+        raw = *reinterpret_cast<const uint4*>(q + (vec0 + lr) * a.rank + d);
+      qf[kk] = __builtin_bit_cast(s16x8_t, raw);
+    }
+  } else {
+    for (int e = threadIdx.x; e < MT * 16 * (RP / 8); e += 256) {
+      const int i = e / (RP / 8), d = e % (RP / 8) * 8;
+      uint4 raw = {0, 0, 0, 0};
+      if (i < cnt && d < a.rank)
+        raw = *reinterpret_cast<const uint4*>(q + (vec0 + i) * a.rank + d);
+      *reinterpret_cast<uint4*>(ql + i * RS + d) = raw;
+    }
+  }
+  int qp[MT];                             // of row lr of each tile
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+    qp[m] = m * 16 + lr < cnt ? qpos(m * 16 + lr) : -1;
+
+  f32x4_t o[MT][NC];
+  float ms[MT], ls[MT];                   // of row lr of each tile
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+#pragma unroll
+    for (int c = 0; c < NC; ++c) o[m][c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    ms[m] = kNegInf;
+    ls[m] = 0.f;
+  }
+
   for (; t * KT < len; t += a.n_split) {
     __syncthreads();                      // the last tile's readers
     stage();
     __syncthreads();
-    if ((t + a.n_split) * KT < len) fetch(t + a.n_split);
-    f32x4_t s[MT];
+    fetch(t + a.n_split);
+    lookup(t + 2 * a.n_split);
+    f32x4_t s[MW];
 #pragma unroll
-    for (int m = 0; m < MT; ++m) s[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int m = 0; m < MW; ++m) s[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int kk = 0; kk < KS; ++kk) {
+    for (int kk = 0; kk < KW; ++kk) {
+      const int d = ((MT == 1 ? half * KW : 0) + kk) * 32 + g * 8;
       const s16x8_t kf = *reinterpret_cast<const s16x8_t*>(
-          cs + (w * 16 + lr) * RS + kk * 32 + g * 8);
+          cs + (kg * 16 + lr) * RS + d);
 #pragma unroll
-      for (int m = 0; m < MT; ++m) {
+      for (int m = 0; m < MW; ++m) {
         s16x8_t qm;
-        if constexpr (QREG) qm = qf[kk];
+        if constexpr (MT == 1) qm = qf[kk];
         else qm = *reinterpret_cast<const s16x8_t*>(
-            ql + (m * 16 + lr) * RS + kk * 32 + g * 8);
+            ql + ((half * MW + m) * 16 + lr) * RS + d);
         s[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qm, kf, s[m], 0, 0, 0);
       }
     }
-    const int key = t * KT + w * 16 + lr;
 #pragma unroll
-    for (int m = 0; m < MT; ++m)
+    for (int m = 0; m < MW; ++m) {
+      const int row = MT == 1 ? half * 16 : (half * MW + m) * 16;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        sc[(m * 16 + g * 4 + r) * SROW + w * 16 + lr] =
-            key <= qp[m][r] ? s[m][r] * a.scale : kNegInf;
+        sc[(row + g * 4 + r) * SROW + kg * 16 + lr] = s[m][r];
+    }
     __syncthreads();
-    // every wave weighs all keys: row lr, keys kb * 32 + g * 8 + j
-    s16x8_t pw[MT][2];
+    s16x8_t pw[MT];                       // row lr, keys g * 8 + j
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
-      float p[16], mx = kNegInf;
+      float p[8], mx = kNegInf;
 #pragma unroll
-      for (int kb = 0; kb < 2; ++kb)
+      for (int j = 0; j < 8; j += 4) {
+        f32x4_t v = *reinterpret_cast<const f32x4_t*>(
+            sc + (m * 16 + lr) * SROW + g * 8 + j);
+        if constexpr (SP == 2) {
+          const f32x4_t u = *reinterpret_cast<const f32x4_t*>(
+              sc + (16 + lr) * SROW + g * 8 + j);
 #pragma unroll
-        for (int j = 0; j < 8; j += 4) {
-          const f32x4_t v = *reinterpret_cast<const f32x4_t*>(
-              sc + (m * 16 + lr) * SROW + kb * 32 + g * 8 + j);
-#pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            p[kb * 8 + j + i] = v[i];
-            mx = fmaxf(mx, v[i]);
-          }
+          for (int i = 0; i < 4; ++i) v[i] += u[i];
         }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          p[j + i] = t * KT + g * 8 + j + i <= qp[m] ? v[i] * a.scale
+                                                     : kNegInf;
+          mx = fmaxf(mx, p[j + i]);
+        }
+      }
       mx = fmaxf(mx, __shfl_xor(mx, 16, kWave));
       mx = fmaxf(mx, __shfl_xor(mx, 32, kWave));
       const float mn = fmaxf(ms[m], mx);
       const float corr = __expf(ms[m] - mn);
       float sum = 0.f;
 #pragma unroll
-      for (int i = 0; i < 16; ++i) {
+      for (int i = 0; i < 8; ++i) {
         p[i] = __expf(p[i] - mn);
         sum += p[i];
       }
       sum += __shfl_xor(sum, 16, kWave);
       sum += __shfl_xor(sum, 32, kWave);
       ls[m] = ls[m] * corr + sum;
-      ms[m] = mn;
+      const uint4 raw = {pack2(p[0], p[1]), pack2(p[2], p[3]),
+                         pack2(p[4], p[5]), pack2(p[6], p[7])};
+      pw[m] = __builtin_bit_cast(s16x8_t, raw);
+      if (!__all(mn == ms[m])) {
+        ms[m] = mn;
+        float cr[4];
 #pragma unroll
-      for (int kb = 0; kb < 2; ++kb) {
-        const uint4 raw = {pack2(p[kb * 8], p[kb * 8 + 1]),
-                           pack2(p[kb * 8 + 2], p[kb * 8 + 3]),
-                           pack2(p[kb * 8 + 4], p[kb * 8 + 5]),
-                           pack2(p[kb * 8 + 6], p[kb * 8 + 7])};
-        pw[m][kb] = __builtin_bit_cast(s16x8_t, raw);
+        for (int r = 0; r < 4; ++r) cr[r] = __shfl(corr, g * 4 + r, kWave);
+#pragma unroll
+        for (int c = 0; c < NC; ++c)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) o[m][c][r] *= cr[r];
       }
-      float cr[4];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) cr[r] = __shfl(corr, g * 4 + r, kWave);
-#pragma unroll
-      for (int c = 0; c < NC; ++c)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) o[m][c][r] *= cr[r];
     }
     // columns in pairs: a dword of a row holds two of them, so eight rows'
     // dwords make the fragments of the even and of the odd columns
 #pragma unroll
-    for (int kb = 0; kb < 2; ++kb)
+    for (int cp = 0; cp < NC / 2; ++cp) {
+      uint32_t d[8];
 #pragma unroll
-      for (int cp = 0; cp < NC / 2; ++cp) {
-        uint32_t d[8];
+      for (int j = 0; j < 8; ++j)
+        d[j] = *reinterpret_cast<const uint32_t*>(
+            cs + (g * 8 + j) * RS + w * NC * 16 + cp * 32 + lr * 2);
+      uint4 ev, od;
+      ev.x = __builtin_amdgcn_perm(d[1], d[0], 0x05040100);
+      ev.y = __builtin_amdgcn_perm(d[3], d[2], 0x05040100);
+      ev.z = __builtin_amdgcn_perm(d[5], d[4], 0x05040100);
+      ev.w = __builtin_amdgcn_perm(d[7], d[6], 0x05040100);
+      od.x = __builtin_amdgcn_perm(d[1], d[0], 0x07060302);
+      od.y = __builtin_amdgcn_perm(d[3], d[2], 0x07060302);
+      od.z = __builtin_amdgcn_perm(d[5], d[4], 0x07060302);
+      od.w = __builtin_amdgcn_perm(d[7], d[6], 0x07060302);
+      const s16x8_t fe = __builtin_bit_cast(s16x8_t, ev);
+      const s16x8_t fo = __builtin_bit_cast(s16x8_t, od);
 #pragma unroll
-        for (int j = 0; j < 8; ++j)
-          d[j] = *reinterpret_cast<const uint32_t*>(
-              cs + (kb * 32 + g * 8 + j) * RS + w * NC * 16 + cp * 32 +
-              lr * 2);
-        uint4 ev, od;
-        ev.x = __builtin_amdgcn_perm(d[1], d[0], 0x05040100);
-        ev.y = __builtin_amdgcn_perm(d[3], d[2], 0x05040100);
-        ev.z = __builtin_amdgcn_perm(d[5], d[4], 0x05040100);
-        ev.w = __builtin_amdgcn_perm(d[7], d[6], 0x05040100);
-        od.x = __builtin_amdgcn_perm(d[1], d[0], 0x07060302);
-        od.y = __builtin_amdgcn_perm(d[3], d[2], 0x07060302);
-        od.z = __builtin_amdgcn_perm(d[5], d[4], 0x07060302);
-        od.w = __builtin_amdgcn_perm(d[7], d[6], 0x07060302);
-        const s16x8_t fe = __builtin_bit_cast(s16x8_t, ev);
-        const s16x8_t fo = __builtin_bit_cast(s16x8_t, od);
-#pragma unroll
-        for (int m = 0; m < MT; ++m) {
-          o[m][2 * cp] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              pw[m][kb], fe, o[m][2 * cp], 0, 0, 0);
-          o[m][2 * cp + 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              pw[m][kb], fo, o[m][2 * cp + 1], 0, 0, 0);
-        }
+      for (int m = 0; m < MT; ++m) {
+        o[m][2 * cp] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            pw[m], fe, o[m][2 * cp], 0, 0, 0);
+        o[m][2 * cp + 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            pw[m], fo, o[m][2 * cp + 1], 0, 0, 0);
       }
+    }
   }
 
 #pragma unroll
@@ -495,7 +509,8 @@ void latent_gather_kernel(GatherArgs a) {
 template <int MT, int NC, typename KC>
 void attn(const LatentAttnArgs& a, hipStream_t st) {
   constexpr int RS = NC * 64 + 8;
-  constexpr size_t smem = size_t(KT) * RS * 2 + MT * 16 * SROW * 4 +
+  constexpr size_t smem = size_t(KT) * RS * 2 +
+                          (MT > 1 ? MT : 2) * 16 * SROW * 4 +
                           (MT > 1 ? size_t(MT) * 16 * RS * 2 : 0);
   auto* k = latent_attn_kernel<MT, NC, KC>;
   if (smem > 65536)
@@ -576,7 +591,8 @@ void launch_head_linear(const HeadLinearArgs& a, hipStream_t st) {
 }
 
 bool latent_fast_ok(int rank, int block_size, bool f32) {
-  return !f32 && rank % 8 == 0 && rank <= 512 && block_size >= 1;
+  return !f32 && rank % 8 == 0 && rank <= 512 && block_size >= 16 &&
+         (block_size & (block_size - 1)) == 0;
 }
 
 int latent_tile(int heads, bool decode) {
