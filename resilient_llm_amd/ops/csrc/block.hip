@@ -39,8 +39,9 @@ DEV_INLINE void store_v(T* p, const float (&in)[V]) {
   else act_store(p, in[0]);
 }
 
-// IT vectors of V columns per thread; IT = 0 walks the row twice
-template <typename T, int WAVES, int IT, int V, bool EMBED>
+// IT vectors of V columns per thread; IT = 0 walks the row twice.  CONV:
+// there are decoded rows, which also convolve
+template <typename T, int WAVES, int IT, int V, bool EMBED, bool CONV>
 __global__ __launch_bounds__(WAVES * 64)
 void block_step_kernel(BlockArgs a) {
   extern __shared__ float sq[];           // [width / V] squares, [groups]
@@ -78,7 +79,7 @@ void block_step_kernel(BlockArgs a) {
   // memory latency covers it; long convolutions and the plain walk load
   // the rest late
   constexpr int ITS = IT > 0 ? IT : 1;
-  constexpr int EARLY = IT == 1 || IT == 2 ? 4 : 0;      // taps
+  constexpr int EARLY = CONV && (IT == 1 || IT == 2) ? 4 : 0;   // taps
   float u[ITS][V], t[ITS][V], gain[ITS][V];
   float tap[ITS][EARLY + 1][V], past[ITS][EARLY + 1][V];
   auto every = [&](auto body) {           // over this thread's vectors
@@ -90,7 +91,7 @@ void block_step_kernel(BlockArgs a) {
       for (int v = threadIdx.x; v < nv; v += NT) body(v, 0);
     }
   };
-  const bool conv = a.hc && n < a.n_decode;
+  const bool conv = CONV && n < a.n_decode;
   const int back = a.n_taps - 1;          // earlier inputs in the ring
   auto load_tap = [&](int k, int c, float (&w)[V]) {
     load_v<float, V>(a.taps + int64_t(back - k) * W + c, w);
@@ -300,24 +301,30 @@ void gate_act_kernel(const T* __restrict__ gu, T* __restrict__ out, int ff,
   }
 }
 
-template <typename T, bool EMBED>
+template <typename T, bool EMBED, bool CONV>
 void step(const BlockArgs& a, hipStream_t st) {
   auto run = [&](auto* k, int threads, int v) {
     hipLaunchKernelGGL(k, dim3(a.n), dim3(threads),
                        (a.width / v + a.groups) * sizeof(float), st, a);
   };
   if (a.width / a.groups % 4 || a.width > 8192)
-    run(block_step_kernel<T, 4, 0, 1, EMBED>, 256, 1);
+    run(block_step_kernel<T, 4, 0, 1, EMBED, CONV>, 256, 1);
   else if (a.width <= 256)
-    run(block_step_kernel<T, 1, 1, 4, EMBED>, 64, 4);
+    run(block_step_kernel<T, 1, 1, 4, EMBED, CONV>, 64, 4);
   else if (a.width <= 1024)
-    run(block_step_kernel<T, 4, 1, 4, EMBED>, 256, 4);
+    run(block_step_kernel<T, 4, 1, 4, EMBED, CONV>, 256, 4);
   else if (a.width <= 2048)
-    run(block_step_kernel<T, 4, 2, 4, EMBED>, 256, 4);
+    run(block_step_kernel<T, 4, 2, 4, EMBED, CONV>, 256, 4);
   else if (a.width <= 4096)
-    run(block_step_kernel<T, 8, 2, 4, EMBED>, 512, 4);
+    run(block_step_kernel<T, 8, 2, 4, EMBED, CONV>, 512, 4);
   else
-    run(block_step_kernel<T, 8, 4, 4, EMBED>, 512, 4);
+    run(block_step_kernel<T, 8, 4, 4, EMBED, CONV>, 512, 4);
+}
+
+template <typename T, bool EMBED>
+void step(const BlockArgs& a, hipStream_t st) {
+  if (a.hc && a.n_decode) step<T, EMBED, true>(a, st);
+  else step<T, EMBED, false>(a, st);
 }
 
 template <typename T>

@@ -215,18 +215,18 @@ void gla_decode_kernel(GlaArgs a) {
 // columns of every 16; MD bounds the key tiles (dpad <= 64 * MD).
 template <typename T, bool FG, int MD>
 __global__ __launch_bounds__(256)
-void gla_intra_kernel(GlaArgs a, bool vec) {
+void gla_intra_kernel(GlaArgs a, bool vec, bool vec_a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   constexpr int NT = 4 * MD;
   const int tile = blockIdx.x, h = blockIdx.y;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int lr = lane & 15, g = lane >> 4;
   const int DP = a.dpad, LR = DP + 4, ndt = DP / 16;
-  float* kl = sm;                        // [64][LR] decayed keys
+  float* kl = sm;                        // [64][LR] keys, then decayed keys
   float* tot = kl + C * LR;              // [4][DP] log-decays of sub-chunks
-  float* EB = tot + 4 * DP;              // [4][DP] e^{B_w}
-  float* ED = EB + 4 * DP;               // [4][DP] e^{B_4 - B_{w+1}}
-  float* EJ = ED + 4 * DP;               // [3][DP] sub-chunks in between
+  float* EB = tot + 4 * DP;              // [3][DP] e^{B_w}, w = 1 .. 3
+  float* ED = EB + 3 * DP;               // [3][DP] e^{B_4 - B_{w+1}}, w < 3
+  float* EJ = ED + 3 * DP;               // [3][DP] sub-chunks in between
   const int row0 = a.tiles[tile];
   const int n = a.tiles[2 * a.n_tiles + tile];
   const int trow = w * 16 + lr;          // this lane's row
@@ -238,20 +238,22 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
   const float* low = FG ? a.lower + h * a.dim : nullptr;
   const float qscale = 1.f / sqrtf(float(a.dim));
 
-  // queries, keys and the running log-decay, all in registers
-  f32x4_t q[NT], k[NT], L[NT];
+  // queries and the running log-decay stay in registers, keys in LDS
+  f32x4_t q[NT], L[NT];
   float wmin = 0.f;
+  // (raw keys wait in the registers of the log-decays)
 #pragma unroll
   for (int dt = 0; dt < NT; ++dt) {
     if (dt >= ndt) continue;
     const int d = dt * 16 + g * 4;
     q[dt] = load4_guard(qrow, d, a.dim, row_ok, vec);
-    k[dt] = load4_guard(krow, d, a.dim, row_ok, vec);
+    L[dt] = load4_guard(krow, d, a.dim, row_ok, vec);
   }
 #pragma unroll
   for (int dt = 0; dt < NT; ++dt) {
     if (dt >= ndt) continue;
     const int d = dt * 16 + g * 4;
+    f32x4_t k = L[dt];
     const f32x4_t bv = load4_guard(bias, d, a.dim, true, a.dim % 4 == 0);
     if constexpr (FG) {
       const f32x4_t lv = load4_guard(low, d, a.dim, true, a.dim % 4 == 0);
@@ -259,8 +261,8 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
       for (int j = 0; j < 4; ++j) {
         const bool ok = row_ok && d + j < a.dim;
         float alpha;
-        const float kk = forget_key<T>(k[dt][j] + bv[j], lv[j], &alpha);
-        k[dt][j] = ok ? kk : 0.f;
+        const float kk = forget_key<T>(k[j] + bv[j], lv[j], &alpha);
+        k[j] = ok ? kk : 0.f;
         L[dt][j] = ok ? log_forget<T>(alpha, kk) : 0.f;
         q[dt][j] = silu<T>(q[dt][j]);
       }
@@ -271,9 +273,9 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
       const T* a2 = reinterpret_cast<const T*>(a.a2) +
                     int64_t(h * a.dim + dt * 16 + lr) * a.rank;
       for (int k0 = 0; k0 < a.rank; k0 += 16) {
-        const f32x4_t av = load4_guard(a1, k0 + g * 4, a.rank, row_ok, false);
+        const f32x4_t av = load4_guard(a1, k0 + g * 4, a.rank, row_ok, vec_a);
         const f32x4_t wv = load4_guard(a2, k0 + g * 4, a.rank,
-                                       dt * 16 + lr < a.dim, false);
+                                       dt * 16 + lr < a.dim, vec_a);
 #pragma unroll
         for (int j = 0; j < 4; ++j) z = mma4(wv[j], av[j], z);
       }
@@ -284,6 +286,7 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
         q[dt][j] *= qscale;
       }
     }
+    *reinterpret_cast<f32x4_t*>(kl + trow * LR + d) = k;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       L[dt][j] = row_prefix(L[dt][j]);
@@ -301,14 +304,14 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
 #pragma unroll
     for (int s = 0; s < 4; ++s) {
       t[s] = tot[s * DP + d];
-      EB[s * DP + d] = gexp<T>(b);
+      if (s > 0) EB[(s - 1) * DP + d] = gexp<T>(b);
       b += t[s];
     }
     a.dec[(int64_t(tile) * a.heads + h) * DP + d] = expf(b);
     float after = 0.f;
 #pragma unroll
     for (int s = 3; s >= 0; --s) {
-      ED[s * DP + d] = gexp<T>(after);
+      if (s < 3) ED[s * DP + d] = gexp<T>(after);
       after += t[s];
     }
     EJ[d] = gexp<T>(t[1]);                // from 0 to 2
@@ -327,9 +330,11 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
 #pragma unroll
     for (int dt = 0; dt < NT; ++dt) {
       if (dt >= ndt) continue;
+      const f32x4_t k = *reinterpret_cast<const f32x4_t*>(
+          kl + trow * LR + dt * 16 + g * 4);
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        const float Lt = L[dt][j], qv = q[dt][j], kv = k[dt][j];
+        const float Lt = L[dt][j], qv = q[dt][j], kv = k[j];
         float ref[4];
 #pragma unroll
         for (int b = 1; b < 4; ++b)
@@ -378,20 +383,21 @@ void gla_intra_kernel(GlaArgs a, bool vec) {
     if (dt >= ndt) continue;
     const int d = dt * 16 + g * 4;
     const f32x4_t tw = *reinterpret_cast<const f32x4_t*>(tot + w * DP + d);
-    const f32x4_t eb = *reinterpret_cast<const f32x4_t*>(EB + w * DP + d);
-    const f32x4_t ed = *reinterpret_cast<const f32x4_t*>(ED + w * DP + d);
-    f32x4_t kt, qo;
+    f32x4_t eb = f32x4_t{1.f, 1.f, 1.f, 1.f}, ed = eb;
+    if (w > 0) eb = *reinterpret_cast<const f32x4_t*>(EB + (w - 1) * DP + d);
+    if (w < 3) ed = *reinterpret_cast<const f32x4_t*>(ED + w * DP + d);
+    f32x4_t kt = *reinterpret_cast<const f32x4_t*>(kl + trow * LR + d), qo;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const float Lt = L[dt][j];
       if (safe) {
         const float Lm = __shfl(Lt, g * 16 + 7, kWave);
-        diag = mma4(q[dt][j] * gexp<T>(Lt - Lm), k[dt][j] * gexp<T>(Lm - Lt),
+        diag = mma4(q[dt][j] * gexp<T>(Lt - Lm), kt[j] * gexp<T>(Lm - Lt),
                     diag);
       }
       q[dt][j] *= gexp<T>(Lt);
       qo[j] = q[dt][j] * eb[j];
-      kt[j] = k[dt][j] * gexp<T>(tw[j] - Lt);
+      kt[j] *= gexp<T>(tw[j] - Lt);
       kd[int64_t(d + j) * C + trow] = kt[j] * ed[j];
     }
     *reinterpret_cast<f32x4_t*>(qd + trow * DP + d) = qo;
@@ -680,15 +686,16 @@ void scan_md(const GlaArgs& a, hipStream_t st) {
 template <typename T, bool FG>
 void prefill(const GlaArgs& a, hipStream_t st) {
   const bool vec = a.dim % 4 == 0 && a.stride % 4 == 0;
+  const bool vec_a = a.rank % 4 == 0 && a.off_a % 4 == 0 && a.stride % 4 == 0;
   const size_t smem =
-      size_t(C * (a.dpad + 4) + 15 * a.dpad) * sizeof(float);
+      size_t(C * (a.dpad + 4) + 13 * a.dpad) * sizeof(float);
   auto intra = [&](auto* k) {
     if (smem > 65536)
       (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k),
                                 hipFuncAttributeMaxDynamicSharedMemorySize,
                                 int(smem));
     hipLaunchKernelGGL(k, dim3(a.n_tiles, a.heads), dim3(256), smem, st, a,
-                       vec);
+                       vec, vec_a);
   };
   if (a.dpad <= 64) intra(gla_intra_kernel<T, FG, 1>);
   else if (a.dpad <= 128) intra(gla_intra_kernel<T, FG, 2>);
