@@ -404,6 +404,7 @@ def moe_experts(h, router, w_up, w_down, top: int, limit: float):
 
 # ------------------------------------------- parallel blocks, latents
 CONV_SPAN = 16        # prompt rows that one convolution workgroup walks
+LATENT_VECTORS = 32   # (row, head) queries of one absorbed prompt tile
 
 
 def block_embed(ids, table, pos_table, positions, x, gain, groups: int,
@@ -501,7 +502,7 @@ def latent_prefill(q, gate, cache, block_tables, prompt, scale: float, w_uk,
         ns.expanded_attn(q, k, vt, gate, prompt.tiles(128), kv_off, heads,
                          scale, out)
         return out
-    tiles = prompt.vectors(64, heads) if fast else prompt.tiles(32)
+    tiles = prompt.vectors(LATENT_VECTORS, heads) if fast else prompt.tiles(32)
     c = ns.latent_attn(head_linear(q, w_uk), cache, block_tables, scale,
                        heads, None, tiles, prompt.pos0())
     return head_linear(c, w_uv, gate, out)

@@ -305,10 +305,8 @@ Tensor latent_attn(const Tensor& q, const Tensor& cache,
   }
   // enough workgroups for the chip, at least 128 keys each
   const int64_t most = int64_t(a.max_blocks) * block / 128;
-  const int64_t aim =
-      rlli::latent_tile(a.heads, tiles == std::nullopt) <= 32 ? 512 : 256;
   a.n_split = int(std::max<int64_t>(
-      1, std::min<int64_t>({32, most, (aim + wgs - 1) /
+      1, std::min<int64_t>({32, most, (512 + wgs - 1) /
                                           std::max<int64_t>(wgs, 1)})));
   Tensor pa, pm;
   if (a.n_split > 1) {

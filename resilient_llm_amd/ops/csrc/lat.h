@@ -93,7 +93,8 @@ struct LatentAttnArgs {
   int cache_kind;
 };
 bool latent_fast_ok(int rank, int block_size, bool f32);
-// query vectors of one workgroup
+// query vectors of one workgroup; a prompt's tile has kLatentVectors
+constexpr int kLatentVectors = 32;
 int latent_tile(int heads, bool decode);
 void launch_latent_attn(const LatentAttnArgs& a, hipStream_t stream);
 void launch_latent_rows(const WindowAttnArgs& a, bool decode,

@@ -190,24 +190,22 @@ DEV_INLINE uint4 to_bf16x8(const typename KC::vec8& raw) {
   }
 }
 
-// MT tiles of 16 query vectors.  Waves pair up over the tile's two groups
-// of 16 keys to score: both of a pair with half of the rank each (MT = 1,
-// the softmax adds the halves) or with half of the query tiles.  Then every
-// wave weighs all keys and accumulates 16 * NC of the output columns.
+// MT (1 or 2) tiles of 16 query vectors.  Waves pair up over the tile's two
+// groups of 16 keys to score: with half of the rank each (MT = 1, the
+// softmax adds the halves) or with a query tile each.  Then every wave
+// weighs all keys and accumulates 16 * NC of the output columns.
 template <int MT, int NC, typename KC>
-__global__ __launch_bounds__(256, MT == 4 ? 1 : MT == 1 ? 3 : 2)
+__global__ __launch_bounds__(256, MT == 1 ? 3 : 2)
 void latent_attn_kernel(LatentAttnArgs a) {
   using vec8 = typename KC::vec8;
   using elem = typename KC::elem;
   constexpr int RP = NC * 64, RS = RP + 8, KS = RP / 32;
   constexpr int PF = KT * RP / 8 / 256;   // vectors a thread stages
-  constexpr int MW = MT > 1 ? MT / 2 : 1; // query tiles a wave scores
   constexpr int KW = MT > 1 ? KS : KS / 2;
   constexpr int SP = MT > 1 ? 1 : 2;      // score parts to add
   extern __shared__ __attribute__((aligned(16))) char smem[];
   uint16_t* cs = reinterpret_cast<uint16_t*>(smem);      // [KT][RS]
-  float* sc = reinterpret_cast<float*>(cs + KT * RS);    // [SP][MT*16][SROW]
-  uint16_t* ql = reinterpret_cast<uint16_t*>(sc + SP * MT * 16 * SROW);
+  float* sc = reinterpret_cast<float*>(cs + KT * RS);    // [32][SROW]
 
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int lr = lane & 15, g = lane >> 4;
@@ -274,27 +272,19 @@ void latent_attn_kernel(LatentAttnArgs a) {
   fetch(t);
   lookup(t + a.n_split);
 
-  // queries: fragments in registers (one tile) or rows in LDS
+  // this wave's queries, as fragments in registers
   const uint16_t* q = reinterpret_cast<const uint16_t*>(a.q);
   const int kg = w & 1, half = w >> 1;    // group of keys, half of the work
-  s16x8_t qf[MT == 1 ? KW : 1];
-  if constexpr (MT == 1) {
+  const int q0 = MT == 1 ? 0 : half * 16, d0 = MT == 1 ? half * KW * 32 : 0;
+  s16x8_t qf[KW];
 #pragma unroll
-    for (int kk = 0; kk < KW; ++kk) {
-      uint4 raw = {0, 0, 0, 0};
-      const int d = (half * KW + kk) * 32 + g * 8;
-      if (lr < cnt && d < a.rank)
-        raw = *reinterpret_cast<const uint4*>(q + (vec0 + lr) * a.rank + d);
-      qf[kk] = __builtin_bit_cast(s16x8_t, raw);
-    }
-  } else {
-    for (int e = threadIdx.x; e < MT * 16 * (RP / 8); e += 256) {
-      const int i = e / (RP / 8), d = e % (RP / 8) * 8;
-      uint4 raw = {0, 0, 0, 0};
-      if (i < cnt && d < a.rank)
-        raw = *reinterpret_cast<const uint4*>(q + (vec0 + i) * a.rank + d);
-      *reinterpret_cast<uint4*>(ql + i * RS + d) = raw;
-    }
+  for (int kk = 0; kk < KW; ++kk) {
+    uint4 raw = {0, 0, 0, 0};
+    const int d = d0 + kk * 32 + g * 8;
+    if (q0 + lr < cnt && d < a.rank)
+      raw = *reinterpret_cast<const uint4*>(q + (vec0 + q0 + lr) * a.rank +
+                                            d);
+    qf[kk] = __builtin_bit_cast(s16x8_t, raw);
   }
   int qp[MT];                             // of row lr of each tile
 #pragma unroll
@@ -317,30 +307,16 @@ void latent_attn_kernel(LatentAttnArgs a) {
     __syncthreads();
     fetch(t + a.n_split);
     lookup(t + 2 * a.n_split);
-    f32x4_t s[MW];
-#pragma unroll
-    for (int m = 0; m < MW; ++m) s[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    f32x4_t s = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int kk = 0; kk < KW; ++kk) {
-      const int d = ((MT == 1 ? half * KW : 0) + kk) * 32 + g * 8;
       const s16x8_t kf = *reinterpret_cast<const s16x8_t*>(
-          cs + (kg * 16 + lr) * RS + d);
-#pragma unroll
-      for (int m = 0; m < MW; ++m) {
-        s16x8_t qm;
-        if constexpr (MT == 1) qm = qf[kk];
-        else qm = *reinterpret_cast<const s16x8_t*>(
-            ql + ((half * MW + m) * 16 + lr) * RS + d);
-        s[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qm, kf, s[m], 0, 0, 0);
-      }
+          cs + (kg * 16 + lr) * RS + d0 + kk * 32 + g * 8);
+      s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[kk], kf, s, 0, 0, 0);
     }
 #pragma unroll
-    for (int m = 0; m < MW; ++m) {
-      const int row = MT == 1 ? half * 16 : (half * MW + m) * 16;
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        sc[(row + g * 4 + r) * SROW + kg * 16 + lr] = s[m][r];
-    }
+    for (int r = 0; r < 4; ++r)
+      sc[(half * 16 + g * 4 + r) * SROW + kg * 16 + lr] = s[r];
     __syncthreads();
     s16x8_t pw[MT];                       // row lr, keys g * 8 + j
 #pragma unroll
@@ -509,14 +485,8 @@ void latent_gather_kernel(GatherArgs a) {
 template <int MT, int NC, typename KC>
 void attn(const LatentAttnArgs& a, hipStream_t st) {
   constexpr int RS = NC * 64 + 8;
-  constexpr size_t smem = size_t(KT) * RS * 2 +
-                          (MT > 1 ? MT : 2) * 16 * SROW * 4 +
-                          (MT > 1 ? size_t(MT) * 16 * RS * 2 : 0);
+  constexpr size_t smem = size_t(KT) * RS * 2 + 32 * SROW * 4;
   auto* k = latent_attn_kernel<MT, NC, KC>;
-  if (smem > 65536)
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k),
-                              hipFuncAttributeMaxDynamicSharedMemorySize,
-                              int(smem));
   const dim3 grid = a.tiles ? dim3(a.n_split, a.n_tiles, 1)
                             : dim3(a.n_split,
                                    (a.heads + MT * 16 - 1) / (MT * 16),
@@ -534,11 +504,8 @@ void attn_rank(const LatentAttnArgs& a, hipStream_t st) {
 
 template <typename KC>
 void attn_tile(const LatentAttnArgs& a, hipStream_t st) {
-  switch (latent_tile(a.heads, a.tiles == nullptr)) {
-    case 16: attn_rank<1, KC>(a, st); break;
-    case 32: attn_rank<2, KC>(a, st); break;
-    default: attn_rank<4, KC>(a, st); break;
-  }
+  if (latent_tile(a.heads, a.tiles == nullptr) == 16) attn_rank<1, KC>(a, st);
+  else attn_rank<2, KC>(a, st);
 }
 
 template <typename T, int KS>
@@ -596,7 +563,7 @@ bool latent_fast_ok(int rank, int block_size, bool f32) {
 }
 
 int latent_tile(int heads, bool decode) {
-  return !decode ? 64 : heads <= 16 ? 16 : heads <= 32 ? 32 : 64;
+  return decode && heads <= 16 ? 16 : kLatentVectors;
 }
 
 void launch_latent_attn(const LatentAttnArgs& a, hipStream_t st) {
