@@ -468,8 +468,9 @@ void latent_gather_kernel(GatherArgs a) {
       reinterpret_cast<const typename KC::elem*>(a.cache);
   uint16_t* out = reinterpret_cast<uint16_t*>(a.out);
   const int nv = a.rank / 8;
-  for (int e = threadIdx.x; e < kGatherRows * nv; e += 256) {
-    const int r = e / nv, d = e % nv * 8;
+  constexpr int kPart = kGatherRows / 8;  // rows of one workgroup
+  for (int e = threadIdx.x; e < kPart * nv; e += 256) {
+    const int r = blockIdx.y * kPart + e / nv, d = e % nv * 8;
     uint4 v = {0, 0, 0, 0};               // rows past the end are zeros
     if (r < cnt) {
       const int p = tok0 + r;
@@ -586,11 +587,11 @@ void launch_latent_rows(const WindowAttnArgs& a, bool decode,
 void launch_latent_gather(const GatherArgs& a, hipStream_t st) {
   if (a.n == 0) return;
   if (a.cache_kind == kCacheFP8)
-    hipLaunchKernelGGL(latent_gather_kernel<CacheFP8>, dim3(a.n), dim3(256),
-                       0, st, a);
+    hipLaunchKernelGGL(latent_gather_kernel<CacheFP8>, dim3(a.n, 8),
+                       dim3(256), 0, st, a);
   else
-    hipLaunchKernelGGL(latent_gather_kernel<CacheBF16>, dim3(a.n), dim3(256),
-                       0, st, a);
+    hipLaunchKernelGGL(latent_gather_kernel<CacheBF16>, dim3(a.n, 8),
+                       dim3(256), 0, st, a);
 }
 
 }  // namespace rlli
