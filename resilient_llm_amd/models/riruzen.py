@@ -4,8 +4,8 @@ Every layer reads one grouped norm h of the residual; its mixer works on
 h + conv(h), a short causal convolution, its feed-forward on h, and both
 are added.  Mixers, in any order: latent attention without positions (one
 normed latent per token is all it caches, queries through a latent of
-their own, sigmoid output gate) and HGRN2 (a linear recurrence whose forget
-gate also decides what is written).  Learned positions are added to the
+their own, sigmoid output gate) and HGRN2 (a linear recurrence without keys:
+a channel takes up as much as it lets go).  Learned positions are added to the
 embedding; the output layer is the embedding.  Sizes, constants and the
 order of layers come from config.json.
 
