@@ -201,7 +201,7 @@ class NesizenForCausalLM(MixedModel):
     the dense and expert widths column-wise, output projections row-wise,
     with an all-reduce after each sublayer; streams are replicated."""
 
-    EXTENSIONS = ("rlli_mix", "rlli_rec")
+    EXTENSIONS = ("rlli_attn", "rlli_mix", "rlli_rec")
 
     def sharded_sizes(self) -> list:
         sizes = []

@@ -172,7 +172,7 @@ class RiruzenForCausalLM(MixedModel):
     per layer; latents, norms, convolutions and the residual are
     replicated."""
 
-    EXTENSIONS = ("rlli_rec", "rlli_lat")
+    EXTENSIONS = ("rlli_attn", "rlli_blk", "rlli_rec", "rlli_lat")
 
     def sharded_sizes(self) -> list:
         return [s for spec in self.config.layers for s in

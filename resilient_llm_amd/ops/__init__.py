@@ -277,14 +277,13 @@ build_cos_sin = ref.build_cos_sin
 
 
 # ----------------------------------------------- mixed-layer model ops
-# f32 or bf16 activations.  The GPU side is torch.ops.rlli_mix (residual
-# streams, windowed attention with kept tokens and a sink, mixture of
-# experts), rlli_rec (gated linear recurrences) and rlli_lat (parallel
-# blocks, latent attention); the CPU side ref_mix.py and ref_lat.py.
-from . import ref_lat, ref_mix  # noqa: E402
-from .ref_mix import GLA_CHUNK  # noqa: E402,F401
+# f32 or bf16 activations.  On the GPU one namespace per kernel library
+# (build.py), on the CPU one ref_*.py each.
+from . import ref_attn, ref_blk, ref_lat, ref_mix, ref_rec  # noqa: E402
+from .ref_rec import REC_CHUNK  # noqa: E402
 
-_CPU_FORMS = {"rlli_mix": ref_mix, "rlli_rec": ref_mix, "rlli_lat": ref_lat}
+_CPU_FORMS = {"rlli_attn": ref_attn, "rlli_mix": ref_mix,
+              "rlli_blk": ref_blk, "rlli_rec": ref_rec, "rlli_lat": ref_lat}
 
 
 def _ns(lib: str, t: torch.Tensor):
@@ -329,23 +328,74 @@ def window_prefill(qkv, k_cache, v_cache, positions, cos_sin, slots,
                    block_tables, prompt, sink, scale: float, n_q: int,
                    window: int, keep_first: int, has_kv: bool):
     """Prompt rows: rotate, append to the cache (``has_kv``), attend."""
-    if qkv.is_cuda:
-        h = window_tile_rows(n_q // k_cache.shape[1], qkv.device)
-        return _mix(qkv).window_prefill(
+    if not qkv.is_cuda:
+        return ref_attn.window_prefill(
             qkv, k_cache, v_cache, positions, cos_sin, slots, block_tables,
-            prompt.tiles(h), h, sink, scale, n_q, window, keep_first, has_kv)
-    return ref_mix.window_prefill(qkv, k_cache, v_cache, positions, cos_sin,
-                                  slots, block_tables, prompt, sink, scale,
-                                  n_q, window, keep_first, has_kv)
+            prompt, sink, scale, n_q, window, keep_first, has_kv, None, None,
+            0.0, 0, None)
+    attn = _ns("rlli_attn", qkv)
+    attn.window_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q,
+                       has_kv, None)
+    mask = (sink, scale, n_q, window, keep_first, has_kv)
+    if attn.window_fast(k_cache, v_cache, qkv.dtype == torch.float32):
+        h = window_tile_rows(n_q // k_cache.shape[1], qkv.device)
+        return _mix(qkv).window_tiled(qkv, k_cache, v_cache, block_tables,
+                                      prompt.tiles(h), h, *mask)
+    return attn.window_rows(qkv, k_cache, v_cache, block_tables,
+                            prompt.tiles(32), 32, *mask, None, None, 0.0, 0)
 
 
 def window_decode(qkv, k_cache, v_cache, positions, cos_sin, slots,
                   block_tables, sink, scale: float, n_q: int, window: int,
                   keep_first: int, has_kv: bool):
     """One new token per sequence: rotation, append and attention fused."""
-    return _mix(qkv).window_decode(
+    return _ns("rlli_attn", qkv).window_decode(
         qkv, k_cache, v_cache, positions, cos_sin, slots, block_tables, sink,
-        scale, n_q, window, keep_first, has_kv)
+        scale, n_q, window, keep_first, has_kv, None, None, 0.0, 0, None)
+
+
+FULL = 1 << 30        # a window that never ends
+
+
+def biased_decode(qkv, k_cache, v_cache, positions, slots, block_tables,
+                  scale: float, n_q: int, r1, r2, temp_coef: float,
+                  temp_every: int, v_eps=None):
+    """Causal attention without rotation: a score loses r1 ln(1 + r2
+    distance), queries are multiplied by 1 + temp_coef ln((p + 1) //
+    temp_every + 1), values cached over their root mean square (``v_eps``).
+    One new token per sequence, append included."""
+    return _ns("rlli_attn", qkv).window_decode(
+        qkv, k_cache, v_cache, positions, None, slots, block_tables, None,
+        scale, n_q, FULL, 0, True, r1, r2, temp_coef, temp_every, v_eps)
+
+
+def biased_prefill(qkv, k_cache, v_cache, positions, slots, block_tables,
+                   prompt, scale: float, n_q: int, r1, r2, temp_coef: float,
+                   temp_every: int, v_eps=None):
+    """The same for prompt rows: append, then attend over the sequence's
+    gathered keys and values (sizes that the tiled kernel does not take:
+    over the pages, row by row)."""
+    score = (r1, r2, temp_coef, temp_every)
+    if not qkv.is_cuda:
+        return ref_attn.window_prefill(
+            qkv, k_cache, v_cache, positions, None, slots, block_tables,
+            prompt, None, scale, n_q, FULL, 0, True, *score, v_eps)
+    attn = _ns("rlli_attn", qkv)
+    attn.window_append(qkv, k_cache, v_cache, positions, None, slots, n_q,
+                       True, v_eps)
+    _, n_kv, _, dim = k_cache.shape
+    vdim = v_cache.shape[3]
+    if qkv.dtype == torch.float32 or not attn.expanded_ok(dim, vdim):
+        return attn.window_rows(qkv, k_cache, v_cache, block_tables,
+                                prompt.tiles(32), 32, None, scale, n_q, FULL,
+                                0, True, *score)
+    blocks, kv_off, tokens = prompt.gathered(64)
+    k, vt = attn.kv_gather(k_cache, v_cache, block_tables, blocks, tokens)
+    out = torch.empty((qkv.shape[0], n_q * vdim), dtype=qkv.dtype,
+                      device=qkv.device)
+    attn.expanded_attn(qkv[:, :n_q * dim], k, vt, None, prompt.tiles(128),
+                       kv_off, n_q, n_kv, scale, out, *score)
+    return out
 
 
 def _out(proj, state, vdim, out):
@@ -369,8 +419,8 @@ def gla_prefill(proj, a2, a2_bias, norm, state, prompt, vdim: int,
                 tau: float, eps: float, out=None):
     out = _out(proj, state, vdim, out)
     _ns("rlli_rec", proj).gla_prefill(
-        proj, a2, a2_bias, norm, state, prompt.tiles(GLA_CHUNK),
-        prompt.seqs(GLA_CHUNK), vdim, tau, eps, out)
+        proj, a2, a2_bias, norm, state, prompt.tiles(REC_CHUNK),
+        prompt.seqs(REC_CHUNK), vdim, tau, eps, out)
     return out
 
 
@@ -388,8 +438,65 @@ def hgrn2_prefill(proj, bias, lower, norm, state, prompt, vdim: int,
                   eps: float, out=None):
     out = _out(proj, state, vdim, out)
     _ns("rlli_rec", proj).hgrn2_prefill(
-        proj, bias, lower, norm, state, prompt.tiles(GLA_CHUNK),
-        prompt.seqs(GLA_CHUNK), vdim, eps, out)
+        proj, bias, lower, norm, state, prompt.tiles(REC_CHUNK),
+        prompt.seqs(REC_CHUNK), vdim, eps, out)
+    return out
+
+
+def rwkv_decode(rkvg, low, w2, w0, bonus, norm, state, slots, positions,
+                eps: float, out):
+    """RWKV-style recurrence, one new token per sequence: ``rkvg`` [4, rows,
+    heads * dim], decay e^(-e^(w2 tanh(low) + w0)), bonus for the present
+    token, norm over a head, silu gate."""
+    _ns("rlli_rec", rkvg).rwkv_decode(rkvg, low, w2, w0, bonus, norm, state,
+                                      slots, positions, eps, out)
+    return out
+
+
+def rwkv_prefill(rkvg, low, w2, w0, bonus, norm, state, prompt, eps: float,
+                 out):
+    _ns("rlli_rec", rkvg).rwkv_prefill(
+        rkvg, low, w2, w0, bonus, norm, state, prompt.tiles(REC_CHUNK),
+        prompt.seqs(REC_CHUNK), eps, out)
+    return out
+
+
+def delta_decode(proj, taps, tail, a_rate, dt_bias, norm, state, slots,
+                 positions, kv_heads: int, vdim: int, eps: float, out):
+    """Gated delta rule, one new token per sequence, convolution of
+    q | k | v included.  ``proj``: q | k | v | gate | beta | decay."""
+    _ns("rlli_rec", proj).delta_decode(
+        proj, taps, tail, a_rate, dt_bias, norm, state, slots, positions,
+        kv_heads, vdim, eps, out)
+    return out
+
+
+def delta_prefill(proj, taps, tail, a_rate, dt_bias, norm, state, prompt,
+                  kv_heads: int, vdim: int, eps: float, out):
+    x = torch.empty((proj.shape[0], taps.shape[1]), dtype=proj.dtype,
+                    device=proj.device)
+    conv_prompt(proj[:, :taps.shape[1]], taps, tail, prompt, x, silu=True)
+    _ns("rlli_rec", proj).delta_prefill(
+        proj, x, a_rate, dt_bias, norm, state, prompt.tiles(REC_CHUNK),
+        prompt.seqs(REC_CHUNK), kv_heads, vdim, eps, out)
+    return out
+
+
+def mlstm_decode(proj, i_bias, f_bias, norm, state, m, slots, positions,
+                 vdim: int, cap: float, eps: float, out):
+    """mLSTM, one new token per sequence.  ``proj``: q | k | v | gate | i |
+    f; the state's last column is the normalizer, ``m`` the running
+    maximum."""
+    _ns("rlli_rec", proj).mlstm_decode(proj, i_bias, f_bias, norm, state, m,
+                                       slots, positions, vdim, cap, eps, out)
+    return out
+
+
+def mlstm_prefill(proj, i_bias, f_bias, norm, state, m, prompt, vdim: int,
+                  cap: float, eps: float, out):
+    _ns("rlli_rec", proj).mlstm_prefill(
+        proj, i_bias, f_bias, norm, state, m, prompt.tiles(REC_CHUNK),
+        prompt.seqs(REC_CHUNK), vdim, cap, eps, out)
     return out
 
 
@@ -402,42 +509,54 @@ def moe_experts(h, router, w_up, w_down, top: int, limit: float):
     return _mix(h).moe_experts(h, router, w_up, w_down, top, limit)
 
 
-# ------------------------------------------- parallel blocks, latents
+# --------------------------------------------------- residual blocks
 CONV_SPAN = 16        # prompt rows that one convolution workgroup walks
-LATENT_VECTORS = 32   # (row, head) queries of one absorbed prompt tile
 
 
 def block_embed(ids, table, pos_table, positions, x, gain, groups: int,
                 eps: float, taps=None, tail=None, slots=None,
-                n_decode: int = 0):
-    """Fill the f32 residual with embedding + position and return its
+                n_decode: int = 0, scale: float = 1.0):
+    """Fill the f32 residual with scaled embedding + position and return its
     grouped norm h and, for the first ``n_decode`` rows (one token per
-    sequence), h + conv(h) from the sequences' tails."""
-    return _ns("rlli_lat", table).block_embed(
+    sequence), h + conv(h) from the sequences' tails.  ``taps`` [branches,
+    taps, width] makes that [branches, rows, width]."""
+    return _ns("rlli_blk", table).block_embed(
         ids, table, pos_table, positions, x, gain, groups, eps, taps, tail,
-        slots, n_decode)
+        slots, n_decode, scale)
 
 
 def block_step(x, y, gain, groups: int, eps: float, positions, taps=None,
                tail=None, slots=None, n_decode: int = 0, rows=None,
-               keep: bool = True):
+               keep: bool = True, y2=None, gain1=None, gain2=None):
     """Add a block's output to the residual; then as block_embed.  ``rows``
-    restricts the result (then keep=False)."""
-    return _ns("rlli_lat", y).block_step(x, y, gain, groups, eps, positions,
+    restricts the result (then keep=False).  With ``y2`` half the sum of
+    both outputs is added, each normed first (``gain1``, ``gain2``)."""
+    return _ns("rlli_blk", y).block_step(x, y, gain, groups, eps, positions,
                                          taps, tail, slots, n_decode, rows,
-                                         keep)
+                                         keep, y2, gain1, gain2)
 
 
-def conv_prompt(h, taps, tail, prompt, out):
-    """out = h + conv(h) for prompt rows, and their sequences' tails."""
-    _ns("rlli_lat", h).conv_prompt(h, taps, tail, prompt.spans(CONV_SPAN),
-                                   prompt.spans(1 << 30), out)
+def conv_prompt(h, taps, tail, prompt, out, silu: bool = False):
+    """out = h + conv(h), or silu(conv(h)), for prompt rows, and their
+    sequences' tails.  Branches as in block_embed."""
+    _ns("rlli_blk", h).conv_prompt(h, taps, tail, prompt.spans(CONV_SPAN),
+                                   prompt.spans(1 << 30), out, silu)
 
 
-def gate_act(gate_up, out, act: str):
-    """out = act(gate) * up of [rows, gate | up]."""
-    _ns("rlli_lat", gate_up).gate_act(gate_up, out, act)
+def gate_act(gate_up, out, act: str, limit: float = 0.0):
+    """out = act(gate) * up of [rows, gate | up]; act 'clamp_glu': g
+    sigmoid(1.702 g) (u + 1) with g <= limit, |u| <= limit."""
+    _ns("rlli_blk", gate_up).gate_act(gate_up, out, act, limit)
     return out
+
+
+def soft_cap(x, cap: float):
+    """cap * tanh(x / cap), 32-bit."""
+    return _ns("rlli_blk", x).soft_cap(x, cap)
+
+
+# ------------------------------------------------------------- latents
+LATENT_VECTORS = 32   # (row, head) queries of one absorbed prompt tile
 
 
 def latent_prep(proj, q_norm, kv_norm, eps: float, cache, slots):
@@ -490,7 +609,8 @@ def latent_prefill(q, gate, cache, block_tables, prompt, scale: float, w_uk,
     vdim = w_uv.shape[1]
     ns = _ns("rlli_lat", q)
     fast = q.is_cuda and ns.latent_fast(cache, q.dtype == torch.float32)
-    ok = fast and ns.expanded_ok(dim, vdim) and all(
+    attn = _ns("rlli_attn", q) if fast else None
+    ok = fast and attn.expanded_ok(dim, vdim) and all(
         t.stride(0) % 4 == 0 and t.data_ptr() % 8 == 0 for t in (gate, out))
     if expand is None:
         expand = ok and expands(prompt, rank, dim, vdim)
@@ -499,8 +619,8 @@ def latent_prefill(q, gate, cache, block_tables, prompt, scale: float, w_uk,
         c = ns.latent_gather(cache, block_tables, blocks, tokens)
         k = torch.nn.functional.linear(c, w_k)
         vt = torch.nn.functional.linear(w_v, c)      # already transposed
-        ns.expanded_attn(q, k, vt, gate, prompt.tiles(128), kv_off, heads,
-                         scale, out)
+        attn.expanded_attn(q, k, vt, gate, prompt.tiles(128), kv_off, heads,
+                           heads, scale, out, None, None, 0.0, 0)
         return out
     tiles = prompt.vectors(LATENT_VECTORS, heads) if fast else prompt.tiles(32)
     c = ns.latent_attn(head_linear(q, w_uk), cache, block_tables, scale,

@@ -30,9 +30,10 @@ SAN_FLAGS = {"asan": ["-Xarch_host", "-fsanitize=address"],
 BUILD = os.path.join(HERE, "build" + (f"-{_SAN}" if _SAN else ""))
 
 # Libraries, so that a process compiles and loads what its model needs:
-# rlli_hip has the Llama-family kernels and the sampler, rlli_mix residual
-# streams, windowed attention and mixture of experts, rlli_rec the gated
-# linear recurrences, rlli_lat parallel blocks and latent attention.
+# rlli_hip has the Llama-family kernels and the sampler, rlli_attn paged
+# softmax attention in its variants, rlli_mix residual streams, windowed
+# prompt attention and mixture of experts, rlli_blk residual blocks and short
+# convolutions, rlli_rec linear recurrences, rlli_lat latent attention.
 LIBRARIES = {
     "rlli_hip": [
         "ext.cpp",
@@ -49,29 +50,41 @@ LIBRARIES = {
         "skinny2.hip",
         "streamprobe.hip",
     ],
+    "rlli_attn": [
+        "ext_attn.cpp",
+        "window_attn.hip",
+        "expanded_attn.hip",
+    ],
     "rlli_mix": [
         "ext_mix.cpp",
         "hyper.hip",
-        "window_attn.hip",
         "window_prefill.hip",
         "moe.hip",
+    ],
+    "rlli_blk": [
+        "ext_blk.cpp",
+        "block.hip",
     ],
     "rlli_rec": [
         "ext_rec.cpp",
         "gla.hip",
+        "delta.hip",
+        "mlstm.hip",
+        "rec_scan.hip",
     ],
     "rlli_lat": [
         "ext_lat.cpp",
-        "block.hip",
         "latent.hip",
-        "latent_prefill.hip",
     ],
 }
-_MIX_HEADERS = ["common.h", "mix.h", "attn_rows.h", "ext_common.h"]
+_ACT = ["common.h", "act.h", "ext_common.h"]
+_ATTN = _ACT + ["attn.h", "attn_rows.h", "ext_window.h"]
 HEADERS = {"rlli_hip": ["common.h", "kernels.h"],
-           "rlli_mix": _MIX_HEADERS,
-           "rlli_rec": _MIX_HEADERS,
-           "rlli_lat": _MIX_HEADERS + ["lat.h"]}
+           "rlli_attn": _ATTN,
+           "rlli_mix": _ATTN + ["mix.h"],
+           "rlli_blk": _ACT + ["blk.h"],
+           "rlli_rec": _ACT + ["rec.h", "rec_math.h"],
+           "rlli_lat": _ATTN + ["lat.h"]}
 # some packed f32 instruction forms have returned wrong results on this
 # hardware; keep the compiler from forming them
 CODEGEN = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]

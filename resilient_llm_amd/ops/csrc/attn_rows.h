@@ -1,10 +1,11 @@
-// Paged attention at any sizes and dtypes, one wave per (row, head),
+// Paged attention (window, kept tokens, sink, distance bias, query
+// temperature) at any sizes and dtypes, one wave per (row, head),
 // scalar everywhere: the 32-bit path, and the shapes that the tiled kernels
 // do not take.  Keys and values may be one tensor (a cached latent that
 // serves as both).
 #pragma once
 
-#include "mix.h"
+#include "attn.h"
 
 namespace rlli {
 namespace {
@@ -42,6 +43,8 @@ void window_rows_kernel(WindowAttnArgs a, bool decode) {
   const CE* kc = reinterpret_cast<const CE*>(a.k_cache);
   const CE* vc = reinterpret_cast<const CE*>(a.v_cache);
 
+  const float scale = a.scale * query_temp(pos, a.temp_coef, a.temp_every);
+  const float r1 = a.r1 ? a.r1[h] : 0.f, r2 = a.r1 ? a.r2[h] : 0.f;
   float m = kNegInf, l = 0.f, acc[MAXV];
 #pragma unroll
   for (int i = 0; i < MAXV; ++i) acc[i] = 0.f;
@@ -61,7 +64,8 @@ void window_rows_kernel(WindowAttnArgs a, bool decode) {
       const CE* kr = kc + rowi * a.dim;
       float dot = 0.f;
       for (int d = 0; d < a.dim; ++d) dot += qs[d] * cache_load(kr + d);
-      s = dot * a.scale;
+      s = dot * scale;
+      if (a.r1) s -= r1 * logf(1.f + r2 * float(pos - j));
       vrow = rowi * a.vdim;
     }
     const float m_new = fmaxf(m, wave_max(s));

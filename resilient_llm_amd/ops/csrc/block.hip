@@ -1,18 +1,24 @@
-// Parallel residual block: the residual and the grouped norm around it,
-// the short causal convolution ahead of a mixer, and a gated activation.
+// Residual blocks: the residual and the (grouped) norm around it, short
+// causal convolutions, gated activations, the output's soft cap.
 //
-// A block reads h = norm(x) once, runs its mixer on h + conv(h) and its
+// A parallel block reads h = norm(x) once, runs its mixer on h + conv(h) and its
 // feed-forward on h, and adds both: their output products are one matrix
 // product over the concatenated activations, so the residual is read and
 // written once per block.  Writing it and norming the next block's input
 // is one pass; for single decoded tokens the convolution and its state are
 // in that pass too.  Residual, norms and convolution sums are 32-bit.
 //
-// The last n_taps - 1 inputs of a sequence sit in a ring by position, so
-// advancing it writes one row and moves nothing.  A used slot needs no
-// clearing: what a row reads before position 0 is zero by position.
+// The last inputs of a sequence sit in a ring by position, so advancing it
+// writes one row and moves nothing.  A used slot needs no clearing: what a
+// row reads before position 0 is zero by position.
+//
+// A convolution may have several branches (its own taps and output each):
+// h + (h' - h) mu with the previous row's h' is the two taps mu, -mu, so
+// mixing a row with the one before it for several projections is one of
+// these.  A block may also end in two outputs, each with a norm of its own,
+// half their sum being what the residual takes (merge).
 
-#include "lat.h"
+#include "blk.h"
 
 namespace rlli {
 namespace {
@@ -21,6 +27,11 @@ DEV_INLINE float round_act(uint16_t, float v) {
   return bf16_to_f32(f32_to_bf16(v));
 }
 DEV_INLINE float round_act(float, float v) { return v; }
+
+template <typename T>
+DEV_INLINE float sigm(float x) {
+  return 1.f / (1.f + (sizeof(T) == 2 ? __expf(-x) : expf(-x)));
+}
 
 template <typename T, int V>
 DEV_INLINE void load_v(const T* p, float (&out)[V]) {
@@ -41,7 +52,8 @@ DEV_INLINE void store_v(T* p, const float (&in)[V]) {
 
 // IT vectors of V columns per thread; IT = 0 walks the row twice.  CONV:
 // there are decoded rows, which also convolve
-template <typename T, int WAVES, int IT, int V, bool EMBED, bool CONV>
+template <typename T, int WAVES, int IT, int V, bool EMBED, bool MERGE,
+          bool CONV>
 __global__ __launch_bounds__(WAVES * 64)
 void block_step_kernel(BlockArgs a) {
   extern __shared__ float sq[];           // [width / V] squares, [groups]
@@ -53,6 +65,16 @@ void block_step_kernel(BlockArgs a) {
   float* xr = a.x + row * W;
   const T* yr = EMBED ? nullptr
                       : reinterpret_cast<const T*>(a.y) + row * W;
+  const T* y2r = MERGE ? reinterpret_cast<const T*>(a.y2) + row * W : nullptr;
+  float s1 = 0.f, s2 = 0.f;               // half over the root mean squares
+  auto merge = [&](int c, const float (&p)[V], const float (&q)[V],
+                   float (&t)[V]) {
+    float g1[V], g2[V];
+    load_v<float, V>(a.gain1 + c, g1);
+    load_v<float, V>(a.gain2 + c, g2);
+#pragma unroll
+    for (int j = 0; j < V; ++j) t[j] = p[j] * s1 * g1[j] + q[j] * s2 * g2[j];
+  };
   const T *er = nullptr, *pr = nullptr;
   if constexpr (EMBED) {
     er = reinterpret_cast<const T*>(a.table) + int64_t(a.ids[n]) * W;
@@ -64,6 +86,8 @@ void block_step_kernel(BlockArgs a) {
   auto summands = [&](int c, float (&u)[V], float (&t)[V]) {
     if constexpr (EMBED) {
       load_v<T, V>(er + c, u);
+#pragma unroll
+      for (int j = 0; j < V; ++j) u[j] *= a.embed_scale;
       if (pr) {
         load_v<T, V>(pr + c, t);
       } else {
@@ -73,6 +97,11 @@ void block_step_kernel(BlockArgs a) {
     } else {
       load_v<float, V>(xr + c, u);
       load_v<T, V>(yr + c, t);
+      if constexpr (MERGE && IT == 0) {
+        float q[V];
+        load_v<T, V>(y2r + c, q);
+        merge(c, t, q, t);
+      }
     }
   };
   // IT > 0: everything a row needs is asked for up front, so that one
@@ -92,18 +121,21 @@ void block_step_kernel(BlockArgs a) {
     }
   };
   const bool conv = CONV && n < a.n_decode;
-  const int back = a.n_taps - 1;          // earlier inputs in the ring
-  auto load_tap = [&](int k, int c, float (&w)[V]) {
-    load_v<float, V>(a.taps + int64_t(back - k) * W + c, w);
+  const int back = a.n_taps - 1;          // earlier inputs that count
+  auto load_tap = [&](int b, int k, int c, float (&w)[V]) {
+    load_v<float, V>(a.taps + (int64_t(b) * a.n_taps + back - k) * W + c, w);
   };
+  float t2[MERGE ? ITS : 1][V];
   if constexpr (IT > 0) {
     every([&](int v, int i) { summands(v * V, u[i], t[i]); });
+    if constexpr (MERGE)
+      every([&](int v, int i) { load_v<T, V>(y2r + v * V, t2[i]); });
     every([&](int v, int i) { load_v<float, V>(a.gain + v * V, gain[i]); });
     if (conv)
       every([&](int v, int i) {
 #pragma unroll
         for (int k = 0; k < EARLY; ++k)
-          if (k <= back) load_tap(k, v * V, tap[i][k]);
+          if (k <= back) load_tap(0, k, v * V, tap[i][k]);
       });
   }
   int pos = 0, at = 0;                    // position, its row of the ring
@@ -111,12 +143,12 @@ void block_step_kernel(BlockArgs a) {
   if (conv) {
     pos = a.positions[n];
     if (back > 0) {
-      ring = reinterpret_cast<T*>(a.tail) + int64_t(a.slots[n]) * back * W;
-      at = pos % back;
+      ring = reinterpret_cast<T*>(a.tail) + int64_t(a.slots[n]) * a.ring * W;
+      at = pos % a.ring;
     }
   }
   auto load_ring = [&](int k, int c, float (&e)[V]) {
-    const int r = at - k < 0 ? at - k + back : at - k;
+    const int r = at - k < 0 ? at - k + a.ring : at - k;
     load_v<T, V>(ring + int64_t(r) * W + c, e);
   };
   if (conv)
@@ -126,6 +158,37 @@ void block_step_kernel(BlockArgs a) {
         if (k <= back && k <= pos) load_ring(k, v * V, past[i][k]);
     });
 
+  if constexpr (MERGE) {
+    __shared__ float part[2][WAVES];
+    every([&](int v, int i) {
+      if constexpr (IT == 0) {
+        load_v<T, V>(yr + v * V, t[0]);
+        load_v<T, V>(y2r + v * V, t2[0]);
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        s1 += t[i][j] * t[i][j];
+        s2 += t2[i][j] * t2[i][j];
+      }
+    });
+    s1 = wave_sum(s1);
+    s2 = wave_sum(s2);
+    if ((threadIdx.x & 63) == 0) {
+      part[0][threadIdx.x >> 6] = s1;
+      part[1][threadIdx.x >> 6] = s2;
+    }
+    __syncthreads();
+    s1 = s2 = 0.f;
+#pragma unroll
+    for (int w = 0; w < WAVES; ++w) {
+      s1 += part[0][w];
+      s2 += part[1][w];
+    }
+    s1 = 0.5f / sqrtf(s1 / W + a.eps);
+    s2 = 0.5f / sqrtf(s2 / W + a.eps);
+    if constexpr (IT > 0)
+      every([&](int v, int i) { merge(v * V, t[i], t2[i], t[i]); });
+  }
   every([&](int v, int i) {
     if constexpr (IT == 0) summands(v * V, u[0], t[0]);
     float s = 0.f;
@@ -164,31 +227,38 @@ void block_step_kernel(BlockArgs a) {
       hv[j] = round_act(T{}, u[i][j] * inv * gain[i][j]);
     store_v<T, V>(hr + c, hv);
     if (conv) {
-      float o[V];
+      for (int b = 0; b < a.branches; ++b) {
+        float o[V];
 #pragma unroll
-      for (int j = 0; j < V; ++j) o[j] = hv[j];
-      auto add = [&](const float (&w)[V], const float (&e)[V]) {
+        for (int j = 0; j < V; ++j) o[j] = hv[j];
+        auto add = [&](const float (&w)[V], const float (&e)[V]) {
 #pragma unroll
-        for (int j = 0; j < V; ++j) o[j] += w[j] * e[j];
-      };
+          for (int j = 0; j < V; ++j) o[j] += w[j] * e[j];
+        };
 #pragma unroll
-      for (int k = 0; k < EARLY; ++k)
-        if (k <= back && k <= pos) add(tap[i][k], k == 0 ? hv : past[i][k]);
-      for (int k = EARLY; k <= back && k <= pos; ++k) {
-        float w[V], e[V];
-        load_tap(k, c, w);
-        if (k > 0) load_ring(k, c, e);
-        add(w, k == 0 ? hv : e);
+        for (int k = 0; k < EARLY; ++k)
+          if (k <= back && k <= pos) {
+            if (b > 0) load_tap(b, k, c, tap[i][k]);
+            add(tap[i][k], k == 0 ? hv : past[i][k]);
+          }
+        for (int k = EARLY; k <= back && k <= pos; ++k) {
+          float w[V], e[V];
+          load_tap(b, k, c, w);
+          if (k > 0) load_ring(k, c, e);
+          add(w, k == 0 ? hv : e);
+        }
+        store_v<T, V>(reinterpret_cast<T*>(a.hc) +
+                          (int64_t(b) * a.n + n) * W + c, o);
       }
-      store_v<T, V>(reinterpret_cast<T*>(a.hc) + int64_t(n) * W + c, o);
       if (back > 0) store_v<T, V>(ring + int64_t(at) * W + c, hv);
     }
   });
 }
 
 // prompt rows of one span, V columns per thread, the window in registers
-// (K taps; K = 0: any number, re-read)
-template <typename T, int K, int V>
+// (K taps; K = 0: any number, re-read).  SILU: silu(conv(h)) instead of
+// h + conv(h)
+template <typename T, int K, int V, bool SILU>
 __global__ __launch_bounds__(256)
 void conv_prompt_kernel(ConvArgs a) {
   const int c = (blockIdx.y * 256 + threadIdx.x) * V;
@@ -197,17 +267,25 @@ void conv_prompt_kernel(ConvArgs a) {
   const int row0 = a.spans[s], pos0 = a.spans[ns + s];
   const int rows = a.spans[2 * ns + s], off = a.spans[3 * ns + s];
   const int taps = K > 0 ? K : a.n_taps, back = taps - 1;
-  const int64_t W = a.width;
+  const int64_t W = a.width, HS = a.h_stride, OS = a.out_stride;
   const T* h = reinterpret_cast<const T*>(a.h) + c;
-  T* out = reinterpret_cast<T*>(a.out) + c;
+  T* out = reinterpret_cast<T*>(a.out) + blockIdx.z * a.branch_stride + c;
+  const float* tap = a.taps + blockIdx.z * taps * W + c;
   const T* ring = reinterpret_cast<const T*>(a.tail) +
-                  int64_t(a.spans[4 * ns + s]) * back * W + c;
+                  int64_t(a.spans[4 * ns + s]) * a.ring * W + c;
+  auto finish = [&](float (&o)[V]) {
+    if constexpr (SILU)
+#pragma unroll
+      for (int j = 0; j < V; ++j)
+        o[j] *= sigm<T>(o[j]);
+  };
   // the input at row r of the span, r may be negative
   auto input = [&](int r, float (&v)[V]) {
     if (off + r >= 0) {
-      load_v<T, V>(h + int64_t(row0 + r) * W, v);
+      load_v<T, V>(h + int64_t(row0 + r) * HS, v);
     } else if (pos0 + r >= 0) {
-      load_v<T, V>(ring + int64_t((pos0 + r) % (back > 0 ? back : 1)) * W, v);
+      load_v<T, V>(ring + int64_t((pos0 + r) % (back > 0 ? a.ring : 1)) * W,
+                   v);
     } else {
 #pragma unroll
       for (int j = 0; j < V; ++j) v[j] = 0.f;
@@ -218,20 +296,21 @@ void conv_prompt_kernel(ConvArgs a) {
     float w[K][V], win[KB][V];
 #pragma unroll
     for (int k = 0; k < K; ++k)
-      load_v<float, V>(a.taps + k * W + c, w[k]);
+      load_v<float, V>(tap + k * W, w[k]);
 #pragma unroll
     for (int k = 0; k < K - 1; ++k) input(k - (K - 1), win[k]);
 #pragma unroll 4
     for (int r = 0; r < rows; ++r) {
       float cur[V], o[V];
-      load_v<T, V>(h + int64_t(row0 + r) * W, cur);
+      load_v<T, V>(h + int64_t(row0 + r) * HS, cur);
 #pragma unroll
       for (int j = 0; j < V; ++j) {
-        o[j] = cur[j] + w[K - 1][j] * cur[j];
+        o[j] = (SILU ? 0.f : cur[j]) + w[K - 1][j] * cur[j];
 #pragma unroll
         for (int k = K - 2; k >= 0; --k) o[j] += w[k][j] * win[k][j];
       }
-      store_v<T, V>(out + int64_t(row0 + r) * W, o);
+      finish(o);
+      store_v<T, V>(out + int64_t(row0 + r) * OS, o);
 #pragma unroll
       for (int k = 0; k < K - 1; ++k)
 #pragma unroll
@@ -242,16 +321,17 @@ void conv_prompt_kernel(ConvArgs a) {
     for (int r = 0; r < rows; ++r) {
       float o[V], e[V], w[V];
       input(r, e);
-      load_v<float, V>(a.taps + int64_t(back) * W + c, w);
+      load_v<float, V>(tap + int64_t(back) * W, w);
 #pragma unroll
-      for (int j = 0; j < V; ++j) o[j] = e[j] + w[j] * e[j];
+      for (int j = 0; j < V; ++j) o[j] = (SILU ? 0.f : e[j]) + w[j] * e[j];
       for (int k = 1; k <= back; ++k) {
         input(r - k, e);
-        load_v<float, V>(a.taps + int64_t(back - k) * W + c, w);
+        load_v<float, V>(tap + int64_t(back - k) * W, w);
 #pragma unroll
         for (int j = 0; j < V; ++j) o[j] += w[j] * e[j];
       }
-      store_v<T, V>(out + int64_t(row0 + r) * W, o);
+      finish(o);
+      store_v<T, V>(out + int64_t(row0 + r) * OS, o);
     }
   }
 }
@@ -263,27 +343,30 @@ __global__ __launch_bounds__(256)
 void conv_tail_kernel(ConvArgs a) {
   const int c = blockIdx.y * 256 + threadIdx.x;
   if (c >= a.width) return;
-  const int s = blockIdx.x, np = a.n_portions, back = a.n_taps - 1;
+  const int s = blockIdx.x, np = a.n_portions, ring_rows = a.ring;
   const int row0 = a.portions[s], pos0 = a.portions[np + s];
   const int rows = a.portions[2 * np + s];
   const T* h = reinterpret_cast<const T*>(a.h) + c;
   T* ring = reinterpret_cast<T*>(a.tail) +
-            int64_t(a.portions[4 * np + s]) * back * a.width + c;
-  for (int r = max(0, rows - back); r < rows; ++r)
-    ring[int64_t((pos0 + r) % back) * a.width] =
-        h[int64_t(row0 + r) * a.width];
+            int64_t(a.portions[4 * np + s]) * ring_rows * a.width + c;
+  for (int r = max(0, rows - ring_rows); r < rows; ++r)
+    ring[int64_t((pos0 + r) % ring_rows) * a.width] =
+        h[int64_t(row0 + r) * a.h_stride];
 }
 
-template <int ACT>
-DEV_INLINE float activate(float x) {
-  if constexpr (ACT == kActRelu) return fmaxf(x, 0.f);
-  return x / (1.f + __expf(-x));
+template <int ACT, typename T>
+DEV_INLINE float gated(float x, float u, float limit) {
+  if constexpr (ACT == kActRelu) return fmaxf(x, 0.f) * u;
+  if constexpr (ACT == kActSilu) return x * sigm<T>(x) * u;
+  x = fminf(x, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return x * sigm<T>(1.702f * x) * (u + 1.f);
 }
 
 template <typename T, int ACT, int V>
 __global__ __launch_bounds__(256)
 void gate_act_kernel(const T* __restrict__ gu, T* __restrict__ out, int ff,
-                     int64_t out_stride, int nb) {
+                     int64_t out_stride, int nb, float limit) {
   const int64_t row = blockIdx.x / nb;
   const int c = ((blockIdx.x % nb) * 256 + threadIdx.x) * V;
   if (c >= ff) return;
@@ -296,53 +379,82 @@ void gate_act_kernel(const T* __restrict__ gu, T* __restrict__ out, int ff,
     load_v<T, P>(g + i * P, a);
     load_v<T, P>(g + ff + i * P, b);
 #pragma unroll
-    for (int j = 0; j < P; ++j) a[j] = activate<ACT>(a[j]) * b[j];
+    for (int j = 0; j < P; ++j) a[j] = gated<ACT, T>(a[j], b[j], limit);
     store_v<T, P>(o + i * P, a);
   }
 }
 
-template <typename T, bool EMBED, bool CONV>
+template <typename T>
+__global__ __launch_bounds__(256)
+void soft_cap_kernel(const T* __restrict__ x, float* __restrict__ out,
+                     int64_t n, float cap) {
+  const int64_t i = (int64_t(blockIdx.x) * 256 + threadIdx.x) * 4;
+  const float inv = 1.f / cap;
+  if (i + 4 <= n) {
+    f32x4_t v = act_load4(x + i);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = cap * tanhf(v[j] * inv);
+    *reinterpret_cast<f32x4_t*>(out + i) = v;
+  } else {
+    for (int64_t k = i; k < n; ++k) out[k] = cap * tanhf(act_load(x + k) * inv);
+  }
+}
+
+template <typename T, bool EMBED, bool MERGE, bool CONV>
 void step(const BlockArgs& a, hipStream_t st) {
   auto run = [&](auto* k, int threads, int v) {
     hipLaunchKernelGGL(k, dim3(a.n), dim3(threads),
                        (a.width / v + a.groups) * sizeof(float), st, a);
   };
   if (a.width / a.groups % 4 || a.width > 8192)
-    run(block_step_kernel<T, 4, 0, 1, EMBED, CONV>, 256, 1);
+    run(block_step_kernel<T, 4, 0, 1, EMBED, MERGE, CONV>, 256, 1);
   else if (a.width <= 256)
-    run(block_step_kernel<T, 1, 1, 4, EMBED, CONV>, 64, 4);
+    run(block_step_kernel<T, 1, 1, 4, EMBED, MERGE, CONV>, 64, 4);
   else if (a.width <= 1024)
-    run(block_step_kernel<T, 4, 1, 4, EMBED, CONV>, 256, 4);
+    run(block_step_kernel<T, 4, 1, 4, EMBED, MERGE, CONV>, 256, 4);
   else if (a.width <= 2048)
-    run(block_step_kernel<T, 4, 2, 4, EMBED, CONV>, 256, 4);
+    run(block_step_kernel<T, 4, 2, 4, EMBED, MERGE, CONV>, 256, 4);
   else if (a.width <= 4096)
-    run(block_step_kernel<T, 8, 2, 4, EMBED, CONV>, 512, 4);
+    run(block_step_kernel<T, 8, 2, 4, EMBED, MERGE, CONV>, 512, 4);
   else
-    run(block_step_kernel<T, 8, 4, 4, EMBED, CONV>, 512, 4);
+    run(block_step_kernel<T, 8, 4, 4, EMBED, MERGE, CONV>, 512, 4);
 }
 
 template <typename T, bool EMBED>
 void step(const BlockArgs& a, hipStream_t st) {
-  if (a.hc && a.n_decode) step<T, EMBED, true>(a, st);
-  else step<T, EMBED, false>(a, st);
+  const bool conv = a.hc && a.n_decode;
+  if constexpr (!EMBED) {
+    if (a.y2) {
+      if (conv) step<T, false, true, true>(a, st);
+      else step<T, false, true, false>(a, st);
+      return;
+    }
+  }
+  if (conv) step<T, EMBED, false, true>(a, st);
+  else step<T, EMBED, false, false>(a, st);
 }
 
-template <typename T>
+template <typename T, bool SILU>
 void conv(const ConvArgs& a, hipStream_t st) {
-  const int v = a.width % 4 ? 1 : 4;
-  const dim3 grid(a.n_spans, (a.width + 256 * v - 1) / (256 * v));
+  const bool vec = a.width % 4 == 0 && a.h_stride % 4 == 0 &&
+                   a.out_stride % 4 == 0 &&
+                   (reinterpret_cast<uintptr_t>(a.h) |
+                    reinterpret_cast<uintptr_t>(a.out)) %
+                           (4 * sizeof(T)) == 0;
+  const int v = vec ? 4 : 1;
+  const dim3 grid(a.n_spans, (a.width + 256 * v - 1) / (256 * v), a.branches);
   auto run = [&](auto* k) {
     hipLaunchKernelGGL(k, grid, dim3(256), 0, st, a);
   };
   if (v == 1) {
-    run(conv_prompt_kernel<T, 0, 1>);
+    run(conv_prompt_kernel<T, 0, 1, SILU>);
   } else {
     switch (a.n_taps) {
-      case 1: run(conv_prompt_kernel<T, 1, 4>); break;
-      case 2: run(conv_prompt_kernel<T, 2, 4>); break;
-      case 3: run(conv_prompt_kernel<T, 3, 4>); break;
-      case 4: run(conv_prompt_kernel<T, 4, 4>); break;
-      default: run(conv_prompt_kernel<T, 0, 4>); break;
+      case 1: run(conv_prompt_kernel<T, 1, 4, SILU>); break;
+      case 2: run(conv_prompt_kernel<T, 2, 4, SILU>); break;
+      case 3: run(conv_prompt_kernel<T, 3, 4, SILU>); break;
+      case 4: run(conv_prompt_kernel<T, 4, 4, SILU>); break;
+      default: run(conv_prompt_kernel<T, 0, 4, SILU>); break;
     }
   }
   if (a.n_taps > 1)
@@ -353,7 +465,7 @@ void conv(const ConvArgs& a, hipStream_t st) {
 
 template <typename T, int ACT>
 void gate_act(const T* gu, T* out, int rows, int ff, int64_t stride,
-              hipStream_t st) {
+              float limit, hipStream_t st) {
   const bool vec = ff % 8 == 0 && stride % 8 == 0 &&
                    reinterpret_cast<uintptr_t>(out) % 16 == 0;
   const int v = vec ? 8 : 1;
@@ -361,10 +473,10 @@ void gate_act(const T* gu, T* out, int rows, int ff, int64_t stride,
   const dim3 grid(uint32_t(rows) * nb);
   if (vec)
     hipLaunchKernelGGL((gate_act_kernel<T, ACT, 8>), grid, dim3(256), 0, st,
-                       gu, out, ff, stride, nb);
+                       gu, out, ff, stride, nb, limit);
   else
     hipLaunchKernelGGL((gate_act_kernel<T, ACT, 1>), grid, dim3(256), 0, st,
-                       gu, out, ff, stride, nb);
+                       gu, out, ff, stride, nb, limit);
 }
 
 }  // namespace
@@ -382,20 +494,42 @@ void launch_block_step(const BlockArgs& a, hipStream_t st) {
 
 void launch_conv_prompt(const ConvArgs& a, hipStream_t st) {
   if (a.n_spans == 0) return;
-  if (a.f32) conv<float>(a, st);
-  else conv<uint16_t>(a, st);
+  auto go = [&](auto t) {
+    using T = decltype(t);
+    if (a.silu) conv<T, true>(a, st);
+    else conv<T, false>(a, st);
+  };
+  if (a.f32) go(float{});
+  else go(uint16_t{});
 }
 
 void launch_gate_act(const void* gu, void* out, int rows, int ff,
-                     int64_t stride, int act, bool f32, hipStream_t st) {
+                     int64_t stride, int act, float limit, bool f32,
+                     hipStream_t st) {
   if (rows == 0) return;
   auto go = [&](auto* g, auto* o) {
     using T = std::remove_pointer_t<decltype(o)>;
-    if (act == kActRelu) gate_act<T, kActRelu>(g, o, rows, ff, stride, st);
-    else gate_act<T, kActSilu>(g, o, rows, ff, stride, st);
+    if (act == kActRelu)
+      gate_act<T, kActRelu>(g, o, rows, ff, stride, limit, st);
+    else if (act == kActSilu)
+      gate_act<T, kActSilu>(g, o, rows, ff, stride, limit, st);
+    else
+      gate_act<T, kActClampGlu>(g, o, rows, ff, stride, limit, st);
   };
   if (f32) go(static_cast<const float*>(gu), static_cast<float*>(out));
   else go(static_cast<const uint16_t*>(gu), static_cast<uint16_t*>(out));
+}
+
+void launch_soft_cap(const void* x, float* out, int64_t n, float cap,
+                     bool f32, hipStream_t st) {
+  if (n == 0) return;
+  const dim3 grid(uint32_t((n + 1023) / 1024));
+  if (f32)
+    hipLaunchKernelGGL(soft_cap_kernel<float>, grid, dim3(256), 0, st,
+                       static_cast<const float*>(x), out, n, cap);
+  else
+    hipLaunchKernelGGL(soft_cap_kernel<uint16_t>, grid, dim3(256), 0, st,
+                       static_cast<const uint16_t*>(x), out, n, cap);
 }
 
 }  // namespace rlli

@@ -1,8 +1,9 @@
-// Prompt attention over expanded keys and values (bf16 matrix cores, f32
-// softmax): every head has its own keys and values, which two matrix
-// products made from a sequence's gathered latents, the values already
-// transposed.  Keys of a sequence start at a multiple of 64 in them and
-// are padded with zeros to a multiple of 64.
+// Prompt attention over a sequence's keys and values in one piece (bf16
+// matrix cores, f32 softmax), values transposed: expanded from gathered
+// latents by two matrix products (a key/value head per query head), or
+// gathered from their pages (kv_gather).  Keys of a sequence start at a
+// multiple of 64 in them and are padded with zeros to a multiple of 64.
+// Optional: a distance bias per head, a query temperature by position.
 //
 // A workgroup owns 128 prompt rows of one head, a wave 32 of them, and
 // walks 64-key tiles through double-buffered LDS, the next tile's loads in
@@ -12,7 +13,7 @@
 // product's operand, in registers, with the keys in the order
 // 0-3, 8-11 | 4-7, 12-15 per 16; the value tile is laid down in that order.
 
-#include "lat.h"
+#include "attn.h"
 
 namespace rlli {
 namespace {
@@ -34,8 +35,9 @@ DEV_INLINE f32x16_t mma32(s16x8_t a, s16x8_t b, f32x16_t c) {
   return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0);
 }
 
-// P: the larger of the key and value widths, rounded up
-template <int P>
+// P: the larger of the key and value widths, rounded up; BIAS: a score
+// loses r1 ln(1 + r2 distance)
+template <int P, bool BIAS>
 __global__ __launch_bounds__(256, P <= 128 ? 2 : 1)
 void expanded_attn_kernel(ExpandedAttnArgs a) {
   constexpr int DC = P / 16;              // contraction steps of a score
@@ -71,10 +73,10 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
   const bool active = sub < nrows;
   const int w_last = pos0 + min(sub + 31, nrows - 1);    // of this wave
 
-  const int64_t qw = int64_t(a.heads) * a.dim;
-  const int64_t vw = int64_t(a.heads) * a.vdim;
+  const int64_t kw = int64_t(a.n_kv) * a.dim;
+  const int kvh = h / (a.heads / a.n_kv);
   const uint16_t* q = reinterpret_cast<const uint16_t*>(a.q) +
-                      (row0 + min(my_row, nrows - 1)) * qw + h * a.dim;
+                      (row0 + min(my_row, nrows - 1)) * a.q_stride + h * a.dim;
   s16x8_t qf[DC];
 #pragma unroll
   for (int c = 0; c < DC; ++c) {
@@ -84,10 +86,10 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
     qf[c] = __builtin_bit_cast(s16x8_t, raw);
   }
 
-  const uint16_t* kp = reinterpret_cast<const uint16_t*>(a.k) + base * qw +
-                       h * a.dim;
+  const uint16_t* kp = reinterpret_cast<const uint16_t*>(a.k) + base * kw +
+                       kvh * a.dim;
   const uint16_t* vp = reinterpret_cast<const uint16_t*>(a.vt) +
-                       int64_t(h) * a.vdim * a.tokens + base;
+                       int64_t(kvh) * a.vdim * a.tokens + base;
   uint4 kr[NK], vr[NK];
   auto fetch = [&](int kv0) {
 #pragma unroll
@@ -96,7 +98,7 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
       const int r = e / (P / 8), d = e % (P / 8) * 8;
       kr[i] = uint4{0, 0, 0, 0};
       if (d < a.dim)
-        kr[i] = *reinterpret_cast<const uint4*>(kp + (kv0 + r) * qw + d);
+        kr[i] = *reinterpret_cast<const uint4*>(kp + (kv0 + r) * kw + d);
       const int vd = e / 8, c = e % 8 * 8;
       vr[i] = uint4{0, 0, 0, 0};
       if (vd < a.vdim)
@@ -124,7 +126,13 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[v][r] = 0.f;
   float m = kNegInf, l = 0.f;
-  const float c2 = a.scale * 1.4426950408889634f;
+  const float c2 = a.scale * query_temp(qpos, a.temp_coef, a.temp_every) *
+                   1.4426950408889634f;
+  float r1 = 0.f, r2 = 0.f;
+  if constexpr (BIAS) {
+    r1 = a.r1[h];
+    r2 = a.r2[h];
+  }
 
   fetch(0);
   stage(lds);
@@ -149,6 +157,19 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
           s[kt] = mma32(kf, qf[c], s[kt]);
         }
       }
+      if constexpr (BIAS) {
+        // r1 ln(x) log2(e) = r1 log2(x)
+        const float at = float(qpos - kv0 - hi * 4);
+#pragma unroll
+        for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) {
+            const float dist = at - float(kt * 32 + (r >> 2) * 8 + (r & 3));
+            s[kt][r] = fmaf(-r1, __builtin_amdgcn_logf(fmaf(r2, fmaxf(dist, 0.f), 1.f)),
+                            s[kt][r] * c2);
+          }
+      }
+      const float c1 = BIAS ? 1.f : c2;
       float mx = kNegInf;
       if (kv0 + KT - 1 > pos0 + sub) {      // some query sees only a part
 #pragma unroll
@@ -156,7 +177,7 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
             const int key = kv0 + kt * 32 + (r >> 2) * 8 + hi * 4 + (r & 3);
-            s[kt][r] = key <= qpos ? s[kt][r] * c2 : kNegInf;
+            s[kt][r] = key <= qpos ? s[kt][r] * c1 : kNegInf;
             mx = fmaxf(mx, s[kt][r]);
           }
       } else {
@@ -164,7 +185,7 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
         for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
-            s[kt][r] *= c2;
+            s[kt][r] *= c1;
             mx = fmaxf(mx, s[kt][r]);
           }
       }
@@ -241,15 +262,81 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
     }
 }
 
-template <int P>
+// one workgroup per (64 tokens, kv head)
+template <typename KC>
+__global__ __launch_bounds__(256)
+void kv_gather_kernel(KvGatherArgs a) {
+  using vec8 = typename KC::vec8;
+  using elem = typename KC::elem;
+  extern __shared__ __attribute__((aligned(16))) uint16_t lds[];   // [vdim][72]
+  const int b = blockIdx.x, kvh = blockIdx.y;
+  const int seq = a.blocks[b], tok0 = a.blocks[a.n + b];
+  const int n = a.blocks[2 * a.n + b];
+  const int64_t row0 = a.blocks[3 * a.n + b];
+  const int32_t* bt = a.block_tables + int64_t(seq) * a.max_blocks;
+  auto cache_row = [&](int r) {
+    const int t = tok0 + r;
+    return (int64_t(bt[t / a.block_size]) * a.n_kv + kvh) * a.block_size +
+           t % a.block_size;
+  };
+  auto bf16 = [](vec8 raw) {
+    float f[8];
+    KC::to_f32(raw, f);
+    bf16x8 o;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o.s[j] = f32_to_bf16(f[j]);
+    return o;
+  };
+  const int k8 = a.dim / 8, v8 = a.vdim / 8;
+  const elem* kc = reinterpret_cast<const elem*>(a.k_cache);
+  const elem* vc = reinterpret_cast<const elem*>(a.v_cache);
+  uint16_t* k = reinterpret_cast<uint16_t*>(a.k) + row0 * a.n_kv * a.dim +
+                kvh * a.dim;
+  for (int e = threadIdx.x; e < kKvGatherRows * v8; e += 256) {
+    const int r = e / v8, d = e % v8 * 8;
+    vec8 raw{};
+    if (r < n) raw = *reinterpret_cast<const vec8*>(vc + cache_row(r) * a.vdim + d);
+    const bf16x8 o = bf16(raw);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) lds[(d + j) * 72 + r] = o.s[j];
+  }
+  for (int e = threadIdx.x; e < kKvGatherRows * k8; e += 256) {
+    const int r = e / k8, d = e % k8 * 8;
+    vec8 raw{};
+    if (r < n) raw = *reinterpret_cast<const vec8*>(kc + cache_row(r) * a.dim + d);
+    *reinterpret_cast<uint4*>(k + int64_t(r) * a.n_kv * a.dim + d) =
+        bf16(raw).u;
+  }
+  __syncthreads();
+  uint16_t* vt = reinterpret_cast<uint16_t*>(a.vt) +
+                 int64_t(kvh) * a.vdim * a.tokens + row0;
+  for (int e = threadIdx.x; e < a.vdim * 8; e += 256) {
+    const int d = e / 8, c = e % 8 * 8;
+    *reinterpret_cast<uint4*>(vt + int64_t(d) * a.tokens + c) =
+        *reinterpret_cast<const uint4*>(lds + d * 72 + c);
+  }
+}
+
+template <int P, bool BIAS>
 void go(const ExpandedAttnArgs& a, hipStream_t st) {
   constexpr size_t smem = size_t(KT * (P + 8) + P * VROW) * 2 * 2;
-  auto* k = expanded_attn_kernel<P>;
+  auto* k = expanded_attn_kernel<P, BIAS>;
   if (smem > 65536)
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k),
                               hipFuncAttributeMaxDynamicSharedMemorySize,
                               int(smem));
   hipLaunchKernelGGL(k, dim3(a.n_tiles * a.heads), dim3(256), smem, st, a);
+}
+
+template <bool BIAS>
+void by_width(const ExpandedAttnArgs& a, hipStream_t st) {
+  const int d = a.dim > a.vdim ? a.dim : a.vdim;
+  if (d <= 32) go<32, BIAS>(a, st);
+  else if (d <= 64) go<64, BIAS>(a, st);
+  else if (d <= 96) go<96, BIAS>(a, st);
+  else if (d <= 128) go<128, BIAS>(a, st);
+  else if (d <= 192) go<192, BIAS>(a, st);
+  else go<256, BIAS>(a, st);
 }
 
 }  // namespace
@@ -260,13 +347,20 @@ bool expanded_ok(int dim, int vdim) {
 
 void launch_expanded_attn(const ExpandedAttnArgs& a, hipStream_t st) {
   if (a.n_tiles == 0) return;
-  const int d = a.dim > a.vdim ? a.dim : a.vdim;
-  if (d <= 32) go<32>(a, st);
-  else if (d <= 64) go<64>(a, st);
-  else if (d <= 96) go<96>(a, st);
-  else if (d <= 128) go<128>(a, st);
-  else if (d <= 192) go<192>(a, st);
-  else go<256>(a, st);
+  if (a.r1) by_width<true>(a, st);
+  else by_width<false>(a, st);
+}
+
+void launch_kv_gather(const KvGatherArgs& a, hipStream_t st) {
+  if (a.n == 0) return;
+  const dim3 grid(a.n, a.n_kv);
+  const size_t smem = size_t(a.vdim) * 72 * 2;
+  if (a.cache_kind == kCacheFP8)
+    hipLaunchKernelGGL(kv_gather_kernel<CacheFP8>, grid, dim3(256), smem, st,
+                       a);
+  else
+    hipLaunchKernelGGL(kv_gather_kernel<CacheBF16>, grid, dim3(256), smem, st,
+                       a);
 }
 
 }  // namespace rlli

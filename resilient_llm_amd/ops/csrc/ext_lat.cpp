@@ -1,5 +1,4 @@
-// Torch bindings (torch.ops.rlli_lat.*) of the parallel-block and latent
-// attention kernels.
+// Torch bindings (torch.ops.rlli_lat.*) of the latent attention kernels.
 
 #include "ext_common.h"
 #include "lat.h"
@@ -19,150 +18,6 @@ int cache_kind(const Tensor& cache, bool f32) {
   TORCH_CHECK(cache.scalar_type() == (f32 ? at::kFloat : at::kBFloat16),
               "cache dtype must match the activations (or be fp8)");
   return f32 ? rlli::kCacheF32 : rlli::kCacheBF16;
-}
-
-// ---------------------------------------------------------------- block
-void check_tail(const OptTensor& tail, const Tensor& like, int n_taps,
-                int width) {
-  if (n_taps == 1) return;
-  TORCH_CHECK(tail.has_value(), "a convolution over time needs its state");
-  same_act(*tail, like, "tail");
-  TORCH_CHECK(tail->dim() == 3 && tail->size(1) == n_taps - 1 &&
-              tail->size(2) == width, "tail must be [slots, taps - 1, width]");
-}
-
-std::tuple<Tensor, Tensor> block_run(rlli::BlockArgs& a, const Tensor& act,
-                                     Tensor x, const Tensor& gain,
-                                     int64_t groups, double eps,
-                                     const Tensor& positions,
-                                     const OptTensor& taps,
-                                     const OptTensor& tail,
-                                     const OptTensor& slots,
-                                     int64_t n_decode) {
-  TORCH_CHECK(x.dim() == 2 && x.is_cuda() && x.is_contiguous() &&
-              x.scalar_type() == at::kFloat, "residual must be f32 [T, W]");
-  a.width = int(x.size(1));
-  TORCH_CHECK(a.width <= 16000, "width out of range");
-  a.groups = int(groups);
-  TORCH_CHECK(groups >= 1 && a.width % groups == 0,
-              "norm groups must divide the width");
-  a.x = x.data_ptr<float>();
-  a.gain = f32_vec(gain, a.width, "gain");
-  a.eps = float(eps);
-  a.positions = i32(positions, "positions");
-  TORCH_CHECK(positions.numel() == x.size(0), "one position per row");
-  Tensor h = at::empty({a.n, a.width}, act.options());
-  Tensor hc;
-  a.h = h.data_ptr();
-  if (taps) {
-    TORCH_CHECK(taps->dim() == 2 && !a.rows, "taps must be [taps, width]");
-    a.n_taps = int(taps->size(0));
-    a.taps = f32_vec(*taps, int64_t(a.n_taps) * a.width, "taps");
-    check_tail(tail, act, a.n_taps, a.width);
-    a.n_decode = int(n_decode);
-    TORCH_CHECK(n_decode >= 0 && n_decode <= a.n);
-    if (a.n_taps > 1) {
-      a.tail = tail->data_ptr();
-      if (a.n_decode) {
-        TORCH_CHECK(slots.has_value());
-        a.slots = i32(*slots, "slots");
-        TORCH_CHECK(slots->numel() == a.n_decode, "one slot per decode row");
-      }
-    }
-    hc = at::empty({a.n, a.width}, act.options());
-    a.hc = hc.data_ptr();
-  } else {
-    a.n_taps = 1;
-    hc = at::empty({0}, act.options());
-  }
-  c10::hip::HIPGuardMasqueradingAsCUDA guard(x.device());
-  rlli::launch_block_step(a, stream_of(x));
-  check_launch("block_step");
-  return {h, hc};
-}
-
-std::tuple<Tensor, Tensor> block_embed(
-    const Tensor& ids, const Tensor& table, const OptTensor& pos_table,
-    const Tensor& positions, Tensor x, const Tensor& gain, int64_t groups,
-    double eps, const OptTensor& taps, const OptTensor& tail,
-    const OptTensor& slots, int64_t n_decode) {
-  rlli::BlockArgs a{};
-  a.f32 = act_f32(table, "table");
-  TORCH_CHECK(table.dim() == 2 && table.size(1) == x.size(-1));
-  a.table = table.data_ptr();
-  if (pos_table) {
-    same_act(*pos_table, table, "pos_table");
-    TORCH_CHECK(pos_table->dim() == 2 &&
-                pos_table->size(1) == table.size(1));
-    a.pos_table = pos_table->data_ptr();
-    a.n_positions = int(pos_table->size(0));
-    TORCH_CHECK(a.n_positions >= 1, "empty position table");
-  }
-  a.ids = i32(ids, "ids");
-  a.n = int(x.size(0));
-  TORCH_CHECK(ids.numel() == a.n, "one id per row");
-  a.keep = true;
-  return block_run(a, table, x, gain, groups, eps, positions, taps, tail,
-                   slots, n_decode);
-}
-
-std::tuple<Tensor, Tensor> block_step(
-    Tensor x, const Tensor& y, const Tensor& gain, int64_t groups, double eps,
-    const Tensor& positions, const OptTensor& taps, const OptTensor& tail,
-    const OptTensor& slots, int64_t n_decode, const OptTensor& rows,
-    bool keep) {
-  rlli::BlockArgs a{};
-  a.f32 = act_f32(y, "y");
-  TORCH_CHECK(y.dim() == 2 && y.sizes() == x.sizes(), "y/residual mismatch");
-  a.y = y.data_ptr();
-  a.n = int(x.size(0));
-  a.keep = keep;
-  if (rows) {
-    TORCH_CHECK(rows->is_cuda() && rows->is_contiguous() &&
-                rows->scalar_type() == at::kLong && !keep);
-    a.rows = rows->data_ptr<int64_t>();
-    a.n = int(rows->numel());
-  }
-  return block_run(a, y, x, gain, groups, eps, positions, taps, tail, slots,
-                   n_decode);
-}
-
-void conv_prompt(const Tensor& h, const Tensor& taps, const OptTensor& tail,
-                 const Tensor& spans, const Tensor& portions, Tensor out) {
-  rlli::ConvArgs a{};
-  a.f32 = act_f32(h, "h");
-  same_act(out, h, "out");
-  TORCH_CHECK(h.dim() == 2 && h.sizes() == out.sizes() && taps.dim() == 2);
-  a.width = int(h.size(1));
-  a.n_taps = int(taps.size(0));
-  a.h = h.data_ptr();
-  a.out = out.data_ptr();
-  a.taps = f32_vec(taps, int64_t(a.n_taps) * a.width, "taps");
-  check_tail(tail, h, a.n_taps, a.width);
-  if (a.n_taps > 1) a.tail = tail->data_ptr();
-  a.spans = i32(spans, "spans");
-  a.portions = i32(portions, "portions");
-  TORCH_CHECK(spans.dim() == 2 && spans.size(0) == 5 &&
-              portions.dim() == 2 && portions.size(0) == 5);
-  a.n_spans = int(spans.size(1));
-  a.n_portions = int(portions.size(1));
-  c10::hip::HIPGuardMasqueradingAsCUDA guard(h.device());
-  rlli::launch_conv_prompt(a, stream_of(h));
-  check_launch("conv_prompt");
-}
-
-void gate_act(const Tensor& gate_up, Tensor out, c10::string_view act) {
-  const bool f32 = act_f32(gate_up, "gate_up");
-  TORCH_CHECK(gate_up.dim() == 2 && gate_up.size(1) % 2 == 0);
-  const int64_t rows = gate_up.size(0), ff = gate_up.size(1) / 2;
-  const int64_t stride = row_stride(out, gate_up, rows, ff, "out");
-  TORCH_CHECK(act == "relu" || act == "silu", "act must be relu or silu");
-  c10::hip::HIPGuardMasqueradingAsCUDA guard(gate_up.device());
-  rlli::launch_gate_act(gate_up.data_ptr(), out.data_ptr(), int(rows),
-                        int(ff), stride,
-                        act == "relu" ? rlli::kActRelu : rlli::kActSilu, f32,
-                        stream_of(gate_up));
-  check_launch("gate_act");
 }
 
 // --------------------------------------------------------------- latent
@@ -345,67 +200,9 @@ Tensor latent_gather(const Tensor& cache, const Tensor& block_tables,
   return out;
 }
 
-bool expanded_ok(int64_t dim, int64_t vdim) {
-  return rlli::expanded_ok(int(dim), int(vdim));
-}
-
-void expanded_attn(const Tensor& q, const Tensor& k, const Tensor& vt,
-                   const OptTensor& gate, const Tensor& tiles,
-                   const Tensor& kv_off, int64_t heads, double scale,
-                   Tensor out) {
-  rlli::ExpandedAttnArgs a{};
-  TORCH_CHECK(!act_f32(q, "q"), "the expanded form is bf16");
-  same_act(k, q, "k");
-  same_act(vt, q, "vt");
-  const int64_t rows = q.size(0);
-  TORCH_CHECK(q.dim() == 2 && k.dim() == 2 && vt.dim() == 2 &&
-              q.size(1) == k.size(1) && q.size(1) % heads == 0 &&
-              vt.size(0) % heads == 0 && vt.size(1) == k.size(0) &&
-              k.size(0) % 64 == 0, "q/k/v mismatch");
-  a.heads = int(heads);
-  a.dim = int(q.size(1) / heads);
-  a.vdim = int(vt.size(0) / heads);
-  a.tokens = int(k.size(0));
-  TORCH_CHECK(rlli::expanded_ok(a.dim, a.vdim), "head sizes out of range");
-  a.out_stride = row_stride(out, q, rows, heads * a.vdim, "out");
-  TORCH_CHECK(a.out_stride % 4 == 0 &&
-              reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0,
-              "out rows must be 8-byte aligned");
-  if (gate) {
-    a.gate_stride = row_stride(*gate, q, rows, heads * a.vdim, "gate");
-    TORCH_CHECK(a.gate_stride % 4 == 0 &&
-                reinterpret_cast<uintptr_t>(gate->data_ptr()) % 8 == 0,
-                "gate rows must be 8-byte aligned");
-    a.gate = gate->data_ptr();
-  }
-  a.q = q.data_ptr();
-  a.k = k.data_ptr();
-  a.vt = vt.data_ptr();
-  a.out = out.data_ptr();
-  a.tiles = i32(tiles, "tiles");
-  a.kv_off = i32(kv_off, "kv_off");
-  TORCH_CHECK(tiles.dim() == 2 && tiles.size(0) == 4);
-  a.n_tiles = int(tiles.size(1));
-  a.scale = float(scale);
-  c10::hip::HIPGuardMasqueradingAsCUDA guard(q.device());
-  rlli::launch_expanded_attn(a, stream_of(q));
-  check_launch("expanded_attn");
-}
-
 }  // namespace
 
 TORCH_LIBRARY(rlli_lat, m) {
-  m.def("block_embed(Tensor ids, Tensor table, Tensor? pos_table, "
-        "Tensor positions, Tensor(a!) x, Tensor gain, int groups, float eps, "
-        "Tensor? taps, Tensor(b!)? tail, Tensor? slots, int n_decode) "
-        "-> (Tensor, Tensor)");
-  m.def("block_step(Tensor(a!) x, Tensor y, Tensor gain, int groups, "
-        "float eps, Tensor positions, Tensor? taps, Tensor(b!)? tail, "
-        "Tensor? slots, int n_decode, Tensor? rows, bool keep) "
-        "-> (Tensor, Tensor)");
-  m.def("conv_prompt(Tensor h, Tensor taps, Tensor(a!)? tail, Tensor spans, "
-        "Tensor portions, Tensor(b!) out) -> ()");
-  m.def("gate_act(Tensor gate_up, Tensor(a!) out, str act) -> ()");
   m.def("latent_prep(Tensor proj, Tensor q_norm, Tensor kv_norm, float eps, "
         "Tensor(a!) cache, Tensor slots) -> Tensor");
   m.def("head_linear(Tensor x, Tensor w, Tensor? gate, Tensor(a!) out) "
@@ -416,21 +213,12 @@ TORCH_LIBRARY(rlli_lat, m) {
         "Tensor? pos0) -> Tensor");
   m.def("latent_gather(Tensor cache, Tensor block_tables, Tensor blocks, "
         "int tokens) -> Tensor");
-  m.def("expanded_ok(int dim, int vdim) -> bool", &expanded_ok);
-  m.def("expanded_attn(Tensor q, Tensor k, Tensor vt, Tensor? gate, "
-        "Tensor tiles, Tensor kv_off, int heads, float scale, "
-        "Tensor(a!) out) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(rlli_lat, CUDA, m) {
-  m.impl("block_embed", &block_embed);
-  m.impl("block_step", &block_step);
-  m.impl("conv_prompt", &conv_prompt);
-  m.impl("gate_act", &gate_act);
   m.impl("latent_prep", &latent_prep);
   m.impl("head_linear", &head_linear);
   m.impl("latent_fast", &latent_fast);
   m.impl("latent_attn", &latent_attn);
   m.impl("latent_gather", &latent_gather);
-  m.impl("expanded_attn", &expanded_attn);
 }

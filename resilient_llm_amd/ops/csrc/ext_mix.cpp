@@ -2,7 +2,7 @@
 // Every shape, dtype and index-table assumption of a kernel is checked
 // here before it is launched.
 
-#include "ext_common.h"
+#include "ext_window.h"
 #include "mix.h"
 
 namespace {
@@ -94,146 +94,31 @@ Tensor relu2(const Tensor& x) {
 }
 
 // --------------------------------------------------------- window attention
-rlli::WindowAttnArgs window_args(const Tensor& qkv, const Tensor& k_cache,
-                                 const Tensor& v_cache,
-                                 const Tensor& positions,
-                                 const Tensor& cos_sin, const Tensor& slots,
-                                 const Tensor& block_tables,
-                                 const OptTensor& sink, double scale,
-                                 int64_t n_q, int64_t window,
-                                 int64_t keep_first, bool has_kv) {
-  rlli::WindowAttnArgs a{};
-  a.f32 = act_f32(qkv, "qkv");
-  TORCH_CHECK(k_cache.dim() == 4 && v_cache.dim() == 4 &&
-              k_cache.is_cuda() && k_cache.is_contiguous() &&
-              v_cache.is_cuda() && v_cache.is_contiguous() &&
-              k_cache.scalar_type() == v_cache.scalar_type() &&
-              k_cache.size(0) == v_cache.size(0) &&
-              k_cache.size(1) == v_cache.size(1) &&
-              k_cache.size(2) == v_cache.size(2), "k/v cache mismatch");
-  if (k_cache.scalar_type() == at::kFloat8_e4m3fn) {
-    TORCH_CHECK(!a.f32, "fp8 cache needs bf16 activations");
-    a.cache = rlli::kCacheFP8;
-  } else {
-    TORCH_CHECK(k_cache.scalar_type() == qkv.scalar_type(),
-                "cache dtype must match the activations (or be fp8)");
-    a.cache = a.f32 ? rlli::kCacheF32 : rlli::kCacheBF16;
-  }
-  a.n_q = int(n_q);
-  a.n_kv = int(k_cache.size(1));
-  a.block_size = int(k_cache.size(2));
-  a.dim = int(k_cache.size(3));
-  a.vdim = int(v_cache.size(3));
-  a.rows = int(qkv.size(0));
-  a.stride = int(qkv.size(1));
-  a.has_kv = has_kv;
-  TORCH_CHECK(a.n_q % a.n_kv == 0, "heads must be a multiple of kv heads");
-  TORCH_CHECK(a.vdim <= 512 && a.dim <= 4096, "head sizes out of range");
-  TORCH_CHECK(a.stride == a.n_q * a.dim +
-              (has_kv ? a.n_kv * (a.dim + a.vdim) : 0), "qkv width mismatch");
-  TORCH_CHECK(window >= 1 && keep_first >= 0);
-  a.window = int(std::min<int64_t>(window, 1 << 30));
-  a.keep_first = int(std::min<int64_t>(keep_first, 1 << 30));
-  a.scale = float(scale);
-  a.qkv = qkv.data_ptr();
-  a.qkv_rw = qkv.data_ptr();
-  a.k_cache = k_cache.data_ptr();
-  a.v_cache = v_cache.data_ptr();
-  a.positions = i32(positions, "positions");
-  a.slots = i32(slots, "slots");
-  TORCH_CHECK(positions.numel() == a.rows && slots.numel() == a.rows,
-              "one position and slot per row");
-  TORCH_CHECK(cos_sin.is_cuda() && cos_sin.is_contiguous() &&
-              cos_sin.scalar_type() == at::kFloat && cos_sin.dim() == 2 &&
-              cos_sin.size(1) % 2 == 0 && cos_sin.size(1) <= a.dim);
-  a.cos_sin = cos_sin.data_ptr<float>();
-  a.rot = int(cos_sin.size(1));
-  a.block_tables = i32(block_tables, "block_tables");
-  TORCH_CHECK(block_tables.dim() == 2);
-  a.max_blocks = int(block_tables.size(1));
-  a.sink = sink ? f32_vec(*sink, a.n_q, "sink") : nullptr;
-  return a;
-}
-
-// prompt rows: rotate + cache, then attend tile by tile; qkv is rotated
-// in place
-Tensor window_prefill(const Tensor& qkv, const Tensor& k_cache,
-                      const Tensor& v_cache, const Tensor& positions,
-                      const Tensor& cos_sin, const Tensor& slots,
-                      const Tensor& block_tables, const Tensor& tiles,
-                      int64_t tile_rows, const OptTensor& sink, double scale,
-                      int64_t n_q, int64_t window, int64_t keep_first,
-                      bool has_kv) {
-  auto a = window_args(qkv, k_cache, v_cache, positions, cos_sin, slots,
-                       block_tables, sink, scale, n_q, window, keep_first,
-                       has_kv);
-  a.tiles = i32(tiles, "tiles");
-  TORCH_CHECK(tiles.dim() == 2 && tiles.size(0) == 4);
-  a.n_tiles = int(tiles.size(1));
-  a.tile_rows = int(tile_rows);
+// tiled prompt rows, rotated and cached before
+Tensor window_tiled(const Tensor& qkv, const Tensor& k_cache,
+                    const Tensor& v_cache, const Tensor& block_tables,
+                    const Tensor& tiles, int64_t tile_rows,
+                    const OptTensor& sink, double scale, int64_t n_q,
+                    int64_t window, int64_t keep_first, bool has_kv) {
+  auto a = window_args(qkv, k_cache, v_cache, n_q, has_kv, scale, window,
+                       keep_first, sink);
+  window_tables(a, block_tables);
+  window_tiles(a, tiles, tile_rows);
+  TORCH_CHECK(!a.f32 && a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= 256 &&
+              a.vdim <= 256, "head sizes out of range");
+  TORCH_CHECK(tile_rows ==
+              32 * rlli::window_prefill_sub_tiles(a.n_q / a.n_kv),
+              "tile height does not fit the head grouping");
   Tensor out = at::empty({a.rows, n_q * a.vdim}, qkv.options());
   a.out = out.data_ptr();
   c10::hip::HIPGuardMasqueradingAsCUDA guard(qkv.device());
-  auto st = stream_of(qkv);
-  rlli::launch_window_rope_append(a, st);
-  if (rlli::window_fast_ok(a)) {
-    TORCH_CHECK(tile_rows ==
-                32 * rlli::window_prefill_sub_tiles(a.n_q / a.n_kv),
-                "tile height does not fit the head grouping");
-    rlli::launch_window_prefill(a, st);
-  } else {
-    rlli::launch_window_rows(a, false, st);
-  }
-  check_launch("window_prefill");
+  rlli::launch_window_prefill(a, stream_of(qkv));
+  check_launch("window_tiled");
   return out;
 }
 
 int64_t window_tile_rows(int64_t group) {
   return 32 * rlli::window_prefill_sub_tiles(int(group));
-}
-
-Tensor window_decode(const Tensor& qkv, const Tensor& k_cache,
-                     const Tensor& v_cache, const Tensor& positions,
-                     const Tensor& cos_sin, const Tensor& slots,
-                     const Tensor& block_tables, const OptTensor& sink,
-                     double scale, int64_t n_q, int64_t window,
-                     int64_t keep_first, bool has_kv) {
-  auto a = window_args(qkv, k_cache, v_cache, positions, cos_sin, slots,
-                       block_tables, sink, scale, n_q, window, keep_first,
-                       has_kv);
-  TORCH_CHECK(block_tables.size(0) == a.rows, "one block table per row");
-  Tensor out = at::empty({a.rows, n_q * a.vdim}, qkv.options());
-  a.out = out.data_ptr();
-  c10::hip::HIPGuardMasqueradingAsCUDA guard(qkv.device());
-  auto st = stream_of(qkv);
-  if (!rlli::window_fast_ok(a)) {
-    rlli::launch_window_rope_append(a, st);
-    rlli::launch_window_rows(a, true, st);
-    check_launch("window_decode");
-    return out;
-  }
-  const int group = a.n_q / a.n_kv;
-  const int hb = rlli::window_decode_heads_per_wg(group);
-  const int64_t wgs = int64_t(std::max(a.rows, 1)) * a.n_kv *
-                      ((group + hb - 1) / hb);
-  // at most one split per 4 visible 16-token steps (one per wave)
-  const int64_t reach = std::min<int64_t>(
-      int64_t(a.max_blocks) * a.block_size,
-      int64_t(a.window) + a.keep_first + 32);
-  const int64_t useful = std::max<int64_t>(1, reach / 64);
-  a.n_split = int(std::min<int64_t>(
-      {16, useful, std::max<int64_t>(1, (512 + wgs - 1) / wgs)}));
-  Tensor pa, pm;
-  if (a.n_split > 1) {
-    auto fo = qkv.options().dtype(at::kFloat);
-    pa = at::empty({a.rows, n_q, a.n_split, a.vdim}, fo);
-    pm = at::empty({a.rows, n_q, a.n_split, 2}, fo);
-    a.part_acc = pa.data_ptr<float>();
-    a.part_ml = pm.data_ptr<float>();
-  }
-  rlli::launch_window_decode(a, st);
-  check_launch("window_decode");
-  return out;
 }
 
 // ------------------------------------------------------------------ moe
@@ -330,15 +215,10 @@ TORCH_LIBRARY(rlli_mix, m) {
         "-> Tensor");
   m.def("relu2(Tensor x) -> Tensor");
   m.def("window_tile_rows(int group) -> int", &window_tile_rows);
-  m.def("window_prefill(Tensor(a!) qkv, Tensor(b!) k_cache, "
-        "Tensor(c!) v_cache, Tensor positions, Tensor cos_sin, Tensor slots, "
+  m.def("window_tiled(Tensor qkv, Tensor k_cache, Tensor v_cache, "
         "Tensor block_tables, Tensor tiles, int tile_rows, Tensor? sink, "
         "float scale, int n_q, int window, int keep_first, bool has_kv) "
         "-> Tensor");
-  m.def("window_decode(Tensor(a!) qkv, Tensor(b!) k_cache, "
-        "Tensor(c!) v_cache, Tensor positions, Tensor cos_sin, Tensor slots, "
-        "Tensor block_tables, Tensor? sink, float scale, int n_q, "
-        "int window, int keep_first, bool has_kv) -> Tensor");
   m.def("moe_route(Tensor h, Tensor router, int top) -> (Tensor, Tensor)");
   m.def("moe_experts(Tensor h, Tensor router, Tensor w_up, Tensor w_down, "
         "int top, float limit) -> Tensor");
@@ -348,8 +228,7 @@ TORCH_LIBRARY_IMPL(rlli_mix, CUDA, m) {
   m.impl("hyper_embed", &hyper_embed);
   m.impl("hyper_step", &hyper_step);
   m.impl("relu2", &relu2);
-  m.impl("window_prefill", &window_prefill);
-  m.impl("window_decode", &window_decode);
+  m.impl("window_tiled", &window_tiled);
   m.impl("moe_route", &moe_route);
   m.impl("moe_experts", &moe_experts);
 }

@@ -1,52 +1,11 @@
-// Launch declarations of the parallel-block kernels (block.hip) and of
-// latent attention (latent.hip, latent_prefill.hip), bound by ext_lat.cpp.
+// Launch declarations of latent attention (latent.hip), bound by
+// ext_lat.cpp.
 #pragma once
 
-#include "mix.h"
+#include "act.h"
+#include "attn.h"
 
 namespace rlli {
-
-// ---- block.hip ---------------------------------------------------------
-struct BlockArgs {
-  const void* table;       // embedding table (embed launch) or null
-  const int32_t* ids;      // token ids (embed launch)
-  const void* pos_table;   // learned positions (embed launch) or null
-  const int32_t* positions;     // [rows]
-  float* x;                // [rows, width] residual
-  const void* y;           // [rows, width] what the last block adds
-  const float* gain;       // [width] gain of the next norm
-  const int64_t* rows;     // row subset (final norm) or null
-  void* h;                 // [n, width] normed
-  void* hc;                // [n, width] normed + convolved, or null
-  const float* taps;       // [n_taps, width], the last meets the own row
-  void* tail;              // [slots, n_taps - 1, width] earlier inputs
-  const int32_t* slots;    // [n_decode]
-  int n, width, groups, n_taps, n_decode;
-  int n_positions;         // rows of pos_table
-  float eps;
-  bool keep;               // write the residual back
-  bool f32;
-};
-// rows [0, n_decode) also get their convolution, from the tail
-void launch_block_step(const BlockArgs& a, hipStream_t stream);
-
-struct ConvArgs {
-  const void* h;           // [rows, width]
-  void* out;               // [rows, width]: h + conv(h)
-  const float* taps;       // [n_taps, width]
-  void* tail;              // [slots, n_taps - 1, width]
-  const int32_t* spans;    // [5, n_spans]: row, position, rows, offset in
-                           // its portion, slot
-  const int32_t* portions; // [5, n_portions], the same for whole portions
-  int n_spans, n_portions, width, n_taps;
-  bool f32;
-};
-void launch_conv_prompt(const ConvArgs& a, hipStream_t stream);
-
-enum ActKind { kActRelu = 0, kActSilu = 1 };
-void launch_gate_act(const void* gate_up, void* out, int rows, int ff,
-                     int64_t out_stride, int act, bool f32,
-                     hipStream_t stream);
 
 // ---- latent.hip --------------------------------------------------------
 struct LatentPrepArgs {
@@ -99,23 +58,6 @@ int latent_tile(int heads, bool decode);
 void launch_latent_attn(const LatentAttnArgs& a, hipStream_t stream);
 void launch_latent_rows(const WindowAttnArgs& a, bool decode,
                         hipStream_t stream);
-
-// ---- latent_prefill.hip ------------------------------------------------
-struct ExpandedAttnArgs {
-  const void* q;           // [rows, heads * dim]
-  const void* k;           // [tokens, heads * dim]
-  const void* vt;          // [heads * vdim, tokens]
-  const void* gate;        // [rows, heads * vdim] or null
-  void* out;               // [rows, heads * vdim], rows out_stride apart
-  const int32_t* tiles;    // [4, n_tiles]: row, position, rows, sequence
-  const int32_t* kv_off;   // [sequences] first token in k / vt, mult. of 64
-  int64_t gate_stride, out_stride;
-  int n_tiles, heads, dim, vdim, tokens;
-  float scale;
-};
-constexpr int kExpandedRows = 128;
-bool expanded_ok(int dim, int vdim);
-void launch_expanded_attn(const ExpandedAttnArgs& a, hipStream_t stream);
 
 struct GatherArgs {
   const void* cache;       // [blocks, 1, block, rank]

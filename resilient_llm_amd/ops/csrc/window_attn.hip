@@ -3,8 +3,11 @@
 // A query at position i sees key j when j <= i and (i - j < window or
 // j < keep_first); the softmax denominator carries one extra exp(sink)
 // per head.  Rotation is the interleaved layout (pairs 2i, 2i+1) over
-// the first `rot` dimensions.  Key and value widths may differ, and a
-// layer may read keys and values that an earlier layer cached.
+// the first `rot` dimensions (0: none).  Key and value widths may differ,
+// and a layer may read keys and values that an earlier layer cached.
+// Optional: a distance bias per head (a score loses r1 ln(1 + r2 distance)),
+// a query temperature by position (in the scale), values cached over their
+// root mean square.
 //
 // Kernels here:
 //   window_rope_append  rotate q in place, rotate and cache k, cache v
@@ -56,6 +59,21 @@ void rope_append_kernel(WindowAttnArgs a) {
                 val);
   }
   const T* v = k + a.n_kv * a.dim;
+  if (a.v_norm) {                         // one wave per head
+    const int lane = threadIdx.x & 63;
+    for (int h = threadIdx.x >> 6; h < a.n_kv; h += 4) {
+      CE* o = vc + ((blk * a.n_kv + h) * a.block_size + off) * a.vdim;
+      float ss = 0.f;
+      for (int d = lane; d < a.vdim; d += 64) {
+        const float x = act_load(v + h * a.vdim + d);
+        ss += x * x;
+      }
+      const float inv = 1.f / sqrtf(wave_sum(ss) / a.vdim + a.v_eps);
+      for (int d = lane; d < a.vdim; d += 64)
+        cache_store(o + d, act_load(v + h * a.vdim + d) * inv);
+    }
+    return;
+  }
   for (int e = threadIdx.x; e < a.n_kv * a.vdim; e += blockDim.x) {
     const int h = e / a.vdim, d = e % a.vdim;
     cache_store(vc + ((blk * a.n_kv + h) * a.block_size + off) * a.vdim + d,
@@ -70,7 +88,7 @@ void rope_append_kernel(WindowAttnArgs a) {
 // the visible steps.  The new token's own term never touches the cache:
 // group 0 of wave 0 of split 0 folds it in from registers while it
 // appends, so no wave waits on a cache write of this launch.
-template <int GW, int HB, typename KC>
+template <int GW, int HB, typename KC, bool BIAS>
 __global__ __launch_bounds__(256)
 void window_decode_kernel(WindowAttnArgs a) {
   constexpr int GPW = 64 / GW;
@@ -120,6 +138,14 @@ void window_decode_kernel(WindowAttnArgs a) {
     }
   };
 
+  const float scale = a.scale * query_temp(pos, a.temp_coef, a.temp_every);
+  float r1[HB], r2[HB];
+  if constexpr (BIAS)
+#pragma unroll
+    for (int h = 0; h < HB; ++h) {
+      r1[h] = h < nh ? a.r1[head0 + h] : 0.f;
+      r2[h] = h < nh ? a.r2[head0 + h] : 0.f;
+    }
   float qv[HB][8], m[HB], l[HB], acc[HB][8];
 #pragma unroll
   for (int h = 0; h < HB; ++h) {
@@ -156,6 +182,14 @@ void window_decode_kernel(WindowAttnArgs a) {
             qrow + (a.n_q + a.n_kv) * a.dim + kvh * a.vdim + d0);
 #pragma unroll
       for (int i = 0; i < 8; ++i) vf[i] = bf16_to_f32(vr.s[i]);
+      if (a.v_norm) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += vf[i] * vf[i];
+        const float inv = 1.f / sqrtf(gsum(ss) / a.vdim + a.v_eps);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) vf[i] *= inv;
+      }
       const int slot = a.slots[seq];
       const int64_t rowi =
           (int64_t(slot / a.block_size) * a.n_kv + kvh) * a.block_size +
@@ -173,7 +207,7 @@ void window_decode_kernel(WindowAttnArgs a) {
         float s = 0.f;
 #pragma unroll
         for (int i = 0; i < 8; ++i) s += qv[h][i] * kf[i];
-        m[h] = gsum(s) * a.scale;
+        m[h] = gsum(s) * scale;
         l[h] = 1.f;
 #pragma unroll
         for (int i = 0; i < 8; ++i) acc[h][i] = vf[i];
@@ -223,7 +257,9 @@ void window_decode_kernel(WindowAttnArgs a) {
         float s = 0.f;
 #pragma unroll
         for (int d = 0; d < 8; ++d) s += qv[h][d] * kf[d];
-        s = gsum(s) * a.scale;
+        s = gsum(s) * scale;
+        if constexpr (BIAS)
+          s -= r1[h] * __logf(fmaf(r2[h], float(max(pos - j, 0)), 1.f));
         sv[h][i] = ok ? s : kNegInf;
       }
       // slots past the end hold whatever an earlier owner left
@@ -417,10 +453,16 @@ void launch_window_decode(const WindowAttnArgs& a, hipStream_t st) {
   const int hb = window_decode_heads_per_wg(group);
   const dim3 grid(a.n_split, a.n_kv * ((group + hb - 1) / hb), a.rows);
   auto go = [&](auto gw, auto hbc, auto kc) {
-    hipLaunchKernelGGL(
-        (window_decode_kernel<decltype(gw)::value, decltype(hbc)::value,
-                              decltype(kc)>),
-        grid, dim3(256), 0, st, a);
+    if (a.r1)
+      hipLaunchKernelGGL(
+          (window_decode_kernel<decltype(gw)::value, decltype(hbc)::value,
+                                decltype(kc), true>),
+          grid, dim3(256), 0, st, a);
+    else
+      hipLaunchKernelGGL(
+          (window_decode_kernel<decltype(gw)::value, decltype(hbc)::value,
+                                decltype(kc), false>),
+          grid, dim3(256), 0, st, a);
   };
   auto by_cache = [&](auto gw, auto hbc) {
     if (a.cache == kCacheFP8) go(gw, hbc, CacheFP8{});

@@ -9,7 +9,7 @@
 // P is the larger of the key and value widths, rounded up; the unused
 // columns are zeros.
 
-#include "mix.h"
+#include "attn.h"
 
 #include <type_traits>
 

@@ -1,79 +1,10 @@
-"""CPU forms of the parallel-block and latent-attention ops (same
-signatures and layouts as torch.ops.rlli_lat), in f32 PyTorch.  Attention
-has the absorbed form only; the expanded one is a GPU choice."""
+"""CPU forms of the latent-attention ops (same signatures and layouts as
+torch.ops.rlli_lat), in f32 PyTorch.  Attention has the absorbed form only;
+the expanded one is a GPU choice."""
 
 from __future__ import annotations
 
 import torch
-
-
-def _group_norm(x, gain, groups, eps):
-    p = x.view(x.shape[0], groups, x.shape[1] // groups)
-    p = p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)
-    return p.view_as(x) * gain
-
-
-def _norm_conv(x, gain, groups, eps, dtype, positions, taps, tail, slots,
-               n_decode):
-    h = _group_norm(x, gain, groups, eps).to(dtype)
-    if taps is None:
-        return h, h.new_empty(0)
-    hc = torch.empty_like(h)
-    back = taps.shape[0] - 1
-    for n in range(n_decode):
-        p = int(positions[n])
-        o = h[n].float() * (1 + taps[back])
-        for k in range(1, min(back, p) + 1):
-            o = o + taps[back - k] * tail[int(slots[n]), (p - k) % back] \
-                .float()
-        hc[n] = o.to(dtype)
-        if back:
-            tail[int(slots[n]), p % back] = h[n]
-    return h, hc
-
-
-def block_embed(ids, table, pos_table, positions, x, gain, groups, eps, taps,
-                tail, slots, n_decode):
-    e = table[ids.long()].float()
-    if pos_table is not None:
-        last = pos_table.shape[0] - 1
-        e = e + pos_table[positions.long().clamp(max=last)].float()
-    x.copy_(e)
-    return _norm_conv(x, gain, groups, eps, table.dtype, positions, taps,
-                      tail, slots, n_decode)
-
-
-def block_step(x, y, gain, groups, eps, positions, taps, tail, slots,
-               n_decode, rows, keep):
-    new = x + y.float()
-    if keep:
-        x.copy_(new)
-    if rows is not None:
-        new = new[rows]
-    return _norm_conv(new, gain, groups, eps, y.dtype, positions, taps, tail,
-                      slots, n_decode)
-
-
-def conv_prompt(h, taps, tail, spans, portions, out):
-    back = taps.shape[0] - 1
-    for row0, pos0, n, _, slot in portions.t().tolist():
-        past = torch.zeros(back, h.shape[1])
-        for k in range(1, min(back, pos0) + 1):
-            past[back - k] = tail[slot, (pos0 - k) % back].float()
-        own = h[row0:row0 + n]
-        seq = torch.cat([past, own.float()])
-        o = own.float()
-        for j in range(back + 1):
-            o = o + taps[j] * seq[j:j + n]
-        out[row0:row0 + n] = o.to(h.dtype)
-        for r in range(max(0, n - back), n):
-            tail[slot, (pos0 + r) % back] = own[r]
-
-
-def gate_act(gate_up, out, act):
-    g, u = gate_up.float().chunk(2, dim=1)
-    f = {"relu": torch.relu, "silu": torch.nn.functional.silu}[act]
-    out.copy_(f(g) * u)
 
 
 def latent_prep(proj, q_norm, kv_norm, eps, cache, slots):
