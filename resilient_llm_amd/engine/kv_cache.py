@@ -66,6 +66,13 @@ class StateLayer:
 
 
 @dataclasses.dataclass(frozen=True)
+class ScalarLayer:
+    """One number per head that a recurrent layer carries beside its state
+    (f32), a running maximum say."""
+    heads: int
+
+
+@dataclasses.dataclass(frozen=True)
 class TailLayer:
     """What a short causal convolution carries per sequence: its last
     ``rows`` inputs, a ring by position (activation dtype)."""
@@ -81,7 +88,8 @@ def layer_parts(spec) -> tuple:
 class RecurrentStates:
     """What live sequences carry from token to token: one slot per live
     sequence, and in each slot a [heads, dim, vdim] f32 state per recurrent
-    layer (rows padded to 16 bytes) and the tail of each convolution.  A
+    layer (rows padded to 16 bytes), its scalars if it has any, and the tail
+    of each convolution.  A
     slot is not cleared when it changes hands: what a sequence's first rows
     would read is zero by position."""
 
@@ -89,6 +97,7 @@ class RecurrentStates:
                  dtype: torch.dtype = torch.bfloat16) -> None:
         self.n_slots = n_slots
         self._layers: dict[int, torch.Tensor] = {}
+        self._scalars: dict[int, torch.Tensor] = {}
         self._tails: dict[int, torch.Tensor] = {}
         for i, spec in enumerate(layers):
             for s in layer_parts(spec):
@@ -96,6 +105,10 @@ class RecurrentStates:
                     self._layers[i] = torch.zeros(
                         (n_slots, s.heads, s.dim, -(-s.vdim // 4) * 4),
                         dtype=torch.float32, device=device)
+                elif isinstance(s, ScalarLayer):
+                    self._scalars[i] = torch.zeros(
+                        (n_slots, s.heads), dtype=torch.float32,
+                        device=device)
                 elif isinstance(s, TailLayer):
                     self._tails[i] = torch.zeros(
                         (n_slots, s.rows, s.width), dtype=dtype,
@@ -104,11 +117,14 @@ class RecurrentStates:
 
     @staticmethod
     def needed(layers: list) -> bool:
-        return any(isinstance(s, (StateLayer, TailLayer))
+        return any(isinstance(s, (StateLayer, ScalarLayer, TailLayer))
                    for spec in layers for s in layer_parts(spec))
 
     def layer(self, i: int) -> torch.Tensor:
         return self._layers[i]
+
+    def scalar(self, i: int) -> torch.Tensor:
+        return self._scalars[i]
 
     def tail(self, i: int) -> Optional[torch.Tensor]:
         return self._tails.get(i)
@@ -128,19 +144,22 @@ class RecurrentStates:
     def cast(self, dtype: torch.dtype) -> None:
         self._tails = {i: t.to(dtype) for i, t in self._tails.items()}
 
+    def _kinds(self) -> dict:
+        return {"states": self._layers, "scalars": self._scalars,
+                "tails": self._tails}
+
     def export(self, slot: int) -> dict:
-        return {"states": {i: t[slot].cpu() for i, t in self._layers.items()},
-                "tails": {i: t[slot].cpu() for i, t in self._tails.items()}}
+        return {kind: {i: t[slot].cpu() for i, t in held.items()}
+                for kind, held in self._kinds().items()}
 
     def import_(self, slot: int, payload: dict) -> None:
-        for i, t in self._layers.items():
-            t[slot].copy_(payload["states"][i])
-        for i, t in self._tails.items():
-            t[slot].copy_(payload["tails"][i])
+        for kind, held in self._kinds().items():
+            for i, t in held.items():
+                t[slot].copy_(payload[kind][i])
 
     def bytes_used(self) -> int:
-        return sum(t.numel() * t.element_size() for t in
-                   (*self._layers.values(), *self._tails.values()))
+        return sum(t.numel() * t.element_size()
+                   for held in self._kinds().values() for t in held.values())
 
 
 class PagedKVCache:

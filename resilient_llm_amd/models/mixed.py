@@ -49,6 +49,18 @@ class MixedConfig:
         self.max_position = n
 
 
+@dataclasses.dataclass
+class Step:
+    """What a step's mixers need besides their input rows."""
+    positions: torch.Tensor
+    slots: torch.Tensor              # cache slot of every row
+    n_decode: int
+    tables_dec: Optional[torch.Tensor]
+    state_slots: Optional[torch.Tensor]
+    tables_pre: Optional[torch.Tensor] = None
+    prompt: object = None            # PromptRows
+
+
 class MixedModel:
     # the engine hands prompt rows and state slots to such a model
     mixed_layers = True
@@ -171,3 +183,36 @@ class MixedModel:
 
     def param_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in self.params.values())
+
+    # ------------------------------------------------------------ compute
+    def _forward(self, input_ids, kv_cache, step: Step, sample_idx):
+        """Logits of ``sample_idx`` rows (None: all) of one step."""
+        raise NotImplementedError
+
+    def _reduce(self, *ys: torch.Tensor):
+        """Sums of row-parallel products over the ranks."""
+        if self.tp_world > 1:
+            import torch.distributed as dist
+            for y in ys:
+                dist.all_reduce(y, group=self.tp_group)
+        return ys if len(ys) > 1 else ys[0]
+
+    def forward_decode(self, input_ids, positions, kv_cache, slot_mapping,
+                       block_tables, seq_lens, state_slots=None):
+        """One token per sequence; returns [batch, vocab] logits."""
+        return self._forward(
+            input_ids, kv_cache, Step(
+                positions, slot_mapping, input_ids.shape[0], block_tables,
+                state_slots), None)
+
+    def forward_mixed(self, input_ids, positions, kv_cache, slot_mapping,
+                      n_decode: int, block_tables_dec, seq_lens_dec,
+                      block_tables_pre, prompt, sample_idx,
+                      state_slots=None):
+        """Rows [0, n_decode) decode one token per sequence, the rest are
+        the portions of ``prompt`` (engine/batch.py).  Returns the logits
+        of ``sample_idx`` rows."""
+        return self._forward(
+            input_ids, kv_cache, Step(
+                positions, slot_mapping, n_decode, block_tables_dec,
+                state_slots, block_tables_pre, prompt), sample_idx)

@@ -7,17 +7,19 @@ import json
 import os
 from typing import Optional
 
+from .bolatar import BOLATAR_PRESETS, BolatarConfig, BolatarForCausalLM
 from .llama import MODEL_PRESETS, LlamaConfig, LlamaForCausalLM
 from .mixed import MixedModel
 from .nesizen import NESIZEN_PRESETS, NesizenConfig, NesizenForCausalLM
 from .riruzen import RIRUZEN_PRESETS, RiruzenConfig, RiruzenForCausalLM
 
 # config.json 'architecture' -> (configuration, model)
-ARCHITECTURES = {"Nesizen": (NesizenConfig, NesizenForCausalLM),
+ARCHITECTURES = {"Bolatar": (BolatarConfig, BolatarForCausalLM),
+                 "Nesizen": (NesizenConfig, NesizenForCausalLM),
                  "Riruzen": (RiruzenConfig, RiruzenForCausalLM)}
 _MODELS = {LlamaConfig: LlamaForCausalLM, **dict(ARCHITECTURES.values())}
 # presets that are made when asked for
-_MADE_PRESETS = {**NESIZEN_PRESETS, **RIRUZEN_PRESETS}
+_MADE_PRESETS = {**BOLATAR_PRESETS, **NESIZEN_PRESETS, **RIRUZEN_PRESETS}
 
 
 def model_names() -> list:

@@ -21,7 +21,6 @@ the convolution tails have the model dtype, which may also be float32.
 from __future__ import annotations
 
 import dataclasses
-from typing import Optional
 
 import torch
 
@@ -265,12 +264,6 @@ class RiruzenForCausalLM(MixedModel):
         P["final.norm"] = vec("final.norm") * self.config.logit_scale
 
     # ------------------------------------------------------------ compute
-    def _reduce(self, y: torch.Tensor) -> torch.Tensor:
-        if self.tp_world > 1:
-            import torch.distributed as dist
-            dist.all_reduce(y, group=self.tp_group)
-        return y
-
     def _latent(self, i, m, proj, kv_cache, step, out) -> None:
         P, p, nd = self.params, f"l{i}.", step.n_decode
         cache, = kv_cache.layer(i)
@@ -341,35 +334,3 @@ class RiruzenForCausalLM(MixedModel):
                     x, y, P["final.norm"], c.norm_groups, c.rms_eps,
                     step.positions, rows=sample_idx, keep=False)
         return _linear(h, P["embed"])
-
-    def forward_decode(self, input_ids, positions, kv_cache, slot_mapping,
-                       block_tables, seq_lens, state_slots=None):
-        """One token per sequence; returns [batch, vocab] logits."""
-        return self._forward(
-            input_ids, kv_cache, _Step(
-                positions, slot_mapping, input_ids.shape[0], block_tables,
-                state_slots), None)
-
-    def forward_mixed(self, input_ids, positions, kv_cache, slot_mapping,
-                      n_decode: int, block_tables_dec, seq_lens_dec,
-                      block_tables_pre, prompt, sample_idx,
-                      state_slots=None):
-        """Rows [0, n_decode) decode one token per sequence, the rest are
-        the portions of ``prompt`` (engine/batch.py).  Returns the logits
-        of ``sample_idx`` rows."""
-        return self._forward(
-            input_ids, kv_cache, _Step(
-                positions, slot_mapping, n_decode, block_tables_dec,
-                state_slots, block_tables_pre, prompt), sample_idx)
-
-
-@dataclasses.dataclass
-class _Step:
-    """What a step's mixers need besides their input rows."""
-    positions: torch.Tensor
-    slots: torch.Tensor              # cache slot of every row
-    n_decode: int
-    tables_dec: Optional[torch.Tensor]
-    state_slots: Optional[torch.Tensor]
-    tables_pre: Optional[torch.Tensor] = None
-    prompt: object = None            # PromptRows
