@@ -19,10 +19,10 @@ Launch (driver):
   python -m torch.distributed.run --nnodes=1 --nproc-per-node N \
       --master-addr 127.0.0.1 bench.py --gpus N --steps K --warmup W
 
-`--design nesizen` measures something else: engine-level prefill and
-decode throughput of Nesizen at layer sizes of real models, beside a
-Llama of equal width, depth and active parameters (one JSON line per
-model and size; see run_design).
+`--design nesizen` (or riruzen, bolatar) measures something else:
+engine-level prefill and decode throughput of that design at layer sizes of
+real models, beside existing models of equal width, depth and active
+parameters (one JSON line per model and size; see run_design).
 """
 
 from __future__ import annotations
@@ -180,9 +180,9 @@ def design_models(design: str) -> dict:
     """size -> {name: configuration}: the design, then existing models of
     equal width, depth, heads and (active) feed-forward size."""
     from resilient_llm_amd.models import (
-        LlamaConfig, NesizenConfig, RiruzenConfig,
+        BolatarConfig, LlamaConfig, NesizenConfig, RiruzenConfig,
     )
-    from resilient_llm_amd.models import nesizen, riruzen
+    from resilient_llm_amd.models import bolatar, nesizen, riruzen
 
     def llama(width, layers, heads, kv, ff):
         return LlamaConfig(name=f"llama-w{width}", hidden_size=width,
@@ -219,8 +219,34 @@ def design_models(design: str) -> dict:
                  {"heads": heads, "dim": 128, "vdim": 128},
                  {"kind": "dense", "ff": ff})}, name=f"riruzen-w{width}")
 
+    def bola(width, layers, heads, kv, ff):
+        return BolatarConfig.from_dict(
+            {"width": width, "vocab": 65536, "logit_softcap": 30.0,
+             "max_positions": 32768, "embedding": {"scale": 1.0},
+             "norm": {"eps": 1e-5},
+             "layers": bolatar.hybrid_layers(
+                 layers, 3,
+                 {"left": {"heads": heads, "kv_heads": kv, "dim": 128,
+                           "vdim": 128, "scale": 128 ** -0.5,
+                           "q_temp": {"coef": 0.1, "every": 4096}},
+                  "right": {"heads": heads, "dim": 64}},
+                 {"heads": heads, "kv_heads": heads // 2, "dim": 128,
+                  "vdim": 128, "conv": 4},
+                 {"heads": heads // 2, "dim": 128, "vdim": 256,
+                  "gate_cap": 15.0},
+                 {"kind": "dense", "ff": ff, "limit": 7.0})},
+            name=f"bolatar-w{width}", decay_rank=64)
+
     def dense(ff):
         return {"kind": "dense", "ff": ff}
+    if design == "bolatar":
+        # two matrices of 3/2 the width are as large as the gated three
+        return {"w2048": {"bolatar": bola(2048, 12, 16, 4, 4096),
+                          "nesizen": nesi(2048, 12, 16, 4, 8, dense(6144)),
+                          "llama": llama(2048, 12, 16, 4, 4096)},
+                "w4096": {"bolatar": bola(4096, 6, 32, 8, 7168),
+                          "nesizen": nesi(4096, 6, 32, 8, 16, dense(10752)),
+                          "llama": llama(4096, 6, 32, 8, 7168)}}
     if design == "nesizen":
         return {"w2048": {"nesizen": nesi(2048, 12, 16, 4, 8,
                                           moe(32, 4, 1024), dense(6144)),
@@ -337,7 +363,7 @@ def main() -> None:
                          "headline metric stays bf16)")
     ap.add_argument("--device", default=None,
                     help="override torch device (tests: cpu)")
-    ap.add_argument("--design", default=None, choices=("nesizen", "riruzen"),
+    ap.add_argument("--design", default=None, choices=("nesizen", "riruzen", "bolatar"),
                     help="measure this design's engine throughput beside "
                          "existing models of equal size instead of serving")
     ap.add_argument("--design-sizes", default="w2048,w4096")

@@ -366,6 +366,7 @@ void prefill(const DeltaArgs& a, hipStream_t st) {
   sa.o = a.o;
   sa.tiles = a.tiles;
   sa.seqs = a.seqs;
+  sa.n_rows = a.rows;
   sa.n_tiles = a.n_tiles;
   sa.n_seqs = a.n_seqs;
   sa.heads = a.heads;

@@ -149,7 +149,7 @@ void prefill(rlli::GlaArgs& a, const Tensor& proj, const Tensor& tiles,
   Tensor kd = at::empty({nh, a.dpad, C}, fo);
   Tensor sc = at::empty({nh, C, C}, fo);
   Tensor dec = at::empty({nh, a.dpad}, fo);
-  Tensor o = at::empty({a.rows, int64_t(a.heads) * a.vdim}, fo);
+  Tensor o = at::empty({a.rows + C, int64_t(a.heads) * a.vdim}, fo);
   a.qd = qd.data_ptr<float>();
   a.kd = kd.data_ptr<float>();
   a.sc = sc.data_ptr<float>();
@@ -292,7 +292,7 @@ void delta_prefill(const Tensor& proj, const Tensor& x, const Tensor& a_rate,
   Tensor row_f = at::empty({nh, 3, C}, fo);
   Tensor w = at::empty({nh, C, a.dpad}, fo);
   Tensor ub = at::empty({nh, C, a.ubp}, fo);
-  Tensor o = at::empty({a.rows, int64_t(a.heads) * a.vdim}, fo);
+  Tensor o = at::empty({a.rows + C, int64_t(a.heads) * a.vdim}, fo);
   a.kt = kt.data_ptr();
   a.sc = sc.data_ptr<float>();
   a.dec = dec.data_ptr<float>();
@@ -363,8 +363,8 @@ void mlstm_prefill(const Tensor& proj, const Tensor& i_bias,
   Tensor kt = at::empty({nh, a.dpad, C}, proj.options());
   Tensor sc = at::empty({nh, C, C}, fo);
   Tensor row_f = at::empty({nh, 3, C}, fo);
-  Tensor o = at::empty({a.rows, a.heads, a.opad}, fo);
-  Tensor mrow = at::empty({a.rows, a.heads}, fo);
+  Tensor o = at::empty({a.rows + C, a.heads, a.opad}, fo);
+  Tensor mrow = at::empty({a.rows + C, a.heads}, fo);
   Tensor m_new = at::empty({a.n_seqs, a.heads}, fo);
   a.kt = kt.data_ptr();
   a.sc = sc.data_ptr<float>();

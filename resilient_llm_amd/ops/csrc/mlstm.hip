@@ -197,6 +197,7 @@ void prefill(const MlstmArgs& a, hipStream_t st) {
   sa.mrow = a.mrow;
   sa.tiles = a.tiles;
   sa.seqs = a.seqs;
+  sa.n_rows = a.rows;
   sa.n_tiles = a.n_tiles;
   sa.n_seqs = a.n_seqs;
   sa.heads = a.heads;

@@ -39,12 +39,12 @@ struct ScanArgs {
   float* state;            // [slots, heads, dim, vpad]
   const float* m;          // [slots, heads] (max)
   float* m_new;            // [n_seqs, heads] (max)
-  float* o;                // [rows, heads, opad]
-  float* mrow;             // [rows, heads] (max)
+  float* o;                // [rows + 64, heads, opad], spare rows behind
+  float* mrow;             // [rows + 64, heads] (max)
   const int32_t* tiles;    // [4, n_tiles] chunks of kRecChunk rows
   const int32_t* seqs;     // [4, n_seqs]: first tile, tiles, pos0, slot
   int64_t v_stride, q_stride;
-  int n_tiles, n_seqs, heads, group, dim, dpad, vdim, vpad, opad, ubp;
+  int n_rows, n_tiles, n_seqs, heads, group, dim, dpad, vdim, vpad, opad, ubp;
   int cols;                // value columns of state and o
   float qscale;            // (max)
   int mode;
@@ -92,7 +92,7 @@ struct GlaArgs {
   float* kd;               // [n_tiles, heads, dpad, 64]
   float* sc;               // [n_tiles, heads, 64, 64]
   float* dec;              // [n_tiles, heads, dpad]
-  float* o;                // [rows, heads * vdim]
+  float* o;                // [rows + 64, heads * vdim]
   void* out;               // [rows, heads * vdim], rows out_stride apart
   int64_t off_k, off_v, off_g;  // from proj
   int64_t stride, a1_stride;
@@ -151,7 +151,7 @@ struct MlstmArgs {
   void* kt;                // scratch, see ScanArgs
   float* sc;
   float* row_f;
-  float* o;                // [rows, heads, opad]
+  float* o;                // [rows + 64, heads, opad]
   float* mrow;
   float* m_new;
   void* out;               // [rows, heads * vdim], rows out_stride apart

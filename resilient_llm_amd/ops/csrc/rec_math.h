@@ -98,6 +98,50 @@ DEV_INLINE f32x4_t load4_guard(const T* p, int d, int dim, bool row_ok,
   return v;
 }
 
+// four columns as they lie in memory: a load's registers are not touched
+// (and so not waited for) until the values are used
+template <typename T> struct Raw4;
+template <> struct Raw4<uint16_t> {
+  uint2 r;
+  DEV_INLINE void zero() { r = uint2{0, 0}; }
+  DEV_INLINE void load(const uint16_t* p) {
+    r = *reinterpret_cast<const uint2*>(p);
+  }
+  DEV_INLINE void put(int j, uint16_t v) {
+    uint32_t& x = j < 2 ? r.x : r.y;
+    x |= uint32_t(v) << (j % 2 * 16);
+  }
+  DEV_INLINE float get(int j) const {
+    const uint32_t x = j < 2 ? r.x : r.y;
+    return __uint_as_float(j % 2 ? x & 0xffff0000u : x << 16);
+  }
+};
+template <> struct Raw4<float> {
+  f32x4_t r;
+  DEV_INLINE void zero() { r = f32x4_t{0.f, 0.f, 0.f, 0.f}; }
+  DEV_INLINE void load(const float* p) {
+    r = *reinterpret_cast<const f32x4_t*>(p);
+  }
+  DEV_INLINE void put(int j, float v) { r[j] = v; }
+  DEV_INLINE float get(int j) const { return r[j]; }
+};
+
+template <typename T>
+DEV_INLINE Raw4<T> raw_guard(const T* p, int d, int dim, bool row_ok,
+                             bool vec) {
+  Raw4<T> v;
+  if (vec && row_ok && d + 4 <= dim) {
+    v.load(p + d);
+    return v;
+  }
+  v.zero();
+  if (!row_ok) return v;
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    if (d + j < dim) v.put(j, p[d + j]);
+  return v;
+}
+
 // eight columns of a row as a matrix operand
 template <typename T>
 DEV_INLINE Frag8<T> frag_guard(const T* p, int d, int dim, bool row_ok,
