@@ -303,7 +303,10 @@ def tensor_shapes(config, rank=8):
 def random_weights(config, seed=0, rank=8):
     """bfloat16 weights that keep every mechanism audible: unit-gain
     linears, norms a little off one, audible taps, decays from slow to
-    fast, input gates of either sign, distance biases that matter."""
+    fast, input gates of either sign, distance biases that matter.  Keys of
+    the recurrences lean towards their queries: a sequence's first read-outs
+    are normed, so a product near zero would decide their sign by rounding.
+    """
     g = torch.Generator().manual_seed(seed)
     out = {}
     for name, shape in tensor_shapes(config, rank).items():
@@ -325,7 +328,7 @@ def random_weights(config, seed=0, rank=8):
         elif leaf.endswith("w0"):
             t = -5 + 5 * u
         elif leaf.endswith(".u"):
-            t = 0.8 * t
+            t = 0.8 + 0.3 * t
         elif leaf == "mix.i.b":
             t = 1.5 * t
         elif leaf == "mix.f.b":
@@ -338,5 +341,9 @@ def random_weights(config, seed=0, rank=8):
             t = 0.5 * t
         elif name != "embed":
             t = t * 1.2 / math.sqrt(shape[-1])
-        out[name] = t.to(torch.bfloat16)
-    return out
+        out[name] = t
+    for name in list(out):
+        q = name[:-1] + ("r" if name.endswith("right.k") else "q")
+        if name.endswith((".mix.k", ".right.k")):
+            out[name] = 0.6 * out[q] + 0.8 * out[name]
+    return {name: t.to(torch.bfloat16) for name, t in out.items()}
