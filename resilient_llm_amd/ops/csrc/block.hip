@@ -111,6 +111,8 @@ void block_step_kernel(BlockArgs a) {
   constexpr int EARLY = CONV && (IT == 1 || IT == 2) ? 4 : 0;   // taps
   float u[ITS][V], t[ITS][V], gain[ITS][V];
   float tap[ITS][EARLY + 1][V], past[ITS][EARLY + 1][V];
+  constexpr int MORE = EARLY > 0 ? 4 : 0; // further branches of two taps
+  float btap[ITS][MORE + 1][2][V];
   auto every = [&](auto body) {           // over this thread's vectors
     if constexpr (IT > 0) {
 #pragma unroll
@@ -136,6 +138,13 @@ void block_step_kernel(BlockArgs a) {
 #pragma unroll
         for (int k = 0; k < EARLY; ++k)
           if (k <= back) load_tap(0, k, v * V, tap[i][k]);
+        if (a.n_taps == 2)
+#pragma unroll
+          for (int b = 0; b < MORE; ++b)
+            if (b + 1 < a.branches) {
+              load_tap(b + 1, 0, v * V, btap[i][b][0]);
+              load_tap(b + 1, 1, v * V, btap[i][b][1]);
+            }
       });
   }
   int pos = 0, at = 0;                    // position, its row of the ring
@@ -227,7 +236,27 @@ void block_step_kernel(BlockArgs a) {
       hv[j] = round_act(T{}, u[i][j] * inv * gain[i][j]);
     store_v<T, V>(hr + c, hv);
     if (conv) {
-      for (int b = 0; b < a.branches; ++b) {
+      int b0 = 0;
+      if (MORE > 0 && a.n_taps == 2 && a.branches > 1) {
+        b0 = min(a.branches, MORE + 1);
+#pragma unroll
+        for (int b = 0; b < MORE + 1; ++b) {
+          if (b >= a.branches) break;
+          float o[V];
+#pragma unroll
+          for (int j = 0; j < V; ++j) {
+            o[j] = hv[j] + (b == 0 ? tap[i][0][j] : btap[i][b - 1][0][j]) *
+                               hv[j];
+            if (pos > 0)
+              o[j] += (b == 0 ? tap[i][MORE > 0 ? 1 : 0][j]
+                              : btap[i][b - 1][1][j]) *
+                      past[i][MORE > 0 ? 1 : 0][j];
+          }
+          store_v<T, V>(reinterpret_cast<T*>(a.hc) +
+                            (int64_t(b) * a.n + n) * W + c, o);
+        }
+      }
+      for (int b = b0; b < a.branches; ++b) {
         float o[V];
 #pragma unroll
         for (int j = 0; j < V; ++j) o[j] = hv[j];

@@ -39,14 +39,14 @@ DEV_INLINE float delta_log_decay(float a, float bias, float rate) {
 }
 
 // REG: a thread's part of the state fits its registers
-template <typename T, bool REG>
-__global__ __launch_bounds__(256)
+// (U rows); NT threads: many when there are few heads to fill the chip with
+template <typename T, bool REG, int NT, int U>
+__global__ __launch_bounds__(NT)
 void delta_decode_kernel(DeltaArgs a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  constexpr int U = 16;
   const int seq = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int group = a.heads / a.kv_heads, kvh = h / group;
-  const int v4n = a.vpad / 4, n_rows = 256 / v4n;
+  const int v4n = a.vpad / 4, n_rows = NT / v4n;
   float* qs = sm;                         // [dim]
   float* ks = qs + a.dpad;                // [dim]
   float* vs = ks + a.dpad;                // [vdim]
@@ -72,7 +72,7 @@ void delta_decode_kernel(DeltaArgs a) {
 
   const int back = a.n_taps - 1, CH = a.channels;
   T* ring = reinterpret_cast<T*>(a.tail) + int64_t(slot) * a.ring * CH;
-  for (int e = tid; e < 2 * a.dim + a.vdim; e += 256) {
+  for (int e = tid; e < 2 * a.dim + a.vdim; e += NT) {
     const int part = e < a.dim ? 0 : e < 2 * a.dim ? 1 : 2;
     const int c = part == 0 ? kvh * a.dim + e
                   : part == 1
@@ -89,15 +89,15 @@ void delta_decode_kernel(DeltaArgs a) {
        : part == 1 ? a.dpad + e - a.dim
                    : 2 * a.dpad + e - 2 * a.dim] = round_act(T{}, silu<T>(y));
   }
-  for (int e = a.vdim + tid; e < a.vpad; e += 256) vs[e] = 0.f;
+  for (int e = a.vdim + tid; e < a.vpad; e += NT) vs[e] = 0.f;
   __syncthreads();
   float qq = 0.f, kk = 0.f, qk = 0.f;
-  for (int d = tid; d < a.dim; d += 256) {
+  for (int d = tid; d < a.dim; d += NT) {
     qq += qs[d] * qs[d];
     kk += ks[d] * ks[d];
     qk += qs[d] * ks[d];
   }
-  __shared__ float part[4][4];
+  __shared__ float part[4][NT / 64];
   qq = wave_sum(qq);
   kk = wave_sum(kk);
   qk = wave_sum(qk);
@@ -131,13 +131,16 @@ void delta_decode_kernel(DeltaArgs a) {
   }
   __syncthreads();
   auto total = [&](int i) {
-    return part[i][0] + part[i][1] + part[i][2] + part[i][3];
+    float s = 0.f;
+#pragma unroll
+    for (int k = 0; k < NT / 64; ++k) s += part[i][k];
+    return s;
   };
   const float kn = 1.f / sqrtf(total(1) + 1e-6f);
   const float qn = 1.f / sqrtf(total(0) + 1e-6f) / sqrtf(float(a.dim));
   const float dot = total(2) * qn * kn;
   float ss = 0.f;
-  for (int e = tid; e < a.vpad; e += 256) {
+  for (int e = tid; e < a.vpad; e += NT) {
     float sk = 0.f, sq = 0.f;
     for (int r = 0; r < n_rows; ++r) {
       sk += rk[r * a.vpad + e];
@@ -172,20 +175,22 @@ void delta_decode_kernel(DeltaArgs a) {
   const float inv = 1.f / sqrtf(total(3) / a.vdim + a.eps);
   T* out = reinterpret_cast<T*>(a.out) + int64_t(seq) * a.out_stride +
            h * a.vdim;
-  for (int e = tid; e < a.vdim; e += 256)
+  for (int e = tid; e < a.vdim; e += NT)
     act_store(out + e, rq[e] * inv * a.norm[e] *
                            silu<T>(act_load(row + a.off_g + h * a.vdim + e)));
 }
 
-template <typename T>
+// ND: 32-column steps of a key (0: any)
+template <typename T, bool VEC, int ND>
 __global__ __launch_bounds__(256)
-void delta_intra_kernel(DeltaArgs a, bool vec) {
+void delta_intra_kernel(DeltaArgs a) {
   __shared__ __attribute__((aligned(16))) float Tm[C * TR];   // [64][TR] below the diagonal
   __shared__ __attribute__((aligned(16))) float Dv[4 * 16 * DR];   // inverted diagonal blocks
   __shared__ float qn[C], kn[C], be[C], G[C];
   const int tile = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int group = a.heads / a.kv_heads, kvh = h / group;
-  const int lane = tid & 63, w = tid >> 6;
+  const int lane = tid & 63;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int lr = lane & 15, g = lane >> 4;
   const int row0 = a.tiles[tile], n = a.tiles[2 * a.n_tiles + tile];
   const T* xb = reinterpret_cast<const T*>(a.x) + int64_t(row0) * a.x_stride;
@@ -194,54 +199,46 @@ void delta_intra_kernel(DeltaArgs a, bool vec) {
   const T* vb = xb + 2 * a.kv_heads * a.dim + h * a.vdim;
   const int64_t ch = int64_t(tile) * a.heads + h;
 
-  // products of the rows as they are: own rows down, block J's rows across
+  // Products of the rows as they are: own rows down, block J's rows across.
+  // Rows behind the last one repeat it; their beta is zero.
   f32x4_t qk[4], kk[4];
 #pragma unroll
   for (int J = 0; J < 4; ++J) qk[J] = kk[J] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  const int trow = w * 16 + lr;
-  for (int d0 = 0; d0 < a.dim; d0 += 32) {
-    const int d = d0 + g * 8;
-    const auto qf = frag_guard(qb + trow * a.x_stride, d, a.dim, trow < n, vec);
-    Frag8<T> kf[4];
+  float sq = 0.f, sk = 0.f;               // squares of row w * 16 + lr
+  const int steps = ND > 0 ? ND : (a.dim + 31) / 32;
+  constexpr int SU = ND > 0 ? ND : 1;
+  for (int st = 0; st < steps; st += SU) {
+    Frag8<T> qf[SU], kf[SU][4];
 #pragma unroll
-    for (int J = 0; J < 4; ++J)
-      if (J <= w)
-        kf[J] = frag_guard(kb + (J * 16 + lr) * a.x_stride, d, a.dim,
-                           J * 16 + lr < n, vec);
-    Frag8<T> own = kf[0];
+    for (int u = 0; u < SU; ++u) {
+      const int d = (st + u) * 32 + g * 8;
+      qf[u] = frag_at<VEC>(qb + min(w * 16 + lr, n - 1) * a.x_stride, d,
+                           a.dim);
 #pragma unroll
-    for (int J = 1; J < 4; ++J)
-      if (J == w) own = kf[J];
+      for (int J = 0; J < 4; ++J)         // (blocks behind w: not used)
+        kf[u][J] = frag_at<VEC>(
+            kb + min(min(J, w) * 16 + lr, n - 1) * a.x_stride, d, a.dim);
+    }
 #pragma unroll
-    for (int J = 0; J < 4; ++J)
-      if (J <= w) {
-        qk[J] = Frag8<T>::mma(qf, kf[J], qk[J]);
-        kk[J] = Frag8<T>::mma(own, kf[J], kk[J]);
-      }
-  }
-  {
-    const int t = tid >> 2, p = tid & 3;  // four threads per row
-    float sq = 0.f, sk = 0.f;
-    for (int d = p * 8; d < a.dim; d += 32) {
+    for (int u = 0; u < SU; ++u) {
+      const Frag8<T> own = kf[u][3];      // min(3, w) = w
+      sq += frag_sq(qf[u]);
+      sk += frag_sq(own);
 #pragma unroll
-      for (int half = 0; half < 8; half += 4) {
-        const f32x4_t qv = load4_guard(qb + t * a.x_stride, d + half, a.dim,
-                                       t < n, vec);
-        const f32x4_t kv = load4_guard(kb + t * a.x_stride, d + half, a.dim,
-                                       t < n, vec);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          sq += qv[j] * qv[j];
-          sk += kv[j] * kv[j];
+      for (int J = 0; J < 4; ++J)
+        if (J <= w) {
+          qk[J] = Frag8<T>::mma(qf[u], kf[u][J], qk[J]);
+          kk[J] = Frag8<T>::mma(own, kf[u][J], kk[J]);
         }
-      }
     }
-    sq = group_sum<4>(sq);
-    sk = group_sum<4>(sk);
-    if (p == 0) {
-      qn[t] = 1.f / sqrtf(sq + 1e-6f) / sqrtf(float(a.dim));
-      kn[t] = 1.f / sqrtf(sk + 1e-6f);
-    }
+  }
+  sq += __shfl_xor(sq, 16, kWave);
+  sk += __shfl_xor(sk, 16, kWave);
+  sq += __shfl_xor(sq, 32, kWave);
+  sk += __shfl_xor(sk, 32, kWave);
+  if (g == 0) {
+    qn[w * 16 + lr] = 1.f / sqrtf(sq + 1e-6f) / sqrtf(float(a.dim));
+    kn[w * 16 + lr] = 1.f / sqrtf(sk + 1e-6f);
   }
   if (tid < C) {
     float lg = 0.f, b = 0.f;
@@ -290,9 +287,9 @@ void delta_intra_kernel(DeltaArgs a, bool vec) {
     }
   }
   if (h % group == 0)
-    keys_down(kb, a.x_stride, n, a.dim, a.dpad, vec,
-              reinterpret_cast<T*>(a.kt) +
-                  (int64_t(tile) * a.kv_heads + kvh) * a.dpad * C);
+    keys_down<VEC>(kb, a.x_stride, n, a.dim, a.dpad,
+                   reinterpret_cast<T*>(a.kt) +
+                       (int64_t(tile) * a.kv_heads + kvh) * a.dpad * C);
   __syncthreads();
   f32x4_t tf[6], df[4];                   // blocks 10 20 21 30 31 32
 #pragma unroll
@@ -310,23 +307,21 @@ void delta_intra_kernel(DeltaArgs a, bool vec) {
   for (int ct = w; ct < nv + nk; ct += 4) {
     const bool val = ct < nv;
     const int c = (val ? ct : ct - nv) * 16 + lr;
-    const T* src = (val ? vb : kb) + c;
-    const bool c_ok = c < (val ? a.vdim : a.dim);
+    // (columns behind the last one meet zeros of the state, or nothing)
+    const T* src = (val ? vb : kb) + min(c, (val ? a.vdim : a.dim) - 1);
+    T raw[16];
+#pragma unroll
+    for (int k = 0; k < 16; ++k)
+      raw[k] = src[min(k / 4 * 16 + g * 4 + k % 4, n - 1) * a.x_stride];
     f32x4_t u[4];
-#pragma unroll
-    for (int I = 0; I < 4; ++I)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = I * 16 + g * 4 + r;
-        u[I][r] = c_ok && t < n ? act_load(src + t * a.x_stride) : 0.f;
-      }
 #pragma unroll
     for (int I = 0; I < 4; ++I) {
       f32x4_t acc;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int t = I * 16 + g * 4 + r;
-        acc[r] = u[I][r] * be[t] * (val ? 1.f : kn[t] * gexp<T>(G[t]));
+        acc[r] = act_load(&raw[I * 4 + r]) * be[t] *
+                 (val ? 1.f : kn[t] * gexp<T>(G[t]));
       }
 #pragma unroll
       for (int K = 0; K < I; ++K)
@@ -347,12 +342,25 @@ void delta_intra_kernel(DeltaArgs a, bool vec) {
   }
 }
 
+// VEC and the number of 32-column steps (0: any) of a chunk kernel
+template <typename F>
+void by_dim(int dim, bool vec, F f) {
+  using std::integral_constant;
+  if (!vec) f(std::false_type{}, integral_constant<int, 0>{});
+  else if (dim == 64) f(std::true_type{}, integral_constant<int, 2>{});
+  else if (dim == 128) f(std::true_type{}, integral_constant<int, 4>{});
+  else f(std::true_type{}, integral_constant<int, 0>{});
+}
+
 template <typename T>
 void prefill(const DeltaArgs& a, hipStream_t st) {
   const bool vec = a.dim % 8 == 0 && a.x_stride % 8 == 0 &&
                    reinterpret_cast<uintptr_t>(a.x) % 16 == 0;
-  hipLaunchKernelGGL(delta_intra_kernel<T>, dim3(a.n_tiles, a.heads),
-                     dim3(256), 0, st, a, vec);
+  by_dim(a.dim, vec, [&](auto v, auto nd) {
+    hipLaunchKernelGGL(
+        (delta_intra_kernel<T, decltype(v)::value, decltype(nd)::value>),
+        dim3(a.n_tiles, a.heads), dim3(256), 0, st, a);
+  });
   ScanArgs sa{};
   sa.q = a.x;
   sa.q_stride = a.x_stride;
@@ -399,19 +407,22 @@ void prefill(const DeltaArgs& a, hipStream_t st) {
 
 void launch_delta_decode(const DeltaArgs& a, hipStream_t st) {
   if (a.rows == 0) return;
-  const int n_rows = 256 / (a.vpad / 4);
-  const size_t smem =
-      size_t(2 * a.dpad + a.vpad + 2 * n_rows * a.vpad) * sizeof(float);
-  const bool reg = a.dim <= 16 * n_rows;
-  auto go = [&](auto* k) {
-    hipLaunchKernelGGL(k, dim3(a.rows, a.heads), dim3(256), smem, st, a);
+  auto go = [&](auto* k, int nt) {
+    const int n_rows = nt / (a.vpad / 4);
+    const size_t smem =
+        size_t(2 * a.dpad + a.vpad + 2 * n_rows * a.vpad) * sizeof(float);
+    hipLaunchKernelGGL(k, dim3(a.rows, a.heads), dim3(nt), smem, st, a);
   };
+  const bool few = int64_t(a.rows) * a.heads < 256;
+  const bool reg = a.dim <= 16 * (256 / (a.vpad / 4));
   if (a.f32) {
-    if (reg) go(delta_decode_kernel<float, true>);
-    else go(delta_decode_kernel<float, false>);
+    if (reg) go(delta_decode_kernel<float, true, 256, 16>, 256);
+    else go(delta_decode_kernel<float, false, 256, 16>, 256);
+  } else if (few && a.dim <= 4 * (1024 / (a.vpad / 4))) {
+    go(delta_decode_kernel<uint16_t, true, 1024, 4>, 1024);
   } else {
-    if (reg) go(delta_decode_kernel<uint16_t, true>);
-    else go(delta_decode_kernel<uint16_t, false>);
+    if (reg) go(delta_decode_kernel<uint16_t, true, 256, 16>, 256);
+    else go(delta_decode_kernel<uint16_t, false, 256, 16>, 256);
   }
 }
 

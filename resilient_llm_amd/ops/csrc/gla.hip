@@ -184,17 +184,20 @@ DEV_INLINE float seen_log(float L) {
 }
 
 // Wave w owns sub-chunk w, lane l its row l & 15 and four neighbouring key
-// columns of every 16; MD bounds the key tiles (dpad <= 64 * MD).
-template <typename T, int KIND, int MD>
+// columns of every 16; MD bounds the key tiles (dpad <= 64 * MD).  FULL: dim
+// is 64 MD, the rank a multiple of 16 and rows are aligned, so that no load
+// is conditional (rows behind the last one are loaded from it).
+template <typename T, int KIND, int MD, bool FULL>
 __global__ __launch_bounds__(256)
 void gla_intra_kernel(GlaArgs a, bool vec, bool vec_a) {
   constexpr bool FG = KIND == kHgrn2, BONUS = KIND == kRwkv;
   extern __shared__ __attribute__((aligned(16))) float sm[];
   constexpr int NT = 4 * MD;
   const int tile = blockIdx.x, h = blockIdx.y;
-  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int lane = threadIdx.x & 63;
+  const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int lr = lane & 15, g = lane >> 4;
-  const int DP = a.dpad, LR = DP + 4, ndt = DP / 16;
+  const int DP = FULL ? 64 * MD : a.dpad, LR = DP + 4, ndt = DP / 16;
   float* kl = sm;                        // [64][LR] keys, then decayed keys
   float* tot = kl + C * LR;              // [4][DP] log-decays of sub-chunks
   float* EB = tot + 4 * DP;              // [3][DP] e^{B_w}, w = 1 .. 3
@@ -204,8 +207,17 @@ void gla_intra_kernel(GlaArgs a, bool vec, bool vec_a) {
   const int n = a.tiles[2 * a.n_tiles + tile];
   const int trow = w * 16 + lr;          // this lane's row
   const bool row_ok = trow < n;
-  const T* qrow = reinterpret_cast<const T*>(a.proj) +
-                  int64_t(row0 + trow) * a.stride + h * a.dim;
+  const int64_t at = row0 + (FULL ? min(trow, n - 1) : trow);
+  const T* qrow = reinterpret_cast<const T*>(a.proj) + at * a.stride +
+                  h * a.dim;
+  auto row4 = [&](const T* p, int d, int width, bool v) {
+    if constexpr (FULL) return act_load4(p + d);
+    else return load4_guard(p, d, width, row_ok, v);
+  };
+  auto vec4 = [&](const float* p, int d) {
+    if constexpr (FULL) return *reinterpret_cast<const f32x4_t*>(p + d);
+    else return load4_guard(p, d, a.dim, true, a.dim % 4 == 0);
+  };
   const T* krow = qrow + a.off_k;
   const float* bias = a.a2_bias + h * a.dim;
   const float* low = FG ? a.lower + h * a.dim : nullptr;
@@ -217,19 +229,21 @@ void gla_intra_kernel(GlaArgs a, bool vec, bool vec_a) {
   // (raw keys wait in the registers of the log-decays)
 #pragma unroll
   for (int dt = 0; dt < NT; ++dt) {
-    if (dt >= ndt) continue;
+    if (!FULL && dt >= ndt) continue;
     const int d = dt * 16 + g * 4;
-    q[dt] = load4_guard(qrow, d, a.dim, row_ok, vec);
-    L[dt] = load4_guard(krow, d, a.dim, row_ok, vec);
+    q[dt] = row4(qrow, d, a.dim, vec);
+    L[dt] = row4(krow, d, a.dim, vec);
   }
 #pragma unroll
   for (int dt = 0; dt < NT; ++dt) {
-    if (dt >= ndt) continue;
+    if (!FULL && dt >= ndt) continue;
     const int d = dt * 16 + g * 4;
     f32x4_t k = L[dt];
-    const f32x4_t bv = load4_guard(bias, d, a.dim, true, a.dim % 4 == 0);
+    if constexpr (FULL && !FG)
+      if (!row_ok) k = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const f32x4_t bv = vec4(bias, d);
     if constexpr (FG) {
-      const f32x4_t lv = load4_guard(low, d, a.dim, true, a.dim % 4 == 0);
+      const f32x4_t lv = vec4(low, d);
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const bool ok = row_ok && d + j < a.dim;
@@ -242,17 +256,18 @@ void gla_intra_kernel(GlaArgs a, bool vec, bool vec_a) {
     } else {
       // z transposed: columns down, rows across the lanes
       f32x4_t z = f32x4_t{0.f, 0.f, 0.f, 0.f};
-      const T* a1 = reinterpret_cast<const T*>(a.a1) +
-                    int64_t(row0 + trow) * a.a1_stride;
+      const T* a1 = reinterpret_cast<const T*>(a.a1) + at * a.a1_stride;
       const T* a2 = reinterpret_cast<const T*>(a.a2) +
                     int64_t(h * a.dim + dt * 16 + lr) * a.rank;
       for (int k0 = 0; k0 < a.rank; k0 += 16) {
-        f32x4_t av = load4_guard(a1, k0 + g * 4, a.rank, row_ok, vec_a);
+        f32x4_t av = row4(a1, k0 + g * 4, a.rank, vec_a);
         if constexpr (BONUS)
 #pragma unroll
           for (int j = 0; j < 4; ++j) av[j] = gtanh<T>(av[j]);
-        const f32x4_t wv = load4_guard(a2, k0 + g * 4, a.rank,
-                                       dt * 16 + lr < a.dim, vec_a);
+        f32x4_t wv;
+        if constexpr (FULL) wv = act_load4(a2 + k0 + g * 4);
+        else wv = load4_guard(a2, k0 + g * 4, a.rank, dt * 16 + lr < a.dim,
+                              vec_a);
 #pragma unroll
         for (int j = 0; j < 4; ++j) z = mma4(wv[j], av[j], z);
       }
@@ -282,11 +297,10 @@ void gla_intra_kernel(GlaArgs a, bool vec, bool vec_a) {
   if constexpr (BONUS) {
 #pragma unroll
     for (int dt = 0; dt < NT; ++dt) {
-      if (dt >= ndt) continue;
+      if (!FULL && dt >= ndt) continue;
       const int d = dt * 16 + g * 4;
       const f32x4_t kv = *reinterpret_cast<const f32x4_t*>(kl + trow * LR + d);
-      const f32x4_t uv = load4_guard(a.bonus + h * a.dim, d, a.dim, true,
-                                     a.dim % 4 == 0);
+      const f32x4_t uv = vec4(a.bonus + h * a.dim, d);
 #pragma unroll
       for (int j = 0; j < 4; ++j) own += q[dt][j] * uv[j] * kv[j];
     }
@@ -324,7 +338,7 @@ void gla_intra_kernel(GlaArgs a, bool vec, bool vec_a) {
     f32x4_t far = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int dt = 0; dt < NT; ++dt) {
-      if (dt >= ndt) continue;
+      if (!FULL && dt >= ndt) continue;
       const f32x4_t k = *reinterpret_cast<const f32x4_t*>(
           kl + trow * LR + dt * 16 + g * 4);
 #pragma unroll
@@ -376,7 +390,7 @@ void gla_intra_kernel(GlaArgs a, bool vec, bool vec_a) {
   f32x4_t diag = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int dt = 0; dt < NT; ++dt) {
-    if (dt >= ndt) continue;
+    if (!FULL && dt >= ndt) continue;
     const int d = dt * 16 + g * 4;
     const f32x4_t tw = *reinterpret_cast<const f32x4_t*>(tot + w * DP + d);
     f32x4_t eb = f32x4_t{1.f, 1.f, 1.f, 1.f}, ed = eb;
@@ -414,7 +428,7 @@ void gla_intra_kernel(GlaArgs a, bool vec, bool vec_a) {
   // rows of the sub-chunks before
 #pragma unroll
   for (int dt = 0; dt < NT; ++dt) {
-    if (dt >= ndt) continue;
+    if (!FULL && dt >= ndt) continue;
     const int d = dt * 16 + g * 4;
 #pragma unroll
     for (int J = 0; J < 3; ++J) {
@@ -462,9 +476,21 @@ void prefill(const GlaArgs& a, hipStream_t st) {
     hipLaunchKernelGGL(k, dim3(a.n_tiles, a.heads), dim3(256), smem, st, a,
                        vec, vec_a);
   };
-  if (a.dpad <= 64) intra(gla_intra_kernel<T, KIND, 1>);
-  else if (a.dpad <= 128) intra(gla_intra_kernel<T, KIND, 2>);
-  else intra(gla_intra_kernel<T, KIND, 4>);
+  bool done = false;                      // (gains nothing for the others)
+  if constexpr (sizeof(T) == 2 && KIND == kRwkv) {
+    done = vec && vec_a && a.rank % 16 == 0 && (a.dim == 64 || a.dim == 128) &&
+           reinterpret_cast<uintptr_t>(a.a2) % 8 == 0;
+    if (done && a.dim == 64) intra(gla_intra_kernel<T, KIND, 1, true>);
+    else if (done) intra(gla_intra_kernel<T, KIND, 2, true>);
+  }
+  if (done) {
+  } else if (a.dpad <= 64) {
+    intra(gla_intra_kernel<T, KIND, 1, false>);
+  } else if (a.dpad <= 128) {
+    intra(gla_intra_kernel<T, KIND, 2, false>);
+  } else {
+    intra(gla_intra_kernel<T, KIND, 4, false>);
+  }
   ScanArgs sa{};
   sa.v = reinterpret_cast<const T*>(a.proj) + a.off_v;
   sa.v_stride = a.stride;

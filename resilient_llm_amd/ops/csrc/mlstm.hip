@@ -22,8 +22,9 @@ DEV_INLINE float soft_cap(float x, float cap) {
   return cap * tanhf(x / cap);
 }
 
-template <typename T>
-__global__ __launch_bounds__(256)
+// NT threads: many when there are few heads to fill the chip with
+template <typename T, int NT>
+__global__ __launch_bounds__(NT)
 void mlstm_decode_kernel(MlstmArgs a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const int seq = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
@@ -41,11 +42,11 @@ void mlstm_decode_kernel(MlstmArgs a) {
   const float m = fmaxf(fm, i);
   const float keep = expf(fm - m), take = expf(i - m);
   const float qscale = 1.f / sqrtf(float(a.dim));
-  for (int d = tid; d < a.dim; d += 256) {
+  for (int d = tid; d < a.dim; d += NT) {
     qs[d] = act_load(row + h * a.dim + d) * qscale;
     ks[d] = act_load(row + a.off_k + h * a.dim + d) * take;
   }
-  const int v4n = a.vpad / 4, n_rows = 256 / v4n;
+  const int v4n = a.vpad / 4, n_rows = NT / v4n;
   const int vr = tid / v4n, vc = tid % v4n;
   const bool live = vr < n_rows;
   f32x4_t v = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -89,32 +90,35 @@ void mlstm_decode_kernel(MlstmArgs a) {
   for (int r = 0; r < n_rows; ++r) nq += red[r * a.vpad + a.vdim];
   const float pre = 1.f / (fmaxf(fabsf(nq), expf(-m)) + 1e-6f);
   float ss = 0.f;
-  for (int e = tid; e < a.vdim; e += 256) {
+  for (int e = tid; e < a.vdim; e += NT) {
     float t = 0.f;
     for (int r = 0; r < n_rows; ++r) t += red[r * a.vpad + e];
     t *= pre;
     red[e] = t;                           // column e is this thread's alone
     ss += t * t;
   }
-  __shared__ float ws[4];
+  __shared__ float ws[NT / 64];
   ss = wave_sum(ss);
   if ((tid & 63) == 0) ws[tid >> 6] = ss;
   __syncthreads();
-  const float inv =
-      1.f / sqrtf((ws[0] + ws[1] + ws[2] + ws[3]) / a.vdim + a.eps);
+  ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < NT / 64; ++k) ss += ws[k];
+  const float inv = 1.f / sqrtf(ss / a.vdim + a.eps);
   T* out = reinterpret_cast<T*>(a.out) + int64_t(seq) * a.out_stride +
            h * a.vdim;
-  for (int e = tid; e < a.vdim; e += 256)
+  for (int e = tid; e < a.vdim; e += NT)
     act_store(out + e, red[e] * inv * a.norm[h * a.vdim + e] *
                            sigm<T>(act_load(row + a.off_g + h * a.vdim + e)));
 }
 
-template <typename T>
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256)
-void mlstm_intra_kernel(MlstmArgs a, bool vec) {
+void mlstm_intra_kernel(MlstmArgs a) {
   __shared__ float A[C], M[C];            // a = i - F and its running maximum
   const int tile = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
-  const int lane = tid & 63, w = tid >> 6;
+  const int lane = tid & 63;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int lr = lane & 15, g = lane >> 4;
   const int row0 = a.tiles[tile], n = a.tiles[2 * a.n_tiles + tile];
   const T* qb = reinterpret_cast<const T*>(a.proj) +
@@ -124,16 +128,15 @@ void mlstm_intra_kernel(MlstmArgs a, bool vec) {
   f32x4_t qk[4];
 #pragma unroll
   for (int J = 0; J < 4; ++J) qk[J] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  const int trow = w * 16 + lr;
   for (int d0 = 0; d0 < a.dim; d0 += 32) {
-    const int d = d0 + g * 8;
-    const auto qf = frag_guard(qb + trow * a.stride, d, a.dim, trow < n, vec);
+    const int d = d0 + g * 8;             // rows behind the last repeat it
+    const auto qf = frag_at<VEC>(qb + min(w * 16 + lr, n - 1) * a.stride, d,
+                                 a.dim);
     Frag8<T> kf[4];
 #pragma unroll
     for (int J = 0; J < 4; ++J)
-      if (J <= w)
-        kf[J] = frag_guard(kb + (J * 16 + lr) * a.stride, d, a.dim,
-                           J * 16 + lr < n, vec);
+      kf[J] = frag_at<VEC>(kb + min(min(J, w) * 16 + lr, n - 1) * a.stride, d,
+                           a.dim);
 #pragma unroll
     for (int J = 0; J < 4; ++J)
       if (J <= w) qk[J] = Frag8<T>::mma(qf, kf[J], qk[J]);
@@ -157,8 +160,8 @@ void mlstm_intra_kernel(MlstmArgs a, bool vec) {
     rf[C + tid] = av;
     rf[2 * C + tid] = mv;
   }
-  keys_down(kb, a.stride, n, a.dim, a.dpad, vec,
-            reinterpret_cast<T*>(a.kt) + ch * a.dpad * C);
+  keys_down<VEC>(kb, a.stride, n, a.dim, a.dpad,
+                 reinterpret_cast<T*>(a.kt) + ch * a.dpad * C);
   __syncthreads();
   const float qscale = 1.f / sqrtf(float(a.dim));
   float* sc = a.sc + ch * C * C;
@@ -180,8 +183,11 @@ void prefill(const MlstmArgs& a, hipStream_t st) {
   const T* p = reinterpret_cast<const T*>(a.proj);
   const bool vec = a.dim % 8 == 0 && a.stride % 8 == 0 && a.off_k % 8 == 0 &&
                    reinterpret_cast<uintptr_t>(p) % 16 == 0;
-  hipLaunchKernelGGL(mlstm_intra_kernel<T>, dim3(a.n_tiles, a.heads),
-                     dim3(256), 0, st, a, vec);
+  auto intra = [&](auto* k) {
+    hipLaunchKernelGGL(k, dim3(a.n_tiles, a.heads), dim3(256), 0, st, a);
+  };
+  if (vec) intra(mlstm_intra_kernel<T, true>);
+  else intra(mlstm_intra_kernel<T, false>);
   ScanArgs sa{};
   sa.v = p + a.off_v;
   sa.v_stride = a.stride;
@@ -239,13 +245,19 @@ void prefill(const MlstmArgs& a, hipStream_t st) {
 
 void launch_mlstm_decode(const MlstmArgs& a, hipStream_t st) {
   if (a.rows == 0) return;
-  const int n_rows = 256 / (a.vpad / 4);
-  const size_t smem = size_t(2 * a.dpad + n_rows * a.vpad) * sizeof(float);
-  auto go = [&](auto* k) {
-    hipLaunchKernelGGL(k, dim3(a.rows, a.heads), dim3(256), smem, st, a);
+  auto go = [&](auto* k, int nt) {
+    const int n_rows = nt / (a.vpad / 4);
+    const size_t smem = size_t(2 * a.dpad + n_rows * a.vpad) * sizeof(float);
+    hipLaunchKernelGGL(k, dim3(a.rows, a.heads), dim3(nt), smem, st, a);
   };
-  if (a.f32) go(mlstm_decode_kernel<float>);
-  else go(mlstm_decode_kernel<uint16_t>);
+  const bool few = int64_t(a.rows) * a.heads < 256;
+  if (a.f32) {
+    go(mlstm_decode_kernel<float, 256>, 256);
+  } else if (few) {
+    go(mlstm_decode_kernel<uint16_t, 1024>, 1024);
+  } else {
+    go(mlstm_decode_kernel<uint16_t, 256>, 256);
+  }
 }
 
 void launch_mlstm_prefill(const MlstmArgs& a, hipStream_t st) {

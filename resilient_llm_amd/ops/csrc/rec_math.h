@@ -142,39 +142,55 @@ DEV_INLINE Raw4<T> raw_guard(const T* p, int d, int dim, bool row_ok,
   return v;
 }
 
-// eight columns of a row as a matrix operand
-template <typename T>
-DEV_INLINE Frag8<T> frag_guard(const T* p, int d, int dim, bool row_ok,
-                               bool vec) {
+// Eight columns of a row as a matrix operand, zeros from ``dim`` on.  The
+// row exists: callers take the last one for those behind it, so that no
+// load is conditional.  VEC: dim is a multiple of 8 and rows are aligned.
+template <bool VEC, typename T>
+DEV_INLINE Frag8<T> frag_at(const T* p, int d, int dim) {
   Frag8<T> f;
-  f.zero();
-  if (!row_ok || d >= dim) return f;
-  if (vec && d + 8 <= dim) {
-    f.load(p + d);
-    return f;
-  }
+  if constexpr (VEC) {
+    f.load(p + min(d, dim - 8));
+    if (d >= dim) f.zero();
+  } else {
+    f.zero();
 #pragma unroll
-  for (int j = 0; j < 8; ++j)
-    if (d + j < dim) {
-      if constexpr (sizeof(T) == 2) f.v[j] = short(p[d + j]);
-      else if (j < 4) f.lo[j] = p[d + j];
-      else f.hi[j - 4] = p[d + j];
-    }
+    for (int j = 0; j < 8; ++j)
+      if (d + j < dim) {
+        if constexpr (sizeof(T) == 2) f.v[j] = short(p[d + j]);
+        else if (j < 4) f.lo[j] = p[d + j];
+        else f.hi[j - 4] = p[d + j];
+      }
+  }
   return f;
 }
 
-// a chunk's keys, columns down: kt [dpad][64], zeros beyond the rows
+DEV_INLINE float frag_get(const Frag8<uint16_t>& f, int j) {
+  return bf16_to_f32(uint16_t(f.v[j]));
+}
+DEV_INLINE float frag_get(const Frag8<float>& f, int j) {
+  return j < 4 ? f.lo[j & 3] : f.hi[j & 3];
+}
 template <typename T>
+DEV_INLINE float frag_sq(const Frag8<T>& f) {
+  float s = 0.f;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) s += frag_get(f, j) * frag_get(f, j);
+  return s;
+}
+
+// a chunk's keys, columns down: kt [dpad][64], zeros from dim on
+template <bool VEC, typename T>
 DEV_INLINE void keys_down(const T* k, int64_t stride, int n, int dim,
-                          int dpad, bool vec, T* kt) {
+                          int dpad, T* kt) {
   const int s = threadIdx.x & 63;
+  const T* row = k + min(s, n - 1) * stride;
   for (int d = (threadIdx.x >> 6) * 8; d < dpad; d += 32) {
-    const Frag8<T> f = frag_guard(k + s * stride, d, dim, s < n, vec);
+    const Frag8<T> f = frag_at<VEC>(row, d, dim);
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       T e;
       if constexpr (sizeof(T) == 2) e = T(f.v[j]);
-      else e = j < 4 ? f.lo[j & 3] : f.hi[j & 3];
+      else e = frag_get(f, j);
       kt[int64_t(d + j) * kRecChunk + s] = e;
     }
   }

@@ -19,6 +19,7 @@
 
 #include "attn_rows.h"
 
+#include <algorithm>
 #include <type_traits>
 
 namespace rlli {
@@ -392,23 +393,24 @@ void window_decode_kernel(WindowAttnArgs a) {
   }
 }
 
-__global__ __launch_bounds__(64)
+// one wave per 64 value columns; lane s holds the weight of split s
+__global__ __launch_bounds__(256)
 void window_combine_kernel(WindowAttnArgs a) {
   const int64_t row = blockIdx.x;               // seq * n_q + head
-  const int h = int(row % a.n_q);
+  const int h = int(row % a.n_q), lane = threadIdx.x & 63;
   const float snk = a.sink ? a.sink[h] : kNegInf;
-  float mm = snk;
-  for (int s = 0; s < a.n_split; ++s)
-    mm = fmaxf(mm, a.part_ml[(row * a.n_split + s) * 2]);
-  float ll = a.sink ? __expf(snk - mm) : 0.f;
-  for (int s = 0; s < a.n_split; ++s)
-    ll += a.part_ml[(row * a.n_split + s) * 2 + 1] *
-          __expf(a.part_ml[(row * a.n_split + s) * 2] - mm);
-  for (int d = threadIdx.x; d < a.vdim; d += 64) {
+  const bool mine = lane < a.n_split;
+  const float2 ml = reinterpret_cast<const float2*>(
+      a.part_ml)[row * a.n_split + (mine ? lane : 0)];
+  const float mm = fmaxf(snk, wave_max(mine ? ml.x : kNegInf));
+  const float c = mine ? __expf(ml.x - mm) : 0.f;
+  const float ll = wave_sum(c * ml.y) + (a.sink ? __expf(snk - mm) : 0.f);
+  for (int d = threadIdx.x; d < a.vdim; d += blockDim.x) {
+    const float* p = a.part_acc + row * a.n_split * a.vdim + d;
     float o = 0.f;
+#pragma unroll 4
     for (int s = 0; s < a.n_split; ++s)
-      o += a.part_acc[(row * a.n_split + s) * a.vdim + d] *
-           __expf(a.part_ml[(row * a.n_split + s) * 2] - mm);
+      o += p[s * a.vdim] * __shfl(c, s, kWave);
     reinterpret_cast<uint16_t*>(a.out)[row * a.vdim + d] =
         f32_to_bf16(o / ll);
   }
@@ -479,8 +481,9 @@ void launch_window_decode(const WindowAttnArgs& a, hipStream_t st) {
   else if (d <= 128) by_heads(std::integral_constant<int, 16>{});
   else by_heads(std::integral_constant<int, 32>{});
   if (a.n_split > 1)
-    hipLaunchKernelGGL(window_combine_kernel, dim3(a.rows * a.n_q), dim3(64),
-                       0, st, a);
+    hipLaunchKernelGGL(window_combine_kernel, dim3(a.rows * a.n_q),
+                       dim3(std::min(256, (a.vdim + 63) / 64 * 64)), 0, st,
+                       a);
 }
 
 }  // namespace rlli
