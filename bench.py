@@ -363,7 +363,8 @@ def main() -> None:
                          "headline metric stays bf16)")
     ap.add_argument("--device", default=None,
                     help="override torch device (tests: cpu)")
-    ap.add_argument("--design", default=None, choices=("nesizen", "riruzen", "bolatar"),
+    ap.add_argument("--design", default=None,
+                    choices=("nesizen", "riruzen", "bolatar"),
                     help="measure this design's engine throughput beside "
                          "existing models of equal size instead of serving")
     ap.add_argument("--design-sizes", default="w2048,w4096")
