@@ -80,20 +80,24 @@ class PromptRows:
             return torch.tensor(pos, dtype=torch.int32).to(self.device)
         return self._once(("pos0",), make)
 
-    def gathered(self, height: int) -> tuple:
+    def gathered(self, height: int, chunk: int = 0) -> tuple:
         """Every portion's sequence up to its last row, one after another,
         each padded to a multiple of ``height`` tokens: (int32 [4, n]
         blocks of that height: sequence, first token, tokens, output row;
-        int32 [sequences] first output row; output rows)."""
+        int32 [sequences] output row of position 0; output rows).  With
+        ``chunk`` a sequence starts with the chunk of its first row (at a
+        multiple of ``height``), so that row may be negative."""
         def make():
             rows, at = [], 0
             off = [0] * (1 + max(p.seq for p in self.portions))
             for p in self.portions:
                 ctx = p.pos0 + p.n
-                off[p.seq] = at
-                rows += [(p.seq, o, min(height, ctx - o), at + o)
-                         for o in range(0, ctx, height)]
-                at += -(-ctx // height) * height
+                start = p.pos0 // chunk * chunk // height * height \
+                    if chunk else 0
+                off[p.seq] = at - start
+                rows += [(p.seq, o, min(height, ctx - o), at - start + o)
+                         for o in range(start, ctx, height)]
+                at += -(-(ctx - start) // height) * height
             return (self._table(rows),
                     torch.tensor(off, dtype=torch.int32).to(self.device), at)
-        return self._once(("gathered", height), make)
+        return self._once(("gathered", height, chunk), make)

@@ -8,6 +8,7 @@ import os
 from typing import Optional
 
 from .bolatar import BOLATAR_PRESETS, BolatarConfig, BolatarForCausalLM
+from .fimunex import FIMUNEX_PRESETS, FimunexConfig, FimunexForCausalLM
 from .llama import MODEL_PRESETS, LlamaConfig, LlamaForCausalLM
 from .mixed import MixedModel
 from .nesizen import NESIZEN_PRESETS, NesizenConfig, NesizenForCausalLM
@@ -15,11 +16,13 @@ from .riruzen import RIRUZEN_PRESETS, RiruzenConfig, RiruzenForCausalLM
 
 # config.json 'architecture' -> (configuration, model)
 ARCHITECTURES = {"Bolatar": (BolatarConfig, BolatarForCausalLM),
+                 "Fimunex": (FimunexConfig, FimunexForCausalLM),
                  "Nesizen": (NesizenConfig, NesizenForCausalLM),
                  "Riruzen": (RiruzenConfig, RiruzenForCausalLM)}
 _MODELS = {LlamaConfig: LlamaForCausalLM, **dict(ARCHITECTURES.values())}
 # presets that are made when asked for
-_MADE_PRESETS = {**BOLATAR_PRESETS, **NESIZEN_PRESETS, **RIRUZEN_PRESETS}
+_MADE_PRESETS = {**BOLATAR_PRESETS, **FIMUNEX_PRESETS, **NESIZEN_PRESETS,
+                 **RIRUZEN_PRESETS}
 
 
 def model_names() -> list:

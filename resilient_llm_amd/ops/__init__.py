@@ -274,6 +274,7 @@ def skinny2_silu_linear(gu: torch.Tensor, w: torch.Tensor,
 
 
 build_cos_sin = ref.build_cos_sin
+yarn_cos_sin = ref.yarn_cos_sin
 
 
 # ----------------------------------------------- mixed-layer model ops
@@ -398,6 +399,52 @@ def biased_prefill(qkv, k_cache, v_cache, positions, slots, block_tables,
     return out
 
 
+def diff_decode(qkv, gate, k_cache, v_cache, positions, cos_sin, slots,
+                block_tables, n_q: int, q_norm, k_norm, scale: float,
+                chunk: int, cap: float, lam: float, out_scale: float,
+                eps: float):
+    """Differential attention, one new token per sequence, append included.
+    ``qkv``: q | k | v | .., a head's query and key being two maps side by
+    side, each normed and rotated (pairs i, i + rot / 2); scores capped; a
+    query sees its chunk of positions; the maps' outputs a1 - lam a2 over
+    their root mean square, times out_scale and the sigmoid of ``gate``
+    [rows, n_q]."""
+    return _ns("rlli_attn", qkv).diff_decode(
+        qkv, k_cache, v_cache, positions, cos_sin, slots, block_tables, gate,
+        scale, n_q, q_norm, k_norm, chunk, cap, lam, out_scale, eps)
+
+
+def diff_prefill(qkv, gate, k_cache, v_cache, positions, cos_sin, slots,
+                 block_tables, prompt, n_q: int, q_norm, k_norm, scale: float,
+                 chunk: int, cap: float, lam: float, out_scale: float,
+                 eps: float):
+    """The same for prompt rows: append, then attend over what the rows'
+    chunks hold, gathered (sizes that the tiled kernel does not take: over
+    the pages, row by row)."""
+    if not qkv.is_cuda:
+        return ref_attn.diff_prefill(
+            qkv, gate, k_cache, v_cache, positions, cos_sin, slots,
+            block_tables, prompt, n_q, q_norm, k_norm, scale, chunk, cap, lam,
+            out_scale, eps)
+    attn = _ns("rlli_attn", qkv)
+    attn.diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q,
+                     q_norm, k_norm, eps)
+    tail = (chunk, cap, lam, out_scale, eps)
+    _, n_kv, _, width = k_cache.shape
+    vdim = v_cache.shape[3]
+    if (qkv.dtype == torch.float32 or qkv.shape[1] % 8
+            or not attn.expanded_ok(width // 2, vdim, 2)):
+        return attn.diff_rows(qkv, k_cache, v_cache, block_tables,
+                              prompt.tiles(32), 32, gate, scale, n_q, *tail)
+    blocks, kv_off, tokens = prompt.gathered(64, chunk)
+    k, vt = attn.kv_gather(k_cache, v_cache, block_tables, blocks, tokens)
+    out = torch.empty((qkv.shape[0], n_q * vdim), dtype=qkv.dtype,
+                      device=qkv.device)
+    attn.diff_expanded(qkv[:, :n_q * width], k, vt, gate, prompt.tiles(128),
+                       kv_off, n_q, n_kv, scale, out, *tail)
+    return out
+
+
 def _out(proj, state, vdim, out):
     if out is not None:
         return out
@@ -509,6 +556,21 @@ def moe_experts(h, router, w_up, w_down, top: int, limit: float):
     return _mix(h).moe_experts(h, router, w_up, w_down, top, limit)
 
 
+def moe_route_softmax(h, router, correction, top: int, groups: int,
+                      keep: int):
+    return _mix(h).moe_route_softmax(h, router, correction, top, groups, keep)
+
+
+def moe_relu2(h, router, correction, w_up, w_down, top: int, groups: int,
+              keep: int):
+    """Squared-relu experts.  Softmax over all routes; ``correction`` shifts
+    the choice, which the best ``keep`` of ``groups`` groups of neighbours
+    hold; weights sum to one.  Returns (y [T, top, W], ids, weights); routes
+    past the experts are identities, whose rows of y are not written."""
+    return _mix(h).moe_relu2(h, router, correction, w_up, w_down, top, groups,
+                             keep)
+
+
 # --------------------------------------------------- residual blocks
 CONV_SPAN = 16        # prompt rows that one convolution workgroup walks
 
@@ -527,13 +589,17 @@ def block_embed(ids, table, pos_table, positions, x, gain, groups: int,
 
 def block_step(x, y, gain, groups: int, eps: float, positions, taps=None,
                tail=None, slots=None, n_decode: int = 0, rows=None,
-               keep: bool = True, y2=None, gain1=None, gain2=None):
+               keep: bool = True, y2=None, gain1=None, gain2=None,
+               part_ids=None, part_w=None, part_h=None, part_limit: int = 0):
     """Add a block's output to the residual; then as block_embed.  ``rows``
     restricts the result (then keep=False).  With ``y2`` half the sum of
-    both outputs is added, each normed first (``gain1``, ``gain2``)."""
+    both outputs is added, each normed first (``gain1``, ``gain2``).  With
+    ``part_ids`` [T, parts] the sum over y [T, parts, W] is added, where a
+    part whose id is ``part_limit`` or more is part_w part_h instead."""
     return _ns("rlli_blk", y).block_step(x, y, gain, groups, eps, positions,
                                          taps, tail, slots, n_decode, rows,
-                                         keep, y2, gain1, gain2)
+                                         keep, y2, gain1, gain2, part_ids,
+                                         part_w, part_h, part_limit)
 
 
 def conv_prompt(h, taps, tail, prompt, out, silu: bool = False):

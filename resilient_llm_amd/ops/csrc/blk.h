@@ -13,7 +13,13 @@ struct BlockArgs {
   const void* pos_table;   // learned positions (embed launch) or null
   const int32_t* positions;     // [rows]
   float* x;                // [rows, width] residual
-  const void* y;           // [rows, width] what the last block adds
+  const void* y;           // [rows, width] what the last block adds, or
+                           // with part_ids [rows, parts, width]: their sum
+  const int32_t* part_ids; // [rows, parts] or null; from part_limit on, a
+                           // part is part_w part_h instead
+  const float* part_w;     // [rows, parts]
+  const void* part_h;      // [rows, width]
+  int parts, part_limit;
   const void* y2;          // its second half (merge), or null
   const float* gain1;      // [width] gains of y's and y2's own norms (merge)
   const float* gain2;

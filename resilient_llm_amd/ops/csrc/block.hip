@@ -16,7 +16,9 @@
 // h + (h' - h) mu with the previous row's h' is the two taps mu, -mu, so
 // mixing a row with the one before it for several projections is one of
 // these.  A block may also end in two outputs, each with a norm of its own,
-// half their sum being what the residual takes (merge).
+// half their sum being what the residual takes (merge), or in one per chosen
+// expert (parts), where identity experts give their weight of the block's
+// input.
 
 #include "blk.h"
 
@@ -53,7 +55,7 @@ DEV_INLINE void store_v(T* p, const float (&in)[V]) {
 // IT vectors of V columns per thread; IT = 0 walks the row twice.  CONV:
 // there are decoded rows, which also convolve
 template <typename T, int WAVES, int IT, int V, bool EMBED, bool MERGE,
-          bool CONV>
+          bool CONV, bool PARTS>
 __global__ __launch_bounds__(WAVES * 64)
 void block_step_kernel(BlockArgs a) {
   extern __shared__ float sq[];           // [width / V] squares, [groups]
@@ -64,7 +66,9 @@ void block_step_kernel(BlockArgs a) {
   float* scale = sq + nv;
   float* xr = a.x + row * W;
   const T* yr = EMBED ? nullptr
-                      : reinterpret_cast<const T*>(a.y) + row * W;
+                      : reinterpret_cast<const T*>(a.y) +
+                            row * (PARTS ? a.parts : 1) * W;
+  const int32_t* part_ids = PARTS ? a.part_ids + row * a.parts : nullptr;
   const T* y2r = MERGE ? reinterpret_cast<const T*>(a.y2) + row * W : nullptr;
   float s1 = 0.f, s2 = 0.f;               // half over the root mean squares
   auto merge = [&](int c, const float (&p)[V], const float (&q)[V],
@@ -96,7 +100,23 @@ void block_step_kernel(BlockArgs a) {
       }
     } else {
       load_v<float, V>(xr + c, u);
-      load_v<T, V>(yr + c, t);
+      if constexpr (PARTS) {
+#pragma unroll
+        for (int j = 0; j < V; ++j) t[j] = 0.f;
+#pragma unroll 4
+        for (int k = 0; k < a.parts; ++k) {
+          const bool own = part_ids[k] < a.part_limit;
+          const T* p = own ? yr + int64_t(k) * W
+                           : reinterpret_cast<const T*>(a.part_h) + row * W;
+          const float w = own ? 1.f : a.part_w[row * a.parts + k];
+          float e[V];
+          load_v<T, V>(p + c, e);
+#pragma unroll
+          for (int j = 0; j < V; ++j) t[j] += w * e[j];
+        }
+      } else {
+        load_v<T, V>(yr + c, t);
+      }
       if constexpr (MERGE && IT == 0) {
         float q[V];
         load_v<T, V>(y2r + c, q);
@@ -429,30 +449,35 @@ void soft_cap_kernel(const T* __restrict__ x, float* __restrict__ out,
   }
 }
 
-template <typename T, bool EMBED, bool MERGE, bool CONV>
+template <typename T, bool EMBED, bool MERGE, bool CONV, bool PARTS = false>
 void step(const BlockArgs& a, hipStream_t st) {
   auto run = [&](auto* k, int threads, int v) {
     hipLaunchKernelGGL(k, dim3(a.n), dim3(threads),
                        (a.width / v + a.groups) * sizeof(float), st, a);
   };
   if (a.width / a.groups % 4 || a.width > 8192)
-    run(block_step_kernel<T, 4, 0, 1, EMBED, MERGE, CONV>, 256, 1);
+    run(block_step_kernel<T, 4, 0, 1, EMBED, MERGE, CONV, PARTS>, 256, 1);
   else if (a.width <= 256)
-    run(block_step_kernel<T, 1, 1, 4, EMBED, MERGE, CONV>, 64, 4);
+    run(block_step_kernel<T, 1, 1, 4, EMBED, MERGE, CONV, PARTS>, 64, 4);
   else if (a.width <= 1024)
-    run(block_step_kernel<T, 4, 1, 4, EMBED, MERGE, CONV>, 256, 4);
+    run(block_step_kernel<T, 4, 1, 4, EMBED, MERGE, CONV, PARTS>, 256, 4);
   else if (a.width <= 2048)
-    run(block_step_kernel<T, 4, 2, 4, EMBED, MERGE, CONV>, 256, 4);
+    run(block_step_kernel<T, 4, 2, 4, EMBED, MERGE, CONV, PARTS>, 256, 4);
   else if (a.width <= 4096)
-    run(block_step_kernel<T, 8, 2, 4, EMBED, MERGE, CONV>, 512, 4);
+    run(block_step_kernel<T, 8, 2, 4, EMBED, MERGE, CONV, PARTS>, 512, 4);
   else
-    run(block_step_kernel<T, 8, 4, 4, EMBED, MERGE, CONV>, 512, 4);
+    run(block_step_kernel<T, 8, 4, 4, EMBED, MERGE, CONV, PARTS>, 512, 4);
 }
 
 template <typename T, bool EMBED>
 void step(const BlockArgs& a, hipStream_t st) {
   const bool conv = a.hc && a.n_decode;
   if constexpr (!EMBED) {
+    if (a.part_ids) {
+      if (conv) step<T, false, false, true, true>(a, st);
+      else step<T, false, false, false, true>(a, st);
+      return;
+    }
     if (a.y2) {
       if (conv) step<T, false, true, true>(a, st);
       else step<T, false, true, false>(a, st);

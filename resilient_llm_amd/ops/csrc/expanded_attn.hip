@@ -4,6 +4,9 @@
 // gathered from their pages (kv_gather).  Keys of a sequence start at a
 // multiple of 64 in them and are padded with zeros to a multiple of 64.
 // Optional: a distance bias per head, a query temperature by position.
+// Differential attention (two maps per head, see attn.h) also has capped
+// scores and chunks; its first waves take map 1 of a row, as many others map
+// 2 over the same tiles, and the difference is made through LDS.
 //
 // A workgroup owns 128 prompt rows of one head, a wave 32 of them, and
 // walks 64-key tiles through double-buffered LDS, the next tile's loads in
@@ -35,16 +38,18 @@ DEV_INLINE f32x16_t mma32(s16x8_t a, s16x8_t b, f32x16_t c) {
   return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0);
 }
 
-// P: the larger of the key and value widths, rounded up; BIAS: a score
-// loses r1 ln(1 + r2 distance)
-template <int P, bool BIAS>
-__global__ __launch_bounds__(256, P <= 128 ? 2 : 1)
+// P: the larger of the key (all maps) and value widths, rounded up; BIAS: a
+// score loses r1 ln(1 + r2 distance)
+template <int P, bool BIAS, int MAPS>
+__global__ __launch_bounds__(256 * MAPS, P <= 128 || MAPS == 2 ? 2 : 1)
 void expanded_attn_kernel(ExpandedAttnArgs a) {
-  constexpr int DC = P / 16;              // contraction steps of a score
+  constexpr int NT = 256 * MAPS;          // threads
+  constexpr int DC = P / MAPS / 16;       // contraction steps of a score
   constexpr int VT = P / 32;              // value tiles
   constexpr int KROW = P + 8;
   constexpr int BUF = KT * KROW + P * VROW;
-  constexpr int NK = KT * (P / 8) / 256;  // vectors a thread stages
+  constexpr int NK = KT * (P / 8) / NT;   // vectors a thread stages
+  static_assert(NK * NT == KT * (P / 8), "a tile is staged whole");
   extern __shared__ __attribute__((aligned(16))) uint16_t lds[];
 
   // heads that share an XCD's L2 walk their tiles together, longest first
@@ -65,18 +70,30 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
   const int seq = a.tiles[3 * a.n_tiles + tile];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int qi = lane & 31, hi = lane >> 5;
-  const int sub = w * 32;
+  const int map = w >> 2, sub = (w & 3) * 32;
   const int64_t base = a.kv_off[seq];
   const int len = pos0 + nrows;
   const int my_row = sub + qi;
   const int qpos = pos0 + min(my_row, nrows - 1);
   const bool active = sub < nrows;
   const int w_last = pos0 + min(sub + 31, nrows - 1);    // of this wave
+  // first visible position: of this lane's query, this wave's first query
+  // and its last
+  int lo = 0, w_lo = 0, w_top = 0, first = 0;
+  if constexpr (MAPS == 2)
+    if (a.chunk > 0) {
+      lo = qpos / a.chunk * a.chunk;
+      w_lo = min(pos0 + sub, w_last) / a.chunk * a.chunk;
+      w_top = w_last / a.chunk * a.chunk;
+      first = pos0 / a.chunk * a.chunk / KT * KT;
+    }
 
-  const int64_t kw = int64_t(a.n_kv) * a.dim;
+  const int64_t kw = int64_t(a.n_kv) * MAPS * a.dim;
+  const int kd = MAPS * a.dim;            // a head's
   const int kvh = h / (a.heads / a.n_kv);
   const uint16_t* q = reinterpret_cast<const uint16_t*>(a.q) +
-                      (row0 + min(my_row, nrows - 1)) * a.q_stride + h * a.dim;
+                      (row0 + min(my_row, nrows - 1)) * a.q_stride +
+                      (h * MAPS + map) * a.dim;
   s16x8_t qf[DC];
 #pragma unroll
   for (int c = 0; c < DC; ++c) {
@@ -87,17 +104,17 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
   }
 
   const uint16_t* kp = reinterpret_cast<const uint16_t*>(a.k) + base * kw +
-                       kvh * a.dim;
+                       kvh * kd;
   const uint16_t* vp = reinterpret_cast<const uint16_t*>(a.vt) +
                        int64_t(kvh) * a.vdim * a.tokens + base;
   uint4 kr[NK], vr[NK];
   auto fetch = [&](int kv0) {
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
-      const int e = i * 256 + threadIdx.x;
+      const int e = i * NT + threadIdx.x;
       const int r = e / (P / 8), d = e % (P / 8) * 8;
       kr[i] = uint4{0, 0, 0, 0};
-      if (d < a.dim)
+      if (d < kd)
         kr[i] = *reinterpret_cast<const uint4*>(kp + (kv0 + r) * kw + d);
       const int vd = e / 8, c = e % 8 * 8;
       vr[i] = uint4{0, 0, 0, 0};
@@ -109,7 +126,7 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
   auto stage = [&](uint16_t* buf) {
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
-      const int e = i * 256 + threadIdx.x;
+      const int e = i * NT + threadIdx.x;
       *reinterpret_cast<uint4*>(buf + e / (P / 8) * KROW + e % (P / 8) * 8) =
           kr[i];
       // keys 0-3 | 4-7 of an octet go eight apart, odd octets four up
@@ -134,16 +151,17 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
     r2 = a.r2[h];
   }
 
-  fetch(0);
+  const float cap2 = MAPS == 2 && a.cap > 0.f ? kTwoLog2e / a.cap : 0.f;
+  fetch(first);
   stage(lds);
   __syncthreads();
   int cur = 0;
-  for (int kv0 = 0; kv0 < len; kv0 += KT) {
+  for (int kv0 = first; kv0 < len; kv0 += KT) {
     const bool more = kv0 + KT < len;
     if (more) fetch(kv0 + KT);
     const uint16_t* ks = lds + cur * BUF;
     const uint16_t* vs = ks + KT * KROW;
-    if (active && kv0 <= w_last) {
+    if (active && kv0 <= w_last && kv0 + KT > w_lo) {
       f32x16_t s[2];
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt) {
@@ -153,7 +171,7 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
         for (int c = 0; c < DC; ++c) {
           if (c * 16 >= a.dim) break;
           const s16x8_t kf = *reinterpret_cast<const s16x8_t*>(
-              ks + (kt * 32 + qi) * KROW + c * 16 + hi * 8);
+              ks + (kt * 32 + qi) * KROW + map * a.dim + c * 16 + hi * 8);
           s[kt] = mma32(kf, qf[c], s[kt]);
         }
       }
@@ -169,15 +187,30 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
                             s[kt][r] * c2);
           }
       }
-      const float c1 = BIAS ? 1.f : c2;
+      float c1 = BIAS ? 1.f : c2;
+      if constexpr (MAPS == 2)
+        if (cap2 > 0.f) {
+          const float in = a.scale * cap2, top = a.cap * 1.4426950408889634f;
+          c1 = 1.f;
+#pragma unroll
+          for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+            for (int r = 0; r < 16; ++r)
+              s[kt][r] = fmaf(
+                  -2.f * top,
+                  __builtin_amdgcn_rcpf(
+                      1.f + __builtin_amdgcn_exp2f(s[kt][r] * in)),
+                  top);
+        }
       float mx = kNegInf;
-      if (kv0 + KT - 1 > pos0 + sub) {      // some query sees only a part
+      // some query sees only a part
+      if (kv0 + KT - 1 > pos0 + sub || kv0 < w_top) {
 #pragma unroll
         for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
             const int key = kv0 + kt * 32 + (r >> 2) * 8 + hi * 4 + (r & 3);
-            s[kt][r] = key <= qpos ? s[kt][r] * c1 : kNegInf;
+            s[kt][r] = key <= qpos && key >= lo ? s[kt][r] * c1 : kNegInf;
             mx = fmaxf(mx, s[kt][r]);
           }
       } else {
@@ -234,6 +267,51 @@ void expanded_attn_kernel(ExpandedAttnArgs a) {
     __syncthreads();
   }
 
+  if constexpr (MAPS == 2) {
+    l += __shfl_xor(l, 32, kWave);
+    const float inv = 1.f / l;
+    // map 2's output through LDS, [value column][32 rows] per pair of waves;
+    // the tiles are done with (a barrier ends the loop)
+    float* side = reinterpret_cast<float*>(lds) + (w & 3) * (P * 32) + qi;
+    if (map == 1) {
+#pragma unroll
+      for (int v = 0; v < VT; ++v)
+#pragma unroll
+        for (int r = 0; r < 16; ++r)
+          side[(v * 32 + (r >> 2) * 8 + hi * 4 + (r & 3)) * 32] =
+              o[v][r] * inv;
+    }
+    __syncthreads();
+    if (map == 1 || my_row >= nrows) return;
+    float ss = 0.f;
+#pragma unroll
+    for (int v = 0; v < VT; ++v)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const int d = v * 32 + (r >> 2) * 8 + hi * 4 + (r & 3);
+        o[v][r] = o[v][r] * inv - a.lambda * side[d * 32];
+        if (d < a.vdim) ss += o[v][r] * o[v][r];
+      }
+    ss += __shfl_xor(ss, 32, kWave);      // both halves have the same row
+    float post = a.out_scale / sqrtf(ss / a.vdim + a.eps);
+    if (a.gate)
+      post /= 1.f + __expf(-bf16_to_f32(
+                        reinterpret_cast<const uint16_t*>(
+                            a.gate)[(row0 + my_row) * a.gate_stride + h]));
+    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) +
+                    (row0 + my_row) * a.out_stride + h * a.vdim;
+#pragma unroll
+    for (int v = 0; v < VT; ++v)
+#pragma unroll
+      for (int r = 0; r < 16; r += 4) {
+        const int d = v * 32 + (r >> 2) * 8 + hi * 4;
+        if (d < a.vdim)
+          *reinterpret_cast<uint2*>(out + d) =
+              uint2{pack2(o[v][r] * post, o[v][r + 1] * post),
+                    pack2(o[v][r + 2] * post, o[v][r + 3] * post)};
+      }
+    return;
+  }
   if (my_row >= nrows) return;
   l += __shfl_xor(l, 32, kWave);
   const float inv = 1.f / l;
@@ -317,38 +395,46 @@ void kv_gather_kernel(KvGatherArgs a) {
   }
 }
 
-template <int P, bool BIAS>
+template <int P, bool BIAS, int MAPS>
 void go(const ExpandedAttnArgs& a, hipStream_t st) {
   constexpr size_t smem = size_t(KT * (P + 8) + P * VROW) * 2 * 2;
-  auto* k = expanded_attn_kernel<P, BIAS>;
+  static_assert(smem >= size_t(4) * 32 * P * sizeof(float),
+                "map 2's output needs the tiles' room");
+  auto* k = expanded_attn_kernel<P, BIAS, MAPS>;
   if (smem > 65536)
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k),
                               hipFuncAttributeMaxDynamicSharedMemorySize,
                               int(smem));
-  hipLaunchKernelGGL(k, dim3(a.n_tiles * a.heads), dim3(256), smem, st, a);
+  hipLaunchKernelGGL(k, dim3(a.n_tiles * a.heads), dim3(256 * MAPS), smem,
+                     st, a);
 }
 
-template <bool BIAS>
+template <bool BIAS, int MAPS>
 void by_width(const ExpandedAttnArgs& a, hipStream_t st) {
-  const int d = a.dim > a.vdim ? a.dim : a.vdim;
-  if (d <= 32) go<32, BIAS>(a, st);
-  else if (d <= 64) go<64, BIAS>(a, st);
-  else if (d <= 96) go<96, BIAS>(a, st);
-  else if (d <= 128) go<128, BIAS>(a, st);
-  else if (d <= 192) go<192, BIAS>(a, st);
-  else go<256, BIAS>(a, st);
+  const int d = MAPS * a.dim > a.vdim ? MAPS * a.dim : a.vdim;
+  if constexpr (MAPS == 1)
+    if (d <= 32) return go<32, BIAS, MAPS>(a, st);
+  if (d <= 64) return go<64, BIAS, MAPS>(a, st);
+  if constexpr (MAPS == 1)
+    if (d <= 96) return go<96, BIAS, MAPS>(a, st);
+  if (d <= 128) go<128, BIAS, MAPS>(a, st);
+  else if (d <= 192) go<192, BIAS, MAPS>(a, st);
+  else go<256, BIAS, MAPS>(a, st);
 }
 
 }  // namespace
 
-bool expanded_ok(int dim, int vdim) {
-  return dim % 8 == 0 && vdim % 8 == 0 && dim <= 256 && vdim <= 256;
+bool expanded_ok(int dim, int vdim, int maps) {
+  // a map's key fragments stop where the next map's begin
+  return dim % (8 * maps) == 0 && vdim % 8 == 0 && maps * dim <= 256 &&
+         vdim <= 256;
 }
 
 void launch_expanded_attn(const ExpandedAttnArgs& a, hipStream_t st) {
   if (a.n_tiles == 0) return;
-  if (a.r1) by_width<true>(a, st);
-  else by_width<false>(a, st);
+  if (a.maps == 2) by_width<false, 2>(a, st);
+  else if (a.r1) by_width<true, 1>(a, st);
+  else by_width<false, 1>(a, st);
 }
 
 void launch_kv_gather(const KvGatherArgs& a, hipStream_t st) {

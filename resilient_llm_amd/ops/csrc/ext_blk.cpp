@@ -108,12 +108,27 @@ std::tuple<Tensor, Tensor> block_step(
     const Tensor& positions, const OptTensor& taps, const OptTensor& tail,
     const OptTensor& slots, int64_t n_decode, const OptTensor& rows,
     bool keep, const OptTensor& y2, const OptTensor& gain1,
-    const OptTensor& gain2) {
+    const OptTensor& gain2, const OptTensor& part_ids,
+    const OptTensor& part_w, const OptTensor& part_h, int64_t part_limit) {
   rlli::BlockArgs a{};
   a.f32 = act_f32(y, "y");
-  TORCH_CHECK(y.dim() == 2 && y.sizes() == x.sizes(), "y/residual mismatch");
-  TORCH_CHECK(y.is_contiguous());
+  TORCH_CHECK(x.dim() == 2 && y.dim() == (part_ids ? 3 : 2) &&
+              y.size(0) == x.size(0) && y.size(-1) == x.size(1),
+              "y/residual mismatch");
   a.y = y.data_ptr();
+  if (part_ids) {
+    TORCH_CHECK(part_w.has_value() && part_h.has_value() && !y2,
+                "parts come with weights and the block's input");
+    a.parts = int(y.size(1));
+    a.part_limit = int(part_limit);
+    a.part_ids = i32(*part_ids, "part_ids");
+    TORCH_CHECK(part_ids->numel() == y.size(0) * y.size(1),
+                "one id per part");
+    a.part_w = f32_vec(*part_w, part_ids->numel(), "part_w");
+    same_act(*part_h, y, "part_h");
+    TORCH_CHECK(part_h->sizes() == x.sizes(), "part_h/residual mismatch");
+    a.part_h = part_h->data_ptr();
+  }
   if (y2) {
     same_act(*y2, y, "y2");
     TORCH_CHECK(y2->sizes() == y.sizes() && gain1.has_value() &&
@@ -219,7 +234,9 @@ TORCH_LIBRARY(rlli_blk, m) {
   m.def("block_step(Tensor(a!) x, Tensor y, Tensor gain, int groups, "
         "float eps, Tensor positions, Tensor? taps, Tensor(b!)? tail, "
         "Tensor? slots, int n_decode, Tensor? rows, bool keep, Tensor? y2, "
-        "Tensor? gain1, Tensor? gain2) -> (Tensor, Tensor)");
+        "Tensor? gain1, Tensor? gain2, Tensor? part_ids=None, "
+        "Tensor? part_w=None, Tensor? part_h=None, int part_limit=0) "
+        "-> (Tensor, Tensor)");
   m.def("conv_prompt(Tensor h, Tensor taps, Tensor(a!)? tail, Tensor spans, "
         "Tensor portions, Tensor(b!) out, bool silu) -> ()");
   m.def("gate_act(Tensor gate_up, Tensor(a!) out, str act, float limit) "

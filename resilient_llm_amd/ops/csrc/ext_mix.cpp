@@ -123,70 +123,59 @@ int64_t window_tile_rows(int64_t group) {
 
 // ------------------------------------------------------------------ moe
 void moe_sizes(rlli::MoeArgs& a, const Tensor& h, const Tensor& router,
-               int64_t top) {
+               int64_t top, int64_t experts) {
   a.f32 = act_f32(h, "h");
   same_act(router, h, "router");
   TORCH_CHECK(h.dim() == 2 && router.dim() == 2 &&
               router.size(1) == h.size(1));
   a.rows = int(h.size(0));
   a.width = int(h.size(1));
-  a.experts = int(router.size(0));
+  a.routes = int(router.size(0));
+  a.experts = int(experts);
   a.top = int(top);
+  a.groups = a.keep = 1;
   TORCH_CHECK(a.width % 8 == 0, "width must be a multiple of 8");
-  TORCH_CHECK(a.experts >= 1 && a.experts <= 256 && a.top >= 1 &&
-              a.top <= a.experts, "1 <= top <= experts <= 256");
+  TORCH_CHECK(a.experts >= 1 && a.experts <= a.routes && a.routes <= 256 &&
+              a.top >= 1 && a.top <= a.routes,
+              "1 <= top <= experts <= 256");
   a.h = h.data_ptr();
   a.router = router.data_ptr();
 }
 
-std::tuple<Tensor, Tensor> moe_route(const Tensor& h, const Tensor& router,
-                                     int64_t top) {
-  rlli::MoeArgs a{};
-  moe_sizes(a, h, router, top);
-  Tensor ids = at::empty({a.rows, top}, h.options().dtype(at::kInt));
-  Tensor w = at::empty({a.rows, top}, h.options().dtype(at::kFloat));
-  a.ids = ids.data_ptr<int32_t>();
-  a.weights = w.data_ptr<float>();
-  c10::hip::HIPGuardMasqueradingAsCUDA guard(h.device());
-  rlli::launch_moe_route(a, stream_of(h));
-  check_launch("moe_route");
-  return {ids, w};
+// softmax scores, a correction of the choice, groups
+void moe_choice(rlli::MoeArgs& a, const OptTensor& correction,
+                int64_t groups, int64_t keep) {
+  a.softmax = true;
+  a.correction = correction ? f32_vec(*correction, a.routes, "correction")
+                            : nullptr;
+  a.groups = int(groups);
+  a.keep = int(keep);
+  TORCH_CHECK(groups >= 1 && a.routes % groups == 0 && keep >= 1 &&
+              keep <= groups && keep * (a.routes / groups) >= a.top,
+              "groups must divide the routes, those kept hold the choice");
 }
 
-// [rows, top, width]: one output row per (token, choice)
-Tensor moe_experts(const Tensor& h, const Tensor& router, const Tensor& w_up,
-                   const Tensor& w_down, int64_t top, double limit) {
-  rlli::MoeArgs a{};
-  moe_sizes(a, h, router, top);
-  same_act(w_up, h, "w_up");
-  same_act(w_down, h, "w_down");
-  TORCH_CHECK(w_up.dim() == 5 && w_up.size(0) == a.experts &&
-              w_up.size(2) == 2 && w_up.size(3) == 16 &&
-              w_up.size(4) == a.width, "w_up layout");
-  a.ffp = int(w_up.size(1)) * 16;
-  TORCH_CHECK(a.ffp % 64 == 0 && w_down.dim() == 3 &&
-              w_down.size(0) == a.experts && w_down.size(1) == a.width &&
-              w_down.size(2) == a.ffp, "w_down layout");
-  a.limit = float(limit);
-  a.w_up = w_up.data_ptr();
-  a.w_down = w_down.data_ptr();
-  const int64_t P = int64_t(a.rows) * top;
+// the two GEMMs over [rows, top] choices: y [rows, top, width]
+Tensor moe_run(rlli::MoeArgs& a, const Tensor& h, Tensor& ids, Tensor& w) {
+  const int64_t P = int64_t(a.rows) * a.top;
   // the tiled GEMMs index rows and one expert's weights with 32 bits
   const int64_t wide = std::max<int64_t>(a.width, a.ffp);
   TORCH_CHECK(P * wide < (int64_t(1) << 31) &&
-              2 * int64_t(a.ffp) * a.width < (int64_t(1) << 31),
+              (a.gated ? 2 : 1) * int64_t(a.ffp) * a.width <
+                  (int64_t(1) << 31),
               "too many rows or too wide an expert for one call");
   // tall tiles once experts have enough rows each to fill them
-  a.tile_m = (a.f32 || a.width % 64 != 0 || P < int64_t(48) * a.experts)
-                 ? 16
-                 : P < int64_t(384) * a.experts ? 128 : 256;
+  const int64_t each = P / a.routes;
+  a.tile_m = (a.f32 || a.width % 64 != 0 || each < 48) ? 16
+             : each < 384                              ? 128
+                                                       : 256;
   a.max_tiles = int(P / a.tile_m + std::min<int64_t>(a.experts, P));
   auto io = h.options().dtype(at::kInt);
-  Tensor ids = at::empty({a.rows, top}, io);
-  Tensor w = at::empty({a.rows, top}, h.options().dtype(at::kFloat));
+  ids = at::empty({a.rows, a.top}, io);
+  w = at::empty({a.rows, a.top}, h.options().dtype(at::kFloat));
   Tensor plan = at::empty({P + 3 * int64_t(a.max_tiles) + 2 * a.experts}, io);
   Tensor act = at::empty({P, a.ffp}, h.options());
-  Tensor y = at::empty({a.rows, top, a.width}, h.options());
+  Tensor y = at::empty({a.rows, a.top, a.width}, h.options());
   a.ids = ids.data_ptr<int32_t>();
   a.weights = w.data_ptr<float>();
   a.perm = plan.data_ptr<int32_t>();
@@ -203,6 +192,82 @@ Tensor moe_experts(const Tensor& h, const Tensor& router, const Tensor& w_up,
   rlli::launch_moe_experts(a, st);
   check_launch("moe_experts");
   return y;
+}
+
+// the router alone
+std::tuple<Tensor, Tensor> moe_pick(rlli::MoeArgs& a, const Tensor& h) {
+  Tensor ids = at::empty({a.rows, a.top}, h.options().dtype(at::kInt));
+  Tensor w = at::empty({a.rows, a.top}, h.options().dtype(at::kFloat));
+  a.ids = ids.data_ptr<int32_t>();
+  a.weights = w.data_ptr<float>();
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(h.device());
+  rlli::launch_moe_route(a, stream_of(h));
+  check_launch("moe_route");
+  return {ids, w};
+}
+
+std::tuple<Tensor, Tensor> moe_route(const Tensor& h, const Tensor& router,
+                                     int64_t top) {
+  rlli::MoeArgs a{};
+  moe_sizes(a, h, router, top, router.size(0));
+  return moe_pick(a, h);
+}
+
+std::tuple<Tensor, Tensor> moe_route_softmax(const Tensor& h,
+                                             const Tensor& router,
+                                             const OptTensor& correction,
+                                             int64_t top, int64_t groups,
+                                             int64_t keep) {
+  rlli::MoeArgs a{};
+  moe_sizes(a, h, router, top, router.size(0));
+  moe_choice(a, correction, groups, keep);
+  return moe_pick(a, h);
+}
+
+void down_sizes(rlli::MoeArgs& a, const Tensor& h, const Tensor& w_down) {
+  same_act(w_down, h, "w_down");
+  TORCH_CHECK(a.ffp % 64 == 0 && w_down.dim() == 3 &&
+              w_down.size(0) == a.experts && w_down.size(1) == a.width &&
+              w_down.size(2) == a.ffp, "w_down layout");
+  a.w_down = w_down.data_ptr();
+}
+
+// [rows, top, width]: one output row per (token, choice)
+Tensor moe_experts(const Tensor& h, const Tensor& router, const Tensor& w_up,
+                   const Tensor& w_down, int64_t top, double limit) {
+  rlli::MoeArgs a{};
+  moe_sizes(a, h, router, top, router.size(0));
+  same_act(w_up, h, "w_up");
+  TORCH_CHECK(w_up.dim() == 5 && w_up.size(0) == a.experts &&
+              w_up.size(2) == 2 && w_up.size(3) == 16 &&
+              w_up.size(4) == a.width, "w_up layout");
+  a.ffp = int(w_up.size(1)) * 16;
+  a.w_up = w_up.data_ptr();
+  down_sizes(a, h, w_down);
+  a.gated = true;
+  a.limit = float(limit);
+  Tensor ids, w;
+  return moe_run(a, h, ids, w);
+}
+
+// the same for squared-relu experts, with the choice: a consumer that sums
+// a token's rows skips identity experts' rows (never written) and adds their
+// weight of h
+std::tuple<Tensor, Tensor, Tensor> moe_relu2(
+    const Tensor& h, const Tensor& router, const OptTensor& correction,
+    const Tensor& w_up, const Tensor& w_down, int64_t top, int64_t groups,
+    int64_t keep) {
+  rlli::MoeArgs a{};
+  moe_sizes(a, h, router, top, w_up.size(0));
+  moe_choice(a, correction, groups, keep);
+  same_act(w_up, h, "w_up");
+  TORCH_CHECK(w_up.dim() == 3 && w_up.size(2) == a.width, "w_up layout");
+  a.ffp = int(w_up.size(1));
+  a.w_up = w_up.data_ptr();
+  down_sizes(a, h, w_down);
+  Tensor ids, w;
+  Tensor y = moe_run(a, h, ids, w);
+  return {y, ids, w};
 }
 
 }  // namespace
@@ -222,6 +287,11 @@ TORCH_LIBRARY(rlli_mix, m) {
   m.def("moe_route(Tensor h, Tensor router, int top) -> (Tensor, Tensor)");
   m.def("moe_experts(Tensor h, Tensor router, Tensor w_up, Tensor w_down, "
         "int top, float limit) -> Tensor");
+  m.def("moe_route_softmax(Tensor h, Tensor router, Tensor? correction, "
+        "int top, int groups, int keep) -> (Tensor, Tensor)");
+  m.def("moe_relu2(Tensor h, Tensor router, Tensor? correction, "
+        "Tensor w_up, Tensor w_down, int top, int groups, int keep) "
+        "-> (Tensor, Tensor, Tensor)");
 }
 
 TORCH_LIBRARY_IMPL(rlli_mix, CUDA, m) {
@@ -231,4 +301,6 @@ TORCH_LIBRARY_IMPL(rlli_mix, CUDA, m) {
   m.impl("window_tiled", &window_tiled);
   m.impl("moe_route", &moe_route);
   m.impl("moe_experts", &moe_experts);
+  m.impl("moe_route_softmax", &moe_route_softmax);
+  m.impl("moe_relu2", &moe_relu2);
 }

@@ -11,7 +11,7 @@ namespace rlli_ext {
 inline rlli::WindowAttnArgs window_args(
     const Tensor& qkv, const Tensor& k_cache, const Tensor& v_cache,
     int64_t n_q, bool has_kv, double scale = 1.0, int64_t window = 1,
-    int64_t keep_first = 0, const OptTensor& sink = {}) {
+    int64_t keep_first = 0, const OptTensor& sink = {}, int maps = 1) {
   rlli::WindowAttnArgs a{};
   a.f32 = act_f32(qkv, "qkv");
   TORCH_CHECK(k_cache.dim() == 4 && v_cache.dim() == 4 &&
@@ -32,7 +32,9 @@ inline rlli::WindowAttnArgs window_args(
   a.n_q = int(n_q);
   a.n_kv = int(k_cache.size(1));
   a.block_size = int(k_cache.size(2));
-  a.dim = int(k_cache.size(3));
+  a.maps = maps;
+  TORCH_CHECK(k_cache.size(3) % maps == 0, "a key per map");
+  a.dim = int(k_cache.size(3)) / maps;
   a.vdim = int(v_cache.size(3));
   TORCH_CHECK(qkv.dim() == 2);
   a.rows = int(qkv.size(0));
@@ -40,8 +42,11 @@ inline rlli::WindowAttnArgs window_args(
   a.has_kv = has_kv;
   TORCH_CHECK(a.n_q % a.n_kv == 0, "heads must be a multiple of kv heads");
   TORCH_CHECK(a.vdim <= 512 && a.dim <= 4096, "head sizes out of range");
-  TORCH_CHECK(a.stride == a.n_q * a.dim +
-              (has_kv ? a.n_kv * (a.dim + a.vdim) : 0), "qkv width mismatch");
+  const int need = a.n_q * maps * a.dim +
+                   (has_kv ? a.n_kv * (maps * a.dim + a.vdim) : 0);
+  // with two maps further columns (a gate) may follow
+  TORCH_CHECK(maps == 1 ? a.stride == need : a.stride >= need,
+              "qkv width mismatch");
   TORCH_CHECK(window >= 1 && keep_first >= 0);
   a.window = int(std::min<int64_t>(window, 1 << 30));
   a.keep_first = int(std::min<int64_t>(keep_first, 1 << 30));

@@ -33,12 +33,14 @@ void launch_relu2(const void* x, void* out, int64_t n, bool f32,
 // ---- moe.hip -----------------------------------------------------------
 struct MoeArgs {
   const void* h;           // [rows, width]
-  const void* router;      // [experts, width]
-  const void* w_up;        // [experts, ffp/16, 2, 16, width] gate | up
+  const void* router;      // [routes, width]
+  const float* correction; // [routes] added for the choice only, or null
+  const void* w_up;        // [experts, ffp/16, 2, 16, width] gate | up, or
+                           // [experts, ffp, width] without a gate
   const void* w_down;      // [experts, width, ffp]
-  int32_t* ids;            // [rows, top]
+  int32_t* ids;            // [rows, top]; from ``experts`` on: identity
   float* weights;          // [rows, top]
-  int32_t* perm;           // [rows * top] pairs in expert order
+  int32_t* perm;           // [rows * top] experts' pairs in expert order
   int32_t* tile_expert;    // [max_tiles]
   int32_t* tile_row0;      // [max_tiles]
   int32_t* tile_rows;      // [max_tiles]
@@ -46,6 +48,13 @@ struct MoeArgs {
   void* act;               // [rows * top, ffp]
   void* y;                 // [rows, top, width]
   int rows, width, experts, top, ffp, tile_m, max_tiles;
+  int routes;              // experts and identity experts
+  int groups, keep;        // only the best ``keep`` groups of neighbouring
+                           // routes can be chosen
+  bool softmax;            // scores: softmax, chosen ones scaled to sum 1
+                           // (else sigmoid as they are)
+  bool gated;              // gated experts, weight on the input; else relu
+                           // squared, weight on the output
   float limit;
   bool f32;
 };

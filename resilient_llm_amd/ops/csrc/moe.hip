@@ -1,16 +1,21 @@
-// Mixture of experts whose routing weight multiplies the expert's INPUT:
-// y = sum over the chosen experts of expert(w * h), sigmoid scores,
-// clamped swish-like gate.
+// Mixture of experts, two kinds.  Gated: the routing weight (a sigmoid)
+// multiplies the expert's INPUT, y = sum over the chosen experts of
+// expert(w * h), clamped swish-like gate.  Squared relu: y = sum of
+// w expert(h), weights a softmax over all routes, scaled to sum to one over
+// the chosen; a correction may shift the choice, routes may be chosen by
+// groups, and the last routes may be identity experts (w h), which run
+// nothing here: whoever sums a token's outputs adds them.
 //
 //   moe_route     router logits (f32 accumulation over the activation's
-//                 own values), sigmoid, top-k
+//                 own values), scores, top-k
 //   moe_plan      (token, choice) pairs in expert order + row tiles; one
 //                 workgroup for decode-sized batches, three small grids
 //                 for prompts; no host round trip, so it is capturable
 //   moe_experts   two grouped GEMMs.  Up: w * (W h) is scaled in the
 //                 accumulator, gated in registers (gate and up rows are
 //                 packed in alternating blocks of 16) and leaves as one
-//                 [pairs, ff] tensor.  Down: scatters every pair's row to
+//                 [pairs, ff] tensor; or w relu(W h)^2, which the down
+//                 product carries through.  Down: scatters every pair's row to
 //                 [token, choice]; the sum over choices happens in the
 //                 residual kernel that reads it anyway.
 // Small row counts stream the weights straight into MFMA fragments, K
@@ -38,8 +43,8 @@ void moe_route_kernel(MoeArgs a) {
   f32x4_t acc[ET];
 #pragma unroll
   for (int e = 0; e < ET; ++e) {
-    // columns past the last expert repeat it; nobody reads them
-    wp[e] = wr + int64_t(min(e * 16 + lr, a.experts - 1)) * a.width;
+    // columns past the last route repeat it; nobody reads them
+    wp[e] = wr + int64_t(min(e * 16 + lr, a.routes - 1)) * a.width;
     acc[e] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   }
   constexpr int U = ET <= 4 ? 4 : 1;      // k steps with loads in flight
@@ -78,30 +83,88 @@ void moe_route_kernel(MoeArgs a) {
     for (int r = 0; r < 4; ++r)
       part[w][g * 4 + r][e * 16 + lr] = acc[e][r];
   __syncthreads();
-  // each wave ranks two rows, lane l holding experts l, l + 64, ...
+  // each wave ranks two rows, lane l holding routes l, l + 64, ...
   constexpr int EL = (E16 + 63) / 64;
+  constexpr float kNone = -INFINITY;      // cannot be chosen
+  auto wave_fence = [] {
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+  };
   for (int t = w * 2; t < w * 2 + 2; ++t) {
     const int row = row0 + t;
     if (row >= a.rows) break;
-    float s[EL];
+    float s[EL], choice[EL];
 #pragma unroll
     for (int i = 0; i < EL; ++i) {
       const int e = i * 64 + lane;
-      s[i] = -1.f;
-      if (e < a.experts) {
-        float z = 0.f;
+      s[i] = kNone;
+      if (e < a.routes) {
+        s[i] = 0.f;
 #pragma unroll
-        for (int p = 0; p < NW; ++p) z += part[p][t][e];
-        s[i] = 1.f / (1.f + expf(-z));
+        for (int p = 0; p < NW; ++p) s[i] += part[p][t][e];
       }
     }
+    if (a.softmax) {
+      float mx = kNone, sum = 0.f;
+#pragma unroll
+      for (int i = 0; i < EL; ++i) mx = fmaxf(mx, s[i]);
+      mx = wave_max(mx);
+#pragma unroll
+      for (int i = 0; i < EL; ++i) {
+        s[i] = expf(s[i] - mx);           // 0 past the last route
+        sum += s[i];
+      }
+      sum = wave_sum(sum);
+#pragma unroll
+      for (int i = 0; i < EL; ++i) s[i] /= sum;
+    } else {
+#pragma unroll
+      for (int i = 0; i < EL; ++i) s[i] = 1.f / (1.f + expf(-s[i]));
+    }
+#pragma unroll
+    for (int i = 0; i < EL; ++i) {
+      const int e = i * 64 + lane;
+      choice[i] = kNone;
+      if (e < a.routes)
+        choice[i] = s[i] + (a.correction ? a.correction[e] : 0.f);
+    }
+    if (a.keep < a.groups) {
+      // this row's part sums are read; their place holds the choice scores,
+      // the groups' best ones, and which groups stay
+      float *cs = part[0][t], *best = part[1][t], *stays = part[2][t];
+      const int size = a.routes / a.groups;
+      wave_fence();
+#pragma unroll
+      for (int i = 0; i < EL; ++i)
+        if (i * 64 + lane < a.routes) cs[i * 64 + lane] = choice[i];
+      wave_fence();
+      for (int g = lane; g < a.groups; g += 64) {
+        float b = kNone;
+        for (int e = g * size; e < (g + 1) * size; ++e) b = fmaxf(b, cs[e]);
+        best[g] = b;
+      }
+      wave_fence();
+      for (int g = lane; g < a.groups; g += 64) {
+        int ahead = 0;
+        for (int o = 0; o < a.groups; ++o)
+          ahead += best[o] > best[g] || (best[o] == best[g] && o < g);
+        stays[g] = ahead < a.keep ? 1.f : 0.f;
+      }
+      wave_fence();
+#pragma unroll
+      for (int i = 0; i < EL; ++i) {
+        const int e = i * 64 + lane;
+        if (e < a.routes && stays[e / size] == 0.f) choice[i] = kNone;
+      }
+    }
+    float won[EL], total = 0.f;           // lane c & 63 keeps weight c
     for (int c = 0; c < a.top; ++c) {
-      float bv = -2.f;
+      float bv = kNone;
       int bi = 0x7fffffff;
 #pragma unroll
       for (int i = 0; i < EL; ++i)
-        if (s[i] > bv) {
-          bv = s[i];
+        if (choice[i] > bv) {
+          bv = choice[i];
           bi = i * 64 + lane;
         }
 #pragma unroll
@@ -115,13 +178,24 @@ void moe_route_kernel(MoeArgs a) {
       }
 #pragma unroll
       for (int i = 0; i < EL; ++i)
-        if (i * 64 + lane == bi) s[i] = -1.f;
-      bi = min(bi, a.experts - 1);      // a NaN row still names an expert
-      if (lane == 0) {
-        a.ids[int64_t(row) * a.top + c] = bi;
-        a.weights[int64_t(row) * a.top + c] = bv;
-      }
+        if (i * 64 + lane == bi) choice[i] = kNone;
+      bi = min(bi, a.routes - 1);       // a NaN row still names a route
+      float mine = s[0];
+#pragma unroll
+      for (int i = 1; i < EL; ++i)
+        if (bi >> 6 == i) mine = s[i];
+      mine = __shfl(mine, bi & 63, kWave);
+      total += mine;
+#pragma unroll
+      for (int i = 0; i < EL; ++i)
+        if (c == i * 64 + lane) won[i] = mine;
+      if (lane == 0) a.ids[int64_t(row) * a.top + c] = bi;
     }
+    const float scale = a.softmax ? 1.f / (total + 1e-20f) : 1.f;
+#pragma unroll
+    for (int i = 0; i < EL; ++i)
+      if (i * 64 + lane < a.top)
+        a.weights[int64_t(row) * a.top + i * 64 + lane] = won[i] * scale;
   }
 }
 
@@ -160,7 +234,8 @@ void moe_plan_one_kernel(MoeArgs a) {
   const int P = a.rows * a.top;
   for (int e = tid; e < a.experts; e += 256) count[e] = 0;
   __syncthreads();
-  for (int p = tid; p < P; p += 256) atomicAdd(&count[a.ids[p]], 1);
+  for (int p = tid; p < P; p += 256)
+    if (a.ids[p] < a.experts) atomicAdd(&count[a.ids[p]], 1);
   __syncthreads();
   if (tid == 0) {
     int s = 0;
@@ -172,7 +247,7 @@ void moe_plan_one_kernel(MoeArgs a) {
   }
   __syncthreads();
   for (int p = tid; p < P; p += 256)
-    a.perm[atomicAdd(&cursor[a.ids[p]], 1)] = p;
+    if (a.ids[p] < a.experts) a.perm[atomicAdd(&cursor[a.ids[p]], 1)] = p;
   write_tiles(a, count, start, tid, 256);
 }
 
@@ -192,7 +267,7 @@ void moe_count_kernel(MoeArgs a) {
   for (int e = tid; e < a.experts; e += 256) count[e] = 0;
   __syncthreads();
   for (int p = p0 + tid; p < min(P, p0 + PLAN_PAIRS); p += 256)
-    atomicAdd(&count[a.ids[p]], 1);
+    if (a.ids[p] < a.experts) atomicAdd(&count[a.ids[p]], 1);
   __syncthreads();
   for (int e = tid; e < a.experts; e += 256)
     if (count[e]) atomicAdd(&a.counters[e], count[e]);
@@ -217,14 +292,14 @@ void moe_scatter_kernel(MoeArgs a) {
     }
   }
   for (int p = p0 + tid; p < min(P, p0 + PLAN_PAIRS); p += 256)
-    atomicAdd(&count[a.ids[p]], 1);
+    if (a.ids[p] < a.experts) atomicAdd(&count[a.ids[p]], 1);
   __syncthreads();
   for (int e = tid; e < a.experts; e += 256)
     base[e] = start[e] +
               (count[e] ? atomicAdd(&a.counters[a.experts + e], count[e]) : 0);
   __syncthreads();
   for (int p = p0 + tid; p < min(P, p0 + PLAN_PAIRS); p += 256)
-    a.perm[atomicAdd(&base[a.ids[p]], 1)] = p;
+    if (a.ids[p] < a.experts) a.perm[atomicAdd(&base[a.ids[p]], 1)] = p;
   if (blockIdx.x == 0) write_tiles(a, total, start, tid, 256);
 }
 
@@ -238,9 +313,14 @@ DEV_INLINE float expert_gate(float g, float u, float limit) {
   return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
 }
 
+DEV_INLINE float relu_squared(float x) {
+  x = fmaxf(x, 0.f);
+  return x * x;
+}
+
 // --------------------------------------- small row counts: stream weights
 // One workgroup per (16-row tile, 32 weight rows); its waves split K.
-template <typename T, bool UP>
+template <typename T, bool UP, bool GATED>
 __global__ __launch_bounds__(256)
 void moe_small_kernel(MoeArgs a) {
   __shared__ float part[4][2][16][17];
@@ -252,7 +332,7 @@ void moe_small_kernel(MoeArgs a) {
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int lr = lane & 15, g = lane >> 4;
   const int K = UP ? a.width : a.ffp;
-  const int N = UP ? 2 * a.ffp : a.width;
+  const int N = UP ? (GATED ? 2 : 1) * a.ffp : a.width;
   const int n0 = blockIdx.x * 32;
 
   const int pr = p0 + min(lr, rows - 1);
@@ -316,9 +396,14 @@ void moe_small_kernel(MoeArgs a) {
   const int pair = a.perm[p0 + row];
   if constexpr (UP) {
     const float wt = a.weights[pair];
-    act_store(reinterpret_cast<T*>(a.act) + int64_t(p0 + row) * a.ffp +
-                  blockIdx.x * 16 + col,
-              expert_gate<T>(s0 * wt, s1 * wt, a.limit));
+    T* o = reinterpret_cast<T*>(a.act) + int64_t(p0 + row) * a.ffp;
+    if constexpr (GATED) {
+      act_store(o + blockIdx.x * 16 + col,
+                expert_gate<T>(s0 * wt, s1 * wt, a.limit));
+    } else {
+      act_store(o + n0 + col, relu_squared(s0) * wt);
+      act_store(o + n0 + 16 + col, relu_squared(s1) * wt);
+    }
   } else {
     T* y = reinterpret_cast<T*>(a.y) + int64_t(pair) * a.width;
     if (n0 + col < N) act_store(y + n0 + col, s0);
@@ -342,7 +427,7 @@ DEV_INLINE void lds_load16(const void* g, void* l) {
       (__attribute__((address_space(3))) void*)l, 16, 0, 0);
 }
 
-template <bool UP, int TT>
+template <bool UP, int TT, bool GATED>
 __global__ __launch_bounds__(TT == 256 ? 512 : 256, 2)
 void moe_tile_kernel(MoeArgs a, int n_blocks) {
   constexpr int NT = TT == 256 ? 512 : 256;       // threads
@@ -362,7 +447,7 @@ void moe_tile_kernel(MoeArgs a, int n_blocks) {
   const int e = a.tile_expert[tile];
   const int p0 = a.tile_row0[tile];
   const int K = UP ? a.width : a.ffp;
-  const int N = UP ? 2 * a.ffp : a.width;
+  const int N = UP ? (GATED ? 2 : 1) * a.ffp : a.width;
   const int n0 = nb * TT;
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
   const int lr = lane & 15, g = lane >> 4;
@@ -470,12 +555,21 @@ void moe_tile_kernel(MoeArgs a, int n_blocks) {
         const float wt = s_weight[tr];
         uint16_t* o = reinterpret_cast<uint16_t*>(a.act) +
                       int64_t(p0 + tr) * a.ffp;
+        if constexpr (GATED) {
 #pragma unroll
-        for (int j = 0; j < 4; j += 2) {
-          const int f = (n0 + wn + j * 16) / 2 + lr;
-          if (f < a.ffp)
-            o[f] = f32_to_bf16(expert_gate<uint16_t>(acc[i][j][r] * wt,
-                                           acc[i][j + 1][r] * wt, a.limit));
+          for (int j = 0; j < 4; j += 2) {
+            const int f = (n0 + wn + j * 16) / 2 + lr;
+            if (f < a.ffp)
+              o[f] = f32_to_bf16(expert_gate<uint16_t>(
+                  acc[i][j][r] * wt, acc[i][j + 1][r] * wt, a.limit));
+          }
+        } else {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const int f = n0 + wn + j * 16 + lr;
+            if (f < a.ffp)
+              o[f] = f32_to_bf16(relu_squared(acc[i][j][r]) * wt);
+          }
         }
       } else {
         uint16_t* o = reinterpret_cast<uint16_t*>(a.y) +
@@ -492,13 +586,13 @@ void moe_tile_kernel(MoeArgs a, int n_blocks) {
 template <typename T>
 void route(const MoeArgs& a, hipStream_t st) {
   const dim3 grid((a.rows + 15) / 16), blk(512);
-  if (a.experts <= 16)
+  if (a.routes <= 16)
     hipLaunchKernelGGL((moe_route_kernel<T, 1>), grid, blk, 0, st, a);
-  else if (a.experts <= 32)
+  else if (a.routes <= 32)
     hipLaunchKernelGGL((moe_route_kernel<T, 2>), grid, blk, 0, st, a);
-  else if (a.experts <= 64)
+  else if (a.routes <= 64)
     hipLaunchKernelGGL((moe_route_kernel<T, 4>), grid, blk, 0, st, a);
-  else if (a.experts <= 128)
+  else if (a.routes <= 128)
     hipLaunchKernelGGL((moe_route_kernel<T, 8>), grid, blk, 0, st, a);
   else
     hipLaunchKernelGGL((moe_route_kernel<T, 16>), grid, blk, 0, st, a);
@@ -506,18 +600,23 @@ void route(const MoeArgs& a, hipStream_t st) {
 
 template <typename T>
 void small(const MoeArgs& a, hipStream_t st) {
-  hipLaunchKernelGGL((moe_small_kernel<T, true>),
-                     dim3(2 * a.ffp / 32, a.max_tiles), dim3(256), 0, st, a);
-  hipLaunchKernelGGL((moe_small_kernel<T, false>),
+  if (a.gated)
+    hipLaunchKernelGGL((moe_small_kernel<T, true, true>),
+                       dim3(2 * a.ffp / 32, a.max_tiles), dim3(256), 0, st,
+                       a);
+  else
+    hipLaunchKernelGGL((moe_small_kernel<T, true, false>),
+                       dim3(a.ffp / 32, a.max_tiles), dim3(256), 0, st, a);
+  hipLaunchKernelGGL((moe_small_kernel<T, false, false>),
                      dim3((a.width + 31) / 32, a.max_tiles), dim3(256), 0, st,
                      a);
 }
 
-template <bool UP, int TT>
+template <bool UP, int TT, bool GATED>
 void tiled_one(const MoeArgs& a, hipStream_t st) {
   const size_t smem = size_t(4) * TT * BK * 2;
-  const int nb = ((UP ? 2 * a.ffp : a.width) + TT - 1) / TT;
-  auto* k = moe_tile_kernel<UP, TT>;
+  const int nb = ((UP ? (GATED ? 2 : 1) * a.ffp : a.width) + TT - 1) / TT;
+  auto* k = moe_tile_kernel<UP, TT, GATED>;
   if (smem > 65536)
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k),
                               hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -528,8 +627,9 @@ void tiled_one(const MoeArgs& a, hipStream_t st) {
 
 template <int TT>
 void tiled(const MoeArgs& a, hipStream_t st) {
-  tiled_one<true, TT>(a, st);
-  tiled_one<false, TT>(a, st);
+  if (a.gated) tiled_one<true, TT, true>(a, st);
+  else tiled_one<true, TT, false>(a, st);
+  tiled_one<false, TT, false>(a, st);
 }
 
 }  // namespace

@@ -9,6 +9,8 @@ kernels round (bf16 storage boundaries), computed in fp32.
 
 from __future__ import annotations
 
+import math
+
 import torch
 
 
@@ -41,6 +43,28 @@ def build_cos_sin(max_pos: int, head_dim: int, theta: float = 500000.0,
     pos = torch.arange(max_pos, dtype=torch.float64)
     ang = torch.outer(pos, inv_freq)
     return torch.cat([ang.cos(), ang.sin()], dim=-1).float().to(device)
+
+
+def yarn_cos_sin(max_pos: int, dims: int, base: float, factor: float,
+                 original: float, fast: float, slow: float,
+                 device="cpu") -> torch.Tensor:
+    """build_cos_sin with frequencies slowed down by ``factor``, as far as
+    they turn fewer than ``slow`` times over ``original`` positions, kept
+    where they turn more than ``fast`` times, a ramp in between; cosines and
+    sines grow with ln(factor)."""
+    def pair_of(turns):
+        return dims * math.log(original / (2 * math.pi * turns)) \
+            / (2 * math.log(base))
+    lo = max(math.floor(pair_of(fast)), 0)
+    hi = min(math.ceil(pair_of(slow)), dims - 1)
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+    freq = base ** (-2 * i / dims)
+    freq = freq / factor * ramp + freq * (1 - ramp)
+    ang = torch.outer(torch.arange(max_pos, dtype=torch.float64), freq)
+    gain = 0.1 * math.log(factor) + 1
+    return (gain * torch.cat([ang.cos(), ang.sin()], dim=-1)).float() \
+        .to(device)
 
 
 def _rotate(x: torch.Tensor, positions: torch.Tensor,

@@ -67,6 +67,99 @@ def _attend(q, qpos, k_cache, v_cache, table, sink, scale, window,
     return torch.einsum("hnm,mhd->nhd", p, v).reshape(q.shape[0], -1)
 
 
+# ---------------------------------------------- differential attention
+def _turn_halves(x, positions, cos_sin):
+    """x [T, ..., D] f32; pairs (i, i + rot / 2)."""
+    if cos_sin is None:
+        return x
+    rot = cos_sin.shape[1]
+    cs = cos_sin[positions.long()].view(-1, *[1] * (x.dim() - 2), rot)
+    c, s = cs.chunk(2, -1)
+    u, v = x[..., :rot // 2], x[..., rot // 2:rot]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., rot:]], -1)
+
+
+def _normed(x, gain, eps):
+    x = x.float()
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * gain
+
+
+def diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q,
+                q_norm, k_norm, eps):
+    T = qkv.shape[0]
+    _, G, bs, D2 = k_cache.shape
+    V, D = v_cache.shape[3], D2 // 2
+    q, k, v = (qkv[:, :n_q * D2].view(T, n_q, 2, D),
+               qkv[:, n_q * D2:(n_q + G) * D2].view(T, G, 2, D),
+               qkv[:, (n_q + G) * D2:(n_q + G) * D2 + G * V])
+    b, o = slots.long() // bs, slots.long() % bs
+    k = _turn_halves(_normed(k, k_norm, eps), positions, cos_sin)
+    k_cache[b, :, o] = k.reshape(T, G, D2).to(k_cache.dtype)
+    v_cache[b, :, o] = v.reshape(T, G, V).to(v_cache.dtype)
+    q.copy_(_turn_halves(_normed(q, q_norm, eps), positions, cos_sin))
+
+
+def _diff_attend(q, gate, qpos, k_cache, v_cache, table, scale, chunk, cap,
+                 lam, out_scale, eps):
+    """q [n, H, 2, D] at positions qpos over one sequence's cache."""
+    _, G, bs, D2 = k_cache.shape
+    n_kv = int(qpos[-1]) + 1
+    blocks = table[:-(-n_kv // bs)].long()
+    k = k_cache[blocks].float().transpose(1, 2).reshape(-1, G, D2)[:n_kv]
+    v = v_cache[blocks].float().transpose(1, 2) \
+        .reshape(-1, G, v_cache.shape[3])[:n_kv]
+    H = q.shape[1]
+    i, j = qpos[:, None].long(), torch.arange(n_kv)[None]
+    ok = (j <= i) & (j >= i // chunk * chunk)
+    seen = ok.any(0)                 # the rest may hold anything
+    k, v, ok = k[seen], v[seen], ok[:, seen]
+    k = k.view(len(k), G, 2, -1).repeat_interleave(H // G, 1)
+    v = v.repeat_interleave(H // G, 1)
+    s = torch.einsum("nhad,mhad->ahnm", q.float(), k) * scale
+    if cap > 0:
+        s = cap * torch.tanh(s / cap)
+    p = torch.softmax(s.masked_fill(~ok, float("-inf")), -1)
+    a1, a2 = torch.einsum("ahnm,mhd->anhd", p, v)
+    o = _normed(a1 - lam * a2, out_scale, eps)
+    if gate is not None:
+        o = o * torch.sigmoid(gate.float())[..., None]
+    return o.reshape(q.shape[0], -1)
+
+
+def _diff_queries(qkv, k_cache, n_q):
+    D2 = k_cache.shape[3]
+    return qkv[:, :n_q * D2].view(-1, n_q, 2, D2 // 2)
+
+
+def diff_prefill(qkv, gate, k_cache, v_cache, positions, cos_sin, slots,
+                 block_tables, prompt, n_q, q_norm, k_norm, scale, chunk, cap,
+                 lam, out_scale, eps):
+    diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q,
+                q_norm, k_norm, eps)
+    q = _diff_queries(qkv, k_cache, n_q)
+    out = torch.empty(qkv.shape[0], n_q * v_cache.shape[3], dtype=qkv.dtype)
+    for p in prompt.portions:
+        r = slice(p.row0, p.row0 + p.n)
+        out[r] = _diff_attend(
+            q[r], None if gate is None else gate[r], positions[r], k_cache,
+            v_cache, block_tables[p.seq], scale, chunk, cap, lam, out_scale,
+            eps).to(qkv.dtype)
+    return out
+
+
+def diff_decode(qkv, k_cache, v_cache, positions, cos_sin, slots,
+                block_tables, gate, scale, n_q, q_norm, k_norm, chunk, cap,
+                lam, out_scale, eps):
+    diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q,
+                q_norm, k_norm, eps)
+    q = _diff_queries(qkv, k_cache, n_q)
+    return torch.cat([
+        _diff_attend(q[b:b + 1], None if gate is None else gate[b:b + 1],
+                     positions[b:b + 1], k_cache, v_cache, block_tables[b],
+                     scale, chunk, cap, lam, out_scale, eps)
+        for b in range(qkv.shape[0])]).to(qkv.dtype)
+
+
 def window_prefill(qkv, k_cache, v_cache, positions, cos_sin, slots,
                    block_tables, prompt, sink, scale, n_q, window,
                    keep_first, has_kv, r1, r2, temp_coef, temp_every, v_eps):

@@ -45,6 +45,33 @@ def moe_route(h, router, top):
     return ids[:, :top].to(torch.int32).contiguous(), w[:, :top].contiguous()
 
 
+def moe_route_softmax(h, router, correction, top, groups, keep):
+    s = torch.softmax(h.float() @ router.float().T, -1)
+    choice = s if correction is None else s + correction
+    g = choice.view(-1, groups, choice.shape[1] // groups)
+    order = torch.sort(g.amax(-1), dim=-1, descending=True,
+                       stable=True).indices[:, :keep]
+    stays = torch.zeros(g.shape[:2], dtype=torch.bool).scatter_(1, order, True)
+    choice = g.masked_fill(~stays[..., None], float("-inf")).flatten(1)
+    ids = torch.sort(choice, dim=-1, descending=True,
+                     stable=True).indices[:, :top]
+    w = s.gather(1, ids)
+    return (ids.to(torch.int32).contiguous(),
+            w / (w.sum(-1, keepdim=True) + 1e-20))
+
+
+def moe_relu2(h, router, correction, w_up, w_down, top, groups, keep):
+    ids, w = moe_route_softmax(h, router, correction, top, groups, keep)
+    # identity experts' rows stay unwritten, as on the GPU
+    y = torch.full((h.shape[0], top, h.shape[1]), float("nan"))
+    for e in range(w_up.shape[0]):
+        t, c = torch.nonzero(ids == e, as_tuple=True)
+        if len(t):
+            r = torch.relu(h[t].float() @ w_up[e].float().T)
+            y[t, c] = (r * r * w[t, c][:, None]) @ w_down[e].float().T
+    return y.to(h.dtype), ids, w
+
+
 def moe_experts(h, router, w_up, w_down, top, limit):
     ids, w = moe_route(h, router, top)
     T, W = h.shape
