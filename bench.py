@@ -180,9 +180,10 @@ def design_models(design: str) -> dict:
     """size -> {name: configuration}: the design, then existing models of
     equal width, depth, heads and (active) feed-forward size."""
     from resilient_llm_amd.models import (
-        BolatarConfig, LlamaConfig, NesizenConfig, RiruzenConfig,
+        BolatarConfig, FimunexConfig, LlamaConfig, NesizenConfig,
+        RiruzenConfig,
     )
-    from resilient_llm_amd.models import bolatar, nesizen, riruzen
+    from resilient_llm_amd.models import bolatar, fimunex, nesizen, riruzen
 
     def llama(width, layers, heads, kv, ff):
         return LlamaConfig(name=f"llama-w{width}", hidden_size=width,
@@ -190,15 +191,16 @@ def design_models(design: str) -> dict:
                            head_dim=128, intermediate_size=ff,
                            vocab_size=65536, max_position=32768)
 
-    def nesi(width, layers, heads, kv, gla_heads, mlp, first=None):
+    def nesi(width, layers, heads, kv, gla_heads, mlp, first=None,
+             attn_every=3, window=1024):
         return NesizenConfig.from_dict(
             {"width": width, "vocab": 65536, "streams": 2,
              "norm": {"eps": 1e-5},
              "layers": nesizen.hybrid_layers(
-                 layers, 3,
+                 layers, attn_every,
                  {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128,
                   "scale": 128 ** -0.5, "rot": {"dims": 64, "base": 1e6},
-                  "mask": {"size": 1024, "keep_first": 4}},
+                  "mask": {"size": window, "keep_first": 4}},
                  {"heads": gla_heads, "dim": 128, "vdim": 256, "tau": 16.0},
                  mlp, first)},
             name=f"nesizen-w{width}")
@@ -237,8 +239,33 @@ def design_models(design: str) -> dict:
                  {"kind": "dense", "ff": ff, "limit": 7.0})},
             name=f"bolatar-w{width}", decay_rank=64)
 
+    def fimu(width, layers, heads, kv, mlp):
+        return FimunexConfig.from_dict(
+            {"width": width, "vocab": 65536, "logit_softcap": 30.0,
+             "canon": {"taps": 4}, "norm": {"eps": 1e-5},
+             "loop": {"start": 0, "stop": layers, "times": 1},
+             "layers": fimunex.uniform_layers(
+                 layers, fimunex.diff_attention(heads, kv, 64, 128, 4096),
+                 mlp)}, name=f"fimunex-w{width}")
+
     def dense(ff):
         return {"kind": "dense", "ff": ff}
+    if design == "fimunex":
+        # attention in every layer, as far as either sees; two matrices of
+        # 3/2 the width are as large as the gated three
+        relu2 = fimunex.relu2_moe
+        return {"w2048": {"fimunex": fimu(2048, 12, 16, 4,
+                                          relu2(32, 8, 4, 1536, 8, 4)),
+                          "nesizen": nesi(2048, 12, 16, 4, 8,
+                                          moe(32, 4, 1024), attn_every=1,
+                                          window=4096),
+                          "llama": llama(2048, 12, 16, 4, 4096)},
+                "w4096": {"fimunex": fimu(4096, 6, 32, 8,
+                                          relu2(16, 4, 2, 5376, 4, 2)),
+                          "nesizen": nesi(4096, 6, 32, 8, 16,
+                                          moe(16, 2, 3584), attn_every=1,
+                                          window=4096),
+                          "llama": llama(4096, 6, 32, 8, 7168)}}
     if design == "bolatar":
         # two matrices of 3/2 the width are as large as the gated three
         return {"w2048": {"bolatar": bola(2048, 12, 16, 4, 4096),
@@ -364,7 +391,7 @@ def main() -> None:
     ap.add_argument("--device", default=None,
                     help="override torch device (tests: cpu)")
     ap.add_argument("--design", default=None,
-                    choices=("nesizen", "riruzen", "bolatar"),
+                    choices=("nesizen", "riruzen", "bolatar", "fimunex"),
                     help="measure this design's engine throughput beside "
                          "existing models of equal size instead of serving")
     ap.add_argument("--design-sizes", default="w2048,w4096")

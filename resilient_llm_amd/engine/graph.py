@@ -29,6 +29,8 @@ exceed the capture envelope (very long sequences) decode eager.
 
 from __future__ import annotations
 
+import gc
+
 import torch
 
 from .. import ops
@@ -121,18 +123,28 @@ class DecodeGraphRunner:
         torch.cuda.current_stream(self.device).wait_stream(s)
         torch.cuda.synchronize(self.device)
 
-        # capture largest-first so the shared pool is sized once
-        for b in sorted(self.buckets, reverse=True):
-            g = torch.cuda.CUDAGraph()
-            if self._pool is None:
-                with torch.cuda.graph(g):
-                    self.logits[b], self.tokens[b] = self._steady_body(b)
-                self._pool = g.pool()
-            else:
-                with torch.cuda.graph(g, pool=self._pool):
-                    self.logits[b], self.tokens[b] = self._steady_body(b)
-            self.graphs[b] = g
-        torch.cuda.synchronize(self.device)
+        # an earlier runner may be garbage by now (it and its engine refer to
+        # each other); were it collected during a capture, destroying its
+        # graphs would be refused and end the process
+        gc.collect()
+        collecting = gc.isenabled()
+        gc.disable()
+        try:
+            # capture largest-first so the shared pool is sized once
+            for b in sorted(self.buckets, reverse=True):
+                g = torch.cuda.CUDAGraph()
+                if self._pool is None:
+                    with torch.cuda.graph(g):
+                        self.logits[b], self.tokens[b] = self._steady_body(b)
+                    self._pool = g.pool()
+                else:
+                    with torch.cuda.graph(g, pool=self._pool):
+                        self.logits[b], self.tokens[b] = self._steady_body(b)
+                self.graphs[b] = g
+            torch.cuda.synchronize(self.device)
+        finally:
+            if collecting:
+                gc.enable()
         # the warmup/captures advanced the state buffers; a load() must
         # precede the first real step()
         self._nb = 0

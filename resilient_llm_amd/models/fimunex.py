@@ -10,9 +10,9 @@ correction of the choice and identity experts.  A range of layers may run
 several times, each pass with a cache of its own.  Sizes, constants and the
 order of layers come from config.json.
 
-Projections that share an input are one product, biases in it.  One pass
-sums a token's expert outputs, writes the residual, norms it and, for
-decoded tokens, convolves.  Residual, norms, angles, scores, router and
+Projections that share an input are one product; its biases are added where
+the product is read.  One pass sums a token's expert outputs, writes the
+residual, norms it and, for decoded tokens, convolves.  Residual, norms, angles, scores, router and
 convolution sums are 32-bit; product inputs, caches and convolution tails
 have the model dtype, which may also be float32.
 """
@@ -322,18 +322,16 @@ class FimunexForCausalLM(MixedModel):
             P[p + "norm.mix"] = 1 + vec(p + "norm1")
             P[p + "taps.mix"] = vec(p + "canon1").t().contiguous()
             w = torch.cat([mat(q + x, rows=True) for x in "qkvg"])
-            b = torch.cat([mat(f"{q}{x}.b", rows=True) for x in "qkv"])
-            rows = -(-w.shape[0] // 8) * 8
-            P[p + "proj"] = F.pad(w, (0, 0, 0, rows - w.shape[0]))
-            P[p + "proj.b"] = F.pad(b, (0, rows - b.shape[0]))
+            P[p + "proj"] = F.pad(w, (0, 0, 0, -w.shape[0] % 8))
+            P[p + "proj.b"] = torch.cat(
+                [vec(f"{q}{x}.b", rows=True) for x in "qkv"])
             P[p + "q_norm"], P[p + "k_norm"] = (vec(q + "q.norm"),
                                                 vec(q + "k.norm"))
             one, two = ((vec(q + "lq" + x) * vec(q + "lk" + x)).sum().exp()
                         for x in "12")
             self._lambda[i] = float(one - two) + m.diff
             P[p + "o"] = mat(q + "o", cols=True)
-            b = mat(q + "o.b")
-            P[p + "o.b"] = b if self.tp_rank == 0 else torch.zeros_like(b)
+            P[p + "o.b"] = vec(q + "o.b")
             if f is None:
                 continue
             q = p + "mlp."
@@ -356,15 +354,17 @@ class FimunexForCausalLM(MixedModel):
 
     # ------------------------------------------------------------ compute
     def _attention(self, i, place, h, kv_cache, step):
+        """(output, what block_step needs to add it)."""
         P, p, nd = self.params, f"l{i}.", step.n_decode
         m, n = self.config.layers[i].mixer, self.tp_world
-        qkv = _linear(h, P[p + "proj"], P[p + "proj.b"])
+        qkv = _linear(h, P[p + "proj"])
         heads, kv = m.heads // n, m.kv_heads // n
         g0 = 2 * (heads + kv) * m.dim + kv * m.vdim
         gate = qkv[:, g0:g0 + heads]
         k, v = kv_cache.layer(place)
-        score = (heads, P[p + "q_norm"], P[p + "k_norm"], m.scale, m.chunk,
-                 m.softcap, self._lambda[i], 1 - m.diff, self.config.rms_eps)
+        score = (heads, P[p + "proj.b"], P[p + "q_norm"], P[p + "k_norm"],
+                 m.scale, m.chunk, m.softcap, self._lambda[i], 1 - m.diff,
+                 self.config.rms_eps)
         parts = []
         if nd:
             parts.append(ops.diff_decode(
@@ -376,10 +376,11 @@ class FimunexForCausalLM(MixedModel):
                 self._rot[m.rot], step.slots[nd:], step.tables_pre,
                 step.prompt, *score))
         out = parts[0] if len(parts) == 1 else torch.cat(parts)
-        return self._reduce(_linear(out, P[p + "o"], P[p + "o.b"]))
+        return (self._reduce(_linear(out, P[p + "o"])),
+                dict(y_bias=P[p + "o.b"]))
 
     def _experts(self, i, h):
-        """(output, what block_step needs to sum it)."""
+        """(output, what block_step needs to add it)."""
         P, f, p = self.params, self.config.layers[i].mlp, f"l{i}."
         W = h.shape[1]
         pad = -W % 8
@@ -421,15 +422,15 @@ class FimunexForCausalLM(MixedModel):
                 ops.conv_prompt(h[nd:], P[f"l{i}.taps.{which}"], tail(n),
                                 step.prompt, hc[nd:])
             if which == "mix":
-                y, parts = self._attention(i, n, hc, kv_cache, step), {}
+                y, more = self._attention(i, n, hc, kv_cache, step)
             else:
-                y, parts = self._experts(i, hc)
+                y, more = self._experts(i, hc)
             if n + 1 < len(self._sublayers):
                 norm, conv = reads(n + 1)
                 h, hc = ops.block_step(x, y, *norm, step.positions, *conv,
-                                       **parts)
+                                       **more)
             else:
                 h, _ = ops.block_step(
                     x, y, P["final.norm"], 1, c.rms_eps, step.positions,
-                    rows=sample_idx, keep=False, **parts)
+                    rows=sample_idx, keep=False, **more)
         return ops.soft_cap(_linear(h, P["head"]), c.logit_softcap)

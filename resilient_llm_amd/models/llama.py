@@ -41,9 +41,7 @@ _USE_SKINNY = os.environ.get("RLLI_SKINNY") == "1"
 _LT_ROWS = frozenset({1, 2, 4, 8, 12, 16, 24, 32, 48, 64, 96, 128})
 
 
-def _linear(x, w, b=None):
-    if b is not None:
-        return F.linear(x, w, b)
+def _linear(x, w):
     if _USE_SKINNY:
         return ops.linear_auto(x, w)
     if x.is_cuda and x.dim() == 2 and x.shape[0] in _LT_ROWS:

@@ -400,35 +400,35 @@ def biased_prefill(qkv, k_cache, v_cache, positions, slots, block_tables,
 
 
 def diff_decode(qkv, gate, k_cache, v_cache, positions, cos_sin, slots,
-                block_tables, n_q: int, q_norm, k_norm, scale: float,
+                block_tables, n_q: int, bias, q_norm, k_norm, scale: float,
                 chunk: int, cap: float, lam: float, out_scale: float,
                 eps: float):
     """Differential attention, one new token per sequence, append included.
-    ``qkv``: q | k | v | .., a head's query and key being two maps side by
-    side, each normed and rotated (pairs i, i + rot / 2); scores capped; a
-    query sees its chunk of positions; the maps' outputs a1 - lam a2 over
-    their root mean square, times out_scale and the sigmoid of ``gate``
-    [rows, n_q]."""
+    ``qkv``: q | k | v | .., ``bias`` added to the three; a head's query and
+    key are two maps side by side, each normed and rotated (pairs i, i + rot
+    / 2); scores capped; a query sees its chunk of positions; the maps'
+    outputs a1 - lam a2 over their root mean square, times out_scale and the
+    sigmoid of ``gate`` [rows, n_q]."""
     return _ns("rlli_attn", qkv).diff_decode(
         qkv, k_cache, v_cache, positions, cos_sin, slots, block_tables, gate,
-        scale, n_q, q_norm, k_norm, chunk, cap, lam, out_scale, eps)
+        scale, n_q, bias, q_norm, k_norm, chunk, cap, lam, out_scale, eps)
 
 
 def diff_prefill(qkv, gate, k_cache, v_cache, positions, cos_sin, slots,
-                 block_tables, prompt, n_q: int, q_norm, k_norm, scale: float,
-                 chunk: int, cap: float, lam: float, out_scale: float,
-                 eps: float):
+                 block_tables, prompt, n_q: int, bias, q_norm, k_norm,
+                 scale: float, chunk: int, cap: float, lam: float,
+                 out_scale: float, eps: float):
     """The same for prompt rows: append, then attend over what the rows'
     chunks hold, gathered (sizes that the tiled kernel does not take: over
     the pages, row by row)."""
     if not qkv.is_cuda:
         return ref_attn.diff_prefill(
             qkv, gate, k_cache, v_cache, positions, cos_sin, slots,
-            block_tables, prompt, n_q, q_norm, k_norm, scale, chunk, cap, lam,
-            out_scale, eps)
+            block_tables, prompt, n_q, bias, q_norm, k_norm, scale, chunk,
+            cap, lam, out_scale, eps)
     attn = _ns("rlli_attn", qkv)
     attn.diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q,
-                     q_norm, k_norm, eps)
+                     bias, q_norm, k_norm, eps)
     tail = (chunk, cap, lam, out_scale, eps)
     _, n_kv, _, width = k_cache.shape
     vdim = v_cache.shape[3]
@@ -590,16 +590,18 @@ def block_embed(ids, table, pos_table, positions, x, gain, groups: int,
 def block_step(x, y, gain, groups: int, eps: float, positions, taps=None,
                tail=None, slots=None, n_decode: int = 0, rows=None,
                keep: bool = True, y2=None, gain1=None, gain2=None,
-               part_ids=None, part_w=None, part_h=None, part_limit: int = 0):
+               part_ids=None, part_w=None, part_h=None, part_limit: int = 0,
+               y_bias=None):
     """Add a block's output to the residual; then as block_embed.  ``rows``
     restricts the result (then keep=False).  With ``y2`` half the sum of
     both outputs is added, each normed first (``gain1``, ``gain2``).  With
     ``part_ids`` [T, parts] the sum over y [T, parts, W] is added, where a
-    part whose id is ``part_limit`` or more is part_w part_h instead."""
+    part whose id is ``part_limit`` or more is part_w part_h instead.
+    ``y_bias`` [W] goes with a single output."""
     return _ns("rlli_blk", y).block_step(x, y, gain, groups, eps, positions,
                                          taps, tail, slots, n_decode, rows,
                                          keep, y2, gain1, gain2, part_ids,
-                                         part_w, part_h, part_limit)
+                                         part_w, part_h, part_limit, y_bias)
 
 
 def conv_prompt(h, taps, tail, prompt, out, silu: bool = False):

@@ -53,6 +53,7 @@ LIBRARIES = {
     "rlli_attn": [
         "ext_attn.cpp",
         "window_attn.hip",
+        "diff_attn.hip",
         "expanded_attn.hip",
     ],
     "rlli_mix": [

@@ -1,5 +1,5 @@
 // Launch declarations of paged softmax attention (window_attn.hip,
-// window_prefill.hip, expanded_attn.hip).
+// window_prefill.hip, diff_attn.hip, expanded_attn.hip).
 #pragma once
 
 #include "act.h"
@@ -46,6 +46,7 @@ struct WindowAttnArgs {
   // map 1 - lambda map 2, over its root mean square, times out_scale and
   // the sigmoid of the head's gate.
   int maps;                // 1 or 2
+  const float* bias;       // [q | k | v] added to them, or null (maps = 2)
   const float* q_norm;     // [dim] norms of queries and keys per head and
   const float* k_norm;     // map, ahead of the rotation (maps = 2)
   float eps;               // of those norms and the output's
@@ -57,19 +58,13 @@ struct WindowAttnArgs {
 DEV_INLINE int first_seen(const WindowAttnArgs& a, int pos) {
   return a.chunk > 0 ? pos / a.chunk * a.chunk : max(0, pos - a.window + 1);
 }
-// cap tanh(s / cap) by hardware exponential and reciprocal; c2 = 2 log2(e)
-// over cap
-DEV_INLINE float fast_cap(float s, float cap, float c2) {
-  return fmaf(-2.f * cap,
-              __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s * c2)),
-              cap);
-}
 constexpr float kTwoLog2e = 2.8853900817779268f;
 void launch_diff_append(const WindowAttnArgs& a, hipStream_t stream);
 void launch_diff_decode(const WindowAttnArgs& a, hipStream_t stream);
 void launch_diff_rows(const WindowAttnArgs& a, bool decode,
                       hipStream_t stream);
 bool diff_fast_ok(const WindowAttnArgs& a);
+int diff_head_blocks(int group);     // workgroups per kv head, sequence, split
 void launch_window_rope_append(const WindowAttnArgs& a, hipStream_t stream);
 void launch_window_decode(const WindowAttnArgs& a, hipStream_t stream);
 void launch_window_rows(const WindowAttnArgs& a, bool decode,

@@ -20,6 +20,7 @@ struct BlockArgs {
   const float* part_w;     // [rows, parts]
   const void* part_h;      // [rows, width]
   int parts, part_limit;
+  const float* y_bias;     // [width] added to y, or null
   const void* y2;          // its second half (merge), or null
   const float* gain1;      // [width] gains of y's and y2's own norms (merge)
   const float* gain2;

@@ -22,6 +22,8 @@
 
 #include "blk.h"
 
+#include <algorithm>
+
 namespace rlli {
 namespace {
 
@@ -64,6 +66,18 @@ void block_step_kernel(BlockArgs a) {
   const int64_t row = a.rows ? a.rows[n] : n;
   const int W = a.width, nv = W / V, gv = nv / a.groups;
   float* scale = sq + nv;
+  // scalar loads that later addresses wait for come first
+  const bool conv = CONV && n < a.n_decode;
+  const int back = a.n_taps - 1;          // earlier inputs that count
+  int pos = 0, at = 0;                    // position, its row of the ring
+  T* ring = nullptr;
+  if (conv) {
+    pos = a.positions[n];
+    if (back > 0) {
+      ring = reinterpret_cast<T*>(a.tail) + int64_t(a.slots[n]) * a.ring * W;
+      at = pos % a.ring;
+    }
+  }
   float* xr = a.x + row * W;
   const T* yr = EMBED ? nullptr
                       : reinterpret_cast<const T*>(a.y) +
@@ -116,6 +130,13 @@ void block_step_kernel(BlockArgs a) {
         }
       } else {
         load_v<T, V>(yr + c, t);
+        if constexpr (!MERGE)
+          if (a.y_bias) {
+            float b[V];
+            load_v<float, V>(a.y_bias + c, b);
+#pragma unroll
+            for (int j = 0; j < V; ++j) t[j] += b[j];
+          }
       }
       if constexpr (MERGE && IT == 0) {
         float q[V];
@@ -142,8 +163,6 @@ void block_step_kernel(BlockArgs a) {
       for (int v = threadIdx.x; v < nv; v += NT) body(v, 0);
     }
   };
-  const bool conv = CONV && n < a.n_decode;
-  const int back = a.n_taps - 1;          // earlier inputs that count
   auto load_tap = [&](int b, int k, int c, float (&w)[V]) {
     load_v<float, V>(a.taps + (int64_t(b) * a.n_taps + back - k) * W + c, w);
   };
@@ -166,15 +185,6 @@ void block_step_kernel(BlockArgs a) {
               load_tap(b + 1, 1, v * V, btap[i][b][1]);
             }
       });
-  }
-  int pos = 0, at = 0;                    // position, its row of the ring
-  T* ring = nullptr;
-  if (conv) {
-    pos = a.positions[n];
-    if (back > 0) {
-      ring = reinterpret_cast<T*>(a.tail) + int64_t(a.slots[n]) * a.ring * W;
-      at = pos % a.ring;
-    }
   }
   auto load_ring = [&](int k, int c, float (&e)[V]) {
     const int r = at - k < 0 ? at - k + a.ring : at - k;
@@ -218,6 +228,7 @@ void block_step_kernel(BlockArgs a) {
     if constexpr (IT > 0)
       every([&](int v, int i) { merge(v * V, t[i], t2[i], t[i]); });
   }
+  float mine = 0.f;                       // one group: this thread's squares
   every([&](int v, int i) {
     if constexpr (IT == 0) summands(v * V, u[0], t[0]);
     float s = 0.f;
@@ -226,19 +237,31 @@ void block_step_kernel(BlockArgs a) {
       u[i][j] += t[i][j];
       s += u[i][j] * u[i][j];
     }
-    sq[v] = s;
+    if (a.groups == 1) mine += s;
+    else sq[v] = s;
     if constexpr (IT > 0)
       if (a.keep) store_v<float, V>(xr + v * V, u[i]);
   });
-  __syncthreads();
-  for (int g = threadIdx.x >> 6; g < a.groups; g += WAVES) {
-    float s = 0.f;
-    for (int v = threadIdx.x & 63; v < gv; v += 64) s += sq[g * gv + v];
-    s = wave_sum(s);
-    if ((threadIdx.x & 63) == 0)
-      scale[g] = 1.f / sqrtf(s / (gv * V) + a.eps);
+  float whole = 0.f;                      // one group: its scale
+  if (a.groups == 1) {
+    // sums of 16 lanes on the VALU, then four per wave through LDS
+    mine = group_sum_dpp<16>(mine);
+    if ((threadIdx.x & 15) == 0) sq[threadIdx.x >> 4] = mine;
+    __syncthreads();
+#pragma unroll
+    for (int w = 0; w < WAVES * 4; ++w) whole += sq[w];
+    whole = 1.f / sqrtf(whole / W + a.eps);
+  } else {
+    __syncthreads();
+    for (int g = threadIdx.x >> 6; g < a.groups; g += WAVES) {
+      float s = 0.f;
+      for (int v = threadIdx.x & 63; v < gv; v += 64) s += sq[g * gv + v];
+      s = wave_sum(s);
+      if ((threadIdx.x & 63) == 0)
+        scale[g] = 1.f / sqrtf(s / (gv * V) + a.eps);
+    }
+    __syncthreads();
   }
-  __syncthreads();
   T* hr = reinterpret_cast<T*>(a.h) + int64_t(n) * W;
   every([&](int v, int i) {
     const int c = v * V;
@@ -250,7 +273,7 @@ void block_step_kernel(BlockArgs a) {
       load_v<float, V>(a.gain + c, gain[0]);
     }
     float hv[V];
-    const float inv = scale[v / gv];
+    const float inv = a.groups == 1 ? whole : scale[v / gv];
 #pragma unroll
     for (int j = 0; j < V; ++j)
       hv[j] = round_act(T{}, u[i][j] * inv * gain[i][j]);
@@ -453,7 +476,8 @@ template <typename T, bool EMBED, bool MERGE, bool CONV, bool PARTS = false>
 void step(const BlockArgs& a, hipStream_t st) {
   auto run = [&](auto* k, int threads, int v) {
     hipLaunchKernelGGL(k, dim3(a.n), dim3(threads),
-                       (a.width / v + a.groups) * sizeof(float), st, a);
+                       std::max(a.width / v + a.groups, threads / 16) *
+                           sizeof(float), st, a);
   };
   if (a.width / a.groups % 4 || a.width > 8192)
     run(block_step_kernel<T, 4, 0, 1, EMBED, MERGE, CONV, PARTS>, 256, 1);

@@ -53,12 +53,11 @@ void window_append(const Tensor& qkv, const Tensor& k_cache,
 
 // splits of a decode step that fill the chip, and room for their results;
 // ``visible``: the most tokens that a query sees
+// ``head_blocks``: workgroups per sequence, kv head and split
 void decode_splits(rlli::WindowAttnArgs& a, const Tensor& qkv,
-                   int64_t visible, Tensor& pa, Tensor& pm) {
-  const int group = a.n_q / a.n_kv;
-  const int hb = rlli::window_decode_heads_per_wg(group);
-  const int64_t wgs = int64_t(std::max(a.rows, 1)) * a.n_kv *
-                      ((group + hb - 1) / hb);
+                   int head_blocks, int64_t visible, Tensor& pa, Tensor& pm) {
+  const int64_t wgs =
+      int64_t(std::max(a.rows, 1)) * a.n_kv * head_blocks;
   // at most one split per 4 visible 16-token steps (one per wave)
   const int64_t reach = std::min<int64_t>(
       int64_t(a.max_blocks) * a.block_size, visible);
@@ -127,8 +126,11 @@ Tensor window_decode(const Tensor& qkv, const Tensor& k_cache,
     check_launch("window_decode");
     return out;
   }
+  const int group = a.n_q / a.n_kv;
+  const int hb = rlli::window_decode_heads_per_wg(group);
   Tensor pa, pm;
-  decode_splits(a, qkv, int64_t(a.window) + a.keep_first + 32, pa, pm);
+  decode_splits(a, qkv, (group + hb - 1) / hb,
+                int64_t(a.window) + a.keep_first + 32, pa, pm);
   rlli::launch_window_decode(a, st);
   check_launch("window_decode");
   return out;
@@ -149,8 +151,11 @@ void diff_score(Args& a, int64_t chunk, double cap, double lambda,
 
 void diff_append_args(rlli::WindowAttnArgs& a, const Tensor& positions,
                       const OptTensor& cos_sin, const Tensor& slots,
-                      const Tensor& q_norm, const Tensor& k_norm, double eps) {
+                      const OptTensor& bias, const Tensor& q_norm, const Tensor& k_norm, double eps) {
   append_args(a, positions, cos_sin, slots, std::nullopt);
+  if (bias)
+    a.bias = f32_vec(*bias, int64_t(a.n_q + a.n_kv) * 2 * a.dim +
+                                int64_t(a.n_kv) * a.vdim, "bias");
   a.q_norm = f32_vec(q_norm, a.dim, "q_norm");
   a.k_norm = f32_vec(k_norm, a.dim, "k_norm");
   a.eps = float(eps);
@@ -166,9 +171,10 @@ void diff_gate(rlli::WindowAttnArgs& a, const Tensor& qkv,
 void diff_append(const Tensor& qkv, const Tensor& k_cache,
                  const Tensor& v_cache, const Tensor& positions,
                  const OptTensor& cos_sin, const Tensor& slots, int64_t n_q,
-                 const Tensor& q_norm, const Tensor& k_norm, double eps) {
+                 const OptTensor& bias, const Tensor& q_norm,
+                 const Tensor& k_norm, double eps) {
   auto a = window_args(qkv, k_cache, v_cache, n_q, true, 1.0, 1, 0, {}, 2);
-  diff_append_args(a, positions, cos_sin, slots, q_norm, k_norm, eps);
+  diff_append_args(a, positions, cos_sin, slots, bias, q_norm, k_norm, eps);
   c10::hip::HIPGuardMasqueradingAsCUDA guard(qkv.device());
   rlli::launch_diff_append(a, stream_of(qkv));
   check_launch("diff_append");
@@ -198,11 +204,11 @@ Tensor diff_decode(const Tensor& qkv, const Tensor& k_cache,
                    const Tensor& v_cache, const Tensor& positions,
                    const OptTensor& cos_sin, const Tensor& slots,
                    const Tensor& block_tables, const OptTensor& gate,
-                   double scale, int64_t n_q, const Tensor& q_norm,
-                   const Tensor& k_norm, int64_t chunk, double cap,
+                   double scale, int64_t n_q, const OptTensor& bias,
+                   const Tensor& q_norm, const Tensor& k_norm, int64_t chunk, double cap,
                    double lambda, double out_scale, double eps) {
   auto a = window_args(qkv, k_cache, v_cache, n_q, true, scale, 1, 0, {}, 2);
-  diff_append_args(a, positions, cos_sin, slots, q_norm, k_norm, eps);
+  diff_append_args(a, positions, cos_sin, slots, bias, q_norm, k_norm, eps);
   diff_score(a, chunk, cap, lambda, out_scale, eps);
   diff_gate(a, qkv, gate);
   window_tables(a, block_tables);
@@ -211,14 +217,15 @@ Tensor diff_decode(const Tensor& qkv, const Tensor& k_cache,
   a.out = out.data_ptr();
   c10::hip::HIPGuardMasqueradingAsCUDA guard(qkv.device());
   auto st = stream_of(qkv);
-  if (!rlli::diff_fast_ok(a) || a.stride % 8) {
+  if (!rlli::diff_fast_ok(a)) {
     rlli::launch_diff_append(a, st);
     rlli::launch_diff_rows(a, true, st);
     check_launch("diff_decode");
     return out;
   }
   Tensor pa, pm;
-  decode_splits(a, qkv, chunk, pa, pm);
+  decode_splits(a, qkv, rlli::diff_head_blocks(a.n_q / a.n_kv), chunk, pa,
+                pm);
   rlli::launch_diff_decode(a, st);
   check_launch("diff_decode");
   return out;
@@ -376,7 +383,8 @@ TORCH_LIBRARY(rlli_attn, m) {
   m.def("expanded_ok(int dim, int vdim, int maps=1) -> bool", &expanded_ok);
   m.def("diff_append(Tensor(a!) qkv, Tensor(b!) k_cache, "
         "Tensor(c!) v_cache, Tensor positions, Tensor? cos_sin, "
-        "Tensor slots, int n_q, Tensor q_norm, Tensor k_norm, float eps) "
+        "Tensor slots, int n_q, Tensor? bias, Tensor q_norm, "
+        "Tensor k_norm, float eps) "
         "-> ()");
   m.def("diff_rows(Tensor qkv, Tensor k_cache, Tensor v_cache, "
         "Tensor block_tables, Tensor tiles, int tile_rows, Tensor? gate, "
@@ -385,7 +393,7 @@ TORCH_LIBRARY(rlli_attn, m) {
   m.def("diff_decode(Tensor(a!) qkv, Tensor(b!) k_cache, Tensor(c!) v_cache, "
         "Tensor positions, Tensor? cos_sin, Tensor slots, "
         "Tensor block_tables, Tensor? gate, float scale, int n_q, "
-        "Tensor q_norm, Tensor k_norm, int chunk, float cap, float lam, "
+        "Tensor? bias, Tensor q_norm, Tensor k_norm, int chunk, float cap, float lam, "
         "float out_scale, float eps) -> Tensor");
   m.def("diff_expanded(Tensor q, Tensor k, Tensor vt, Tensor? gate, "
         "Tensor tiles, Tensor kv_off, int heads, int kv_heads, float scale, "

@@ -109,13 +109,18 @@ std::tuple<Tensor, Tensor> block_step(
     const OptTensor& slots, int64_t n_decode, const OptTensor& rows,
     bool keep, const OptTensor& y2, const OptTensor& gain1,
     const OptTensor& gain2, const OptTensor& part_ids,
-    const OptTensor& part_w, const OptTensor& part_h, int64_t part_limit) {
+    const OptTensor& part_w, const OptTensor& part_h, int64_t part_limit,
+    const OptTensor& y_bias) {
   rlli::BlockArgs a{};
   a.f32 = act_f32(y, "y");
   TORCH_CHECK(x.dim() == 2 && y.dim() == (part_ids ? 3 : 2) &&
               y.size(0) == x.size(0) && y.size(-1) == x.size(1),
               "y/residual mismatch");
   a.y = y.data_ptr();
+  if (y_bias) {
+    TORCH_CHECK(!part_ids && !y2, "a bias goes with a single output");
+    a.y_bias = f32_vec(*y_bias, x.size(1), "y_bias");
+  }
   if (part_ids) {
     TORCH_CHECK(part_w.has_value() && part_h.has_value() && !y2,
                 "parts come with weights and the block's input");
@@ -235,8 +240,8 @@ TORCH_LIBRARY(rlli_blk, m) {
         "float eps, Tensor positions, Tensor? taps, Tensor(b!)? tail, "
         "Tensor? slots, int n_decode, Tensor? rows, bool keep, Tensor? y2, "
         "Tensor? gain1, Tensor? gain2, Tensor? part_ids=None, "
-        "Tensor? part_w=None, Tensor? part_h=None, int part_limit=0) "
-        "-> (Tensor, Tensor)");
+        "Tensor? part_w=None, Tensor? part_h=None, int part_limit=0, "
+        "Tensor? y_bias=None) -> (Tensor, Tensor)");
   m.def("conv_prompt(Tensor h, Tensor taps, Tensor(a!)? tail, Tensor spans, "
         "Tensor portions, Tensor(b!) out, bool silu) -> ()");
   m.def("gate_act(Tensor gate_up, Tensor(a!) out, str act, float limit) "

@@ -27,6 +27,37 @@ namespace rlli {
 namespace {
 
 // ------------------------------------------------------------- router
+// Wave-wide reductions on the VALU, the result in every lane: rows of 16,
+// then across rows, then out of the last lane.
+template <int CTRL>
+DEV_INLINE float dpp_or_own(float v) {
+  const int b = __builtin_bit_cast(int, v);
+  return __builtin_bit_cast(
+      float, __builtin_amdgcn_update_dpp(b, b, CTRL, 0xf, 0xf, false));
+}
+DEV_INLINE float last_lane(float v) {
+  return __builtin_bit_cast(
+      float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), 63));
+}
+DEV_INLINE float wave_sum_dpp(float v) {
+  v = group_sum_dpp<16>(v);
+  // rows 0 + 1 | 2 + 3, then all four, in the last lane
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
+           0, __builtin_bit_cast(int, v), 0x142, 0xa, 0xf, false));
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
+           0, __builtin_bit_cast(int, v), 0x143, 0xc, 0xf, false));
+  return last_lane(v);
+}
+DEV_INLINE float wave_max_dpp(float v) {
+  v = fmaxf(v, dpp_or_own<0x111>(v));     // row_shr 1, 2, 4, 8
+  v = fmaxf(v, dpp_or_own<0x112>(v));
+  v = fmaxf(v, dpp_or_own<0x114>(v));
+  v = fmaxf(v, dpp_or_own<0x118>(v));
+  v = fmaxf(v, dpp_or_own<0x142>(v));     // row_bcast 15, 31
+  v = fmaxf(v, dpp_or_own<0x143>(v));
+  return last_lane(v);
+}
+
 // 16 rows per workgroup, K split over eight waves
 template <typename T, int ET>
 __global__ __launch_bounds__(512)
@@ -108,13 +139,13 @@ void moe_route_kernel(MoeArgs a) {
       float mx = kNone, sum = 0.f;
 #pragma unroll
       for (int i = 0; i < EL; ++i) mx = fmaxf(mx, s[i]);
-      mx = wave_max(mx);
+      mx = wave_max_dpp(mx);
 #pragma unroll
       for (int i = 0; i < EL; ++i) {
         s[i] = expf(s[i] - mx);           // 0 past the last route
         sum += s[i];
       }
-      sum = wave_sum(sum);
+      sum = wave_sum_dpp(sum);
 #pragma unroll
       for (int i = 0; i < EL; ++i) s[i] /= sum;
     } else {
@@ -159,22 +190,16 @@ void moe_route_kernel(MoeArgs a) {
     }
     float won[EL], total = 0.f;           // lane c & 63 keeps weight c
     for (int c = 0; c < a.top; ++c) {
-      float bv = kNone;
+      // the best score left, and the first route that has it
+      float bv = choice[0];
+#pragma unroll
+      for (int i = 1; i < EL; ++i) bv = fmaxf(bv, choice[i]);
+      bv = wave_max_dpp(bv);
       int bi = 0x7fffffff;
 #pragma unroll
-      for (int i = 0; i < EL; ++i)
-        if (choice[i] > bv) {
-          bv = choice[i];
-          bi = i * 64 + lane;
-        }
-#pragma unroll
-      for (int off = 32; off > 0; off >>= 1) {
-        const float ov = __shfl_xor(bv, off, kWave);
-        const int oi = __shfl_xor(bi, off, kWave);
-        if (ov > bv || (ov == bv && oi < bi)) {
-          bv = ov;
-          bi = oi;
-        }
+      for (int i = EL - 1; i >= 0; --i) {
+        const uint64_t has = __ballot(choice[i] == bv);
+        if (has) bi = i * 64 + __builtin_ctzll(has);
       }
 #pragma unroll
       for (int i = 0; i < EL; ++i)
@@ -184,7 +209,9 @@ void moe_route_kernel(MoeArgs a) {
 #pragma unroll
       for (int i = 1; i < EL; ++i)
         if (bi >> 6 == i) mine = s[i];
-      mine = __shfl(mine, bi & 63, kWave);
+      mine = __builtin_bit_cast(
+          float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, mine),
+                                           bi & 63));
       total += mine;
 #pragma unroll
       for (int i = 0; i < EL; ++i)
@@ -590,6 +617,8 @@ void route(const MoeArgs& a, hipStream_t st) {
     hipLaunchKernelGGL((moe_route_kernel<T, 1>), grid, blk, 0, st, a);
   else if (a.routes <= 32)
     hipLaunchKernelGGL((moe_route_kernel<T, 2>), grid, blk, 0, st, a);
+  else if (a.routes <= 48)
+    hipLaunchKernelGGL((moe_route_kernel<T, 3>), grid, blk, 0, st, a);
   else if (a.routes <= 64)
     hipLaunchKernelGGL((moe_route_kernel<T, 4>), grid, blk, 0, st, a);
   else if (a.routes <= 128)

@@ -84,19 +84,23 @@ def _normed(x, gain, eps):
     return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * gain
 
 
-def diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q,
+def diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q, bias,
                 q_norm, k_norm, eps):
     T = qkv.shape[0]
     _, G, bs, D2 = k_cache.shape
     V, D = v_cache.shape[3], D2 // 2
-    q, k, v = (qkv[:, :n_q * D2].view(T, n_q, 2, D),
-               qkv[:, n_q * D2:(n_q + G) * D2].view(T, G, 2, D),
-               qkv[:, (n_q + G) * D2:(n_q + G) * D2 + G * V])
+    n_k, n_v = (n_q + G) * D2, (n_q + G) * D2 + G * V
+    x = qkv[:, :n_v].float()
+    if bias is not None:
+        x = x + bias
+    q, k, v = (x[:, :n_q * D2].view(T, n_q, 2, D),
+               x[:, n_q * D2:n_k].view(T, G, 2, D), x[:, n_k:])
     b, o = slots.long() // bs, slots.long() % bs
     k = _turn_halves(_normed(k, k_norm, eps), positions, cos_sin)
     k_cache[b, :, o] = k.reshape(T, G, D2).to(k_cache.dtype)
     v_cache[b, :, o] = v.reshape(T, G, V).to(v_cache.dtype)
-    q.copy_(_turn_halves(_normed(q, q_norm, eps), positions, cos_sin))
+    qkv[:, :n_q * D2] = _turn_halves(_normed(q, q_norm, eps), positions,
+                                     cos_sin).flatten(1).to(qkv.dtype)
 
 
 def _diff_attend(q, gate, qpos, k_cache, v_cache, table, scale, chunk, cap,
@@ -132,9 +136,9 @@ def _diff_queries(qkv, k_cache, n_q):
 
 
 def diff_prefill(qkv, gate, k_cache, v_cache, positions, cos_sin, slots,
-                 block_tables, prompt, n_q, q_norm, k_norm, scale, chunk, cap,
-                 lam, out_scale, eps):
-    diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q,
+                 block_tables, prompt, n_q, bias, q_norm, k_norm, scale,
+                 chunk, cap, lam, out_scale, eps):
+    diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q, bias,
                 q_norm, k_norm, eps)
     q = _diff_queries(qkv, k_cache, n_q)
     out = torch.empty(qkv.shape[0], n_q * v_cache.shape[3], dtype=qkv.dtype)
@@ -148,9 +152,9 @@ def diff_prefill(qkv, gate, k_cache, v_cache, positions, cos_sin, slots,
 
 
 def diff_decode(qkv, k_cache, v_cache, positions, cos_sin, slots,
-                block_tables, gate, scale, n_q, q_norm, k_norm, chunk, cap,
-                lam, out_scale, eps):
-    diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q,
+                block_tables, gate, scale, n_q, bias, q_norm, k_norm, chunk,
+                cap, lam, out_scale, eps):
+    diff_append(qkv, k_cache, v_cache, positions, cos_sin, slots, n_q, bias,
                 q_norm, k_norm, eps)
     q = _diff_queries(qkv, k_cache, n_q)
     return torch.cat([

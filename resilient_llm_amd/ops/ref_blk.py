@@ -45,13 +45,15 @@ def block_embed(ids, table, pos_table, positions, x, gain, groups, eps, taps,
 
 def block_step(x, y, gain, groups, eps, positions, taps, tail, slots,
                n_decode, rows, keep, y2, gain1, gain2, part_ids=None,
-               part_w=None, part_h=None, part_limit=0):
+               part_w=None, part_h=None, part_limit=0, y_bias=None):
     if part_ids is not None:
         own = (part_ids < part_limit)[..., None]
         new = x + torch.where(own, y.float(), part_w[..., None]
                               * part_h.float()[:, None]).sum(1)
     elif y2 is None:
         new = x + y.float()
+        if y_bias is not None:
+            new = new + y_bias
     else:
         new = x + 0.5 * (_group_norm(y.float(), gain1, 1, eps)
                          + _group_norm(y2.float(), gain2, 1, eps))

@@ -188,3 +188,73 @@ def run(config, weights, tokens, dtype=torch.float64):
         after.append(x)
     h = rms(x, eps) * (1 + W["final.norm"])
     return soft_cap(h @ W["head"].T, config["logit_softcap"]), after
+
+
+# ------------------------------------------------------------ test models
+def make_config(layers, width=64, vocab=97, eps=1e-5, taps=3, softcap=9.0,
+                loop=(0, 0, 1)):
+    return {"architecture": "Fimunex", "canon": {"taps": taps},
+            "layers": layers, "logit_softcap": softcap,
+            "loop": dict(zip(("start", "stop", "times"), loop)),
+            "norm": {"eps": eps}, "vocab": vocab, "width": width}
+
+
+def tensor_shapes(config):
+    """Checkpoint names and shapes that a configuration implies."""
+    d, taps = config["width"], config["canon"]["taps"]
+    out = {"embed": (config["vocab"], d), "head": (config["vocab"], d),
+           "final.norm": (d,)}
+    for n, layer in enumerate(config["layers"]):
+        m, f, p = layer["mixer"], layer["mlp"], f"l{n}."
+        H, G, dim, vdim = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        out.update({p + "norm1": (d,), p + "canon1": (d, taps)})
+        p += "mix."
+        out.update({p + "q": (2 * H * dim, d), p + "q.b": (2 * H * dim,),
+                    p + "k": (2 * G * dim, d), p + "k.b": (2 * G * dim,),
+                    p + "v": (G * vdim, d), p + "v.b": (G * vdim,),
+                    p + "o": (d, H * vdim), p + "o.b": (d,),
+                    p + "g": (H, d)})
+        out.update({p + x: (dim,) for x in (
+            "q.norm", "k.norm", "lq1", "lk1", "lq2", "lk2")})
+        if f is None:
+            continue
+        p, r, ff = f"l{n}.", f["router"], f["expert"]["ff"]
+        out.update({p + "norm2": (d,), p + "canon2": (d, taps)})
+        p += "mlp."
+        routes = r["experts"] + r["identity"]
+        out.update({p + "router": (routes, d), p + "correction": (routes,)})
+        for e in range(r["experts"]):
+            out[f"{p}e{e}.up"], out[f"{p}e{e}.down"] = (ff, d), (d, ff)
+    return out
+
+
+def random_weights(config, seed=0, decisive=False):
+    """bfloat16 weights that keep every mechanism audible: unit-gain
+    linears, biases and taps that matter, sharp queries and keys, routers
+    that spread, corrections of either sign.  ``decisive``: corrections far
+    apart, so that no rounding changes a choice."""
+    g = torch.Generator().manual_seed(seed)
+    out = {}
+    for name, shape in tensor_shapes(config).items():
+        t = torch.randn(shape, generator=g)
+        leaf = name.split(".", 1)[-1]
+        if leaf in ("mix.q.norm", "mix.k.norm"):
+            t = 1.4 + 0.4 * t
+        elif leaf.endswith(("norm", "norm1", "norm2")):
+            t = 0.25 * t
+        elif leaf.startswith("canon"):
+            t = 0.4 * t
+        elif leaf.endswith(".b"):
+            t = 0.5 * t
+        elif leaf.startswith("mix.l"):
+            t = 0.3 * t
+        elif leaf == "mlp.correction":
+            t = -0.3 + 0.4 * t
+            if decisive:
+                t = -10 + 2.0 * torch.randperm(shape[0], generator=g).float()
+        elif leaf == "mlp.router":
+            t = t * 1.5 / math.sqrt(shape[-1])
+        elif name != "embed":
+            t = t * 1.2 / math.sqrt(shape[-1])
+        out[name] = t.to(torch.bfloat16)
+    return out
