@@ -82,7 +82,22 @@ void block_step_kernel(BlockArgs a) {
   const T* yr = EMBED ? nullptr
                       : reinterpret_cast<const T*>(a.y) +
                             row * (PARTS ? a.parts : 1) * W;
-  const int32_t* part_ids = PARTS ? a.part_ids + row * a.parts : nullptr;
+  // the first parts: where they come from and what they count
+  constexpr int PE = PARTS ? 4 : 1;
+  const T* part[PE];
+  float part_w[PE];
+  auto find_part = [&](int k, const T*& p, float& w) {
+    const bool own = a.part_ids[row * a.parts + k] < a.part_limit;
+    p = own ? yr + int64_t(k) * W
+            : reinterpret_cast<const T*>(a.part_h) + row * W;
+    w = own ? 1.f : a.part_w[row * a.parts + k];
+  };
+  if constexpr (PARTS)
+#pragma unroll
+    for (int k = 0; k < PE; ++k) {
+      find_part(min(k, a.parts - 1), part[k], part_w[k]);
+      if (k >= a.parts) part_w[k] = 0.f;
+    }
   const T* y2r = MERGE ? reinterpret_cast<const T*>(a.y2) + row * W : nullptr;
   float s1 = 0.f, s2 = 0.f;               // half over the root mean squares
   auto merge = [&](int c, const float (&p)[V], const float (&q)[V],
@@ -100,6 +115,14 @@ void block_step_kernel(BlockArgs a) {
       pr = reinterpret_cast<const T*>(a.pos_table) +
            int64_t(min(a.positions[n], a.n_positions - 1)) * W;
   }
+  const bool biased = !EMBED && !MERGE && !PARTS && a.y_bias;
+  auto add_bias = [&](int c, float (&t)[V]) {
+    if (!biased) return;
+    float b[V];
+    load_v<float, V>(a.y_bias + c, b);
+#pragma unroll
+    for (int j = 0; j < V; ++j) t[j] += b[j];
+  };
   // the two summands of a row's new value
   auto summands = [&](int c, float (&u)[V], float (&t)[V]) {
     if constexpr (EMBED) {
@@ -115,28 +138,26 @@ void block_step_kernel(BlockArgs a) {
     } else {
       load_v<float, V>(xr + c, u);
       if constexpr (PARTS) {
+        float e[PE][V];
 #pragma unroll
-        for (int j = 0; j < V; ++j) t[j] = 0.f;
-#pragma unroll 4
-        for (int k = 0; k < a.parts; ++k) {
-          const bool own = part_ids[k] < a.part_limit;
-          const T* p = own ? yr + int64_t(k) * W
-                           : reinterpret_cast<const T*>(a.part_h) + row * W;
-          const float w = own ? 1.f : a.part_w[row * a.parts + k];
-          float e[V];
-          load_v<T, V>(p + c, e);
+        for (int k = 0; k < PE; ++k) load_v<T, V>(part[k] + c, e[k]);
 #pragma unroll
-          for (int j = 0; j < V; ++j) t[j] += w * e[j];
+        for (int j = 0; j < V; ++j) {
+          t[j] = 0.f;
+#pragma unroll
+          for (int k = 0; k < PE; ++k) t[j] += part_w[k] * e[k][j];
+        }
+        for (int k = PE; k < a.parts; ++k) {
+          const T* p;
+          float w;
+          find_part(k, p, w);
+          load_v<T, V>(p + c, e[0]);
+#pragma unroll
+          for (int j = 0; j < V; ++j) t[j] += w * e[0][j];
         }
       } else {
         load_v<T, V>(yr + c, t);
-        if constexpr (!MERGE)
-          if (a.y_bias) {
-            float b[V];
-            load_v<float, V>(a.y_bias + c, b);
-#pragma unroll
-            for (int j = 0; j < V; ++j) t[j] += b[j];
-          }
+        if constexpr (!MERGE && IT == 0) add_bias(c, t);
       }
       if constexpr (MERGE && IT == 0) {
         float q[V];
@@ -150,7 +171,7 @@ void block_step_kernel(BlockArgs a) {
   // the rest late
   constexpr int ITS = IT > 0 ? IT : 1;
   constexpr int EARLY = CONV && (IT == 1 || IT == 2) ? 4 : 0;   // taps
-  float u[ITS][V], t[ITS][V], gain[ITS][V];
+  float u[ITS][V], t[ITS][V], gain[ITS][V], bias[ITS][V];
   float tap[ITS][EARLY + 1][V], past[ITS][EARLY + 1][V];
   constexpr int MORE = EARLY > 0 ? 4 : 0; // further branches of two taps
   float btap[ITS][MORE + 1][2][V];
@@ -172,6 +193,8 @@ void block_step_kernel(BlockArgs a) {
     if constexpr (MERGE)
       every([&](int v, int i) { load_v<T, V>(y2r + v * V, t2[i]); });
     every([&](int v, int i) { load_v<float, V>(a.gain + v * V, gain[i]); });
+    if (biased)
+      every([&](int v, int i) { load_v<float, V>(a.y_bias + v * V, bias[i]); });
     if (conv)
       every([&](int v, int i) {
 #pragma unroll
@@ -235,6 +258,8 @@ void block_step_kernel(BlockArgs a) {
 #pragma unroll
     for (int j = 0; j < V; ++j) {
       u[i][j] += t[i][j];
+      if constexpr (IT > 0)
+        if (biased) u[i][j] += bias[i][j];
       s += u[i][j] * u[i][j];
     }
     if (a.groups == 1) mine += s;
@@ -485,8 +510,12 @@ void step(const BlockArgs& a, hipStream_t st) {
     run(block_step_kernel<T, 1, 1, 4, EMBED, MERGE, CONV, PARTS>, 64, 4);
   else if (a.width <= 1024)
     run(block_step_kernel<T, 4, 1, 4, EMBED, MERGE, CONV, PARTS>, 256, 4);
+  else if (a.width <= 2048 && CONV)       // few rows: latency counts
+    run(block_step_kernel<T, 8, 1, 4, EMBED, MERGE, CONV, PARTS>, 512, 4);
   else if (a.width <= 2048)
     run(block_step_kernel<T, 4, 2, 4, EMBED, MERGE, CONV, PARTS>, 256, 4);
+  else if (a.width <= 4096 && CONV)
+    run(block_step_kernel<T, 16, 1, 4, EMBED, MERGE, CONV, PARTS>, 1024, 4);
   else if (a.width <= 4096)
     run(block_step_kernel<T, 8, 2, 4, EMBED, MERGE, CONV, PARTS>, 512, 4);
   else

@@ -28,16 +28,16 @@ DEV_INLINE uint32_t pack2(float a, float b) {
   return __builtin_bit_cast(uint32_t, v);
 }
 
+// eight neighbours at ``p + off``, zeros unless ``ok``; p itself can always be
+// read, so that no load waits behind a branch
 template <typename T>
-DEV_INLINE void load8(const T* p, bool ok, float (&x)[8]) {
-#pragma unroll
-  for (int j = 0; j < 8; ++j) x[j] = 0.f;
-  if (!ok) return;
+DEV_INLINE void load8(const T* p, int off, bool ok, float (&x)[8]) {
+  p += ok ? off : 0;
   const f32x4_t lo = act_load4(p), hi = act_load4(p + 4);
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
-    x[j] = lo[j];
-    x[4 + j] = hi[j];
+    x[j] = ok ? lo[j] : 0.f;
+    x[4 + j] = ok ? hi[j] : 0.f;
   }
 }
 
@@ -76,6 +76,7 @@ void diff_append_kernel(WindowAttnArgs a) {
   if (unit >= int64_t(a.rows) * per_row) return;    // whole groups leave
   const int row = int(unit / per_row), u = int(unit % per_row);
   const int lane = threadIdx.x & 63, gl = lane & (W - 1), d0 = gl * 8;
+  const float* bias = a.bias ? a.bias : a.q_norm;
   T* x = reinterpret_cast<T*>(a.qkv_rw) + int64_t(row) * a.stride;
   const int slot = a.slots[row];
   const int64_t blk = slot / a.block_size, off = slot % a.block_size;
@@ -84,11 +85,10 @@ void diff_append_kernel(WindowAttnArgs a) {
     const T* v = x + (nq + nk) * a.dim + h * a.vdim;
     CE* o = reinterpret_cast<CE*>(a.v_cache) +
             ((blk * a.n_kv + h) * a.block_size + off) * a.vdim;
-    const float* b = a.bias + (nq + nk) * a.dim + h * a.vdim;
     for (int d = d0; d < a.vdim; d += W * 8) {
       float e[8], eb[8];
-      load8(v + d, true, e);
-      load8(b + d, a.bias != nullptr, eb);
+      load8(v, d, true, e);
+      load8(bias, (nq + nk) * a.dim + h * a.vdim + d, a.bias, eb);
 #pragma unroll
       for (int j = 0; j < 8; ++j) e[j] += eb[j];
       store8(o + d, e);
@@ -99,15 +99,16 @@ void diff_append_kernel(WindowAttnArgs a) {
   const int half = a.rot / 2;
   // this lane's dimensions and their pairs' other halves
   const int p0 = d0 < half ? d0 + half : d0 < a.rot ? d0 - half : -1;
-  const float* cs = a.cos_sin + int64_t(a.positions[row]) * a.rot +
-                    (d0 < half ? d0 : d0 - half);
+  const int i0 = d0 < half ? d0 : d0 - half;
+  const float* cs = a.rot ? a.cos_sin + int64_t(a.positions[row]) * a.rot
+                          : a.q_norm;
   const float* w = u < nq ? a.q_norm : a.k_norm;
   float e[8], eb[8], ew[8], o[8], c[8], s[8];
-  load8(x + u * a.dim + d0, ok, e);
-  load8(a.bias + u * a.dim + d0, ok && a.bias, eb);
-  load8(w + d0, ok, ew);
-  load8(cs, p0 >= 0, c);
-  load8(cs + half, p0 >= 0, s);
+  load8(x + u * a.dim, d0, ok, e);
+  load8(bias, u * a.dim + d0, ok && a.bias, eb);
+  load8(w, d0, ok, ew);
+  load8(cs, i0, p0 >= 0, c);
+  load8(cs, half + i0, p0 >= 0, s);
   float ss = 0.f;
 #pragma unroll
   for (int j = 0; j < 8; ++j) {
@@ -232,17 +233,26 @@ void diff_decode_kernel(WindowAttnArgs a) {
   // this lane's pieces of a vector of ``dim``, normed, times w, rotated, as
   // 16-bit
   const int half = a.rot / 2;
-  const float* cs = a.cos_sin + int64_t(pos) * a.rot;
+  const float* cs = a.rot ? a.cos_sin + int64_t(pos) * a.rot : a.q_norm;
+  const float* bias = a.bias ? a.bias : a.q_norm;
   auto normed = [&](int at, const float* w, bool live, uint4 (&out)[DC]) {
     const uint16_t* x = row + at;
-    const float* b = a.bias + at;
-    const bool biased = live && a.bias;
-    float e[DC][8], eb[DC][8], ss = 0.f;
+    float e[DC][8], eb[DC][8], o[DC][8], ob[DC][8], ew[DC][8], ow[DC][8];
+    float ec[DC][8], es[DC][8], ss = 0.f;
 #pragma unroll
     for (int c = 0; c < DC; ++c) {
+      // a piece and its pairs' other halves
       const int d = c * 32 + g * 8;
-      load8(x + d, live && d < a.dim, e[c]);
-      load8(b + d, biased && d < a.dim, eb[c]);
+      const int p = d < half ? d + half : d - half, i = d < half ? d : p;
+      const bool turns = d < a.rot, in = live && d < a.dim;
+      load8(x, d, in, e[c]);
+      load8(bias, at + d, in && a.bias, eb[c]);
+      load8(x, p, live && turns, o[c]);
+      load8(bias, at + p, live && turns && a.bias, ob[c]);
+      load8(w, d, d < a.dim, ew[c]);
+      load8(w, p, turns, ow[c]);
+      load8(cs, i, turns, ec[c]);
+      load8(cs, half + i, turns, es[c]);
     }
 #pragma unroll
     for (int c = 0; c < DC; ++c)
@@ -257,21 +267,12 @@ void diff_decode_kernel(WindowAttnArgs a) {
 #pragma unroll
     for (int c = 0; c < DC; ++c) {
       const int d = c * 32 + g * 8;
-      const int p = d < half ? d + half : d - half;
-      const bool turns = d < a.rot, in = d < a.dim;
-      const int i = d < half ? d : p;
-      float o[8], ob[8], ew[8], ow[8], ec[8], es[8];
-      load8(w + d, in, ew);
-      load8(x + p, live && turns, o);
-      load8(b + p, biased && turns, ob);
-      load8(w + p, turns, ow);
-      load8(cs + i, turns, ec);
-      load8(cs + half + i, turns, es);
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
-        const float u = e[c][j] * inv * ew[j];
-        const float v = (o[j] + ob[j]) * inv * ow[j];
-        e[c][j] = turns ? u * ec[j] + (d < half ? -v : v) * es[j] : u;
+        const float u = e[c][j] * inv * ew[c][j];
+        const float v = (o[c][j] + ob[c][j]) * inv * ow[c][j];
+        e[c][j] = d < a.rot
+                      ? u * ec[c][j] + (d < half ? -v : v) * es[c][j] : u;
       }
       out[c] = uint4{pack2(e[c][0], e[c][1]), pack2(e[c][2], e[c][3]),
                      pack2(e[c][4], e[c][5]), pack2(e[c][6], e[c][7])};
@@ -414,8 +415,8 @@ void diff_decode_kernel(WindowAttnArgs a) {
     for (int h = 0; h < VH; ++h) {
       const int d = h * 128 + col * 8;
       float f[8], b[8];
-      load8(row + v_at + d, d < a.vdim, f);
-      load8(a.bias + v_at + d, d < a.vdim && a.bias, b);
+      load8(row, v_at + d, d < a.vdim, f);
+      load8(bias, v_at + d, d < a.vdim && a.bias, b);
 #pragma unroll
       for (int j = 0; j < 8; ++j) f[j] += b[j];
       const vec8 raw = KC::from_f32(f);
@@ -431,6 +432,8 @@ void diff_decode_kernel(WindowAttnArgs a) {
   const int step0 = lo / 16, n_steps = (len + 15) / 16 - step0;
   const int32_t* bt = a.block_tables + int64_t(seq) * a.max_blocks;
   auto fetch_phys = [&](int b) { return bt[(b * 16) / a.block_size]; };
+  // past a key's or value's end a lane loads its first piece: there the
+  // queries are zero, and nobody reads the output columns
   auto issue = [&](int b, int phys, vec8 (&kr)[2][DC], vec8 (&vr)[VH][4]) {
     const int64_t base = (int64_t(phys) * a.n_kv + kvh) * a.block_size +
                          (b * 16) % a.block_size;
@@ -441,19 +444,16 @@ void diff_decode_kernel(WindowAttnArgs a) {
 #pragma unroll
       for (int c = 0; c < DC; ++c) {
         const int d = c * 32 + g * 8;
-        kr[mp][c] = vec8{};
-        if (d < a.dim)
-          kr[mp][c] = *reinterpret_cast<const vec8*>(kp + mp * a.dim + d);
+        kr[mp][c] = *reinterpret_cast<const vec8*>(
+            kp + mp * a.dim + (d < a.dim ? d : 0));
       }
 #pragma unroll
     for (int h = 0; h < VH; ++h) {
       const int d = h * 128 + col * 8;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        vr[h][r] = vec8{};
-        if (d < a.vdim)
-          vr[h][r] = *reinterpret_cast<const vec8*>(vp + r * a.vdim + d);
-      }
+      for (int r = 0; r < 4; ++r)
+        vr[h][r] = *reinterpret_cast<const vec8*>(
+            vp + r * a.vdim + (d < a.vdim ? d : 0));
     }
   };
   auto take = [&](int b, const vec8 (&kr)[2][DC], const vec8 (&vr)[VH][4]) {
