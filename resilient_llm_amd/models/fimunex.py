@@ -12,9 +12,10 @@ order of layers come from config.json.
 
 Projections that share an input are one product; its biases are added where
 the product is read.  One pass sums a token's expert outputs, writes the
-residual, norms it and, for decoded tokens, convolves.  Residual, norms, angles, scores, router and
-convolution sums are 32-bit; product inputs, caches and convolution tails
-have the model dtype, which may also be float32.
+residual, norms it and, for decoded tokens, convolves.  Residual, norms,
+angles, scores, router and convolution sums are 32-bit; product inputs,
+caches and convolution tails have the model dtype, which may also be
+float32.
 """
 
 from __future__ import annotations

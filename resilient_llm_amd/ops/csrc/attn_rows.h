@@ -125,7 +125,8 @@ void window_rows_kernel(WindowAttnArgs a, bool decode) {
 #pragma unroll
     for (int i = 0; i < MAXV; ++i) {
       const int d = i * 64 + lane;
-      if (d < a.vdim) act_store(out + d, MAPS == 2 ? acc[i] * post : acc[i] / l);
+      if (d < a.vdim)
+        act_store(out + d, MAPS == 2 ? acc[i] * post : acc[i] / l);
     }
   }
 }

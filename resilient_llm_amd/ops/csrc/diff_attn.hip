@@ -578,7 +578,8 @@ void diff_decode_kernel(WindowAttnArgs a) {
                     (int64_t(seq) * a.n_q + head0 + h) * a.vdim;
 #pragma unroll
     for (int i = 0; i < NV; ++i)
-      if (i * 64 + lane < a.vdim) act_store(out + i * 64 + lane, x[0][i] * post);
+      if (i * 64 + lane < a.vdim)
+        act_store(out + i * 64 + lane, x[0][i] * post);
   }
 }
 

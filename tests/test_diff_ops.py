@@ -36,7 +36,7 @@ def i32(x, device):
 
 
 # ----------------------------------------------------------------- angles
-YARN = [(32, 10000.0, 4.0, 1024, 32.0, 1.0), (8, 500.0, 1.0, 64, 4.0, 0.5),
+YARN = [(32, 10000.0, 5.0, 2048, 24.0, 1.5), (8, 500.0, 1.0, 64, 4.0, 0.5),
         (64, 1e6, 16.0, 4096, 32.0, 1.0), (2, 100.0, 3.0, 50, 2.0, 1.0),
         # both ends beyond the pairs, and a ramp of no width
         (16, 1000.0, 8.0, 1 << 20, 1e5, 1e4), (16, 1000.0, 8.0, 2, 8.0, 4.0),
